@@ -21,13 +21,35 @@ NEG, SIN, COS, EXP, LOG, FLOOR, ROUND = range(7)
 ADD, SUB, MUL, DIV, POW, LT, GT, GTE, LTE, EQ = range(10)
 
 # enum cg_kernel_class
-K_GEMM_MFMA, K_GEMM_SKINNY, K_GEMM_SIMPLE, K_ELEMENTWISE, K_REDUCE, K_GATHER, K_ATTENTION, K_PACK = range(8)
+K_GEMM_MFMA, K_GEMM_SKINNY, K_GEMM_SIMPLE, K_ELEMENTWISE, K_REDUCE, K_GATHER, K_ATTENTION, K_PACK, K_RECURRENCE = range(9)
 
 _P = C.c_void_p
 _PP = C.POINTER(C.c_void_p)
 _SZ = C.c_size_t
 _SZP = C.POINTER(C.c_size_t)
 _I = C.c_int
+
+
+# cg_linear_args, cg_branch, cg_attention_args, cg_channel_delta_args
+class LinearArgs(C.Structure):
+    _fields_ = [(n, _P) for n in ("x", "x2", "gamma", "w", "bias")] + [("eps", C.c_float), ("scale", C.c_float)]
+
+
+class Branch(C.Structure):
+    _fields_ = [(n, _P) for n in ("y", "w", "gate", "gate_bias", "poly")]
+
+
+class AttentionArgs(C.Structure):
+    _fields_ = ([(n, _P) for n in ("q", "k", "v", "q_norm", "k_norm", "talk", "k_cache", "v_cache")]
+                + [(n, _SZ) for n in ("heads", "kv_heads", "dim", "vdim", "position", "window", "temp_every")]
+                + [("scale", C.c_float), ("norm_eps", C.c_float), ("temp_coef", C.c_float), ("distance_bias", C.c_int)])
+
+
+class ChannelDeltaArgs(C.Structure):
+    _fields_ = ([(n, _P) for n in ("q", "k", "v", "conv_q", "conv_k", "conv_v", "beta", "decay", "decay_w", "a_log", "dt_bias",
+                                   "gate", "gate_w", "norm", "state", "conv_state")]
+                + [(n, _SZ) for n in ("heads", "kv_heads", "dim", "vdim")] + [("eps", C.c_float)])
+
 
 # name -> (restype, argtypes); every symbol the header declares.
 SIGNATURES = {
@@ -74,6 +96,10 @@ SIGNATURES = {
     "cg_slice": (_I, [_P, _P, _SZ, _SZ, _SZ, _PP]),
     "cg_concat": (_I, [_P, _P, _P, _SZ, _PP]),
     "cg_index": (_I, [_P, _P, _SZ, _P, _PP]),
+    "cg_block_linear": (_I, [_P, C.POINTER(LinearArgs), _PP]),
+    "cg_block_residual": (_I, [_P, _P, C.POINTER(Branch), _SZ, C.c_float, _PP]),
+    "cg_block_attention": (_I, [_P, C.POINTER(AttentionArgs), _PP, _PP, _PP]),
+    "cg_block_channel_delta": (_I, [_P, C.POINTER(ChannelDeltaArgs), _PP, _PP, _PP]),
 }
 
 

@@ -319,6 +319,40 @@ class Backend:
     def index(self, x, dim: int, indices) -> Tensor:
         return self._op(lambda b, o: self._lib.cg_index(b, self._take(x), dim, self._take(indices), o))
 
+    # ---- decoder blocks (the last section of include/catgrad_hip.h) --------------------------
+    def _block(self, cls, tensors: dict, options: dict):
+        known = {n for n, _ in cls._fields_}
+        unknown = (set(tensors) | set(options)) - known
+        if unknown:
+            raise TypeError(f"unknown arguments {sorted(unknown)}")
+        a = cls(**options)
+        for name, t in tensors.items():
+            if t is not None:
+                setattr(a, name, self._take(t))
+        return a
+
+    def block_linear(self, x, w, x2=None, gamma=None, bias=None, eps=0.0, scale=1.0) -> Tensor:
+        a = self._block(A.LinearArgs, dict(x=x, w=w, x2=x2, gamma=gamma, bias=bias), dict(eps=eps, scale=scale))
+        return self._op(lambda b, o: self._lib.cg_block_linear(b, C.byref(a), o))
+
+    def block_residual(self, x, branches, eps=0.0) -> Tensor:
+        """branches: dictionaries with y, w and optionally gate, gate_bias, poly."""
+        br = (A.Branch * max(len(branches), 1))(*[self._block(A.Branch, d, {}) for d in branches])
+        return self._op(lambda b, o: self._lib.cg_block_residual(b, self._take(x), br, len(branches), eps, o))
+
+    def _three(self, fn, a):
+        o = [C.c_void_p() for _ in range(3)]
+        self._check(fn(self._b, C.byref(a), *[C.byref(p) for p in o]))
+        return tuple(Tensor(self, p.value) for p in o)
+
+    def block_attention(self, tensors: dict, **options):
+        """-> (output, k cache, v cache); tensors: q, k, v, k_cache, v_cache and optionally q_norm, k_norm, talk."""
+        return self._three(self._lib.cg_block_attention, self._block(A.AttentionArgs, tensors, options))
+
+    def block_channel_delta(self, tensors: dict, **options):
+        """-> (output, state, convolution state)."""
+        return self._three(self._lib.cg_block_channel_delta, self._block(A.ChannelDeltaArgs, tensors, options))
+
 
 _hip_lib = None
 

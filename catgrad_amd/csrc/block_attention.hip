@@ -1,0 +1,316 @@
+// Causal attention of new tokens behind a cache, with a window, a distance bias, a query temperature, norms over whole
+// projections and head mixing after the soft-max (cg_block_attention).
+//
+//   attention_prepare_kernel  a workgroup per token: the query row normed and scaled, the key and value rows into the cache
+//   attention_scores_kernel   a workgroup per (token, kv head, 128 keys): scores, and their maximum and sum per head
+//   attention_mix_kernel      the same split: soft-max weights of every head, mixed, times the values of the kv head
+//   attention_sum_kernel      partial results of a token's key segments added up
+#include "blocks.hpp"
+#include "device_utils.hpp"
+
+#include <algorithm>
+
+namespace cg {
+namespace {
+
+constexpr int kThreads = 256, kWaves = 4;
+constexpr uint32_t kSeg = 128; // keys of a segment
+
+__device__ __forceinline__ float wave_sum(float v) {
+#pragma unroll
+    for (int d = 32; d > 0; d >>= 1) v += __shfl_xor(v, d, 64);
+    return v;
+}
+__device__ __forceinline__ float block_sum(float v, float *red) {
+    v = wave_sum(v);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return (red[0] + red[1]) + (red[2] + red[3]);
+}
+__device__ __forceinline__ float slope_of(uint32_t h, uint32_t heads) { return exp2f(-8.0f * (float)(h + 1) / (float)heads); }
+
+// Visible keys of the token in row s: [lo, hi) of the cached and new keys together.
+__device__ __forceinline__ void visible(const AttentionPlan &p, uint32_t s, uint32_t *lo, uint32_t *hi) {
+    const uint32_t i = p.cached + s;
+    *hi = i + 1;
+    *lo = p.window && i + 1 > p.window ? i + 1 - p.window : 0;
+}
+
+__global__ __launch_bounds__(kThreads) void attention_prepare_kernel(const AttentionPlan p, float *__restrict__ q) {
+    __shared__ float red[kWaves];
+    const uint32_t r = blockIdx.x, b = r / p.S, s = r - b * p.S;
+    const uint32_t nq = p.heads * p.dim, nk = p.kv_heads * p.dim, nv = p.kv_heads * p.vdim;
+    const float *qr = p.q.p + (int64_t)r * p.q.pitch, *kr = p.k.p + (int64_t)r * p.k.pitch, *vr = p.v.p + (int64_t)r * p.v.pitch;
+    float mq = 0.0f, mk = 0.0f;
+    if (p.q_norm)
+        for (uint32_t i = threadIdx.x; i < nq; i += kThreads) mq = fmaf(qr[i], qr[i], mq);
+    if (p.k_norm)
+        for (uint32_t i = threadIdx.x; i < nk; i += kThreads) mk = fmaf(kr[i], kr[i], mk);
+    float fq = 1.0f, fk = 1.0f;
+    if (p.q_norm) fq = 1.0f / sqrtf(block_sum(mq, red) / (float)nq + p.eps);
+    if (p.k_norm) fk = 1.0f / sqrtf(block_sum(mk, red) / (float)nk + p.eps);
+    float temp = p.scale;
+    if (p.temp_every) temp *= 1.0f + p.temp_coef * logf((float)((p.position + s + 1) / p.temp_every + 1));
+    for (uint32_t i = threadIdx.x; i < nq; i += kThreads) {
+        float v = qr[i];
+        if (p.q_norm) v = v * fq * p.q_norm[i];
+        q[(int64_t)r * nq + i] = v * temp;
+    }
+    float *kc = p.keys + (int64_t)b * p.kv_heads * p.k_block + (int64_t)(p.cached + s) * p.dim;
+    float *vc = p.values + (int64_t)b * p.kv_heads * p.v_block + (int64_t)(p.cached + s) * p.vdim;
+    for (uint32_t i = threadIdx.x; i < nk; i += kThreads) {
+        const uint32_t g = i / p.dim, d = i - g * p.dim;
+        float v = kr[i];
+        if (p.k_norm) v = v * fk * p.k_norm[i];
+        kc[(int64_t)g * p.k_block + d] = v;
+    }
+    for (uint32_t i = threadIdx.x; i < nv; i += kThreads) {
+        const uint32_t g = i / p.vdim, d = i - g * p.vdim;
+        vc[(int64_t)g * p.v_block + d] = vr[i];
+    }
+}
+
+// Four lanes share a key; REP query heads of the kv head at a time (blockIdx.y = kv head and which of its head groups).
+template <int REP, int VW>
+__global__ __launch_bounds__(kThreads) void attention_scores_kernel(const AttentionPlan p, const float *__restrict__ q, const uint32_t row0, const uint32_t nseg,
+                                                                    float *__restrict__ scores, float2 *__restrict__ stats) {
+    extern __shared__ float lds[]; // [REP][dim] queries, then [REP][kSeg] scores
+    const uint32_t rep = p.heads / p.kv_heads, groups = (rep + REP - 1) / REP;
+    const uint32_t g = blockIdx.y / groups, h0 = g * rep + (blockIdx.y - g * groups) * REP, nh = min((uint32_t)REP, (g + 1) * rep - h0);
+    const uint32_t r = row0 + blockIdx.z, b = r / p.S, s = r - b * p.S, seg = blockIdx.x;
+    float *sc = lds + REP * p.dim;
+    for (uint32_t i = threadIdx.x; i < REP * p.dim; i += kThreads) {
+        const uint32_t h = i / p.dim, d = i - h * p.dim;
+        lds[i] = h < nh ? q[((int64_t)r * p.heads + h0 + h) * p.dim + d] : 0.0f;
+    }
+    __syncthreads();
+    uint32_t lo, hi;
+    visible(p, s, &lo, &hi);
+    const float *K = p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block;
+    const uint32_t sub = threadIdx.x & 3, nd = p.dim / VW;
+    for (uint32_t key = threadIdx.x >> 2; key < kSeg; key += kThreads / 4) {
+        const uint32_t j = lo + seg * kSeg + key;
+        float acc[REP] = {};
+        if (j < hi) {
+            const float *kp = K + (int64_t)j * p.dim;
+            for (uint32_t i = sub; i < nd; i += 4) {
+                float kv[VW];
+                if constexpr (VW == 4) {
+                    const float4 t = *reinterpret_cast<const float4 *>(kp + 4 * i);
+                    kv[0] = t.x, kv[1] = t.y, kv[2] = t.z, kv[3] = t.w;
+                } else {
+                    kv[0] = kp[i];
+                }
+#pragma unroll
+                for (int h = 0; h < REP; h++)
+#pragma unroll
+                    for (int e = 0; e < VW; e++) acc[h] = fmaf(kv[e], lds[h * p.dim + VW * i + e], acc[h]);
+            }
+        }
+#pragma unroll
+        for (int h = 0; h < REP; h++) {
+            float v = acc[h];
+            v += __shfl_xor(v, 1, 64);
+            v += __shfl_xor(v, 2, 64);
+            if (sub == 0) {
+                if (p.bias) v -= slope_of(h0 + h, p.heads) * (float)(int)(p.cached + s - j);
+                sc[h * kSeg + key] = j < hi ? v : -INFINITY;
+            }
+        }
+    }
+    __syncthreads();
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    for (uint32_t h = wave; h < nh; h += kWaves) {
+        const float a = sc[h * kSeg + lane], c = sc[h * kSeg + 64 + lane];
+        float m = fmaxf(a, c);
+#pragma unroll
+        for (int d = 32; d > 0; d >>= 1) m = fmaxf(m, __shfl_xor(m, d, 64));
+        const float l = m == -INFINITY ? 0.0f : wave_sum(expf(a - m) + expf(c - m));
+        const int64_t head = (int64_t)blockIdx.z * p.heads + h0 + h;
+        float *o = scores + (head * nseg + seg) * kSeg;
+        o[lane] = a;
+        o[64 + lane] = c;
+        if (lane == 0) stats[head * nseg + seg] = make_float2(m, l);
+    }
+}
+
+template <int REP, int VW>
+__global__ __launch_bounds__(kThreads) void attention_mix_kernel(const AttentionPlan p, const uint32_t row0, const uint32_t nseg, const float *__restrict__ scores,
+                                                                 const float2 *__restrict__ stats, float *__restrict__ dst, const bool partial) {
+    // [H'] maxima, [REP][H'] mixing factors over the sums, [H'][kSeg] exponentials, [REP][kSeg] weights, [256 * VW] results;
+    // H': all heads when they are mixed, else the heads of this workgroup
+    extern __shared__ float lds[];
+    const uint32_t rep = p.heads / p.kv_heads, groups = (rep + REP - 1) / REP;
+    const uint32_t g = blockIdx.y / groups, h0 = g * rep + (blockIdx.y - g * groups) * REP, nh = min((uint32_t)REP, (g + 1) * rep - h0);
+    const uint32_t r = row0 + blockIdx.z, b = r / p.S, s = r - b * p.S, seg = blockIdx.x;
+    const uint32_t first = p.talk ? 0 : h0, nm = p.talk ? p.heads : nh, slots = p.talk ? p.heads : REP;
+    float *mx = lds, *tm = mx + slots, *ex = tm + REP * slots, *wt = ex + slots * kSeg, *red = wt + REP * kSeg;
+    for (uint32_t h = threadIdx.x; h < nm; h += kThreads) {
+        const float2 *st = stats + ((int64_t)blockIdx.z * p.heads + first + h) * nseg;
+        float m = -INFINITY, l = 0.0f;
+        for (uint32_t i = 0; i < nseg; i++) m = fmaxf(m, st[i].x);
+        for (uint32_t i = 0; i < nseg; i++)
+            if (st[i].y > 0.0f) l = fmaf(st[i].y, expf(st[i].x - m), l);
+        mx[h] = m;
+        for (uint32_t o = 0; o < REP; o++) {
+            const float f = o >= nh ? 0.0f : p.talk ? p.talk[(int64_t)(h0 + o) * p.heads + h] : (o == h ? 1.0f : 0.0f);
+            tm[o * slots + h] = f / l;
+        }
+    }
+    __syncthreads();
+    for (uint32_t i = threadIdx.x; i < nm * kSeg; i += kThreads) {
+        const uint32_t h = i / kSeg, k = i - h * kSeg;
+        ex[i] = expf(scores[(((int64_t)blockIdx.z * p.heads + first + h) * nseg + seg) * kSeg + k] - mx[h]); // (beyond the last key: 0)
+    }
+    __syncthreads();
+    for (uint32_t i = threadIdx.x; i < REP * kSeg; i += kThreads) {
+        const uint32_t o = i / kSeg, k = i - o * kSeg;
+        float w = 0.0f;
+        for (uint32_t h = 0; h < nm; h++) w = fmaf(tm[o * slots + h], ex[h * kSeg + k], w);
+        wt[i] = w;
+    }
+    __syncthreads();
+    uint32_t lo, hi;
+    visible(p, s, &lo, &hi);
+    const uint32_t j0 = lo + seg * kSeg, keys = j0 < hi ? min(kSeg, hi - j0) : 0;
+    const float *Vp = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)j0 * p.vdim;
+    uint32_t lanes = 1; // lanes side by side along vdim; the others take keys in turn
+    while (lanes < kThreads && lanes * VW < p.vdim) lanes *= 2;
+    const uint32_t across = threadIdx.x & (lanes - 1), turn = threadIdx.x / lanes, turns = kThreads / lanes;
+    for (uint32_t d0 = 0; d0 < p.vdim; d0 += lanes * VW) {
+        const uint32_t d = d0 + across * VW;
+        float acc[REP][VW] = {};
+        if (d < p.vdim)
+            for (uint32_t k = turn; k < keys; k += turns) {
+                float v[VW];
+                const float *vp = Vp + (int64_t)k * p.vdim + d;
+                if constexpr (VW == 4) {
+                    const float4 t = *reinterpret_cast<const float4 *>(vp);
+                    v[0] = t.x, v[1] = t.y, v[2] = t.z, v[3] = t.w;
+                } else {
+                    v[0] = *vp;
+                }
+#pragma unroll
+                for (int o = 0; o < REP; o++)
+#pragma unroll
+                    for (int e = 0; e < VW; e++) acc[o][e] = fmaf(wt[o * kSeg + k], v[e], acc[o][e]);
+            }
+        for (uint32_t o = 0; o < nh; o++) {
+#pragma unroll
+            for (int e = 0; e < VW; e++) {
+                float mine = 0.0f;
+#pragma unroll
+                for (int c = 0; c < REP; c++)
+                    if (c == (int)o) mine = acc[c][e];
+                red[e * kThreads + threadIdx.x] = mine;
+            }
+            __syncthreads();
+            if (turn == 0 && d < p.vdim) {
+                const uint32_t h = h0 + o;
+                float *out = partial ? dst + (((int64_t)blockIdx.z * nseg + seg) * p.heads + h) * p.vdim : dst + ((int64_t)r * p.heads + h) * p.vdim;
+#pragma unroll
+                for (int e = 0; e < VW; e++) {
+                    float sum = 0.0f;
+                    for (uint32_t t = 0; t < turns; t++) sum += red[e * kThreads + t * lanes + across];
+                    out[d + e] = sum;
+                }
+            }
+            __syncthreads();
+        }
+    }
+}
+
+__global__ __launch_bounds__(kThreads) void attention_sum_kernel(const float *__restrict__ parts, const uint32_t nseg, const uint32_t n, float *__restrict__ out) {
+    const uint32_t i = blockIdx.x * kThreads + threadIdx.x;
+    if (i >= n) return;
+    const float *p = parts + (int64_t)blockIdx.y * nseg * n + i;
+    float s = 0.0f;
+    for (uint32_t k = 0; k < nseg; k++) s += p[(int64_t)k * n];
+    out[(int64_t)blockIdx.y * n + i] = s;
+}
+
+int launched(const char *what) {
+    const hipError_t e = hipGetLastError();
+    return e == hipSuccess ? CG_OK : hip_fail(e, what);
+}
+
+constexpr size_t kMaxLds = 128 << 10;
+template <class F> int allow_lds(F *kernel, size_t bytes) {
+    if (bytes > kMaxLds) return fail(CG_ERR_UNSUPPORTED, "block_attention: heads or sizes beyond what the kernels hold");
+    if (bytes <= (64 << 10)) return CG_OK;
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds);
+    return e == hipSuccess ? CG_OK : hip_fail(e, "hipFuncSetAttribute");
+}
+
+struct Scratch {
+    cg_backend *be;
+    void *p = nullptr;
+    size_t cls = 0;
+    explicit Scratch(cg_backend *b) : be(b) {}
+    int get(size_t bytes) { return be->pool.alloc(bytes ? bytes : 4, &p, &cls); }
+    ~Scratch() {
+        if (p) be->pool.free(p, cls);
+    }
+};
+
+template <int REP, int SVW, int MVW>
+int rows_kernels(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t row0, uint32_t rows, uint32_t nseg, float *scores, float2 *stats, float *parts) {
+    const uint32_t rep = p.heads / p.kv_heads, groups = (rep + REP - 1) / REP, slots = p.talk ? p.heads : REP;
+    const size_t lds1 = ((size_t)REP * p.dim + REP * kSeg) * 4;
+    const size_t lds2 = ((size_t)slots + REP * slots + (size_t)slots * kSeg + REP * kSeg + kThreads * MVW) * 4;
+    if (int rc = allow_lds(attention_scores_kernel<REP, SVW>, lds1)) return rc;
+    if (int rc = allow_lds(attention_mix_kernel<REP, MVW>, lds2)) return rc;
+    const dim3 grid(nseg, p.kv_heads * groups, rows);
+    hipLaunchKernelGGL((attention_scores_kernel<REP, SVW>), grid, dim3(kThreads), lds1, be->stream, p, q, row0, nseg, scores, stats);
+    hipLaunchKernelGGL((attention_mix_kernel<REP, MVW>), grid, dim3(kThreads), lds2, be->stream, p, row0, nseg, scores, stats, nseg > 1 ? parts : p.out, nseg > 1);
+    if (nseg > 1) {
+        const uint32_t n = p.heads * p.vdim;
+        hipLaunchKernelGGL(attention_sum_kernel, dim3((n + kThreads - 1) / kThreads, rows), dim3(kThreads), 0, be->stream, parts, nseg, n,
+                           p.out + (int64_t)row0 * n);
+    }
+    return launched("block_attention");
+}
+
+template <int REP>
+int rows_kernels(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t row0, uint32_t rows, uint32_t nseg, float *scores, float2 *stats, float *parts) {
+    const bool dv = p.dim % 4 == 0, vv = p.vdim % 4 == 0; // (cache rows begin at multiples of their length: 16-byte loads then)
+    if (dv && vv) return rows_kernels<REP, 4, 4>(be, p, q, row0, rows, nseg, scores, stats, parts);
+    if (dv) return rows_kernels<REP, 4, 1>(be, p, q, row0, rows, nseg, scores, stats, parts);
+    if (vv) return rows_kernels<REP, 1, 4>(be, p, q, row0, rows, nseg, scores, stats, parts);
+    return rows_kernels<REP, 1, 1>(be, p, q, row0, rows, nseg, scores, stats, parts);
+}
+
+} // namespace
+
+int launch_attention(cg_backend *be, const AttentionPlan &p) {
+    const uint32_t rows = p.B * p.S, all = p.cached + p.S;
+    Scratch qbuf(be);
+    if (int rc = qbuf.get((size_t)rows * p.heads * p.dim * 4)) return rc;
+    float *q = static_cast<float *>(qbuf.p);
+    hipLaunchKernelGGL(attention_prepare_kernel, dim3(rows), dim3(kThreads), 0, be->stream, p, q);
+    if (int rc = launched("attention_prepare")) return rc;
+    const uint32_t most = p.window ? std::min(p.window, all) : all, nseg = (most + kSeg - 1) / kSeg, rep = p.heads / p.kv_heads;
+    double pairs = 0.0; // visible (query, key) pairs
+    for (uint32_t s = 0; s < p.S; s++) pairs += (double)std::min(p.window ? p.window : ~0u, p.cached + s + 1);
+    ProfScope prof(be, CG_K_ATTENTION, pairs * p.B * p.heads * (2.0 * p.dim + 2.0 * p.vdim + (p.talk ? 2.0 * p.heads : 0.0)));
+    // rows in parts that keep the scores within 64 MB
+    const size_t per_row = (size_t)p.heads * nseg * (kSeg * 4 + sizeof(float2)) + (nseg > 1 ? (size_t)nseg * p.heads * p.vdim * 4 : 0);
+    const uint32_t part = (uint32_t)std::max<size_t>(1, std::min<size_t>(std::min<size_t>(rows, 65535), (64u << 20) / per_row));
+    Scratch mem(be);
+    if (int rc = mem.get((size_t)part * per_row)) return rc;
+    float *scores = static_cast<float *>(mem.p);
+    float2 *stats = reinterpret_cast<float2 *>(scores + (size_t)part * p.heads * nseg * kSeg);
+    float *parts = reinterpret_cast<float *>(stats + (size_t)part * p.heads * nseg);
+    for (uint32_t r0 = 0; r0 < rows; r0 += part) {
+        const uint32_t n = std::min(part, rows - r0);
+        int rc = rep <= 1   ? rows_kernels<1>(be, p, q, r0, n, nseg, scores, stats, parts)
+                 : rep <= 2 ? rows_kernels<2>(be, p, q, r0, n, nseg, scores, stats, parts)
+                 : rep <= 4 ? rows_kernels<4>(be, p, q, r0, n, nseg, scores, stats, parts)
+                            : rows_kernels<8>(be, p, q, r0, n, nseg, scores, stats, parts);
+        if (rc) return rc;
+    }
+    return CG_OK;
+}
+
+} // namespace cg

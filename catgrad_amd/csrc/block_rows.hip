@@ -1,0 +1,525 @@
+// Row-wise kernels of the decoder blocks: products of a few rows with streamed weight matrices (the norms of their left
+// operand in the loads, the gated residual sum in the store), and for many rows the operand and the sum on their own.
+#include "blocks.hpp"
+#include "device_utils.hpp"
+
+namespace cg {
+namespace {
+
+constexpr int kThreads = 256, kWaves = 4;
+
+__device__ __forceinline__ float wave_sum(float v) {
+#pragma unroll
+    for (int d = 32; d > 0; d >>= 1) v += __shfl_xor(v, d, 64);
+    return v;
+}
+// sum over the 256 threads of a workgroup, for every thread; `red` has a slot per wave
+__device__ __forceinline__ float block_sum(float v, float *red) {
+    v = wave_sum(v);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return (red[0] + red[1]) + (red[2] + red[3]);
+}
+__device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float bf16_lo(uint32_t w) { return asf(w << 16); }
+__device__ __forceinline__ float bf16_hi(uint32_t w) { return asf(w & 0xFFFF0000u); }
+
+__device__ __forceinline__ float input_at(const ProductInput &in, uint32_t r, uint32_t k) {
+    return k < in.k1 ? in.x.p[(int64_t)r * in.x.pitch + k] : in.x2.p[(int64_t)r * in.x2.pitch + (k - in.k1)];
+}
+
+// What a row of the input is multiplied by / turned into, from sums over the row.
+struct RowScale {
+    float s1 = 1.0f, s2 = 0.0f, s3 = 0.0f, c = 0.0f; // gamma: s1 = 1 / rms; poly: z -> s1 z + s2 z^2 + s3 z^3 + c
+};
+__device__ __forceinline__ RowScale row_scale(const ProductInput &in, float m1, float m2, float m3) {
+    RowScale o;
+    const float n = (float)in.k;
+    if (in.gamma) {
+        o.s1 = 1.0f / sqrtf(m1 / n + in.eps);
+    } else if (in.poly) {
+        o.s1 = in.poly[0] / sqrtf(m1 / n + in.eps);
+        o.s2 = in.poly[1] / sqrtf(m2 / n + in.eps);
+        o.s3 = in.poly[2] / sqrtf(m3 / n + in.eps);
+        o.c = in.poly[3];
+    }
+    return o;
+}
+__device__ __forceinline__ float scaled(const ProductInput &in, const RowScale &o, float z, uint32_t k) {
+    if (in.gamma) return z * o.s1 * in.gamma[k];
+    if (in.poly) return fmaf(z, fmaf(z, fmaf(z, o.s3, o.s2), o.s1), o.c);
+    return z;
+}
+
+// Where column k of a staged row lies in LDS: for bfloat16 weights, which a lane takes eight columns at a time, the two
+// halves of every eight apart, so that both 16-byte reads of a wave are contiguous.
+template <bool BF16> __device__ __forceinline__ uint32_t lds_at(uint32_t k, uint32_t half) {
+    return BF16 ? ((k >> 2) & 1) * half + ((k >> 3) << 2) + (k & 3) : k;
+}
+
+// The rows of the product's left operand into LDS, [M][pitch]; columns up to the pitch are zero.
+template <int M, bool BF16> __device__ void stage_input(const ProductInput &in, uint32_t rows, uint32_t pitch, float *lds, float *red) {
+    const uint32_t half = pitch / 2;
+    float m1[M], m2[M], m3[M];
+#pragma unroll
+    for (int m = 0; m < M; m++) m1[m] = m2[m] = m3[m] = 0.0f;
+    for (uint32_t k = threadIdx.x; k < pitch; k += kThreads) {
+        const uint32_t at = lds_at<BF16>(k, half);
+#pragma unroll
+        for (int m = 0; m < M; m++) {
+            const float z = k < in.k && m < (int)rows ? input_at(in, m, k) : 0.0f;
+            lds[m * pitch + at] = z;
+            const float z2 = z * z;
+            m1[m] += z2;
+            if (in.poly) {
+                m2[m] = fmaf(z2, z2, m2[m]);
+                m3[m] = fmaf(z2 * z2, z2, m3[m]);
+            }
+        }
+    }
+    if (!in.gamma && !in.poly) return; // (the caller's barrier follows)
+    RowScale o[M];
+#pragma unroll
+    for (int m = 0; m < M; m++) {
+        const float a = block_sum(m1[m], red), b = in.poly ? block_sum(m2[m], red) : 0.0f, c = in.poly ? block_sum(m3[m], red) : 0.0f;
+        o[m] = row_scale(in, a, b, c);
+    }
+    for (uint32_t k = threadIdx.x; k < in.k; k += kThreads) { // every thread its own columns again
+        const uint32_t at = lds_at<BF16>(k, half);
+#pragma unroll
+        for (int m = 0; m < M; m++) lds[m * pitch + at] = scaled(in, o[m], lds[m * pitch + at], k);
+    }
+}
+
+// What a lane holds of NC weight rows: 16 bytes of each, or one element.
+template <int NC, bool BF16, bool VEC> struct WeightRegs {
+    uint4 v[NC];
+    __device__ __forceinline__ void load(const Weight &w, const uint32_t (&n)[NC], uint32_t k) {
+        if constexpr (VEC) {
+            constexpr uint32_t EB = BF16 ? 2 : 4;
+#pragma unroll
+            for (int c = 0; c < NC; c++) {
+                typedef uint32_t u4 __attribute__((ext_vector_type(4)));
+                const u4 t = __builtin_nontemporal_load(reinterpret_cast<const u4 *>(static_cast<const char *>(w.p) + ((int64_t)n[c] * w.pitch + k) * EB));
+                v[c] = make_uint4(t[0], t[1], t[2], t[3]);
+            }
+        } else {
+#pragma unroll
+            for (int c = 0; c < NC; c++)
+                v[c].x = BF16 ? (uint32_t)static_cast<const uint16_t *>(w.p)[(int64_t)n[c] * w.pitch + k] << 16
+                              : static_cast<const uint32_t *>(w.p)[(int64_t)n[c] * w.pitch + k];
+        }
+    }
+};
+
+// acc[c][m] += w[n_c, :] . lds[m, :]; a wave walks all of K.  `first` holds the first trip's weights already.
+template <int M, int NC, bool BF16, bool VEC>
+__device__ __forceinline__ void dot_rows(const Weight &w, const uint32_t (&n)[NC], const float *lds, uint32_t pitch, WeightRegs<NC, BF16, VEC> cur,
+                                         float (&acc)[NC][M]) {
+    constexpr uint32_t VW = VEC ? (BF16 ? 8 : 4) : 1, STEP = 64 * VW;
+    const uint32_t half = pitch / 2;
+    uint32_t k = (threadIdx.x & 63) * VW;
+    while (k < w.k) {
+        WeightRegs<NC, BF16, VEC> next;
+        if (k + STEP < w.k) next.load(w, n, k + STEP);
+        if constexpr (!VEC) {
+#pragma unroll
+            for (int m = 0; m < M; m++) {
+                const float x = lds[m * pitch + lds_at<BF16>(k, half)];
+#pragma unroll
+                for (int c = 0; c < NC; c++) acc[c][m] = fmaf(asf(cur.v[c].x), x, acc[c][m]);
+            }
+        } else if constexpr (BF16) {
+#pragma unroll
+            for (int m = 0; m < M; m++) {
+                const float4 a = *reinterpret_cast<const float4 *>(lds + m * pitch + (k >> 1)), b = *reinterpret_cast<const float4 *>(lds + m * pitch + half + (k >> 1));
+#pragma unroll
+                for (int c = 0; c < NC; c++) {
+                    float s = acc[c][m];
+                    s = fmaf(bf16_lo(cur.v[c].x), a.x, s);
+                    s = fmaf(bf16_hi(cur.v[c].x), a.y, s);
+                    s = fmaf(bf16_lo(cur.v[c].y), a.z, s);
+                    s = fmaf(bf16_hi(cur.v[c].y), a.w, s);
+                    s = fmaf(bf16_lo(cur.v[c].z), b.x, s);
+                    s = fmaf(bf16_hi(cur.v[c].z), b.y, s);
+                    s = fmaf(bf16_lo(cur.v[c].w), b.z, s);
+                    s = fmaf(bf16_hi(cur.v[c].w), b.w, s);
+                    acc[c][m] = s;
+                }
+            }
+        } else {
+#pragma unroll
+            for (int m = 0; m < M; m++) {
+                const float4 a = *reinterpret_cast<const float4 *>(lds + m * pitch + k);
+#pragma unroll
+                for (int c = 0; c < NC; c++) {
+                    float s = acc[c][m];
+                    s = fmaf(asf(cur.v[c].x), a.x, s);
+                    s = fmaf(asf(cur.v[c].y), a.y, s);
+                    s = fmaf(asf(cur.v[c].z), a.z, s);
+                    s = fmaf(asf(cur.v[c].w), a.w, s);
+                    acc[c][m] = s;
+                }
+            }
+        }
+        cur = next;
+        k += STEP;
+    }
+}
+
+template <int NC> __device__ __forceinline__ void wave_columns(uint32_t N, uint32_t (&n)[NC], uint32_t *n0) {
+    *n0 = (blockIdx.x * kWaves + (threadIdx.x >> 6)) * NC;
+#pragma unroll
+    for (int c = 0; c < NC; c++) n[c] = min(*n0 + c, N - 1);
+}
+
+template <int M, int NC, bool BF16, bool VEC>
+__global__ __launch_bounds__(kThreads) void few_rows_linear_kernel(const ProductInput in, const uint32_t rows, const Weight w, const uint32_t pitch,
+                                                                   const float *__restrict__ bias, const float scale, float *__restrict__ out) {
+    extern __shared__ float lds[];
+    __shared__ float red[kWaves];
+    uint32_t n[NC], n0;
+    wave_columns<NC>(w.n, n, &n0);
+    constexpr uint32_t VW = VEC ? (BF16 ? 8 : 4) : 1;
+    WeightRegs<NC, BF16, VEC> first;
+    if ((threadIdx.x & 63) * VW < w.k) first.load(w, n, (threadIdx.x & 63) * VW); // on its way while the operand is staged
+    stage_input<M, BF16>(in, rows, pitch, lds, red);
+    __syncthreads();
+    float acc[NC][M] = {};
+    dot_rows<M, NC, BF16, VEC>(w, n, lds, pitch, first, acc);
+#pragma unroll
+    for (int c = 0; c < NC; c++) {
+#pragma unroll
+        for (int m = 0; m < M; m++) {
+            const float s = wave_sum(acc[c][m]);
+            if ((threadIdx.x & 63) == (uint32_t)m && m < (int)rows && n0 + c < w.n)
+                out[(int64_t)m * w.n + n0 + c] = s * scale + (bias ? bias[n0 + c] : 0.0f);
+        }
+    }
+}
+
+template <int M, bool BF16, bool VEC, int NB>
+__global__ __launch_bounds__(kThreads) void few_rows_residual_kernel(const Rows x, const ResidualBranch b0, const ResidualBranch b1, const uint32_t rows,
+                                                                     const uint32_t width, const uint32_t pitch0, const uint32_t pitch1,
+                                                                     float *__restrict__ out) {
+    extern __shared__ float lds[];
+    __shared__ float red[kWaves];
+    uint32_t n[1], n0;
+    wave_columns<1>(width, n, &n0);
+    constexpr uint32_t VW = VEC ? (BF16 ? 8 : 4) : 1;
+    const uint32_t k0 = (threadIdx.x & 63) * VW;
+    WeightRegs<1, BF16, VEC> f0, f1;
+    if (k0 < b0.w.k) f0.load(b0.w, n, k0);
+    if (NB > 1 && k0 < b1.w.k) f1.load(b1.w, n, k0);
+    float *lds1 = lds + M * pitch0;
+    stage_input<M, BF16>(b0.in, rows, pitch0, lds, red);
+    if (NB > 1) stage_input<M, BF16>(b1.in, rows, pitch1, lds1, red);
+    // the lane that stores row m asks for the rest of the sum now
+    const uint32_t lane = threadIdx.x & 63, m_of = min(lane, rows - 1);
+    const float xs = x.p[(int64_t)m_of * x.pitch + n[0]];
+    const float g0 = b0.gate.p ? b0.gate.p[(int64_t)m_of * b0.gate.pitch + n[0]] + (b0.gate_bias ? b0.gate_bias[n[0]] : 0.0f) : 0.0f;
+    const float g1 = NB > 1 && b1.gate.p ? b1.gate.p[(int64_t)m_of * b1.gate.pitch + n[0]] + (b1.gate_bias ? b1.gate_bias[n[0]] : 0.0f) : 0.0f;
+    __syncthreads();
+    float a0[1][M] = {}, a1[1][M] = {};
+    dot_rows<M, 1, BF16, VEC>(b0.w, n, lds, pitch0, f0, a0);
+    if (NB > 1) dot_rows<M, 1, BF16, VEC>(b1.w, n, lds1, pitch1, f1, a1);
+    float s0 = 0.0f, s1 = 0.0f;
+#pragma unroll
+    for (int m = 0; m < M; m++) {
+        const float t0 = wave_sum(a0[0][m]), t1 = NB > 1 ? wave_sum(a1[0][m]) : 0.0f;
+        if (lane == (uint32_t)m) {
+            s0 = t0;
+            s1 = t1;
+        }
+    }
+    if (lane < rows && n0 < width) {
+        float o = b0.gate.p ? sigmoid(g0) * s0 : s0;
+        if (NB > 1) o += b1.gate.p ? sigmoid(g1) * s1 : s1;
+        out[(int64_t)lane * width + n0] = xs + o;
+    }
+}
+
+// ---- many rows -------------------------------------------------------------------------------------------------------
+__device__ __forceinline__ uint32_t round_bf16(float v) { return asu(v) + 0x7FFFu + ((asu(v) >> 16) & 1u); } // (bits above 15 hold the pattern)
+
+// A workgroup per row: the row's sums, then the row as the product reads it.  FMT: 0 f32 words, 1 words rounded to
+// bfloat16, 2 bfloat16 patterns.
+template <int FMT> __global__ __launch_bounds__(kThreads) void product_input_kernel(const ProductInput in, void *__restrict__ dst) {
+    __shared__ float red[kWaves];
+    const uint32_t r = blockIdx.x;
+    RowScale o;
+    if (in.gamma || in.poly) {
+        float m1 = 0.0f, m2 = 0.0f, m3 = 0.0f;
+        for (uint32_t k = threadIdx.x; k < in.k; k += kThreads) {
+            const float z = input_at(in, r, k), z2 = z * z;
+            m1 += z2;
+            if (in.poly) {
+                m2 = fmaf(z2, z2, m2);
+                m3 = fmaf(z2 * z2, z2, m3);
+            }
+        }
+        m1 = block_sum(m1, red);
+        if (in.poly) {
+            m2 = block_sum(m2, red);
+            m3 = block_sum(m3, red);
+        }
+        o = row_scale(in, m1, m2, m3);
+    }
+    const int64_t base = (int64_t)r * in.k;
+    for (uint32_t k = threadIdx.x; k < in.k; k += kThreads) {
+        const float v = scaled(in, o, input_at(in, r, k), k);
+        if constexpr (FMT == 0) static_cast<float *>(dst)[base + k] = v;
+        if constexpr (FMT == 1) static_cast<uint32_t *>(dst)[base + k] = round_bf16(v) & 0xFFFF0000u;
+        if constexpr (FMT == 2) static_cast<uint16_t *>(dst)[base + k] = (uint16_t)(round_bf16(v) >> 16);
+    }
+}
+
+// The same with every row held in registers between the two walks, four columns at a time: one part, k a multiple of 4,
+// at most 4 * 256 * TRIPS columns.
+template <int FMT, int TRIPS> __global__ __launch_bounds__(kThreads) void product_input_vec_kernel(const ProductInput in, void *__restrict__ dst) {
+    __shared__ float red[kWaves];
+    const uint32_t r = blockIdx.x;
+    const float *x = in.x.p + (int64_t)r * in.x.pitch;
+    float4 z[TRIPS];
+    float m1 = 0.0f, m2 = 0.0f, m3 = 0.0f;
+#pragma unroll
+    for (int t = 0; t < TRIPS; t++) {
+        const uint32_t k = (t * kThreads + threadIdx.x) * 4;
+        z[t] = k < in.k ? *reinterpret_cast<const float4 *>(x + k) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    }
+    if (in.gamma || in.poly) {
+#pragma unroll
+        for (int t = 0; t < TRIPS; t++) {
+            const float v[4] = {z[t].x, z[t].y, z[t].z, z[t].w};
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                const float z2 = v[j] * v[j];
+                m1 += z2;
+                if (in.poly) {
+                    m2 = fmaf(z2, z2, m2);
+                    m3 = fmaf(z2 * z2, z2, m3);
+                }
+            }
+        }
+        m1 = block_sum(m1, red);
+        if (in.poly) {
+            m2 = block_sum(m2, red);
+            m3 = block_sum(m3, red);
+        }
+    }
+    const RowScale o = row_scale(in, m1, m2, m3);
+    const int64_t base = (int64_t)r * in.k;
+#pragma unroll
+    for (int t = 0; t < TRIPS; t++) {
+        const uint32_t k = (t * kThreads + threadIdx.x) * 4;
+        if (k >= in.k) continue;
+        const float v[4] = {scaled(in, o, z[t].x, k), scaled(in, o, z[t].y, k + 1), scaled(in, o, z[t].z, k + 2), scaled(in, o, z[t].w, k + 3)};
+        if constexpr (FMT == 0) *reinterpret_cast<float4 *>(static_cast<float *>(dst) + base + k) = make_float4(v[0], v[1], v[2], v[3]);
+        if constexpr (FMT == 1)
+            *reinterpret_cast<uint4 *>(static_cast<uint32_t *>(dst) + base + k) =
+                make_uint4(round_bf16(v[0]) & 0xFFFF0000u, round_bf16(v[1]) & 0xFFFF0000u, round_bf16(v[2]) & 0xFFFF0000u, round_bf16(v[3]) & 0xFFFF0000u);
+        if constexpr (FMT == 2)
+            *reinterpret_cast<uint2 *>(static_cast<uint16_t *>(dst) + base + k) =
+                make_uint2((round_bf16(v[0]) >> 16) | (round_bf16(v[1]) & 0xFFFF0000u), (round_bf16(v[2]) >> 16) | (round_bf16(v[3]) & 0xFFFF0000u));
+    }
+}
+
+__global__ __launch_bounds__(kThreads) void affine_rows_kernel(float *__restrict__ y, const uint32_t n, const float *__restrict__ bias, const float scale) {
+    const uint32_t k = blockIdx.x * kThreads + threadIdx.x;
+    if (k >= n) return;
+    float *p = y + (int64_t)blockIdx.y * n + k;
+    *p = *p * scale + (bias ? bias[k] : 0.0f);
+}
+
+struct GatedSumArgs {
+    Rows x;
+    GatedTerm t[2];
+    int n;
+    uint32_t width;
+};
+template <int VW> __global__ __launch_bounds__(kThreads) void gated_sum_kernel(const GatedSumArgs a, float *__restrict__ out) {
+    const uint32_t k = (blockIdx.x * kThreads + threadIdx.x) * VW, r = blockIdx.y;
+    if (k >= a.width) return;
+    float x[VW], s[VW] = {}, y[VW], g[VW];
+    auto load = [&](const float *p, float(&v)[VW]) {
+        if constexpr (VW == 4) {
+            const float4 t = *reinterpret_cast<const float4 *>(p);
+            v[0] = t.x, v[1] = t.y, v[2] = t.z, v[3] = t.w;
+        } else {
+            v[0] = *p;
+        }
+    };
+    load(a.x.p + (int64_t)r * a.x.pitch + k, x);
+#pragma unroll
+    for (int i = 0; i < 2; i++) {
+        if (i >= a.n) break;
+        load(a.t[i].y + (int64_t)r * a.width + k, y);
+        if (a.t[i].gate.p) load(a.t[i].gate.p + (int64_t)r * a.t[i].gate.pitch + k, g);
+#pragma unroll
+        for (int j = 0; j < VW; j++)
+            s[j] += a.t[i].gate.p ? sigmoid(g[j] + (a.t[i].gate_bias ? a.t[i].gate_bias[k + j] : 0.0f)) * y[j] : y[j];
+    }
+#pragma unroll
+    for (int j = 0; j < VW; j++) x[j] += s[j];
+    float *o = out + (int64_t)r * a.width + k;
+    if constexpr (VW == 4) *reinterpret_cast<float4 *>(o) = make_float4(x[0], x[1], x[2], x[3]);
+    else *o = x[0];
+}
+
+bool aligned16(const void *p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
+
+int launched(const char *what) {
+    const hipError_t e = hipGetLastError();
+    return e == hipSuccess ? CG_OK : hip_fail(e, what);
+}
+
+// Kernels with more than 64 KB of dynamic LDS say so once.
+template <class F> int allow_lds(F *kernel, size_t bytes) {
+    if (bytes <= (64 << 10)) return CG_OK;
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, kFewRowsLds);
+    return e == hipSuccess ? CG_OK : hip_fail(e, "hipFuncSetAttribute");
+}
+
+bool vector_rows(const Weight &w) {
+    const int64_t vw = w.fmt == kFmtBF16 ? 8 : 4;
+    return w.k % vw == 0 && w.pitch % vw == 0 && aligned16(w.p);
+}
+
+template <int M, int NC, bool BF16, bool VEC>
+int few_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows, const Weight &w, const float *bias, float scale, float *out) {
+    const uint32_t pitch = staged_pitch(in.k);
+    const size_t bytes = (size_t)M * pitch * 4;
+    if (int rc = allow_lds(few_rows_linear_kernel<M, NC, BF16, VEC>, bytes)) return rc;
+    hipLaunchKernelGGL((few_rows_linear_kernel<M, NC, BF16, VEC>), dim3((w.n + kWaves * NC - 1) / (kWaves * NC)), dim3(kThreads), bytes, be->stream, in, rows, w,
+                       pitch, bias, scale, out);
+    return CG_OK;
+}
+
+template <int M, bool BF16, bool VEC, int NB>
+int few_rows_residual(cg_backend *be, const Rows &x, const ResidualBranch *br, uint32_t rows, uint32_t width, float *out) {
+    const uint32_t p0 = staged_pitch(br[0].in.k), p1 = NB > 1 ? staged_pitch(br[1].in.k) : 0;
+    const size_t bytes = (size_t)M * (p0 + p1) * 4;
+    if (int rc = allow_lds(few_rows_residual_kernel<M, BF16, VEC, NB>, bytes)) return rc;
+    hipLaunchKernelGGL((few_rows_residual_kernel<M, BF16, VEC, NB>), dim3((width + kWaves - 1) / kWaves), dim3(kThreads), bytes, be->stream, x, br[0],
+                       br[NB > 1 ? 1 : 0], rows, width, p0, p1, out);
+    return CG_OK;
+}
+
+} // namespace
+
+int launch_few_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows, const Weight &w, const float *bias, float scale, float *out) {
+    const uint32_t m = few_rows_slots(rows, (uint64_t)staged_pitch(in.k) * 4);
+    if (!m) return fail(CG_ERR_ARG, "internal error: too many rows for the streaming product");
+    const bool bf16 = w.fmt == kFmtBF16, vec = vector_rows(w);
+    ProfScope prof(be, CG_K_GEMM_SKINNY, (double)w.n * w.k * (bf16 ? 2.0 : 4.0) + 4.0 * rows * ((double)in.k + w.n));
+    const int nc = !vec ? 1 : w.n >= 8192 ? 4 : w.n >= 4096 ? 2 : 1;
+    int rc = CG_OK;
+#define CG_LIN(M, NC, BF, VE) rc = few_rows_linear<M, NC, BF, VE>(be, in, rows, w, bias, scale, out)
+#define CG_LIN_NC(M, BF)              \
+    if (!vec) CG_LIN(M, 1, BF, false); \
+    else if (nc == 4) CG_LIN(M, 4, BF, true); \
+    else if (nc == 2) CG_LIN(M, 2, BF, true); \
+    else CG_LIN(M, 1, BF, true)
+#define CG_LIN_M(M)              \
+    if (bf16) { CG_LIN_NC(M, true); } \
+    else { CG_LIN_NC(M, false); }
+    if (m == 1) { CG_LIN_M(1) }
+    else if (m == 2) { CG_LIN_M(2) }
+    else if (m == 4) { CG_LIN_M(4) }
+    else { CG_LIN_M(8) }
+#undef CG_LIN_M
+#undef CG_LIN_NC
+#undef CG_LIN
+    return rc ? rc : launched("few_rows_linear");
+}
+
+int launch_few_rows_residual(cg_backend *be, const Rows &x, const ResidualBranch *br, int n, uint32_t rows, uint32_t width, float *out) {
+    uint64_t per_row = 0;
+    double bytes = 8.0 * rows * width;
+    bool vec = true;
+    for (int i = 0; i < n; i++) {
+        per_row += (uint64_t)staged_pitch(br[i].in.k) * 4;
+        bytes += (double)br[i].w.n * br[i].w.k * (br[i].w.fmt == kFmtBF16 ? 2.0 : 4.0) + 4.0 * rows * ((double)br[i].in.k + width);
+        vec = vec && vector_rows(br[i].w);
+    }
+    const uint32_t m = few_rows_slots(rows, per_row);
+    if (!m || n < 1) return fail(CG_ERR_ARG, "internal error: too many rows for the streaming product");
+    ResidualBranch same[2] = {br[0], br[n > 1 ? 1 : 0]};
+    if (n > 1 && same[0].w.fmt != same[1].w.fmt) { // one small matrix in words, the other in patterns: one branch after the other
+        if (int rc = launch_few_rows_residual(be, x, br, 1, rows, width, out)) return rc;
+        Rows o{out, (int64_t)width};
+        return launch_few_rows_residual(be, o, br + 1, 1, rows, width, out);
+    }
+    const bool bf16 = br[0].w.fmt == kFmtBF16;
+    ProfScope prof(be, CG_K_GEMM_SKINNY, bytes);
+    int rc = CG_OK;
+#define CG_RES(M, BF, VE)                                                                       \
+    rc = n > 1 ? few_rows_residual<M, BF, VE, 2>(be, x, same, rows, width, out) : few_rows_residual<M, BF, VE, 1>(be, x, same, rows, width, out)
+#define CG_RES_M(M)                       \
+    if (bf16 && vec) CG_RES(M, true, true);       \
+    else if (bf16) CG_RES(M, true, false);        \
+    else if (vec) CG_RES(M, false, true);         \
+    else CG_RES(M, false, false)
+    if (m == 1) { CG_RES_M(1); }
+    else if (m == 2) { CG_RES_M(2); }
+    else if (m == 4) { CG_RES_M(4); }
+    else { CG_RES_M(8); }
+#undef CG_RES_M
+#undef CG_RES
+    return rc ? rc : launched("few_rows_residual");
+}
+
+int launch_product_input(cg_backend *be, const ProductInput &in, uint32_t rows, void *dst, bool round_bf16, int fmt) {
+    ProfScope prof(be, CG_K_REDUCE, (double)rows * in.k * (4.0 + (fmt == kFmtBF16 ? 2.0 : 4.0)));
+    const int f = fmt == kFmtBF16 ? 2 : round_bf16 ? 1 : 0;
+    const bool vec = !in.x2.p && in.k % 4 == 0 && in.x.pitch % 4 == 0 && aligned16(in.x.p) && in.k <= 4 * kThreads * 16;
+    const int trips = (int)((in.k + 4 * kThreads - 1) / (4 * kThreads));
+    hipStream_t s = be->stream;
+#define CG_IN(F)                                                                                                                       \
+    if (!vec) hipLaunchKernelGGL((product_input_kernel<F>), dim3(rows), dim3(kThreads), 0, s, in, dst);                                 \
+    else if (trips <= 1) hipLaunchKernelGGL((product_input_vec_kernel<F, 1>), dim3(rows), dim3(kThreads), 0, s, in, dst);               \
+    else if (trips <= 2) hipLaunchKernelGGL((product_input_vec_kernel<F, 2>), dim3(rows), dim3(kThreads), 0, s, in, dst);               \
+    else if (trips <= 4) hipLaunchKernelGGL((product_input_vec_kernel<F, 4>), dim3(rows), dim3(kThreads), 0, s, in, dst);               \
+    else if (trips <= 8) hipLaunchKernelGGL((product_input_vec_kernel<F, 8>), dim3(rows), dim3(kThreads), 0, s, in, dst);               \
+    else hipLaunchKernelGGL((product_input_vec_kernel<F, 16>), dim3(rows), dim3(kThreads), 0, s, in, dst)
+    if (f == 0) { CG_IN(0); }
+    else if (f == 1) { CG_IN(1); }
+    else { CG_IN(2); }
+#undef CG_IN
+    return launched("product_input");
+}
+
+int launch_affine_rows(cg_backend *be, float *y, uint32_t rows, uint32_t n, const float *bias, float scale) {
+    for (uint32_t r0 = 0; r0 < rows; r0 += 65535) { // (the grid's y extent)
+        const uint32_t nr = rows - r0 < 65535 ? rows - r0 : 65535;
+        ProfScope prof(be, CG_K_ELEMENTWISE, 8.0 * nr * n);
+        hipLaunchKernelGGL(affine_rows_kernel, dim3((n + kThreads - 1) / kThreads, nr), dim3(kThreads), 0, be->stream, y + (int64_t)r0 * n, n, bias, scale);
+    }
+    return launched("affine_rows");
+}
+
+int launch_gated_sum(cg_backend *be, const Rows &x, const GatedTerm *t, int n, uint32_t rows, uint32_t width, float *out) {
+    bool vec = width % 4 == 0 && x.pitch % 4 == 0 && aligned16(x.p) && aligned16(out);
+    for (int i = 0; i < n; i++) vec = vec && (!t[i].gate.p || (t[i].gate.pitch % 4 == 0 && aligned16(t[i].gate.p))) && aligned16(t[i].y);
+    for (uint32_t r0 = 0; r0 < rows; r0 += 65535) {
+        const uint32_t nr = rows - r0 < 65535 ? rows - r0 : 65535;
+        ProfScope prof(be, CG_K_ELEMENTWISE, (2.0 + 2.0 * n) * 4.0 * nr * width);
+        GatedSumArgs a{};
+        a.x = {x.p + (int64_t)r0 * x.pitch, x.pitch};
+        a.n = n;
+        a.width = width;
+        for (int i = 0; i < n; i++) {
+            a.t[i] = t[i];
+            a.t[i].y += (int64_t)r0 * width;
+            if (a.t[i].gate.p) a.t[i].gate.p += (int64_t)r0 * a.t[i].gate.pitch;
+        }
+        const uint32_t per = kThreads * (vec ? 4 : 1);
+        const dim3 grid((width + per - 1) / per, nr);
+        if (vec) hipLaunchKernelGGL((gated_sum_kernel<4>), grid, dim3(kThreads), 0, be->stream, a, out + (int64_t)r0 * width);
+        else hipLaunchKernelGGL((gated_sum_kernel<1>), grid, dim3(kThreads), 0, be->stream, a, out + (int64_t)r0 * width);
+    }
+    return launched("gated_sum");
+}
+
+} // namespace cg

@@ -284,6 +284,34 @@ int new_dense(cg_backend *be, cg_dtype dt, const int64_t *dims, int rank, cg_ten
 // The narrowest format that results of dtype dt with n elements are stored in (small results stay words: the kernels of a
 // decode step address words).
 int result_fmt(const cg_backend *be, cg_dtype dt, int64_t n);
+// A handle of this backend, counted in it, everything else unset.
+cg_tensor *alloc_tensor(cg_backend *be);
+// Turns a deferred tensor into a concrete one, in place (every holder of the handle sees it).
+int ensure_concrete(cg_tensor *t);
+// A dense copy of any view.
+int materialize(cg_backend *be, const cg_tensor *x, cg_tensor **out);
+
+// ---- helpers for the entry points -------------------------------------------------------
+struct Consume { // the consumed reference of a tensor argument (move semantics of the ABI)
+    cg_tensor *t;
+    explicit Consume(cg_tensor *t) : t(t) {}
+    ~Consume() { release(t); }
+};
+// Every entry point that touches a backend's state holds the backend's lock for its whole duration
+// (declared first, so the tensor arguments it consumes are released under the lock too): handles may be
+// cloned, moved between threads and used from several threads; calls on one backend then run one at a time.
+struct Enter {
+    explicit Enter(cg_backend *b) : b_(b) {
+        if (b_) b_->mu.lock();
+    }
+    ~Enter() {
+        if (b_) b_->mu.unlock();
+    }
+    Enter(const Enter &) = delete;
+    Enter &operator=(const Enter &) = delete;
+    cg_backend *b_;
+};
+
 // Fresh uniform tensor (no memory).
 cg_tensor *new_uniform(cg_backend *be, cg_dtype dt, const int64_t *dims, int rank, uint32_t bits);
 // New handle sharing t's buffer and metadata.

@@ -21,7 +21,7 @@ namespace cg {
 
 static thread_local std::string g_err;
 static std::recursive_mutex g_lazy_mu; // guards lazy backing of uniform tensors and of deferred ones (computing one may compute another)
-static int ensure_concrete(cg_tensor *t);
+
 static int run_pending(cg_backend *be, const cg_tensor *dst, const Pending &p, bool fresh);
 
 int fail(int code, const char *fmt, ...) {
@@ -327,7 +327,7 @@ int lazy_mm_force(cg_backend *be, LazyMm *m) {
 
 // Every handle that can leave the library is counted in its backend: the backend's memory pool, stream and lock
 // outlive cg_backend_destroy for as long as such a handle exists (see there).
-static cg_tensor *alloc_tensor(cg_backend *be) {
+cg_tensor *alloc_tensor(cg_backend *be) {
     cg_tensor *t = new cg_tensor;
     t->be = be;
     be->live_tensors.fetch_add(1, std::memory_order_relaxed);
@@ -668,12 +668,6 @@ double distinct_bytes(const cg_tensor *t) {
 }
 
 // ---- helpers for the entry points -------------------------------------------------------
-struct Consume { // the consumed reference of a tensor argument (move semantics of the ABI)
-    cg_tensor *t;
-    explicit Consume(cg_tensor *t) : t(t) {}
-    ~Consume() { release(t); }
-};
-
 static const char *kTodo = "unknown dtype";
 static bool supported(cg_dtype d) { return d == CG_F32 || d == CG_U32 || d == CG_F16 || d == CG_BF16 || d == CG_F8; }
 // bytes of one element at the boundary (from_vec / to_vec)
@@ -793,7 +787,7 @@ static int run_pending(cg_backend *be, const cg_tensor *dst, const Pending &p, b
 static int run_pending(cg_backend *be, const cg_tensor *dst, const Pending &p) { return run_pending(be, dst, p, false); }
 
 // Row-major copy of a view (the materialising half of reshape / to_vec).
-static int materialize(cg_backend *be, const cg_tensor *x, cg_tensor **out) {
+int materialize(cg_backend *be, const cg_tensor *x, cg_tensor **out) {
     cg_tensor *o;
     // a copy of a view of a narrow buffer keeps the buffer's format (whatever dtype tags the view); a program without row
     // reductions stores the format of its dtype
@@ -1412,7 +1406,7 @@ static bool may_wait(const cg_backend *be, const cg_tensor *dst, const Pending *
 }
 
 // Turns a deferred tensor into a concrete one, in place (every holder of the handle sees it).
-static int ensure_concrete(cg_tensor *t) {
+int ensure_concrete(cg_tensor *t) {
     if (t->split >= 0) { // a split-axis view becomes a plain dense tensor, in place
         std::lock_guard<std::recursive_mutex> lk(g_lazy_mu);
         if (t->split < 0) return CG_OK;
@@ -2106,21 +2100,6 @@ using namespace cg;
 extern "C" {
 
 // ---- backend lifetime ----------------------------------------------------------------
-// Every entry point that touches a backend's state holds the backend's lock for its whole duration
-// (declared first, so the tensor arguments it consumes are released under the lock too): handles may be
-// cloned, moved between threads and used from several threads; calls on one backend then run one at a time.
-struct Enter {
-    explicit Enter(cg_backend *b) : b_(b) {
-        if (b_) b_->mu.lock();
-    }
-    ~Enter() {
-        if (b_) b_->mu.unlock();
-    }
-    Enter(const Enter &) = delete;
-    Enter &operator=(const Enter &) = delete;
-    cg_backend *b_;
-};
-
 int cg_backend_create(int device, cg_backend **out) {
     if (!out) return fail(CG_ERR_ARG, "null out");
     int count = 0;

@@ -42,6 +42,7 @@ struct Abi {
     CGH_FN(cg_binary) CGH_FN(cg_where) CGH_FN(cg_matmul) CGH_FN(cg_sum) CGH_FN(cg_max) CGH_FN(cg_argmax)
     CGH_FN(cg_topk) CGH_FN(cg_broadcast) CGH_FN(cg_reshape) CGH_FN(cg_transpose) CGH_FN(cg_slice)
     CGH_FN(cg_concat) CGH_FN(cg_index) CGH_FN(cg_profile_enable) CGH_FN(cg_profile_read)
+    CGH_FN(cg_block_linear) CGH_FN(cg_block_residual) CGH_FN(cg_block_attention) CGH_FN(cg_block_channel_delta)
 #undef CGH_FN
     void *handle = nullptr;
 
@@ -60,6 +61,7 @@ struct Abi {
         CGH_LOAD(cg_max) CGH_LOAD(cg_argmax) CGH_LOAD(cg_topk) CGH_LOAD(cg_broadcast) CGH_LOAD(cg_reshape)
         CGH_LOAD(cg_transpose) CGH_LOAD(cg_slice) CGH_LOAD(cg_concat) CGH_LOAD(cg_index)
         CGH_LOAD(cg_profile_enable) CGH_LOAD(cg_profile_read)
+        CGH_LOAD(cg_block_linear) CGH_LOAD(cg_block_residual) CGH_LOAD(cg_block_attention) CGH_LOAD(cg_block_channel_delta)
 #undef CGH_LOAD
     }
     Abi(const Abi &) = delete;
@@ -257,6 +259,21 @@ class Backend {
     Tensor arange(size_t end) {
         return out([&](cg_tensor **o) { return abi_.cg_arange(b_, end, o); });
     }
+    // A tensor that takes over a reference given up with into_raw.
+    Tensor adopt(cg_tensor *h) { return Tensor(&abi_, h); }
+    // Decoder blocks (include/catgrad_hip.h): the argument structures hold raw references, which the call consumes.
+    Tensor block_linear(const cg_linear_args &a) {
+        return out([&](cg_tensor **o) { return abi_.cg_block_linear(b_, &a, o); });
+    }
+    Tensor block_residual(Tensor x, const std::vector<cg_branch> &br, float eps) {
+        return out([&](cg_tensor **o) { return abi_.cg_block_residual(b_, x.into_raw(), br.data(), br.size(), eps, o); });
+    }
+    std::vector<Tensor> block_attention(const cg_attention_args &a) {
+        return out3([&](cg_tensor **o) { return abi_.cg_block_attention(b_, &a, &o[0], &o[1], &o[2]); });
+    }
+    std::vector<Tensor> block_channel_delta(const cg_channel_delta_args &a) {
+        return out3([&](cg_tensor **o) { return abi_.cg_block_channel_delta(b_, &a, &o[0], &o[1], &o[2]); });
+    }
     bool to_bool(const Tensor &x) {
         calls++;
         int r = 0;
@@ -313,6 +330,17 @@ class Backend {
             check(f(&o));
         }
         return Tensor(&abi_, o);
+    }
+    template <class F> std::vector<Tensor> out3(F &&f) {
+        calls++;
+        cg_tensor *o[3] = {nullptr, nullptr, nullptr};
+        const auto t0 = std::chrono::steady_clock::now();
+        const int rc = f(o);
+        if (time_calls) seconds_in_backend += std::chrono::duration<double>(std::chrono::steady_clock::now() - t0).count();
+        check(rc);
+        std::vector<Tensor> r;
+        for (cg_tensor *t : o) r.emplace_back(&abi_, t);
+        return r;
     }
     Tensor from_vec(cg_dtype dt, const void *data, size_t len, const Shape &shape) {
         calls++;

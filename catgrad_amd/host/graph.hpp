@@ -94,6 +94,7 @@ struct Term : WireTable, OpRecorder {
         auto dt = [&](size_t i) { return a[i].tensor.dtype(); };
         switch (op.op) {
         case TensorOp::Probe: return {};
+        case TensorOp::Block: return op.block->types;
         case TensorOp::Where: return {{sh(1), dt(1)}}; // [mask, x, y]: the type of the values, not of the mask
         case TensorOp::NatToU32: return {{Shape{}, CG_U32}};
         case TensorOp::ScalarF32: return {{Shape{}, CG_F32}};

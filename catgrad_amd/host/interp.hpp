@@ -14,7 +14,9 @@
 #include <cmath>
 #include <cstdio>
 #include <cstdlib>
+#include <functional>
 #include <map>
+#include <memory>
 #include <string>
 #include <vector>
 
@@ -45,7 +47,13 @@ struct InterpreterError : std::runtime_error { // abstract_interpreter/types.rs:
 enum class TensorOp {
     Add, Sub, Mul, Div, Neg, Pow, LT, GT, GTE, LTE, EQ, Cos, Sin, Exp, Log, Floor, Round, Where,
     NatToU32, Cast, MatMul, ScalarF32, ScalarU32, Sum, Max, Argmax, TopK, Broadcast, Reshape, Transpose,
-    Slice, Concat, Arange, Index, Probe
+    Slice, Concat, Arange, Index, Probe, Block
+};
+
+// A step of a decoder layer that is one backend call of its own (blocks.hpp), not one of the trait's operations.
+struct BlockOp {
+    std::function<std::vector<Tensor>(Backend &, std::vector<Tensor>)> run;
+    std::vector<std::pair<Shape, cg_dtype>> types; // of its results
 };
 
 struct Op {
@@ -53,6 +61,7 @@ struct Op {
     float f32 = 0.0f;   // payload of ScalarF32
     uint32_t u32 = 0;   // payload of ScalarU32
     std::string label;  // payload of Probe
+    std::shared_ptr<const BlockOp> block; // payload of Block
     Op(TensorOp o) : op(o) {}
     static Op scalar(float v) { Op o(TensorOp::ScalarF32); o.f32 = v; return o; }
     static Op scalar(uint32_t v) { Op o(TensorOp::ScalarU32); o.u32 = v; return o; }
@@ -189,6 +198,13 @@ inline std::vector<Value> tensor_op(Backend &b, const Op &op, std::vector<Value>
             std::fflush(stdout);
         }
         return {};
+    }
+    case TensorOp::Block: {
+        std::vector<Tensor> in;
+        for (Value &v : args) in.push_back(to_tensor(v));
+        std::vector<Value> r;
+        for (Tensor &t : op.block->run(b, std::move(in))) r.emplace_back(std::move(t));
+        return r;
     }
     }
     throw InterpreterError("unknown tensor op");

@@ -2,13 +2,9 @@
 //   LlamaModel  catgrad-llm-models/src/models/llama.rs:144-386
 //   Qwen3Model  catgrad-llm-models/src/models/qwen3.rs:100-123,196-434 (dense path)
 //   HiddenMlp   catgrad/examples/hidden.rs:103-132 with nn::linear + nn::Sigmoid
-// plus the greedy generate loop and its timing protocol
-// (catgrad-llm/examples/llama/main.rs:876-940,955-1037; catgrad-llm/src/utils/mod.rs:528-583).
 #pragma once
 
-#include <chrono>
-
-#include "graph.hpp"
+#include "model.hpp"
 #include "nn.hpp"
 
 namespace cgh {
@@ -21,53 +17,26 @@ struct LlmConfig { // the fields of LlamaConfig / Qwen3Config that the dense gra
     int tie_word_embeddings = 0;
 };
 
-struct ForwardOut {
-    Tensor tokens, out_k, out_v;
-};
-
-class LlmModel {
+class LlmModel : public Model {
   public:
-    LlmModel(Interpreter &i, const LlmConfig &c) : i_(i), c_(c) {}
+    LlmModel(Interpreter &i, const LlmConfig &c) : Model(i), c_(c) {}
     const LlmConfig &config() const { return c_; }
     std::string root() const { return c_.arch == 0 ? "llama" : "qwen3"; }
-
-    // `Interpreter::run(term, inputs)` for the model's term.  With Interpreter::schedule 0 the operations run as the
-    // graph builder issues them; with 1 the pass is first recorded as a term and then evaluated in the layers of the
-    // reference's evaluator, with its value map (graph.hpp); with 2 recorded and evaluated in the order of recording.
-    ForwardOut forward(Tensor x, Tensor in_k, Tensor in_v, size_t max_positions, Tensor *logits = nullptr) {
-        if (i_.schedule == 0 || i_.recorder) return def(std::move(x), std::move(in_k), std::move(in_v), max_positions, logits);
-        Term term;
-        Tensor sx = term.source(x.shape(), x.dtype()), sk = term.source(in_k.shape(), in_k.dtype()),
-               sv = term.source(in_v.shape(), in_v.dtype());
-        ForwardOut o;
-        Tensor lg;
-        i_.recorder = &term;
-        try {
-            o = def(std::move(sx), std::move(sk), std::move(sv), max_positions, logits ? &lg : nullptr);
-        } catch (...) {
-            i_.recorder = nullptr;
-            throw;
-        }
-        i_.recorder = nullptr;
-        std::vector<Tensor> outs;
-        outs.push_back(std::move(o.tokens));
-        outs.push_back(std::move(o.out_k));
-        outs.push_back(std::move(o.out_v));
-        if (logits) outs.push_back(std::move(lg));
-        term.finish(std::move(outs));
-        std::vector<Tensor> in;
-        in.push_back(std::move(x));
-        in.push_back(std::move(in_k));
-        in.push_back(std::move(in_v));
-        std::vector<Tensor> r = term.run(i_, std::move(in), i_.schedule == 2);
-        if (logits) *logits = std::move(r[3]);
-        return {std::move(r[0]), std::move(r[1]), std::move(r[2])};
+    size_t vocab_size() const override { return c_.vocab_size; }
+    State empty_state(size_t B) override { // empty_state_cache (utils/mod.rs:570-583) with the batch axis set to B
+        Shape kv{c_.num_hidden_layers, B, c_.num_key_value_heads, 0, c_.head_dim};
+        State s;
+        s.tensors.push_back(i_.backend.zeros(kv, CG_F32));
+        s.tensors.push_back(i_.backend.zeros(kv, CG_F32));
+        return s;
     }
 
+  protected:
     // `DynModule::def` for inputs [x u32[B,S], in_k, in_v f32[L,B,kvH,P,hd], Nat(max_positions)]
-    // `logits`, when given, receives a clone of the lm_head output (for parity checks).
-    ForwardOut def(Tensor x, Tensor in_k, Tensor in_v, size_t max_positions, Tensor *logits = nullptr) {
+    // The logits, when asked for, are a clone of the lm_head output (for parity checks).
+    Parts def(Tensor x, std::vector<Tensor> state, size_t, size_t max_positions, const Want &want) override {
         using namespace nn;
+        Tensor in_k = std::move(state[0]), in_v = std::move(state[1]);
         I &i = i_;
         const std::string model = root() + ".model";
         // rope tables + per-layer cache views: Cache::init (helpers/cache.rs:86-103)
@@ -85,10 +54,19 @@ class LlmModel {
         x = rmsnorm(i, c_.rms_norm_eps, model + ".norm", std::move(x));
         const std::string lm_head = c_.tie_word_embeddings ? model + ".embed_tokens" : root() + ".lm_head";
         x = linear_no_bias(i, c_.hidden_size, c_.vocab_size, lm_head, std::move(x));
-        if (logits) *logits = x;
-        x = argmax(i, std::move(x));
+        if (want.rows) { // [B, S, vocab] -> [1, rows, vocab]: the graph projects every position, the chosen ones are gathered
+            Shape ls = shape(x);
+            x = reshape(i, Shape{ls[0] * ls[1], ls[2]}, std::move(x));
+            Tensor ids = i.backend.ndarray_from_vec_u32(want.rows->data(), want.rows->size(), Shape{want.rows->size()});
+            x = unsqueeze(i, 0, index(i, 0, std::move(ids), std::move(x)));
+        }
+        Parts p;
+        if (want.logits) p.out.logits = x;
+        if (want.tokens) p.out.tokens = argmax(i, std::move(x));
         auto kv = cache.output(i);
-        return {std::move(x), std::move(kv.first), std::move(kv.second)};
+        p.state.push_back(std::move(kv.first));
+        p.state.push_back(std::move(kv.second));
+        return p;
     }
 
   private:
@@ -164,7 +142,6 @@ class LlmModel {
         return linear_no_bias(i, nh * hd, dim, p + ".o_proj", std::move(attn));
     }
 
-    Interpreter &i_;
     LlmConfig c_;
 };
 
@@ -173,56 +150,6 @@ inline Tensor hidden_mlp(Interpreter &i, size_t in_dim, size_t hidden, size_t ou
     x = nn::linear(i, in_dim, hidden, "mlp.l1", std::move(x));
     x = nn::sigmoid_module(i, std::move(x));
     return nn::linear(i, hidden, out_dim, "mlp.l2", std::move(x));
-}
-
-struct GenerateStats {
-    double prefill_s = 0, decode_s = 0;
-    uint64_t prefill_calls = 0, decode_calls = 0;
-};
-
-// Greedy generation with KV cache for a batch of B equal-length prompts.  One prefill
-// run, then `steps` decode runs; each run ends with the only device-to-host read of
-// the step, `to_vec` of the argmax tokens, of which the last position of every sequence
-// is the next input (main.rs:1031-1037 generalised from batch 1 to B rows).
-// out_tokens receives (steps + 1) x B ids: the token produced by the prefill, then one
-// per decode run.  Prefill time includes the first read-back, as in main.rs:914-917.
-// prefill_logits, when given, receives the lm_head output [B, S, vocab] of the prefill run (read back after the
-// timed part of that run; for parity checks).
-inline void generate(LlmModel &m, Interpreter &i, const uint32_t *prompt, size_t B, size_t S, size_t steps,
-                     size_t max_positions, uint32_t *out_tokens, GenerateStats *st, std::vector<uint32_t> *prefill_logits = nullptr) {
-    const LlmConfig &c = m.config();
-    // empty_state_cache (utils/mod.rs:570-583) with the batch axis set to B
-    Shape kv{c.num_hidden_layers, B, c.num_key_value_heads, 0, c.head_dim};
-    Tensor state_k = i.backend.zeros(kv, CG_F32), state_v = i.backend.zeros(kv, CG_F32);
-    std::vector<uint32_t> ids(prompt, prompt + B * S);
-    size_t cur = S;
-    auto t0 = std::chrono::steady_clock::now();
-    uint64_t calls0 = i.backend.calls;
-    for (size_t it = 0; it <= steps; it++) {
-        Tensor x = i.backend.ndarray_from_vec_u32(ids.data(), ids.size(), Shape{B, cur});
-        // the run's inputs are clones of the caller's state (main.rs:1007)
-        Tensor logits;
-        ForwardOut o = m.forward(std::move(x), state_k, state_v, max_positions, it == 0 && prefill_logits ? &logits : nullptr);
-        std::vector<uint32_t> tok = i.backend.to_vec_bits(std::move(o.tokens));
-        ids.resize(B);
-        for (size_t b = 0; b < B; b++) {
-            ids[b] = tok[b * cur + (cur - 1)];
-            out_tokens[it * B + b] = ids[b];
-        }
-        state_k = std::move(o.out_k);
-        state_v = std::move(o.out_v);
-        cur = 1;
-        if (it == 0) {
-            auto t1 = std::chrono::steady_clock::now();
-            st->prefill_s = std::chrono::duration<double>(t1 - t0).count();
-            st->prefill_calls = i.backend.calls - calls0;
-            if (prefill_logits) *prefill_logits = i.backend.to_vec_bits(std::move(logits));
-            calls0 = i.backend.calls;
-            t0 = std::chrono::steady_clock::now();
-        }
-    }
-    st->decode_s = std::chrono::duration<double>(std::chrono::steady_clock::now() - t0).count();
-    st->decode_calls = i.backend.calls - calls0;
 }
 
 } // namespace cgh

@@ -6,15 +6,27 @@
 #include <cstring>
 #include <memory>
 
-#include "models.hpp"
+#include "registry.hpp"
 #include "weights.hpp"
 
 using namespace cgh;
 
 struct cgm_session {
     std::unique_ptr<Interpreter> interp;
-    LlmConfig config;
+    std::unique_ptr<Model> model;
+    std::map<uint64_t, State> requests; // what requests in progress hold: caches, recurrent states
     std::string name;
+    Model &loaded() {
+        if (!model) throw InterpreterError("no model configuration has been set");
+        return *model;
+    }
+    void set_model(std::unique_ptr<Model> m) {
+        requests.clear();
+        model = std::move(m);
+    }
+    void parameters_changed() {
+        if (model) model->parameters_changed();
+    }
 };
 
 static thread_local std::string g_err;
@@ -64,6 +76,7 @@ int cgm_open(const char *backend_library, int device, cgm_session **out) {
 
 void cgm_close(cgm_session *s) {
     if (!s) return;
+    s->requests.clear();
     s->interp->parameters.clear();
     delete s;
 }
@@ -76,12 +89,14 @@ int cgm_set_param(cgm_session *s, const char *path, const float *data, const siz
         size_t n = 1;
         for (size_t d : shape) n *= d;
         s->interp->parameters[path] = s->interp->backend.ndarray_from_vec_f32(data, n, shape);
+        s->parameters_changed();
     });
 }
 
 int cgm_load_safetensors(cgm_session *s, const char *const *paths, size_t npaths, double *stats4) {
     return guarded([&] {
         std::vector<std::string> files(paths, paths + npaths);
+        s->parameters_changed();
         LoadStats st = load_safetensors(*s->interp, files);
         stats4[0] = (double)st.tensors;
         stats4[1] = (double)st.params;
@@ -91,14 +106,17 @@ int cgm_load_safetensors(cgm_session *s, const char *const *paths, size_t npaths
 }
 
 int cgm_clear_params(cgm_session *s) {
-    return guarded([&] { s->interp->parameters.clear(); });
+    return guarded([&] {
+        s->interp->parameters.clear();
+        s->parameters_changed();
+    });
 }
 
 int cgm_set_config(cgm_session *s, int arch, size_t hidden_size, size_t num_hidden_layers, size_t num_attention_heads,
                    size_t num_key_value_heads, size_t head_dim, size_t intermediate_size, size_t vocab_size,
                    float rms_norm_eps, float rope_theta, int tie_word_embeddings) {
     return guarded([&] {
-        LlmConfig &c = s->config;
+        LlmConfig c;
         c.arch = arch;
         c.hidden_size = hidden_size;
         c.num_hidden_layers = num_hidden_layers;
@@ -110,7 +128,55 @@ int cgm_set_config(cgm_session *s, int arch, size_t hidden_size, size_t num_hidd
         c.rms_norm_eps = rms_norm_eps;
         c.rope_theta = rope_theta;
         c.tie_word_embeddings = tie_word_embeddings;
+        s->set_model(std::make_unique<LlmModel>(*s->interp, c));
     });
+}
+
+int cgm_load_config(cgm_session *s, const char *json, int weights_dtype) {
+    return guarded([&] {
+        if (weights_dtype != CG_F32 && weights_dtype != CG_BF16) throw ConfigError("weights are held in f32 or bf16");
+        s->set_model(make_model(*s->interp, Json::parse(json), (cg_dtype)weights_dtype));
+    });
+}
+
+int cgm_vocab_size(cgm_session *s, size_t *out) {
+    return guarded([&] { *out = s->loaded().vocab_size(); });
+}
+
+int cgm_request_step(cgm_session *s, uint64_t id, const uint32_t *tokens, size_t n, size_t max_positions, const uint32_t *rows,
+                     size_t nrows, float *out_logits, uint32_t *out_next) {
+    return guarded([&] {
+        Interpreter &i = *s->interp;
+        Model &m = s->loaded();
+        if (!n) throw InterpreterError("a step of no tokens");
+        const size_t vocab = m.vocab_size();
+        for (size_t k = 0; k < nrows; k++)
+            if (rows[k] >= n) throw InterpreterError("a wanted place lies outside the step");
+        auto it = s->requests.find(id);
+        if (it == s->requests.end()) it = s->requests.emplace(id, m.empty_state(1)).first;
+        std::vector<uint32_t> want_rows(rows, rows + nrows);
+        if (out_next) want_rows.push_back((uint32_t)n - 1);
+        Want want;
+        want.rows = &want_rows;
+        want.logits = nrows > 0;
+        want.tokens = out_next != nullptr;
+        Tensor x = i.backend.ndarray_from_vec_u32(tokens, n, Shape{1, n});
+        RunOut o = m.run(std::move(x), it->second, max_positions, want);
+        if (want.logits) {
+            std::vector<uint32_t> lg = i.backend.to_vec_bits(std::move(o.logits));
+            memcpy(out_logits, lg.data(), nrows * vocab * 4);
+        }
+        if (out_next) *out_next = i.backend.to_vec_bits(std::move(o.tokens)).back();
+        if (!want.logits && !out_next) i.backend.sync();
+    });
+}
+
+int cgm_request_end(cgm_session *s, uint64_t id) {
+    return guarded([&] { s->requests.erase(id); });
+}
+
+int cgm_request_count(cgm_session *s, size_t *out) {
+    return guarded([&] { *out = s->requests.size(); });
 }
 
 int cgm_set_schedule(cgm_session *s, int schedule) {
@@ -192,7 +258,7 @@ int cgm_helper(cgm_session *s, int which, const float *x, const size_t *dims, si
 int cgm_generate(cgm_session *s, const uint32_t *prompt, size_t B, size_t S, size_t steps, size_t max_positions,
                  uint32_t *out_tokens, double *stats4) {
     return guarded([&] {
-        LlmModel m(*s->interp, s->config);
+        Model &m = s->loaded();
         GenerateStats st;
         const char *tc = getenv("CGH_TIME_CALLS");
         s->interp->backend.time_calls = tc && tc[0] == '1';
@@ -211,7 +277,7 @@ int cgm_generate(cgm_session *s, const uint32_t *prompt, size_t B, size_t S, siz
 int cgm_generate_with_logits(cgm_session *s, const uint32_t *prompt, size_t B, size_t S, size_t steps, size_t max_positions,
                              uint32_t *out_tokens, double *stats4, float *prefill_logits) {
     return guarded([&] {
-        LlmModel m(*s->interp, s->config);
+        Model &m = s->loaded();
         GenerateStats st;
         std::vector<uint32_t> lg;
         generate(m, *s->interp, prompt, B, S, steps, max_positions, out_tokens, &st, &lg);
@@ -227,17 +293,16 @@ int cgm_forward(cgm_session *s, const uint32_t *tokens, size_t B, size_t S, size
                 float *out_logits) {
     return guarded([&] {
         Interpreter &i = *s->interp;
-        LlmModel m(i, s->config);
-        const LlmConfig &c = s->config;
-        Shape kv{c.num_hidden_layers, B, c.num_key_value_heads, 0, c.head_dim};
+        Model &m = s->loaded();
         Tensor x = i.backend.ndarray_from_vec_u32(tokens, B * S, Shape{B, S});
-        Tensor logits;
-        ForwardOut o = m.forward(std::move(x), i.backend.zeros(kv, CG_F32), i.backend.zeros(kv, CG_F32), max_positions,
-                                 out_logits ? &logits : nullptr);
+        State st = m.empty_state(B);
+        Want want;
+        want.logits = out_logits != nullptr;
+        RunOut o = m.run(std::move(x), st, max_positions, want);
         std::vector<uint32_t> tok = i.backend.to_vec_bits(std::move(o.tokens));
         memcpy(out_tokens, tok.data(), tok.size() * 4);
         if (out_logits) {
-            std::vector<uint32_t> lg = i.backend.to_vec_bits(std::move(logits));
+            std::vector<uint32_t> lg = i.backend.to_vec_bits(std::move(o.logits));
             memcpy(out_logits, lg.data(), lg.size() * 4);
         }
     });
@@ -247,15 +312,15 @@ int cgm_forward_rows(cgm_session *s, const uint32_t *tokens, size_t B, size_t S,
                      const uint32_t *rows, size_t nrows, float *out_logits) {
     return guarded([&] {
         Interpreter &i = *s->interp;
-        LlmModel m(i, s->config);
-        const LlmConfig &c = s->config;
-        Shape kv{c.num_hidden_layers, B, c.num_key_value_heads, 0, c.head_dim};
+        Model &m = s->loaded();
         Tensor x = i.backend.ndarray_from_vec_u32(tokens, B * S, Shape{B, S});
-        Tensor logits;
-        ForwardOut o = m.forward(std::move(x), i.backend.zeros(kv, CG_F32), i.backend.zeros(kv, CG_F32), max_positions, &logits);
+        State st = m.empty_state(B);
+        Want want;
+        want.logits = true;
+        RunOut o = m.run(std::move(x), st, max_positions, want);
         std::vector<uint32_t> tok = i.backend.to_vec_bits(std::move(o.tokens));
         memcpy(out_tokens, tok.data(), tok.size() * 4);
-        Tensor flat = i.backend.reshape(std::move(logits), Shape{B * S, c.vocab_size});
+        Tensor flat = i.backend.reshape(std::move(o.logits), Shape{B * S, m.vocab_size()});
         Tensor idx = i.backend.ndarray_from_vec_u32(rows, nrows, Shape{nrows});
         Tensor picked = i.backend.index(std::move(flat), 0, std::move(idx));
         std::vector<uint32_t> lg = i.backend.to_vec_bits(std::move(picked));

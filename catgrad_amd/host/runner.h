@@ -29,6 +29,20 @@ int cgm_set_config(cgm_session *s, int arch, size_t hidden_size, size_t num_hidd
                    size_t num_key_value_heads, size_t head_dim, size_t intermediate_size, size_t vocab_size,
                    float rms_norm_eps, float rope_theta, int tie_word_embeddings);
 
+/* The model a config.json describes (its text): Loretar, or a Llama / Qwen3 checkpoint's.  weights_dtype: CG_F32, or
+ * CG_BF16 for matrices held and multiplied at bfloat16 precision (Loretar).  Ends every request in progress. */
+int cgm_load_config(cgm_session *s, const char *json, int weights_dtype);
+int cgm_vocab_size(cgm_session *s, size_t *out);
+
+/* Requests in progress, each a sequence with its own caches and recurrent states under an id of the caller's.
+ * A step runs the request's next n tokens (the first step of an id begins it): a whole prompt, a portion of any length,
+ * or one token.  rows[nrows]: the places among them whose logits are read back to out_logits [nrows, vocab];
+ * out_next (may be null): the arg-max after the last of them.  `end` gives back what the request holds. */
+int cgm_request_step(cgm_session *s, uint64_t id, const uint32_t *tokens, size_t n, size_t max_positions, const uint32_t *rows,
+                     size_t nrows, float *out_logits, uint32_t *out_next);
+int cgm_request_end(cgm_session *s, uint64_t id);
+int cgm_request_count(cgm_session *s, size_t *out);
+
 /* Order of evaluation of the model runs and of cgm_cond_kat: 0 = the operations run as the graph builder issues
  * them; 1 = every run is first recorded as a term and evaluated in the layers of the reference's evaluator
  * (catgrad/src/abstract_interpreter/eval.rs:38-66, catgrad/src/ssa/mod.rs:24-76) with its move / clone value map;

@@ -7,11 +7,13 @@ exports the same C ABI (the CPU oracle) as `backend_library`."""
 from __future__ import annotations
 
 import ctypes as C
+import json
 import os
 from dataclasses import dataclass
 
 import numpy as np
 
+from . import _abi as A
 from .backend import HIP_LIBRARY, load_hip_library
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
@@ -36,6 +38,11 @@ def _host():
             "cgm_clear_params": (C.c_int, [P]),
             "cgm_load_safetensors": (C.c_int, [P, C.POINTER(C.c_char_p), SZ, C.POINTER(C.c_double)]),
             "cgm_set_config": (C.c_int, [P, C.c_int] + [SZ] * 7 + [C.c_float, C.c_float, C.c_int]),
+            "cgm_load_config": (C.c_int, [P, C.c_char_p, C.c_int]),
+            "cgm_vocab_size": (C.c_int, [P, SZP]),
+            "cgm_request_step": (C.c_int, [P, C.c_uint64, P, SZ, SZ, P, SZ, P, C.POINTER(C.c_uint32)]),
+            "cgm_request_end": (C.c_int, [P, C.c_uint64]),
+            "cgm_request_count": (C.c_int, [P, SZP]),
             "cgm_set_schedule": (C.c_int, [P, C.c_int]),
             "cgm_cond_kat": (C.c_int, [P, C.c_float, C.c_float, C.POINTER(C.c_float)]),
             "cgm_cond_mismatch": (C.c_int, [P]),
@@ -169,7 +176,48 @@ class Session:
             self._s, 0 if config.arch == "llama" else 1, config.hidden_size, config.num_hidden_layers,
             config.num_attention_heads, config.num_key_value_heads, config.hd, config.intermediate_size,
             config.vocab_size, config.rms_norm_eps, config.rope_theta, int(config.tie_word_embeddings)))
-        self.config = config
+        self.vocab_size = config.vocab_size
+
+    WEIGHT_DTYPES = {"float32": A.F32, "bfloat16": A.BF16}
+
+    def load_config(self, config: dict | str, dtype: str = "float32"):
+        """The model a config.json describes (a dictionary, or its text).  dtype "bfloat16": matrices are held and
+        multiplied at bfloat16 precision (architectures that have such a form)."""
+        text = config if isinstance(config, str) else json.dumps(config)
+        self._check(self._lib.cgm_load_config(self._s, text.encode(), self.WEIGHT_DTYPES[dtype]))
+        n = C.c_size_t()
+        self._check(self._lib.cgm_vocab_size(self._s, C.byref(n)))
+        self.vocab_size = int(n.value)
+
+    def load_pretrained(self, folder, dtype: str = "float32"):
+        """A model folder: config.json and model.safetensors (or the *.safetensors files in it)."""
+        with open(os.path.join(folder, "config.json")) as f:
+            self.load_config(f.read(), dtype)
+        files = sorted(f for f in os.listdir(folder) if f.endswith(".safetensors"))
+        if not files:
+            raise RuntimeError(f"{folder} holds no .safetensors file")
+        return self.load_safetensors([os.path.join(folder, f) for f in files])
+
+    def step(self, request: int, tokens, rows=(), want_next: bool = False, max_positions: int = 0):
+        """Runs the next tokens of a request (its first step begins it).  Returns the logits [len(rows), vocab] at the
+        places `rows` among them; with `want_next` also the arg-max after the last one."""
+        tokens = np.ascontiguousarray(tokens, dtype=np.uint32)
+        rows = np.ascontiguousarray(rows, dtype=np.uint32)
+        logits = np.zeros((rows.size, self.vocab_size), dtype=np.float32)
+        nxt = C.c_uint32()
+        self._check(self._lib.cgm_request_step(
+            self._s, request, tokens.ctypes.data_as(C.c_void_p), tokens.size, max_positions, rows.ctypes.data_as(C.c_void_p),
+            rows.size, logits.ctypes.data_as(C.c_void_p), C.byref(nxt) if want_next else None))
+        return (logits, int(nxt.value)) if want_next else logits
+
+    def end(self, request: int):
+        """Gives back what a request holds in caches and states."""
+        self._check(self._lib.cgm_request_end(self._s, request))
+
+    def requests_in_progress(self) -> int:
+        n = C.c_size_t()
+        self._check(self._lib.cgm_request_count(self._s, C.byref(n)))
+        return int(n.value)
 
     def load_safetensors(self, paths, config: LlmConfig = None):
         """Parameters from safetensors files (F32 and BF16 tensors become f32, I64 is skipped), as
@@ -189,11 +237,7 @@ class Session:
         self.clear_params()
         for name, w in (params if params is not None else random_params(config, seed)):
             self.set_param(name, w)
-        self._check(self._lib.cgm_set_config(
-            self._s, 0 if config.arch == "llama" else 1, config.hidden_size, config.num_hidden_layers,
-            config.num_attention_heads, config.num_key_value_heads, config.hd, config.intermediate_size,
-            config.vocab_size, config.rms_norm_eps, config.rope_theta, int(config.tie_word_embeddings)))
-        self.config = config
+        self.set_config(config)
 
     def set_schedule(self, schedule: int):
         """0: operations run as the graph builder issues them (default); 1: every model run is recorded as a term and
@@ -237,7 +281,7 @@ class Session:
         stats = (C.c_double * 4)()
         logits = None
         if want_logits:
-            logits = np.zeros((B, S, self.config.vocab_size), dtype=np.float32)
+            logits = np.zeros((B, S, self.vocab_size), dtype=np.float32)
             self._check(self._lib.cgm_generate_with_logits(self._s, prompt.ctypes.data_as(C.c_void_p), B, S, steps,
                                                            max_positions, out.ctypes.data_as(C.c_void_p), stats,
                                                            logits.ctypes.data_as(C.c_void_p)))
@@ -251,7 +295,7 @@ class Session:
         tokens = np.ascontiguousarray(tokens, dtype=np.uint32)
         B, S = tokens.shape
         out = np.zeros((B, S), dtype=np.uint32)
-        logits = np.zeros((B, S, self.config.vocab_size), dtype=np.float32) if want_logits else None
+        logits = np.zeros((B, S, self.vocab_size), dtype=np.float32) if want_logits else None
         self._check(self._lib.cgm_forward(self._s, tokens.ctypes.data_as(C.c_void_p), B, S, max_positions or S,
                                           out.ctypes.data_as(C.c_void_p),
                                           logits.ctypes.data_as(C.c_void_p) if want_logits else None))
@@ -264,7 +308,7 @@ class Session:
         rows = np.ascontiguousarray(rows, dtype=np.uint32)
         B, S = tokens.shape
         out = np.zeros((B, S), dtype=np.uint32)
-        logits = np.zeros((rows.size, self.config.vocab_size), dtype=np.float32)
+        logits = np.zeros((rows.size, self.vocab_size), dtype=np.float32)
         self._check(self._lib.cgm_forward_rows(self._s, tokens.ctypes.data_as(C.c_void_p), B, S, max_positions or S,
                                                out.ctypes.data_as(C.c_void_p), rows.ctypes.data_as(C.c_void_p), rows.size,
                                                logits.ctypes.data_as(C.c_void_p)))

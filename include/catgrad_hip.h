@@ -144,7 +144,8 @@ typedef enum cg_kernel_class {
     CG_K_GATHER = 5,      /* work = bytes gathered + written */
     CG_K_ATTENTION = 6,   /* one-pass causal attention of a prefill; work = flop of the visible scores and sums */
     CG_K_PACK = 7,        /* an operand narrowed to 2- / 1-byte patterns in memory for a product; work = bytes read + written */
-    CG_K_CLASSES = 8
+    CG_K_RECURRENCE = 8,  /* cg_block_channel_delta: the recurrence itself; work = flop of decay, read, write and read-out */
+    CG_K_CLASSES = 9
 } cg_kernel_class;
 int cg_profile_enable(cg_backend *b, cg_kernel_class cls, unsigned sample_every);
 /* Element-wise results are computed lazily (fused into their consumer); cg_realize queues
@@ -249,6 +250,69 @@ int cg_slice(cg_backend *b, cg_tensor *x, size_t dim, size_t start, size_t len, 
 int cg_concat(cg_backend *b, cg_tensor *x, cg_tensor *y, size_t dim, cg_tensor **out);
 /* `Backend::index` (mod.rs:94-99; ndarray.rs:466-487,571-579): gather along dim. */
 int cg_index(cg_backend *b, cg_tensor *x, size_t dim, cg_tensor *indices, cg_tensor **out);
+
+/* ---- decoder blocks (no counterpart in the reference) ---------------------------
+ * Steps of a decoder layer that the trait's ops cannot express without writing every intermediate out, or not at all
+ * without an op per token (a recurrence).  Each is one call with its mechanisms as parameters; an absent mechanism is a
+ * null tensor or a zero parameter.  Tensor arguments are consumed like those of the trait's methods, activations are
+ * f32 [B, S, features] views whose last axis has unit stride (parts of one wider product's rows are taken as they lie),
+ * B sequences of S new tokens each.  Weight matrices ([out, in]) may be CG_F32, or CG_BF16: then the activations of a
+ * product are taken at bfloat16 precision, or better, and the sums are f32.  Everything else is computed in f32. */
+
+/* out[.., n] = scale * sum_k norm(x | x2)[.., k] * w[n, k] + bias[n], where (x | x2) is x, followed by x2 along the last
+ * axis when given, and norm is the RMS norm v / sqrt(mean(v^2) + eps) * gamma when gamma is given. */
+typedef struct cg_linear_args {
+    cg_tensor *x, *x2, *gamma, *w, *bias; /* x2, gamma, bias: may be null */
+    float eps, scale;
+} cg_linear_args;
+int cg_block_linear(cg_backend *b, const cg_linear_args *a, cg_tensor **out);
+
+/* out = x + sum_i sigmoid(gate_i + gate_bias_i) * (act_i(y_i) . w_i^T): the residual stream after up to two sublayers that
+ * read the same input.  act is the identity, or with poly = [a, b, c, e] the polynomial norm
+ * a N(z) + b N(z^2) + c N(z^3) + e, where N divides a row by its root mean square (eps inside the root). */
+typedef struct cg_branch {
+    cg_tensor *y, *w, *gate, *gate_bias, *poly; /* gate (with gate_bias) and poly: may be null */
+} cg_branch;
+int cg_block_residual(cg_backend *b, cg_tensor *x, const cg_branch *branches, size_t n, float eps, cg_tensor **out);
+
+/* Causal attention of S new tokens (positions position .. position + S - 1) behind a cache.
+ *  q [B, S, heads * dim], k [B, S, kv_heads * dim], v [B, S, kv_heads * vdim]; query head h reads key / value head
+ *  h / (heads / kv_heads).
+ *  q_norm / k_norm: RMS norm over a token's whole projection (all heads at once).
+ *  temp_every > 0: the query at position p is multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1).
+ *  score(i, j) = scale * q_i . k_j, minus 2^(-8 (h + 1) / heads) * (i - j) with distance_bias.
+ *  window > 0: position i sees 0 <= i - j < window; window == 0: every j <= i.
+ *  talk [heads, heads]: after the soft-max, weight_h <- sum_g talk[h, g] weight_g.
+ *  k_cache [B, kv_heads, T, dim], v_cache [B, kv_heads, T, vdim]: the keys (as they enter the scores) and values of the T
+ *  positions before `position`, at least min(position, window - 1) of them.  The results k_out / v_out hold the last
+ *  min(T + S, window - 1) positions (all of them without a window) and are appended in place when they end at the
+ *  frontier of the cache's memory. */
+typedef struct cg_attention_args {
+    cg_tensor *q, *k, *v, *q_norm, *k_norm, *talk, *k_cache, *v_cache; /* q_norm, k_norm, talk: may be null */
+    size_t heads, kv_heads, dim, vdim, position, window, temp_every;
+    float scale, norm_eps, temp_coef;
+    int distance_bias;
+} cg_attention_args;
+int cg_block_attention(cg_backend *b, const cg_attention_args *a, cg_tensor **out, cg_tensor **k_out, cg_tensor **v_out);
+
+/* Gated delta rule with a decay per key channel.
+ *  q, k [B, S, kv_heads * dim], v [B, S, heads * vdim]: each through a causal convolution over time per channel
+ *  (conv_* [channels, taps], last column = the current token) and silu; q and k are then unit vectors per head,
+ *  x / sqrt(sum(x^2) + 1e-6), and q is multiplied by dim^(-1/2); head h uses q / k head h / (heads / kv_heads).
+ *  beta [B, S, heads]: through a sigmoid.  decay [B, S, r] . decay_w^T [heads * dim, r] = a, and the factor on the state's
+ *  row (h, d) is exp(-exp(a_log[h]) * softplus(a + dt_bias)).
+ *  Per head: S <- g * S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.
+ *  o is divided by its root mean square over vdim (eps inside the root), times norm [vdim], times
+ *  sigmoid(gate [B, S, r2] . gate_w^T [heads * vdim, r2]).
+ *  state [B, heads, dim, vdim] f32, conv_state [B, taps - 1, channels of q, k, v]: the convolutions' last inputs. */
+typedef struct cg_channel_delta_args {
+    cg_tensor *q, *k, *v, *conv_q, *conv_k, *conv_v, *beta, *decay, *decay_w, *a_log, *dt_bias, *gate, *gate_w, *norm, *state,
+        *conv_state;
+    size_t heads, kv_heads, dim, vdim;
+    float eps;
+} cg_channel_delta_args;
+int cg_block_channel_delta(cg_backend *b, const cg_channel_delta_args *a, cg_tensor **out, cg_tensor **state_out,
+                           cg_tensor **conv_out);
 
 #ifdef __cplusplus
 }

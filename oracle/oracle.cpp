@@ -1370,3 +1370,274 @@ int cg_index(cg_backend *, cg_tensor *x, size_t dim, cg_tensor *indices, cg_tens
 }
 
 } // extern "C"
+
+// ---- decoder blocks (include/catgrad_hip.h, last section): plain loops in double, one sequence position at a time ----
+namespace {
+
+struct Owned { // the consumed references of a block's tensor arguments
+    std::vector<cg_tensor *> t;
+    ~Owned() {
+        for (cg_tensor *x : t) release(x);
+    }
+};
+
+std::vector<double> wide(const cg_tensor *t) {
+    Vec<float> v = dense<float>(t);
+    return std::vector<double>(v.begin(), v.end());
+}
+
+// the activations of a product with a bfloat16 weight matrix
+double operand(double v, const cg_tensor *w) { return w->dt == CG_BF16 ? (double)float_of(round_to(CG_BF16, bits_of((float)v))) : v; }
+
+double sigmoid(double z) { return 1.0 / (1.0 + std::exp(-z)); }
+double softplus(double z) { return z > 30.0 ? z : std::log1p(std::exp(z)); }
+
+double mean_square(const double *x, size_t n) {
+    double s = 0;
+    for (size_t i = 0; i < n; i++) s += x[i] * x[i];
+    return s / (double)n;
+}
+
+// y[rows, n] = x[rows, k] . w[n, k]^T
+std::vector<double> product(const std::vector<double> &x, size_t rows, size_t k, const cg_tensor *w) {
+    const size_t n = w->dims[0];
+    std::vector<double> wv = wide(w), xv(x.size()), y(rows * n);
+    for (size_t i = 0; i < x.size(); i++) xv[i] = operand(x[i], w);
+    for (size_t r = 0; r < rows; r++)
+        for (size_t j = 0; j < n; j++) {
+            double s = 0;
+            for (size_t i = 0; i < k; i++) s += xv[r * k + i] * wv[j * k + i];
+            y[r * n + j] = s;
+        }
+    return y;
+}
+
+cg_tensor *result(const std::vector<double> &v, std::vector<size_t> dims) {
+    cg_tensor *t = new_tensor(CG_F32, dims.data(), (int)dims.size());
+    float *p = data_of<float>(t);
+    for (size_t i = 0; i < v.size(); i++) p[i] = (float)v[i];
+    return t;
+}
+
+std::vector<size_t> dims_of(const cg_tensor *t) { return std::vector<size_t>(t->dims, t->dims + t->rank); }
+
+} // namespace
+
+extern "C" {
+
+int cg_block_linear(cg_backend *, const cg_linear_args *a, cg_tensor **out) {
+    if (!a) return fail(CG_ERR_ARG, "null argument");
+    Owned own{{a->x, a->x2, a->gamma, a->w, a->bias}};
+    if (!a->x || !a->w || !out) return fail(CG_ERR_ARG, "null argument");
+    const size_t k1 = a->x->dims[a->x->rank - 1], k2 = a->x2 ? a->x2->dims[a->x2->rank - 1] : 0, k = k1 + k2;
+    const size_t rows = k1 ? numel(a->x) / k1 : 0, n = a->w->dims[0];
+    if (a->w->rank != 2 || a->w->dims[1] != k || (a->x2 && k2 * rows != numel(a->x2)) || (a->gamma && numel(a->gamma) != k) ||
+        (a->bias && numel(a->bias) != n))
+        return fail(CG_ERR_SHAPE, "block_linear: incompatible shapes");
+    std::vector<double> x1 = wide(a->x), x2, x(rows * k);
+    if (a->x2) x2 = wide(a->x2);
+    for (size_t r = 0; r < rows; r++) {
+        for (size_t i = 0; i < k1; i++) x[r * k + i] = x1[r * k1 + i];
+        for (size_t i = 0; i < k2; i++) x[r * k + k1 + i] = x2[r * k2 + i];
+    }
+    if (a->gamma) {
+        std::vector<double> g = wide(a->gamma);
+        for (size_t r = 0; r < rows; r++) {
+            const double d = std::sqrt(mean_square(&x[r * k], k) + a->eps);
+            for (size_t i = 0; i < k; i++) x[r * k + i] = x[r * k + i] / d * g[i];
+        }
+    }
+    std::vector<double> y = product(x, rows, k, a->w);
+    std::vector<double> bias = a->bias ? wide(a->bias) : std::vector<double>(n, 0.0);
+    for (size_t r = 0; r < rows; r++)
+        for (size_t j = 0; j < n; j++) y[r * n + j] = y[r * n + j] * a->scale + bias[j];
+    std::vector<size_t> od = dims_of(a->x);
+    od.back() = n;
+    *out = result(y, od);
+    return CG_OK;
+}
+
+int cg_block_residual(cg_backend *, cg_tensor *x, const cg_branch *br, size_t n, float eps, cg_tensor **out) {
+    Owned own{{x}};
+    for (size_t i = 0; i < n; i++) own.t.insert(own.t.end(), {br[i].y, br[i].w, br[i].gate, br[i].gate_bias, br[i].poly});
+    if (!x || !out || n > 2) return fail(CG_ERR_ARG, "bad argument");
+    const size_t width = x->dims[x->rank - 1], rows = numel(x) / width;
+    std::vector<double> o = wide(x);
+    for (size_t i = 0; i < n; i++) {
+        const cg_branch &b = br[i];
+        const size_t k = b.y->dims[b.y->rank - 1];
+        if (b.w->rank != 2 || b.w->dims[0] != width || b.w->dims[1] != k || numel(b.y) != rows * k || (b.gate && numel(b.gate) != rows * width))
+            return fail(CG_ERR_SHAPE, "block_residual: incompatible shapes");
+        std::vector<double> y = wide(b.y);
+        if (b.poly) {
+            std::vector<double> c = wide(b.poly);
+            for (size_t r = 0; r < rows; r++) {
+                double *z = &y[r * k], m[3] = {0, 0, 0};
+                for (size_t j = 0; j < k; j++)
+                    for (int e = 0; e < 3; e++) m[e] += std::pow(z[j], 2.0 * (e + 1));
+                for (int e = 0; e < 3; e++) m[e] = std::sqrt(m[e] / (double)k + eps);
+                for (size_t j = 0; j < k; j++) z[j] = c[0] * z[j] / m[0] + c[1] * z[j] * z[j] / m[1] + c[2] * z[j] * z[j] * z[j] / m[2] + c[3];
+            }
+        }
+        std::vector<double> p = product(y, rows, k, b.w), g, gb;
+        if (b.gate) g = wide(b.gate);
+        if (b.gate_bias) gb = wide(b.gate_bias);
+        for (size_t r = 0; r < rows; r++)
+            for (size_t j = 0; j < width; j++)
+                o[r * width + j] += p[r * width + j] * (b.gate ? sigmoid(g[r * width + j] + (b.gate_bias ? gb[j] : 0.0)) : 1.0);
+    }
+    *out = result(o, dims_of(x));
+    return CG_OK;
+}
+
+int cg_block_attention(cg_backend *, const cg_attention_args *a, cg_tensor **out, cg_tensor **k_out, cg_tensor **v_out) {
+    if (!a) return fail(CG_ERR_ARG, "null argument");
+    Owned own{{a->q, a->k, a->v, a->q_norm, a->k_norm, a->talk, a->k_cache, a->v_cache}};
+    if (!a->q || !a->k || !a->v || !a->k_cache || !a->v_cache || !out || !k_out || !v_out) return fail(CG_ERR_ARG, "null argument");
+    const size_t H = a->heads, G = a->kv_heads, D = a->dim, V = a->vdim, B = a->q->dims[0], S = a->q->dims[1], T = a->k_cache->dims[2], rep = H / G;
+    if (numel(a->q) != B * S * H * D || numel(a->k) != B * S * G * D || numel(a->v) != B * S * G * V || numel(a->k_cache) != B * G * T * D ||
+        numel(a->v_cache) != B * G * T * V)
+        return fail(CG_ERR_SHAPE, "block_attention: incompatible shapes");
+    const size_t need = a->window ? std::min(a->position, a->window - 1) : a->position;
+    if (T < need || T > a->position) return fail(CG_ERR_SHAPE, "block_attention: the cache does not hold the visible positions");
+    std::vector<double> q = wide(a->q), k = wide(a->k), v = wide(a->v), kc = wide(a->k_cache), vc = wide(a->v_cache);
+    auto norm = [&](std::vector<double> &x, size_t n, const cg_tensor *g) {
+        if (!g) return;
+        std::vector<double> w = wide(g);
+        for (size_t r = 0; r < B * S; r++) {
+            const double d = std::sqrt(mean_square(&x[r * n], n) + a->norm_eps);
+            for (size_t i = 0; i < n; i++) x[r * n + i] = x[r * n + i] / d * w[i];
+        }
+    };
+    norm(q, H * D, a->q_norm);
+    norm(k, G * D, a->k_norm);
+    std::vector<double> talk;
+    if (a->talk) talk = wide(a->talk);
+    const size_t all = T + S, keep = a->window ? std::min(all, a->window - 1) : all, first = a->position - T;
+    std::vector<double> o(B * S * H * V, 0.0), K(B * G * all * D), Vv(B * G * all * V);
+    for (size_t b = 0; b < B; b++)
+        for (size_t g = 0; g < G; g++)
+            for (size_t j = 0; j < all; j++) {
+                for (size_t d = 0; d < D; d++)
+                    K[((b * G + g) * all + j) * D + d] = j < T ? kc[((b * G + g) * T + j) * D + d] : (double)(float)k[((b * S + j - T) * G + g) * D + d];
+                for (size_t d = 0; d < V; d++)
+                    Vv[((b * G + g) * all + j) * V + d] = j < T ? vc[((b * G + g) * T + j) * V + d] : v[((b * S + j - T) * G + g) * V + d];
+            }
+    std::vector<double> w(H * all), mixed(H);
+    for (size_t b = 0; b < B; b++)
+        for (size_t s = 0; s < S; s++) {
+            const size_t p = a->position + s, lo = a->window && p + 1 > a->window ? p + 1 - a->window : 0;
+            const size_t j0 = lo > first ? lo - first : 0, j1 = T + s + 1;
+            const double temp = a->temp_every ? 1.0 + a->temp_coef * std::log(std::floor((double)(p + 1) / (double)a->temp_every) + 1.0) : 1.0;
+            for (size_t h = 0; h < H; h++) {
+                const double slope = a->distance_bias ? std::pow(2.0, -8.0 * (double)(h + 1) / (double)H) : 0.0;
+                double m = -std::numeric_limits<double>::infinity(), sum = 0;
+                for (size_t j = j0; j < j1; j++) {
+                    double x = 0;
+                    for (size_t d = 0; d < D; d++) x += q[((b * S + s) * H + h) * D + d] * K[((b * G + h / rep) * all + j) * D + d];
+                    x = x * temp * a->scale - slope * (double)(p - (first + j));
+                    w[h * all + j] = x;
+                    m = std::max(m, x);
+                }
+                for (size_t j = j0; j < j1; j++) sum += w[h * all + j] = std::exp(w[h * all + j] - m);
+                for (size_t j = j0; j < j1; j++) w[h * all + j] /= sum;
+            }
+            for (size_t j = j0; j < j1; j++) {
+                for (size_t h = 0; h < H; h++) {
+                    mixed[h] = a->talk ? 0.0 : w[h * all + j];
+                    if (a->talk)
+                        for (size_t g = 0; g < H; g++) mixed[h] += talk[h * H + g] * w[g * all + j];
+                }
+                for (size_t h = 0; h < H; h++)
+                    for (size_t d = 0; d < V; d++) o[((b * S + s) * H + h) * V + d] += mixed[h] * Vv[((b * G + h / rep) * all + j) * V + d];
+            }
+        }
+    auto tail = [&](const std::vector<double> &x, size_t n) {
+        std::vector<double> r(B * G * keep * n);
+        for (size_t g = 0; g < B * G; g++)
+            for (size_t j = 0; j < keep; j++)
+                for (size_t d = 0; d < n; d++) r[(g * keep + j) * n + d] = x[(g * all + all - keep + j) * n + d];
+        return result(r, {B, G, keep, n});
+    };
+    *out = result(o, {B, S, H * V});
+    *k_out = tail(K, D);
+    *v_out = tail(Vv, V);
+    return CG_OK;
+}
+
+int cg_block_channel_delta(cg_backend *, const cg_channel_delta_args *a, cg_tensor **out, cg_tensor **state_out, cg_tensor **conv_out) {
+    if (!a) return fail(CG_ERR_ARG, "null argument");
+    Owned own{{a->q, a->k, a->v, a->conv_q, a->conv_k, a->conv_v, a->beta, a->decay, a->decay_w, a->a_log, a->dt_bias, a->gate, a->gate_w,
+               a->norm, a->state, a->conv_state}};
+    for (const cg_tensor *t : own.t)
+        if (!t) return fail(CG_ERR_ARG, "null argument");
+    if (!out || !state_out || !conv_out) return fail(CG_ERR_ARG, "null argument");
+    const size_t H = a->heads, G = a->kv_heads, D = a->dim, V = a->vdim, B = a->q->dims[0], S = a->q->dims[1], rep = H / G;
+    const size_t taps = a->conv_q->dims[1], Cq = G * D, Cv = H * V, C = 2 * Cq + Cv, past = taps - 1;
+    if (numel(a->q) != B * S * Cq || numel(a->k) != B * S * Cq || numel(a->v) != B * S * Cv || numel(a->state) != B * H * D * V ||
+        numel(a->conv_state) != B * past * C || numel(a->beta) != B * S * H || a->decay_w->dims[0] != H * D || a->gate_w->dims[0] != H * V)
+        return fail(CG_ERR_SHAPE, "block_channel_delta: incompatible shapes");
+    std::vector<double> raw[3] = {wide(a->q), wide(a->k), wide(a->v)}, tap[3] = {wide(a->conv_q), wide(a->conv_k), wide(a->conv_v)};
+    std::vector<double> beta = wide(a->beta), a_log = wide(a->a_log), bias = wide(a->dt_bias), norm = wide(a->norm), st = wide(a->state),
+                        cs = wide(a->conv_state);
+    std::vector<double> dec = product(wide(a->decay), B * S, a->decay_w->dims[1], a->decay_w);
+    std::vector<double> gate = product(wide(a->gate), B * S, a->gate_w->dims[1], a->gate_w);
+    const size_t width[3] = {Cq, Cq, Cv}, at[3] = {0, Cq, 2 * Cq};
+    // inputs of the convolutions, the kept ones first
+    std::vector<double> in(B * (past + S) * C), act(B * S * C), o(B * S * H * V), keep(B * past * C);
+    for (size_t b = 0; b < B; b++)
+        for (size_t t = 0; t < past + S; t++)
+            for (int w = 0; w < 3; w++)
+                for (size_t c = 0; c < width[w]; c++)
+                    in[(b * (past + S) + t) * C + at[w] + c] =
+                        t < past ? cs[(b * past + t) * C + at[w] + c] : raw[w][(b * S + t - past) * width[w] + c];
+    for (size_t b = 0; b < B; b++)
+        for (size_t t = 0; t < S; t++)
+            for (int w = 0; w < 3; w++)
+                for (size_t c = 0; c < width[w]; c++) {
+                    double s = 0;
+                    for (size_t i = 0; i < taps; i++) s += in[(b * (past + S) + t + i) * C + at[w] + c] * tap[w][c * taps + i];
+                    act[(b * S + t) * C + at[w] + c] = s * sigmoid(s);
+                }
+    for (size_t b = 0; b < B; b++)
+        for (size_t t = 0; t < S; t++)
+            for (size_t h = 0; h < H; h++) {
+                const double *row = &act[(b * S + t) * C];
+                std::vector<double> q(row + h / rep * D, row + (h / rep + 1) * D), k(row + Cq + h / rep * D, row + Cq + (h / rep + 1) * D);
+                const double *v = row + 2 * Cq + h * V;
+                const double dq = std::sqrt(mean_square(q.data(), D) * (double)D + 1e-6) * std::sqrt((double)D),
+                             dk = std::sqrt(mean_square(k.data(), D) * (double)D + 1e-6);
+                for (size_t d = 0; d < D; d++) {
+                    q[d] /= dq;
+                    k[d] /= dk;
+                }
+                double *s = &st[(b * H + h) * D * V];
+                for (size_t d = 0; d < D; d++) {
+                    const double g = std::exp(-std::exp(a_log[h]) * softplus(dec[(b * S + t) * H * D + h * D + d] + bias[h * D + d]));
+                    for (size_t c = 0; c < V; c++) s[d * V + c] *= g;
+                }
+                const double bt = sigmoid(beta[(b * S + t) * H + h]);
+                std::vector<double> y(V, 0.0);
+                for (size_t c = 0; c < V; c++) {
+                    double read = 0;
+                    for (size_t d = 0; d < D; d++) read += s[d * V + c] * k[d];
+                    const double u = bt * (v[c] - read);
+                    for (size_t d = 0; d < D; d++) {
+                        s[d * V + c] += k[d] * u;
+                        y[c] += s[d * V + c] * q[d];
+                    }
+                }
+                const double m = std::sqrt(mean_square(y.data(), V) + a->eps);
+                for (size_t c = 0; c < V; c++)
+                    o[((b * S + t) * H + h) * V + c] = y[c] / m * norm[c] * sigmoid(gate[(b * S + t) * H * V + h * V + c]);
+            }
+    for (size_t b = 0; b < B; b++)
+        for (size_t t = 0; t < past; t++)
+            for (size_t c = 0; c < C; c++) keep[(b * past + t) * C + c] = in[(b * (past + S) + S + t) * C + c];
+    *out = result(o, {B, S, H * V});
+    *state_out = result(st, {B, H, D, V});
+    *conv_out = result(keep, {B, past, C});
+    return CG_OK;
+}
+
+} // extern "C"
