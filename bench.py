@@ -342,6 +342,84 @@ def other_config_line(config, steps=2, warmup=1):
     }
 
 
+# Loretar at the sizes of BASELINE configs 5 and 4: same width, depth (layer runs), heads, feed-forward, vocabulary, batch and
+# lengths; half of the layer runs attend (window 1024), half run the recurrence, and the middle half of the layers runs twice.
+def loretar_config(size):
+    from catgrad_amd.loretar import attention_layer, config_of, delta_layer
+
+    if size == 5:
+        width, ff, vocab, runs, at, de = 2048, 8192, 128256, 16, (32, 8, 64, 64), (16, 16, 128, 128)
+    else:
+        width, ff, vocab, runs, at, de = 1024, 3072, 151936, 28, (16, 8, 128, 128), (8, 8, 128, 128)
+    once = runs // 4                       # layers before and behind the loop together, and half as many layer runs in each pass
+    twice = (runs - 2 * once) // 2
+    layers = [attention_layer(*at, 1024, ff) if i % 2 else delta_layer(*de, ff) for i in range(2 * once + twice)]
+    return config_of(layers, vocab, width, loop={"start": once, "stop": once + twice, "times": 2})
+
+
+def measure_loretar(size, dtype, steps, warmup, seed=0):
+    """Prefill + greedy decode of Loretar at the size of a BASELINE configuration: the whole job, then the kernel classes of
+    one more pass (event records around every launch, untimed)."""
+    from catgrad_amd import _abi as A
+    from catgrad_amd.loretar import random_params
+    from catgrad_amd.runner import Session
+
+    B, S, T, _ = CONFIGS[size]
+    config = loretar_config(size)
+    sess = Session()
+    sess.load_config(config, dtype)
+    weights = 0
+    lp = config["loop"]
+    for name, w in random_params(config, seed, low_rank=64):
+        sess.set_param(name, w)
+        if w.ndim == 2 and not name.startswith(("embed", "loop.step")) and not name.endswith((".conv", ".talk")):
+            i = int(name[1:].split(".")[0]) if name[0] == "l" and name[1].isdigit() else None
+            n = lp["times"] if name == "loop.in" or (i is not None and lp["start"] <= i < lp["stop"]) else 1
+            weights += n * w.size
+    prompt = np.random.default_rng(seed).integers(0, config["vocab"], size=(B, S), dtype=np.uint32)
+    for _ in range(max(warmup, 1)):
+        sess.generate(prompt, steps=T, max_positions=S + T)
+    pp = tg = 0.0
+    for _ in range(steps):
+        tokens, st = sess.generate(prompt, steps=T, max_positions=S + T)
+        pp += st["prefill_s"] / steps
+        tg += st["decode_s"] / steps
+    classes = {"gemm": (A.K_GEMM_MFMA, "flop"), "streamed_products": (A.K_GEMM_SKINNY, "byte"), "attention": (A.K_ATTENTION, "flop"),
+               "recurrence": (A.K_RECURRENCE, "flop"), "row_kernels": (A.K_REDUCE, "byte"), "elementwise": (A.K_ELEMENTWISE, "byte")}
+    per_class = {}
+    for phase, n in (("prefill", 0), ("decode", 32)):
+        if phase == "decode":                # a prompt of one token: every launch is a decode launch
+            args = (prompt[:, :1], n)
+        else:
+            args = (prompt, 0)
+        for c, _ in classes.values():
+            sess.profile_enable(c, 1)
+            sess.profile_read(c, reset=True)
+        sess.generate(args[0], steps=args[1], max_positions=S + T)
+        sess.sync()
+        per_class[phase] = {}
+        for label, (c, unit) in classes.items():
+            k, ms, work = sess.profile_read(c)
+            sess.profile_enable(c, 0)
+            if k:
+                per_class[phase][label] = {"launches": k, "ms": round(ms, 3),
+                                           "rate": f"{work / (ms * 1e-3) / 1e12:.2f} T{unit}/s" if ms else None}
+    sess.close()
+    wb = 2 if dtype == "bfloat16" else 4
+    at = [l["mixer"] for l in config["layers"] if l["type"] == "attention"]
+    linear_flop = 2.0 * B * S * (weights - config["vocab"] * config["width"])
+    out = {
+        "workload": f"Loretar, {dtype}, batch {B}, prefill {S} + {T} decode steps, sizes of BASELINE config {size}",
+        "tok_s": round(B * (S + T) / (pp + tg), 1), "prefill_ms": round(pp * 1e3, 3), "prefill_tok_s": round(B * S / pp, 1),
+        "decode_ms_per_step": round(tg / T * 1e3, 4), "decode_tok_s": round(B * T / tg, 1),
+        "weight_bytes_per_step": int(weights * wb), "decode_hbm_frac_weights": round(weights * wb / (tg / T) / HBM_PEAK, 4),
+        "prefill_linear_flop": linear_flop,
+        "prefill_linear_peak_frac": round(linear_flop / pp / (2.5e15 if dtype == "bfloat16" else MFMA_F32_PEAK), 4),
+        "window": at[0]["mask"]["size"], "kernel_classes": per_class, "first_tokens": tokens[:2].tolist(),
+    }
+    return out
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -361,6 +439,9 @@ def main():
                     help="skip the short runs of BASELINE configs 3 and 4 that the default line carries as `other_configs`")
     ap.add_argument("--cpu-sample", type=int, nargs=3, default=None, metavar=("BATCH", "PREFILL", "DECODE"),
                     help="the CPU baseline's sample (default: the measured batch, prefill 8, 1 decode step)")
+    ap.add_argument("--loretar", choices=["float32", "bfloat16", "both"], default=None,
+                    help="only the Loretar model at the size of --config 5 or 4, beside that configuration's own model "
+                         "(one JSON line of their own)")
     ap.add_argument("--micro-only", action="store_true", help="only the op micro-benchmarks (one JSON line of their own)")
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="only run a strided copy of known size (268435456 B read + 268435456 B written per launch), "
@@ -385,6 +466,17 @@ def main():
 
     if args.micro_only:
         print(json.dumps({"micro": micro_bench()}))
+        return
+
+    if args.loretar:
+        if args.config == 3:
+            ap.error("--loretar takes --config 5 or 4")
+        line = {}
+        for dt in ("float32", "bfloat16") if args.loretar == "both" else (args.loretar,):
+            line[f"loretar_{dt}"] = measure_loretar(args.config, dt, args.steps, args.warmup, args.seed)
+            print(f"loretar {dt} measured", file=sys.stderr, flush=True)
+        line["closest_model"] = other_config_line(args.config, args.steps, args.warmup)
+        print(json.dumps({"loretar": line}))
         return
 
     import torch  # device-wide synchronisation around the timed region

@@ -294,6 +294,7 @@ int launch_attention(cg_backend *be, const AttentionPlan &p) {
     double pairs = 0.0; // visible (query, key) pairs
     for (uint32_t s = 0; s < p.S; s++) pairs += (double)std::min(p.window ? p.window : ~0u, p.cached + s + 1);
     ProfScope prof(be, CG_K_ATTENTION, pairs * p.B * p.heads * (2.0 * p.dim + 2.0 * p.vdim + (p.talk ? 2.0 * p.heads : 0.0)));
+    if (int rc = launch_attention_tiles(be, p, q); rc != kDeclined) return rc;
     // rows in parts that keep the scores within 64 MB
     const size_t per_row = (size_t)p.heads * nseg * (kSeg * 4 + sizeof(float2)) + (nseg > 1 ? (size_t)nseg * p.heads * p.vdim * 4 : 0);
     const uint32_t part = (uint32_t)std::max<size_t>(1, std::min<size_t>(std::min<size_t>(rows, 65535), (64u << 20) / per_row));

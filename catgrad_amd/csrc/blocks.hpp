@@ -77,6 +77,8 @@ struct AttentionPlan {
     float *out;                 // [B * S, heads * vdim]
 };
 int launch_attention(cg_backend *be, const AttentionPlan &p);
+// More than a few new tokens, on the matrix instructions (q: the prepared queries); kDeclined: sizes it does not take.
+int launch_attention_tiles(cg_backend *be, const AttentionPlan &p, const float *q);
 
 // ---- gated delta rule ------------------------------------------------------------------------------------------------
 struct DeltaPlan {
