@@ -2,8 +2,8 @@
 // v_mfma_f32_16x16x4.  Head mixing after the soft-max needs the finished weights of every head for the same (query, key),
 // so the row maxima and sums come first, from a launch of their own:
 //
-//   attention_row_stats_kernel  a wave per (16 query rows, up to 4 heads): maximum and sum of every row's scores
-//   attention_tiles_kernel      8 waves per 16 query rows, a few heads each: scores again, weights to LDS, mixed there over
+//   attention_row_stats_kernel  a wave per (16 query rows, one or two heads): maximum and sum of every row's scores
+//   attention_tiles_kernel      8 or 16 waves per 16 query rows, one or two heads each: scores again, weights to LDS, mixed there over
 //                               the heads (as the product talk . weights, a column per (query, key)), times the values.
 //                               The keys of a row tile may be cut over several workgroups: finished weights only add up.
 //
@@ -21,7 +21,7 @@ namespace {
 
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
-constexpr int kTileWaves = 8, kStatWaves = 4;
+constexpr int kStatWaves = 4;
 constexpr uint32_t kRowsT = 16, kKeysT = 32;
 constexpr uint32_t kRowPitch = kKeysT + 4;                // floats; 16-byte rows off each other's banks
 constexpr uint32_t kHeadPitch = kRowsT * kRowPitch + 4;   // heads four apart lie 16 banks apart
@@ -101,25 +101,23 @@ __global__ __launch_bounds__(kStatWaves * 64) void attention_row_stats_kernel(co
     }
     uint32_t lo, hi;
     tile_keys(p, at.s0, &lo, &hi);
-    for (uint32_t j0 = lo; j0 < hi; j0 += kKeysT) {
-        f32x4 k0[DT], k1[DT];
-        uint32_t have = ~0u;
+    const uint32_t g0 = h0 / rep;
+    const bool shared = min(h0 + HPW - 1, p.heads - 1) / rep == g0; // one kv head for all of this wave's heads
+    for (uint32_t j0 = lo; j0 < hi; j0 += 16) {
+        f32x4 k[DT];
+        load_k<DT>(p, at, g0, j0, k);
 #pragma unroll
         for (int i = 0; i < HPW; i++) {
-            const uint32_t g = min(h0 + i, p.heads - 1) / rep;
-            if (g != have) {
-                load_k<DT>(p, at, g, j0, k0);
-                load_k<DT>(p, at, g, j0 + 16, k1);
-                have = g;
-            }
-            const f32x4 a = scores<DT>(qf[i], k0), b = scores<DT>(qf[i], k1);
+            if (i > 0 && !shared) load_k<DT>(p, at, min(h0 + i, p.heads - 1) / rep, j0, k);
+            const f32x4 a = scores<DT>(qf[i], k);
 #pragma unroll
             for (int r = 0; r < 4; r++) {
-                const uint32_t s = at.s0 + 4 * at.lg + r;
-                const float x = visible_score(p, a[r], slope[i], s, j0 + at.li, hi), y = visible_score(p, b[r], slope[i], s, j0 + 16 + at.li, hi);
-                const float top = fmaxf(m[i][r], fmaxf(x, y));
-                l[i][r] = fmaf(l[i][r], exp_of(m[i][r] - top), exp_of(x - top) + exp_of(y - top));
-                m[i][r] = top;
+                const float x = visible_score(p, a[r], slope[i], at.s0 + 4 * at.lg + r, j0 + at.li, hi);
+                const float up = fmaxf(m[i][r], x);
+                // one of the two factors is 1
+                const float e = exp_of(fminf(m[i][r], x) - up);
+                l[i][r] = x > m[i][r] ? fmaf(l[i][r], e, 1.0f) : l[i][r] + e;
+                m[i][r] = up;
             }
         }
     }
@@ -140,11 +138,11 @@ __global__ __launch_bounds__(kStatWaves * 64) void attention_row_stats_kernel(co
 }
 
 // QREG: the queries stay in registers; else they are read again for every key tile.
-template <int HPW, int DT, bool QREG, bool TALK>
-__global__ __launch_bounds__(kTileWaves * 64) void attention_tiles_kernel(const AttentionPlan p, const float *__restrict__ q, const float2 *__restrict__ stats,
+template <int NW, int HPW, int DT, bool QREG, bool TALK>
+__global__ __launch_bounds__(NW * 64) void attention_tiles_kernel(const AttentionPlan p, const float *__restrict__ q, const float2 *__restrict__ stats,
                                                                           const uint32_t splits, float *__restrict__ dst) {
     extern __shared__ float lds[]; // weights [heads rounded up to 16][16][32]
-    constexpr int RT = (HPW * kTileWaves + 15) / 16; // row tiles of the mixing product
+    constexpr int RT = (HPW * NW + 15) / 16; // row tiles of the mixing product
     const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const uint32_t tile = blockIdx.x / splits, split = blockIdx.x - tile * splits;
     const Place at{blockIdx.y, tile * kRowsT, lane & 15, lane >> 4};
@@ -156,6 +154,8 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_tiles_kernel(const 
     const uint32_t end = hi;
     hi = min(hi, lo + (split + 1) * per * kKeysT);
     lo += split * per * kKeysT;
+
+    const bool shared = min(h0 + HPW - 1, p.heads - 1) / rep == min(h0, p.heads - 1) / rep; // one kv head for all of this wave's heads
 
     f32x4 qf[QREG ? HPW : 1][DT], out[HPW][DT], talk[TALK ? RT : 1][TALK ? RT : 1];
     float slope[HPW], top[HPW][4], scale[HPW][4];
@@ -183,38 +183,34 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_tiles_kernel(const 
                     const uint32_t h = 16 * a + at.li, g = 16 * c + 4 * at.lg + t;
                     talk[a][c][t] = h < p.heads && g < p.heads ? p.talk[(int64_t)h * p.heads + g] : 0.0f;
                 }
-        for (uint32_t i = p.heads * kHeadPitch + threadIdx.x; i < tiles16 * 16 * kHeadPitch; i += kTileWaves * 64) lds[i] = 0.0f; // heads that are not there
+        for (uint32_t i = p.heads * kHeadPitch + threadIdx.x; i < tiles16 * 16 * kHeadPitch; i += NW * 64) lds[i] = 0.0f; // heads that are not there
     }
     for (uint32_t j0 = lo; j0 < hi; j0 += kKeysT) {
         // scores -> weights of this wave's heads
-        f32x4 k0[DT], k1[DT];
-        uint32_t have = ~0u;
 #pragma unroll
-        for (int i = 0; i < HPW; i++) {
-            const uint32_t h = h0 + i;
-            if (h >= p.heads) break;
-            const uint32_t g = h / rep;
-            if (g != have) {
-                load_k<DT>(p, at, g, j0, k0);
-                load_k<DT>(p, at, g, j0 + 16, k1);
-                have = g;
-            }
-            if constexpr (!QREG) load_q<DT>(p, q, at, h, qf[0]);
-            const f32x4 a = scores<DT>(qf[QREG ? i : 0], k0), b = scores<DT>(qf[QREG ? i : 0], k1);
-            float *w = lds + h * kHeadPitch + at.li;
+        for (int half = 0; half < 2; half++) {
+            f32x4 k[DT];
+            if (h0 < p.heads) load_k<DT>(p, at, h0 / rep, j0 + 16 * half, k);
 #pragma unroll
-            for (int r = 0; r < 4; r++) {
-                const uint32_t s = at.s0 + 4 * at.lg + r;
-                w[(4 * at.lg + r) * kRowPitch] = exp_of(visible_score(p, a[r], slope[i], s, j0 + at.li, end) - top[i][r]) * scale[i][r];
-                w[(4 * at.lg + r) * kRowPitch + 16] = exp_of(visible_score(p, b[r], slope[i], s, j0 + 16 + at.li, end) - top[i][r]) * scale[i][r];
+            for (int i = 0; i < HPW; i++) {
+                const uint32_t h = h0 + i;
+                if (h >= p.heads) break;
+                if (i > 0 && !shared) load_k<DT>(p, at, h / rep, j0 + 16 * half, k);
+                if constexpr (!QREG) load_q<DT>(p, q, at, h, qf[0]);
+                const f32x4 a = scores<DT>(qf[QREG ? i : 0], k);
+                float *w = lds + h * kHeadPitch + 16 * half + at.li;
+#pragma unroll
+                for (int r = 0; r < 4; r++)
+                    w[(4 * at.lg + r) * kRowPitch] =
+                        exp_of(visible_score(p, a[r], slope[i], at.s0 + 4 * at.lg + r, j0 + 16 * half + at.li, end) - top[i][r]) * scale[i][r];
             }
         }
         if constexpr (TALK) {
             __syncthreads();
             // talk [heads, heads] . weights [heads, 512 columns]: a wave owns whole columns and writes them back in place
 #pragma unroll
-            for (uint32_t n = 0; n < kRowsT * kKeysT / 16 / kTileWaves; n++) {
-                const uint32_t col = (wave * (kRowsT * kKeysT / 16 / kTileWaves) + n) * 16; // of 512
+            for (uint32_t n = 0; n < kRowsT * kKeysT / 16 / NW; n++) {
+                const uint32_t col = (wave * (kRowsT * kKeysT / 16 / NW) + n) * 16; // of 512
                 float *w = lds + (col / kKeysT) * kRowPitch + (col % kKeysT) + at.li;
                 f32x4 acc[RT];
 #pragma unroll
@@ -240,7 +236,6 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_tiles_kernel(const 
             __syncthreads();
         }
         // weights . values
-        have = ~0u;
 #pragma unroll
         for (int half = 0; half < 2; half++) {
             float v[4][DT];
@@ -249,7 +244,7 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_tiles_kernel(const 
                 const uint32_t h = h0 + i;
                 if (h >= p.heads) break;
                 const uint32_t g = h / rep;
-                if (i == 0 || g != have) {
+                if (i == 0 || !shared) {
 #pragma unroll
                     for (int t = 0; t < 4; t++) {
                         const float *row = p.values + ((int64_t)at.b * p.kv_heads + g) * p.v_block +
@@ -257,7 +252,6 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_tiles_kernel(const 
 #pragma unroll
                         for (int c = 0; c < DT; c++) v[t][c] = 16 * c + at.li < p.vdim ? row[16 * c] : 0.0f;
                     }
-                    have = g;
                 }
                 const f32x4 w = *reinterpret_cast<const f32x4 *>(lds + h * kHeadPitch + at.li * kRowPitch + 16 * half + 4 * at.lg);
 #pragma unroll
@@ -302,29 +296,33 @@ __global__ __launch_bounds__(256) void attention_parts_kernel(const float *__res
     }
 }
 
-template <int HPW, int DT, bool QREG> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, float2 *stats, uint32_t splits, float *dst) {
-    const uint32_t tiles = (p.S + kRowsT - 1) / kRowsT;
-    constexpr int SH = QREG ? HPW : 1; // heads of a stats wave
-    hipLaunchKernelGGL((attention_row_stats_kernel<SH, DT>), dim3(tiles, (p.heads + SH * kStatWaves - 1) / (SH * kStatWaves), p.B), dim3(kStatWaves * 64), 0,
-                       be->stream, p, q, stats);
+template <int NW, int HPW, int DT, bool QREG> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, float2 *stats, uint32_t splits, float *dst) {
+    const uint32_t tiles = (p.S + kRowsT - 1) / kRowsT, rep = p.heads / p.kv_heads;
+    // heads of a stats wave: two that share their keys, or one
+    if (rep % 2 == 0 && DT <= 4)
+        hipLaunchKernelGGL((attention_row_stats_kernel<2, DT>), dim3(tiles, (p.heads + 2 * kStatWaves - 1) / (2 * kStatWaves), p.B), dim3(kStatWaves * 64), 0,
+                           be->stream, p, q, stats);
+    else
+        hipLaunchKernelGGL((attention_row_stats_kernel<1, DT>), dim3(tiles, (p.heads + kStatWaves - 1) / kStatWaves, p.B), dim3(kStatWaves * 64), 0, be->stream, p,
+                           q, stats);
     const size_t lds = (size_t)(p.heads + 15) / 16 * 16 * kHeadPitch * 4;
-    const void *f = p.talk ? reinterpret_cast<const void *>(&attention_tiles_kernel<HPW, DT, QREG, true>)
-                           : reinterpret_cast<const void *>(&attention_tiles_kernel<HPW, DT, QREG, false>);
+    const void *f = p.talk ? reinterpret_cast<const void *>(&attention_tiles_kernel<NW, HPW, DT, QREG, true>)
+                           : reinterpret_cast<const void *>(&attention_tiles_kernel<NW, HPW, DT, QREG, false>);
     if (lds > (64 << 10)) {
         const hipError_t e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return hip_fail(e, "hipFuncSetAttribute");
     }
     const dim3 grid(tiles * splits, p.B);
-    if (p.talk) hipLaunchKernelGGL((attention_tiles_kernel<HPW, DT, QREG, true>), grid, dim3(kTileWaves * 64), lds, be->stream, p, q, stats, splits, dst);
-    else hipLaunchKernelGGL((attention_tiles_kernel<HPW, DT, QREG, false>), grid, dim3(kTileWaves * 64), lds, be->stream, p, q, stats, splits, dst);
+    if (p.talk) hipLaunchKernelGGL((attention_tiles_kernel<NW, HPW, DT, QREG, true>), grid, dim3(NW * 64), lds, be->stream, p, q, stats, splits, dst);
+    else hipLaunchKernelGGL((attention_tiles_kernel<NW, HPW, DT, QREG, false>), grid, dim3(NW * 64), lds, be->stream, p, q, stats, splits, dst);
     return CG_OK;
 }
-template <int HPW> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, float2 *stats, uint32_t splits, float *dst) {
+template <int NW, int HPW> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, float2 *stats, uint32_t splits, float *dst) {
     const uint32_t d = std::max(p.dim, p.vdim);
-    if (d <= 32) return run_tiles<HPW, 2, true>(be, p, q, stats, splits, dst);
-    if (d <= 64) return run_tiles<HPW, 4, true>(be, p, q, stats, splits, dst);
-    if (d <= 96) return run_tiles<HPW, 6, (HPW < 4)>(be, p, q, stats, splits, dst);
-    return run_tiles<HPW, 8, (HPW < 4)>(be, p, q, stats, splits, dst);
+    if (d <= 32) return run_tiles<NW, HPW, 2, true>(be, p, q, stats, splits, dst);
+    if (d <= 64) return run_tiles<NW, HPW, 4, true>(be, p, q, stats, splits, dst);
+    if (d <= 96) return run_tiles<NW, HPW, 6, (HPW < 2)>(be, p, q, stats, splits, dst);
+    return run_tiles<NW, HPW, 8, (HPW < 2)>(be, p, q, stats, splits, dst);
 }
 
 } // namespace
@@ -343,9 +341,9 @@ int launch_attention_tiles(cg_backend *be, const AttentionPlan &p, const float *
     float *dst = splits > 1 ? static_cast<float *>(parts) : p.out;
     float2 *stats = static_cast<float2 *>(mem);
     if (!rc)
-        rc = p.heads <= 8    ? run_tiles<1>(be, p, q, stats, splits, dst)
-             : p.heads <= 16 ? run_tiles<2>(be, p, q, stats, splits, dst)
-                             : run_tiles<4>(be, p, q, stats, splits, dst);
+        rc = p.heads <= 8    ? run_tiles<8, 1>(be, p, q, stats, splits, dst)
+             : p.heads <= 16 ? run_tiles<16, 1>(be, p, q, stats, splits, dst)
+                             : run_tiles<16, 2>(be, p, q, stats, splits, dst);
     if (!rc && splits > 1)
         hipLaunchKernelGGL(attention_parts_kernel, dim3((uint32_t)((n + 1023) / 1024)), dim3(256), 0, be->stream, dst, splits, n, p.out);
     if (mem) be->pool.free(mem, mem_cls);

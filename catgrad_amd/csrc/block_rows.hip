@@ -3,6 +3,8 @@
 #include "blocks.hpp"
 #include "device_utils.hpp"
 
+#include <algorithm>
+
 namespace cg {
 namespace {
 
@@ -240,6 +242,270 @@ __global__ __launch_bounds__(kThreads) void few_rows_residual_kernel(const Rows 
     }
 }
 
+// ---- at most four rows -----------------------------------------------------------------------------------------------
+// The 4x4x4 (bfloat16) and 4x4x1 (f32) matrix instructions multiply 16 independent blocks of four columns and four rows:
+// lane (block = lane / 4, j = lane % 4) supplies weights of column n0 + j and activations of row j at the block's values of
+// k, 16 bytes of weights at a time, and finds rows 0 .. 3 ... of its column j's sums in its registers — the sums over the
+// blocks, and over the waves of the workgroup, which take k in turn, come at the end.  Nothing is staged and nothing waits:
+// the factors of a norm are the same for a whole row, so they are applied to the sums, and the row sums they need are formed
+// from what a wave loads anyway.  The polynomial norm is linear in z, z^2, z^3 and 1: four sums instead of one.
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef short bf16x4 __attribute__((ext_vector_type(4)));
+typedef __bf16 bfx2 __attribute__((ext_vector_type(2)));
+
+template <bool BF16> struct Frag { // a lane's weights, or its activations in the form the instruction takes
+    static constexpr uint32_t W = BF16 ? 8 : 4; // values of k
+    uint32_t v[4];
+};
+
+template <bool BF16> __device__ __forceinline__ Frag<BF16> load_weights(const Weight &w, uint32_t n, uint32_t k) {
+    typedef uint32_t u4 __attribute__((ext_vector_type(4)));
+    Frag<BF16> f;
+    u4 t = {0, 0, 0, 0};
+    if (k < w.k) t = __builtin_nontemporal_load(reinterpret_cast<const u4 *>(static_cast<const char *>(w.p) + ((int64_t)n * w.pitch + k) * (BF16 ? 2 : 4)));
+#pragma unroll
+    for (int i = 0; i < 4; i++) f.v[i] = t[i];
+    return f;
+}
+template <bool BF16> __device__ __forceinline__ Frag<BF16> pack(const float (&x)[Frag<BF16>::W]) {
+    Frag<BF16> f;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        if constexpr (BF16) {
+            typedef float f2 __attribute__((ext_vector_type(2)));
+            const f2 t = {x[2 * i], x[2 * i + 1]};
+            f.v[i] = __builtin_bit_cast(uint32_t, __builtin_convertvector(t, bfx2));
+        } else {
+            f.v[i] = asu(x[i]);
+        }
+    }
+    return f;
+}
+template <bool BF16> __device__ __forceinline__ f32x4 multiply(const Frag<BF16> &w, const Frag<BF16> &x, f32x4 acc) {
+    if constexpr (BF16) {
+#pragma unroll
+        for (int i = 0; i < 4; i += 2) {
+            typedef uint32_t u2 __attribute__((ext_vector_type(2)));
+            const u2 a = {w.v[i], w.v[i + 1]}, b = {x.v[i], x.v[i + 1]};
+            acc = __builtin_amdgcn_mfma_f32_4x4x4bf16_1k(__builtin_bit_cast(bf16x4, a), __builtin_bit_cast(bf16x4, b), acc, 0, 0, 0);
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; i++) acc = __builtin_amdgcn_mfma_f32_4x4x1f32(asf(w.v[i]), asf(x.v[i]), acc, 0, 0, 0);
+    }
+    return acc;
+}
+// W consecutive activations of row r (zeros behind the last column and for rows that are not there)
+template <bool BF16> __device__ __forceinline__ void load_input(const ProductInput &in, uint32_t r, bool there, uint32_t k, float (&x)[Frag<BF16>::W]) {
+#pragma unroll
+    for (uint32_t i = 0; i < Frag<BF16>::W; i += 4) {
+        f32x4 t = {0.0f, 0.0f, 0.0f, 0.0f};
+        if (there && k + i < in.k)
+            t = k + i < in.k1 ? *reinterpret_cast<const f32x4 *>(in.x.p + (int64_t)r * in.x.pitch + k + i)
+                              : *reinterpret_cast<const f32x4 *>(in.x2.p + (int64_t)r * in.x2.pitch + (k + i - in.k1));
+#pragma unroll
+        for (int j = 0; j < 4; j++) x[i + j] = t[j];
+    }
+}
+// over the 16 lanes that share j
+__device__ __forceinline__ float blocks_sum(float v) {
+#pragma unroll
+    for (int d = 4; d < 64; d <<= 1) v += __shfl_xor(v, d, 64);
+    return v;
+}
+
+// A workgroup holds all of its waves' activations in registers (STEPS of 64 lanes' worth each) and walks column groups.
+template <bool BF16, int STEPS, int WAVES>
+__global__ __launch_bounds__(WAVES * 64) void four_rows_linear_kernel(const ProductInput in, const uint32_t rows, const Weight w, const uint32_t iters,
+                                                                      const float *__restrict__ bias, const float scale, float *__restrict__ out) {
+    constexpr uint32_t W = Frag<BF16>::W, SPAN = 16 * W;
+    __shared__ f32x4 sums[2][WAVES][4];
+    __shared__ float squares[WAVES][4];
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, j = lane & 3, k0 = wave * SPAN + (lane >> 2) * W;
+    const uint32_t g0 = blockIdx.x * iters, groups = (w.n + 3) / 4, g1 = min(g0 + iters, groups);
+    Frag<BF16> wt[STEPS];
+    auto ask = [&](uint32_t g) {
+        const uint32_t n = min(g * 4 + j, w.n - 1);
+#pragma unroll
+        for (int s = 0; s < STEPS; s++) wt[s] = load_weights<BF16>(w, n, k0 + s * WAVES * SPAN);
+    };
+    ask(g0);
+    Frag<BF16> x[STEPS];
+    float ss = 0.0f;
+#pragma unroll
+    for (int s = 0; s < STEPS; s++) {
+        const uint32_t k = k0 + s * WAVES * SPAN;
+        float z[W];
+        load_input<BF16>(in, j, j < rows, k, z);
+        if (in.gamma) {
+#pragma unroll
+            for (uint32_t i = 0; i < W; i++) {
+                ss = fmaf(z[i], z[i], ss);
+                z[i] = k + i < in.k ? z[i] * in.gamma[k + i] : 0.0f;
+            }
+        }
+        x[s] = pack<BF16>(z);
+    }
+    if (in.gamma) {
+        ss = blocks_sum(ss);
+        if (lane < 4) squares[wave][lane] = ss;
+    }
+    float rstd = scale;
+    for (uint32_t g = g0; g < g1; g++) {
+        f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+        for (int s = 0; s < STEPS; s++) acc = multiply<BF16>(wt[s], x[s], acc);
+        if (g + 1 < g1) ask(g + 1);
+#pragma unroll
+        for (int r = 0; r < 4; r++) acc[r] = blocks_sum(acc[r]);
+        f32x4(&mine)[WAVES][4] = sums[g & 1];
+        if (lane < 4) mine[wave][lane] = acc;
+        __syncthreads(); // (two buffers: the next group's sums do not wait for these to be read)
+        if (wave == (g - g0) % WAVES && lane < 16) { // lane (j, r): row j, column r of the group
+            const uint32_t m = lane >> 2, c = lane & 3, n = g * 4 + c;
+            float s = 0.0f;
+#pragma unroll
+            for (int i = 0; i < WAVES; i++) s += mine[i][m][c];
+            if (in.gamma) {
+                float q = 0.0f;
+#pragma unroll
+                for (int i = 0; i < WAVES; i++) q += squares[i][m];
+                rstd = scale / sqrtf(q / (float)in.k + in.eps);
+            }
+            if (m < rows && n < w.n) out[(int64_t)m * w.n + n] = s * rstd + (bias ? bias[n] : 0.0f);
+        }
+    }
+}
+
+// One branch of the residual sum: the sums of the polynomial's terms (or the plain sum) and the row sums they are scaled by.
+template <int NG> struct BranchSums {
+    f32x4 acc[NG][4]; // of z, z^2, z^3, 1
+    float m[3];
+};
+template <bool BF16, int NG, int WAVES, bool POLY>
+__device__ __forceinline__ void walk_branch(const ResidualBranch &b, uint32_t rows, uint32_t width, uint32_t n0, BranchSums<NG> &o) {
+    constexpr uint32_t W = Frag<BF16>::W, SPAN = 16 * W, STEP = WAVES * SPAN;
+    constexpr int AHEAD = 4;
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, j = lane & 3;
+    uint32_t n[NG];
+#pragma unroll
+    for (int g = 0; g < NG; g++) n[g] = min(n0 + 4 * g + j, width - 1);
+    float one[W];
+#pragma unroll
+    for (uint32_t i = 0; i < W; i++) one[i] = 1.0f;
+    const Frag<BF16> ones = pack<BF16>(one);
+    for (uint32_t base = wave * SPAN; base < b.w.k; base += AHEAD * STEP) { // (the same trips for every lane: the instruction does not mask)
+        const uint32_t k0 = base + (lane >> 2) * W;
+        Frag<BF16> wt[AHEAD][NG];
+        float z[AHEAD][W];
+#pragma unroll
+        for (int a = 0; a < AHEAD; a++)
+#pragma unroll
+            for (int g = 0; g < NG; g++) wt[a][g] = load_weights<BF16>(b.w, n[g], k0 + a * STEP);
+#pragma unroll
+        for (int a = 0; a < AHEAD; a++) load_input<BF16>(b.in, j, j < rows, k0 + a * STEP, z[a]);
+#pragma unroll
+        for (int a = 0; a < AHEAD; a++) {
+            Frag<BF16> x = pack<BF16>(z[a]);
+#pragma unroll
+            for (int g = 0; g < NG; g++) o.acc[g][0] = multiply<BF16>(wt[a][g], x, o.acc[g][0]);
+            if constexpr (POLY) {
+                float p[W], c[W];
+#pragma unroll
+                for (uint32_t i = 0; i < W; i++) {
+                    p[i] = z[a][i] * z[a][i];
+                    c[i] = p[i] * z[a][i];
+                    o.m[0] += p[i];
+                    o.m[1] = fmaf(p[i], p[i], o.m[1]);
+                    o.m[2] = fmaf(c[i], c[i], o.m[2]);
+                }
+                x = pack<BF16>(p);
+#pragma unroll
+                for (int g = 0; g < NG; g++) o.acc[g][1] = multiply<BF16>(wt[a][g], x, o.acc[g][1]);
+                x = pack<BF16>(c);
+#pragma unroll
+                for (int g = 0; g < NG; g++) o.acc[g][2] = multiply<BF16>(wt[a][g], x, o.acc[g][2]);
+#pragma unroll
+                for (int g = 0; g < NG; g++) o.acc[g][3] = multiply<BF16>(wt[a][g], ones, o.acc[g][3]);
+            }
+        }
+    }
+}
+
+// NG groups of four columns per workgroup.  POLY: branch 1 (or the only one) goes through the polynomial norm.
+template <bool BF16, int NB, int NG, int WAVES, bool POLY0, bool POLY1>
+__global__ __launch_bounds__(WAVES * 64) void four_rows_residual_kernel(const Rows x, const ResidualBranch b0, const ResidualBranch b1, const uint32_t rows,
+                                                                        const uint32_t width, float *__restrict__ out) {
+    __shared__ f32x4 sums[NB][WAVES][NG][4][4]; // [branch][wave][group][term][row]
+    __shared__ float squares[NB][WAVES][3][4];
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, n0 = blockIdx.x * NG * 4;
+    BranchSums<NG> s[NB];
+#pragma unroll
+    for (int b = 0; b < NB; b++) {
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int g = 0; g < NG; g++) s[b].acc[g][t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+        s[b].m[0] = s[b].m[1] = s[b].m[2] = 0.0f;
+    }
+    // thread e of the first 16 * NG: row m, column n; what it needs besides the sums is asked for first
+    const uint32_t e = threadIdx.x, m = e / (4 * NG), c = e % (4 * NG), n = min(n0 + c, width - 1), mr = min(m, rows - 1);
+    float xs = 0.0f, gate[NB] = {};
+    if (e < 16 * NG) {
+        xs = x.p[(int64_t)mr * x.pitch + n];
+        if (b0.gate.p) gate[0] = b0.gate.p[(int64_t)mr * b0.gate.pitch + n] + (b0.gate_bias ? b0.gate_bias[n] : 0.0f);
+        if (NB > 1 && b1.gate.p) gate[NB - 1] = b1.gate.p[(int64_t)mr * b1.gate.pitch + n] + (b1.gate_bias ? b1.gate_bias[n] : 0.0f);
+    }
+    walk_branch<BF16, NG, WAVES, POLY0>(b0, rows, width, n0, s[0]);
+    if (NB > 1) walk_branch<BF16, NG, WAVES, POLY1>(b1, rows, width, n0, s[NB - 1]);
+#pragma unroll
+    for (int b = 0; b < NB; b++) {
+        const bool poly = b == 0 ? POLY0 : POLY1;
+#pragma unroll
+        for (int t = 0; t < 4; t++) {
+            if (t > 0 && !poly) break;
+#pragma unroll
+            for (int g = 0; g < NG; g++) {
+                f32x4 v;
+#pragma unroll
+                for (int r = 0; r < 4; r++) v[r] = blocks_sum(s[b].acc[g][t][r]);
+                if (lane < 4) sums[b][wave][g][t][lane] = v;
+            }
+            if (t < 3 && poly) {
+                const float q = blocks_sum(s[b].m[t]);
+                if (lane < 4) squares[b][wave][t][lane] = q;
+            }
+        }
+    }
+    __syncthreads();
+    if (e >= 16 * NG || m >= rows || n0 + c >= width) return;
+#pragma unroll
+    for (int b = 0; b < NB; b++) {
+        const ResidualBranch &br = b == 0 ? b0 : b1;
+        const bool poly = b == 0 ? POLY0 : POLY1;
+        float y = 0.0f;
+#pragma unroll
+        for (int t = 0; t < 4; t++) {
+            if (t > 0 && !poly) break;
+            float v = 0.0f, q = 0.0f;
+#pragma unroll
+            for (int i = 0; i < WAVES; i++) v += sums[b][i][c / 4][t][m][c % 4];
+            if (poly) {
+                if (t < 3) {
+#pragma unroll
+                    for (int i = 0; i < WAVES; i++) q += squares[b][i][t][m];
+                    v *= br.in.poly[t] / sqrtf(q / (float)br.in.k + br.in.eps);
+                } else {
+                    v *= br.in.poly[3];
+                }
+            }
+            y += v;
+        }
+        xs += br.gate.p ? sigmoid(gate[b]) * y : y;
+    }
+    out[(int64_t)m * width + n0 + c] = xs;
+}
+
 // ---- many rows -------------------------------------------------------------------------------------------------------
 __device__ __forceinline__ uint32_t round_bf16(float v) { return asu(v) + 0x7FFFu + ((asu(v) >> 16) & 1u); } // (bits above 15 hold the pattern)
 
@@ -408,7 +674,37 @@ int few_rows_residual(cg_backend *be, const Rows &x, const ResidualBranch *br, u
 
 } // namespace
 
+// The kernels for at most four rows read activations and weights 16 bytes at a time.
+static bool four_rows(const ProductInput &in, uint32_t rows, const Weight &w) {
+    const uint32_t vw = w.fmt == kFmtBF16 ? 8 : 4;
+    return rows <= 4 && vector_rows(w) && in.k1 % vw == 0 && in.k % vw == 0 && in.x.pitch % 4 == 0 && aligned16(in.x.p) &&
+           (!in.x2.p || (in.x2.pitch % 4 == 0 && aligned16(in.x2.p)));
+}
+
+template <bool BF16, int STEPS, int WAVES>
+static void four_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows, const Weight &w, const float *bias, float scale, float *out) {
+    const uint32_t groups = (w.n + 3) / 4, resident = (uint32_t)be->compute_units * 8; // workgroups that walk several groups when there are many
+    const uint32_t iters = std::max(1u, (groups + resident - 1) / resident);
+    hipLaunchKernelGGL((four_rows_linear_kernel<BF16, STEPS, WAVES>), dim3((groups + iters - 1) / iters), dim3(WAVES * 64), 0, be->stream, in, rows, w, iters,
+                       bias, scale, out);
+}
+
 int launch_few_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows, const Weight &w, const float *bias, float scale, float *out) {
+    if (four_rows(in, rows, w) && !in.poly && in.k <= (w.fmt == kFmtBF16 ? 8192u : 4096u)) {
+        const bool bf16 = w.fmt == kFmtBF16;
+        ProfScope prof(be, CG_K_GEMM_SKINNY, (double)w.n * w.k * (bf16 ? 2.0 : 4.0) + 4.0 * rows * ((double)in.k + w.n));
+        const uint32_t steps = (in.k + (bf16 ? 511 : 255)) / (bf16 ? 512 : 256); // of a workgroup of four waves
+#define CG_FOUR(BF)                                                                              \
+    if (steps <= 1) four_rows_linear<BF, 1, 4>(be, in, rows, w, bias, scale, out);               \
+    else if (steps <= 2) four_rows_linear<BF, 2, 4>(be, in, rows, w, bias, scale, out);          \
+    else if (steps <= 4) four_rows_linear<BF, 4, 4>(be, in, rows, w, bias, scale, out);          \
+    else if (steps <= 8) four_rows_linear<BF, 4, 8>(be, in, rows, w, bias, scale, out);          \
+    else four_rows_linear<BF, 8, 8>(be, in, rows, w, bias, scale, out)
+        if (bf16) { CG_FOUR(true); }
+        else { CG_FOUR(false); }
+#undef CG_FOUR
+        return launched("four_rows_linear");
+    }
     const uint32_t m = few_rows_slots(rows, (uint64_t)staged_pitch(in.k) * 4);
     if (!m) return fail(CG_ERR_ARG, "internal error: too many rows for the streaming product");
     const bool bf16 = w.fmt == kFmtBF16, vec = vector_rows(w);
@@ -434,7 +730,42 @@ int launch_few_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows
     return rc ? rc : launched("few_rows_linear");
 }
 
+template <bool BF16, int NG> static bool four_rows_residual(cg_backend *be, const Rows &x, const ResidualBranch *br, int n, uint32_t rows, uint32_t width, float *out) {
+    constexpr int WAVES = 8;
+    const dim3 grid((width + 4 * NG - 1) / (4 * NG)), block(WAVES * 64);
+    const bool p0 = br[0].in.poly != nullptr, p1 = n > 1 && br[1].in.poly != nullptr;
+    const ResidualBranch &b1 = br[n > 1 ? 1 : 0];
+    hipStream_t s = be->stream;
+    if (n == 2 && !p0 && p1) hipLaunchKernelGGL((four_rows_residual_kernel<BF16, 2, NG, WAVES, false, true>), grid, block, 0, s, x, br[0], b1, rows, width, out);
+    else if (n == 2 && !p0 && !p1) hipLaunchKernelGGL((four_rows_residual_kernel<BF16, 2, NG, WAVES, false, false>), grid, block, 0, s, x, br[0], b1, rows, width, out);
+    else if (n == 1 && p0) hipLaunchKernelGGL((four_rows_residual_kernel<BF16, 1, NG, WAVES, true, false>), grid, block, 0, s, x, br[0], b1, rows, width, out);
+    else if (n == 1) hipLaunchKernelGGL((four_rows_residual_kernel<BF16, 1, NG, WAVES, false, false>), grid, block, 0, s, x, br[0], b1, rows, width, out);
+    else return false;
+    return true;
+}
+
+bool takes_few_rows_residual(const ResidualBranch *br, int n, uint32_t rows) {
+    uint64_t per_row = 0;
+    bool four = n > 0;
+    for (int i = 0; i < n; i++) {
+        per_row += (uint64_t)staged_pitch(br[i].in.k) * 4;
+        four = four && four_rows(br[i].in, rows, br[i].w);
+    }
+    return n > 0 && (four || few_rows_slots(rows, per_row));
+}
+
 int launch_few_rows_residual(cg_backend *be, const Rows &x, const ResidualBranch *br, int n, uint32_t rows, uint32_t width, float *out) {
+    bool four = n > 0 && (n == 1 || br[0].w.fmt == br[1].w.fmt) && !(n == 2 && br[0].in.poly);
+    for (int i = 0; i < n; i++) four = four && four_rows(br[i].in, rows, br[i].w);
+    if (four) {
+        double work = 8.0 * rows * width;
+        for (int i = 0; i < n; i++) work += (double)br[i].w.n * br[i].w.k * (br[i].w.fmt == kFmtBF16 ? 2.0 : 4.0) + 4.0 * rows * ((double)br[i].in.k + width);
+        ProfScope prof(be, CG_K_GEMM_SKINNY, work);
+        const bool bf16 = br[0].w.fmt == kFmtBF16, two = width >= (uint32_t)be->compute_units * 8;
+        if (two) bf16 ? four_rows_residual<true, 2>(be, x, br, n, rows, width, out) : four_rows_residual<false, 2>(be, x, br, n, rows, width, out);
+        else bf16 ? four_rows_residual<true, 1>(be, x, br, n, rows, width, out) : four_rows_residual<false, 1>(be, x, br, n, rows, width, out);
+        return launched("four_rows_residual");
+    }
     uint64_t per_row = 0;
     double bytes = 8.0 * rows * width;
     bool vec = true;

@@ -347,7 +347,6 @@ int cg_block_residual(cg_backend *b, cg_tensor *x, const cg_branch *br, size_t n
     cg_tensor *wv[2] = {nullptr, nullptr};
     Rows xr;
     if (int rc = rows_of(b, h, x, rows, width, &xr, "block_residual x")) return rc;
-    uint64_t lds = 0;
     for (size_t i = 0; i < n; i++) {
         if (!br[i].y || !br[i].w || br[i].y->rank < 1) return fail(CG_ERR_ARG, "block_residual: null argument");
         const int64_t K = br[i].y->dims[br[i].y->rank - 1];
@@ -363,14 +362,13 @@ int cg_block_residual(cg_backend *b, cg_tensor *x, const cg_branch *br, size_t n
             if (int rc = rows_of(b, h, br[i].gate, rows, width, &r[i].gate, "block_residual gate")) return rc;
         if (br[i].gate_bias)
             if (int rc = dense_of(b, h, br[i].gate_bias, width, &r[i].gate_bias, "block_residual gate bias")) return rc;
-        lds += (uint64_t)staged_pitch((uint32_t)K) * 4;
     }
     cg_tensor *o = nullptr;
     if (int rc = new_dense(b, CG_F32, x->dims, x->rank, &o)) return rc;
     int rc = CG_OK;
     if (rows > 0 && width > 0) {
         float *y = static_cast<float *>(o->buf->ptr);
-        if (n > 0 && few_rows_slots((uint64_t)rows, lds)) {
+        if (takes_few_rows_residual(r, (int)n, (uint32_t)rows)) {
             rc = launch_few_rows_residual(b, xr, r, (int)n, (uint32_t)rows, (uint32_t)width, y);
         } else {
             Scratch tmp(b);

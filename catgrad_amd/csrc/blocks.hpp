@@ -47,6 +47,8 @@ struct ResidualBranch {
     Rows gate; // p null: none
     const float *gate_bias = nullptr;
 };
+// Whether launch_few_rows_residual takes these branches (one of them with 16-byte rows at most four rows deep, or LDS for all)
+bool takes_few_rows_residual(const ResidualBranch *br, int n, uint32_t rows);
 int launch_few_rows_residual(cg_backend *be, const Rows &x, const ResidualBranch *br, int n, uint32_t rows, uint32_t width, float *out);
 
 // dst[r, 0 .. k) = the product input of row r, as 32-bit words (bf16: rounded to it first) or bfloat16 patterns
