@@ -1,8 +1,10 @@
 // Causal attention of new tokens behind a cache, with a window, a distance bias, a query temperature, norms over whole
 // projections and head mixing after the soft-max (cg_block_attention).
 //
-//   attention_prepare_kernel  a workgroup per token: the query row normed and scaled, the key and value rows into the cache
-//   attention_scores_kernel   a workgroup per (token, kv head, 128 keys): scores, and their maximum and sum per head
+//   attention_prepare_kernel  more than a few new tokens, a workgroup per token: the query row normed and scaled, the key and
+//                             value rows into the cache (then block_attention_tiles.hip, for the sizes it takes)
+//   attention_scores_kernel   a workgroup per (token, kv head, 128 keys): scores, and their maximum and sum per head; with a
+//                             few new tokens the preparation as well
 //   attention_mix_kernel      the same split: soft-max weights of every head, mixed, times the values of the kv head
 //   attention_sum_kernel      partial results of a token's key segments added up
 #include "blocks.hpp"
@@ -71,42 +73,94 @@ __global__ __launch_bounds__(kThreads) void attention_prepare_kernel(const Atten
     }
 }
 
+// n consecutive floats of a row, 16 bytes at a time where they lie so
+__device__ __forceinline__ float row_squares(const float *__restrict__ x, uint32_t n) {
+    float m = 0.0f;
+    if (n % 4 == 0 && (reinterpret_cast<uintptr_t>(x) & 15) == 0) {
+#pragma unroll 4
+        for (uint32_t i = threadIdx.x; i < n / 4; i += kThreads) {
+            const float4 v = reinterpret_cast<const float4 *>(x)[i];
+            m = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, m))));
+        }
+    } else {
+        for (uint32_t i = threadIdx.x; i < n; i += kThreads) m = fmaf(x[i], x[i], m);
+    }
+    return m;
+}
+
 // Four lanes share a key; REP query heads of the kv head at a time (blockIdx.y = kv head and which of its head groups).
-template <int REP, int VW>
+// FRESH (a few new tokens): the queries and the new keys are normed here, from the projections as they are, and a token's
+// own workgroups of the last segment write its key and value rows into the cache; the cache is not read at new positions.
+template <int REP, int VW, bool FRESH>
 __global__ __launch_bounds__(kThreads) void attention_scores_kernel(const AttentionPlan p, const float *__restrict__ q, const uint32_t row0, const uint32_t nseg,
                                                                     float *__restrict__ scores, float2 *__restrict__ stats) {
-    extern __shared__ float lds[]; // [REP][dim] queries, then [REP][kSeg] scores
+    extern __shared__ float lds[]; // [REP][dim] queries, [REP][kSeg] scores, FRESH: [S][dim] new keys
+    __shared__ float red[kWaves];
     const uint32_t rep = p.heads / p.kv_heads, groups = (rep + REP - 1) / REP;
     const uint32_t g = blockIdx.y / groups, h0 = g * rep + (blockIdx.y - g * groups) * REP, nh = min((uint32_t)REP, (g + 1) * rep - h0);
     const uint32_t r = row0 + blockIdx.z, b = r / p.S, s = r - b * p.S, seg = blockIdx.x;
-    float *sc = lds + REP * p.dim;
-    for (uint32_t i = threadIdx.x; i < REP * p.dim; i += kThreads) {
-        const uint32_t h = i / p.dim, d = i - h * p.dim;
-        lds[i] = h < nh ? q[((int64_t)r * p.heads + h0 + h) * p.dim + d] : 0.0f;
-    }
-    __syncthreads();
+    float *sc = lds + REP * p.dim, *fresh = sc + REP * kSeg;
     uint32_t lo, hi;
     visible(p, s, &lo, &hi);
+    const uint32_t j0 = lo + seg * kSeg;
+    if constexpr (FRESH) {
+        const uint32_t nq = p.heads * p.dim, nk = p.kv_heads * p.dim;
+        const float *qr = p.q.p + (int64_t)r * p.q.pitch;
+        float f = p.scale;
+        if (p.temp_every) f *= 1.0f + p.temp_coef * logf((float)((p.position + s + 1) / p.temp_every + 1));
+        const float rms = p.q_norm ? 1.0f / sqrtf(block_sum(row_squares(qr, nq), red) / (float)nq + p.eps) : 1.0f;
+        for (uint32_t i = threadIdx.x; i < REP * p.dim; i += kThreads) {
+            const uint32_t h = i / p.dim, e = h0 * p.dim + i;
+            float v = 0.0f;
+            if (h < nh) v = p.q_norm ? qr[e] * rms * p.q_norm[e] : qr[e];
+            lds[i] = v * f;
+        }
+        for (uint32_t t = 0; t <= s; t++) { // the new keys among this workgroup's
+            const uint32_t j = p.cached + t;
+            if (j < j0 || j >= j0 + kSeg) continue;
+            const float *kr = p.k.p + ((int64_t)b * p.S + t) * p.k.pitch;
+            const float fk = p.k_norm ? 1.0f / sqrtf(block_sum(row_squares(kr, nk), red) / (float)nk + p.eps) : 1.0f;
+            float *kc = p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)j * p.dim;
+            for (uint32_t d = threadIdx.x; d < p.dim; d += kThreads) {
+                const float v = p.k_norm ? kr[g * p.dim + d] * fk * p.k_norm[g * p.dim + d] : kr[g * p.dim + d];
+                fresh[t * p.dim + d] = v;
+                if (t == s && h0 == g * rep) kc[d] = v;
+            }
+            if (t == s && h0 == g * rep)
+                for (uint32_t d = threadIdx.x; d < p.vdim; d += kThreads)
+                    p.values[((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)j * p.vdim + d] = p.v.p[(int64_t)r * p.v.pitch + g * p.vdim + d];
+        }
+    } else {
+        for (uint32_t i = threadIdx.x; i < REP * p.dim; i += kThreads) {
+            const uint32_t h = i / p.dim, d = i - h * p.dim;
+            lds[i] = h < nh ? q[((int64_t)r * p.heads + h0 + h) * p.dim + d] : 0.0f;
+        }
+    }
+    __syncthreads();
     const float *K = p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block;
     const uint32_t sub = threadIdx.x & 3, nd = p.dim / VW;
     for (uint32_t key = threadIdx.x >> 2; key < kSeg; key += kThreads / 4) {
-        const uint32_t j = lo + seg * kSeg + key;
+        const uint32_t j = j0 + key;
         float acc[REP] = {};
         if (j < hi) {
-            const float *kp = K + (int64_t)j * p.dim;
-            for (uint32_t i = sub; i < nd; i += 4) {
-                float kv[VW];
-                if constexpr (VW == 4) {
-                    const float4 t = *reinterpret_cast<const float4 *>(kp + 4 * i);
-                    kv[0] = t.x, kv[1] = t.y, kv[2] = t.z, kv[3] = t.w;
-                } else {
-                    kv[0] = kp[i];
+            auto walk = [&](const float *kp) {
+#pragma unroll 4
+                for (uint32_t i = sub; i < nd; i += 4) {
+                    float kv[VW];
+                    if constexpr (VW == 4) {
+                        const float4 t = *reinterpret_cast<const float4 *>(kp + 4 * i);
+                        kv[0] = t.x, kv[1] = t.y, kv[2] = t.z, kv[3] = t.w;
+                    } else {
+                        kv[0] = kp[i];
+                    }
+#pragma unroll
+                    for (int h = 0; h < REP; h++)
+#pragma unroll
+                        for (int e = 0; e < VW; e++) acc[h] = fmaf(kv[e], lds[h * p.dim + VW * i + e], acc[h]);
                 }
-#pragma unroll
-                for (int h = 0; h < REP; h++)
-#pragma unroll
-                    for (int e = 0; e < VW; e++) acc[h] = fmaf(kv[e], lds[h * p.dim + VW * i + e], acc[h]);
-            }
+            };
+            if (FRESH && j >= p.cached) walk(fresh + (j - p.cached) * p.dim);
+            else walk(K + (int64_t)j * p.dim);
         }
 #pragma unroll
         for (int h = 0; h < REP; h++) {
@@ -135,42 +189,21 @@ __global__ __launch_bounds__(kThreads) void attention_scores_kernel(const Attent
     }
 }
 
+// LDS of the mixing kernel, in floats: with H' all heads when they are mixed, else the heads of a workgroup.
+// [H'] maxima, [REP][H'] mixing factors over the sums, [H'][kSeg] exponentials, [REP][kSeg] weights, [REP][VW][256] results
+__host__ __device__ constexpr uint32_t mix_floats(uint32_t rep, uint32_t slots, uint32_t vw) {
+    return slots + rep * slots + slots * kSeg + rep * kSeg + rep * vw * kThreads;
+}
+
 template <int REP, int VW>
 __global__ __launch_bounds__(kThreads) void attention_mix_kernel(const AttentionPlan p, const uint32_t row0, const uint32_t nseg, const float *__restrict__ scores,
                                                                  const float2 *__restrict__ stats, float *__restrict__ dst, const bool partial) {
-    // [H'] maxima, [REP][H'] mixing factors over the sums, [H'][kSeg] exponentials, [REP][kSeg] weights, [256 * VW] results;
-    // H': all heads when they are mixed, else the heads of this workgroup
     extern __shared__ float lds[];
     const uint32_t rep = p.heads / p.kv_heads, groups = (rep + REP - 1) / REP;
     const uint32_t g = blockIdx.y / groups, h0 = g * rep + (blockIdx.y - g * groups) * REP, nh = min((uint32_t)REP, (g + 1) * rep - h0);
     const uint32_t r = row0 + blockIdx.z, b = r / p.S, s = r - b * p.S, seg = blockIdx.x;
     const uint32_t first = p.talk ? 0 : h0, nm = p.talk ? p.heads : nh, slots = p.talk ? p.heads : REP;
     float *mx = lds, *tm = mx + slots, *ex = tm + REP * slots, *wt = ex + slots * kSeg, *red = wt + REP * kSeg;
-    for (uint32_t h = threadIdx.x; h < nm; h += kThreads) {
-        const float2 *st = stats + ((int64_t)blockIdx.z * p.heads + first + h) * nseg;
-        float m = -INFINITY, l = 0.0f;
-        for (uint32_t i = 0; i < nseg; i++) m = fmaxf(m, st[i].x);
-        for (uint32_t i = 0; i < nseg; i++)
-            if (st[i].y > 0.0f) l = fmaf(st[i].y, expf(st[i].x - m), l);
-        mx[h] = m;
-        for (uint32_t o = 0; o < REP; o++) {
-            const float f = o >= nh ? 0.0f : p.talk ? p.talk[(int64_t)(h0 + o) * p.heads + h] : (o == h ? 1.0f : 0.0f);
-            tm[o * slots + h] = f / l;
-        }
-    }
-    __syncthreads();
-    for (uint32_t i = threadIdx.x; i < nm * kSeg; i += kThreads) {
-        const uint32_t h = i / kSeg, k = i - h * kSeg;
-        ex[i] = expf(scores[(((int64_t)blockIdx.z * p.heads + first + h) * nseg + seg) * kSeg + k] - mx[h]); // (beyond the last key: 0)
-    }
-    __syncthreads();
-    for (uint32_t i = threadIdx.x; i < REP * kSeg; i += kThreads) {
-        const uint32_t o = i / kSeg, k = i - o * kSeg;
-        float w = 0.0f;
-        for (uint32_t h = 0; h < nm; h++) w = fmaf(tm[o * slots + h], ex[h * kSeg + k], w);
-        wt[i] = w;
-    }
-    __syncthreads();
     uint32_t lo, hi;
     visible(p, s, &lo, &hi);
     const uint32_t j0 = lo + seg * kSeg, keys = j0 < hi ? min(kSeg, hi - j0) : 0;
@@ -178,46 +211,82 @@ __global__ __launch_bounds__(kThreads) void attention_mix_kernel(const Attention
     uint32_t lanes = 1; // lanes side by side along vdim; the others take keys in turn
     while (lanes < kThreads && lanes * VW < p.vdim) lanes *= 2;
     const uint32_t across = threadIdx.x & (lanes - 1), turn = threadIdx.x / lanes, turns = kThreads / lanes;
+    // the values of the first columns are asked for before the weights are known
+    constexpr int AHEAD = 16;
+    float v[AHEAD][VW];
+    auto load = [&](uint32_t d, uint32_t k, float(&t)[VW]) {
+        const bool there = d < p.vdim && k < keys;
+        if constexpr (VW == 4) {
+            const float4 x = there ? *reinterpret_cast<const float4 *>(Vp + (int64_t)k * p.vdim + d) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+            t[0] = x.x, t[1] = x.y, t[2] = x.z, t[3] = x.w;
+        } else {
+            t[0] = there ? Vp[(int64_t)k * p.vdim + d] : 0.0f;
+        }
+    };
+#pragma unroll
+    for (int i = 0; i < AHEAD; i++) load(across * VW, turn + i * turns, v[i]);
+    const uint32_t key = threadIdx.x % kSeg; // two threads share a key's column of scores
+    for (uint32_t h = threadIdx.x / kSeg; h < nm; h += kThreads / kSeg) ex[h * kSeg + key] = scores[(((int64_t)blockIdx.z * p.heads + first + h) * nseg + seg) * kSeg + key];
+    for (uint32_t h = threadIdx.x; h < nm; h += kThreads) {
+        const float2 *st = stats + ((int64_t)blockIdx.z * p.heads + first + h) * nseg;
+        float m = -INFINITY, l = 0.0f;
+#pragma unroll 4
+        for (uint32_t i = 0; i < nseg; i++) { // the running pair: one walk along the segments
+            const float2 t = st[i];
+            const float up = fmaxf(m, t.x);
+            if (t.y > 0.0f) l = (m == -INFINITY ? 0.0f : l * expf(m - up)) + t.y * expf(t.x - up);
+            m = up;
+        }
+        mx[h] = m;
+        for (uint32_t o = 0; o < REP; o++) {
+            const float f = o >= nh ? 0.0f : p.talk ? p.talk[(int64_t)(h0 + o) * p.heads + h] : (o == h ? 1.0f : 0.0f);
+            tm[o * slots + h] = f / l;
+        }
+    }
+    __syncthreads();
+    for (uint32_t h = threadIdx.x / kSeg; h < nm; h += kThreads / kSeg) ex[h * kSeg + key] = expf(ex[h * kSeg + key] - mx[h]); // (beyond the last key: 0)
+    __syncthreads();
+    for (uint32_t o = threadIdx.x / kSeg; o < REP; o += kThreads / kSeg) {
+        float w = 0.0f;
+#pragma unroll 4
+        for (uint32_t h = 0; h < nm; h++) w = fmaf(tm[o * slots + h], ex[h * kSeg + key], w);
+        wt[o * kSeg + key] = w;
+    }
+    __syncthreads();
     for (uint32_t d0 = 0; d0 < p.vdim; d0 += lanes * VW) {
         const uint32_t d = d0 + across * VW;
         float acc[REP][VW] = {};
-        if (d < p.vdim)
-            for (uint32_t k = turn; k < keys; k += turns) {
-                float v[VW];
-                const float *vp = Vp + (int64_t)k * p.vdim + d;
-                if constexpr (VW == 4) {
-                    const float4 t = *reinterpret_cast<const float4 *>(vp);
-                    v[0] = t.x, v[1] = t.y, v[2] = t.z, v[3] = t.w;
-                } else {
-                    v[0] = *vp;
-                }
+        for (uint32_t k0 = turn; k0 < keys; k0 += AHEAD * turns) {
+            if (d0 > 0 || k0 > turn)
 #pragma unroll
-                for (int o = 0; o < REP; o++)
+                for (int i = 0; i < AHEAD; i++) load(d, k0 + i * turns, v[i]);
 #pragma unroll
-                    for (int e = 0; e < VW; e++) acc[o][e] = fmaf(wt[o * kSeg + k], v[e], acc[o][e]);
+            for (int i = 0; i < AHEAD; i++) {
+                const uint32_t k = k0 + i * turns;
+                if (k < keys)
+#pragma unroll
+                    for (int o = 0; o < REP; o++) {
+                        const float w = wt[o * kSeg + k];
+#pragma unroll
+                        for (int e = 0; e < VW; e++) acc[o][e] = fmaf(w, v[i][e], acc[o][e]);
+                    }
             }
-        for (uint32_t o = 0; o < nh; o++) {
-#pragma unroll
-            for (int e = 0; e < VW; e++) {
-                float mine = 0.0f;
-#pragma unroll
-                for (int c = 0; c < REP; c++)
-                    if (c == (int)o) mine = acc[c][e];
-                red[e * kThreads + threadIdx.x] = mine;
-            }
-            __syncthreads();
-            if (turn == 0 && d < p.vdim) {
-                const uint32_t h = h0 + o;
-                float *out = partial ? dst + (((int64_t)blockIdx.z * nseg + seg) * p.heads + h) * p.vdim : dst + ((int64_t)r * p.heads + h) * p.vdim;
-#pragma unroll
-                for (int e = 0; e < VW; e++) {
-                    float sum = 0.0f;
-                    for (uint32_t t = 0; t < turns; t++) sum += red[e * kThreads + t * lanes + across];
-                    out[d + e] = sum;
-                }
-            }
-            __syncthreads();
         }
+#pragma unroll
+        for (int o = 0; o < REP; o++)
+#pragma unroll
+            for (int e = 0; e < VW; e++) red[(o * VW + e) * kThreads + threadIdx.x] = acc[o][e];
+        __syncthreads();
+        const uint32_t cols = min(lanes * VW, p.vdim - d0);
+        for (uint32_t i = threadIdx.x; i < nh * cols; i += kThreads) {
+            const uint32_t o = i / cols, c = i - o * cols, h = h0 + o;
+            float sum = 0.0f;
+#pragma unroll 4
+            for (uint32_t t = 0; t < turns; t++) sum += red[(o * VW + c % VW) * kThreads + t * lanes + c / VW];
+            float *out = partial ? dst + (((int64_t)blockIdx.z * nseg + seg) * p.heads + h) * p.vdim : dst + ((int64_t)r * p.heads + h) * p.vdim;
+            out[d0 + c] = sum;
+        }
+        __syncthreads();
     }
 }
 
@@ -257,12 +326,14 @@ struct Scratch {
 template <int REP, int SVW, int MVW>
 int rows_kernels(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t row0, uint32_t rows, uint32_t nseg, float *scores, float2 *stats, float *parts) {
     const uint32_t rep = p.heads / p.kv_heads, groups = (rep + REP - 1) / REP, slots = p.talk ? p.heads : REP;
-    const size_t lds1 = ((size_t)REP * p.dim + REP * kSeg) * 4;
-    const size_t lds2 = ((size_t)slots + REP * slots + (size_t)slots * kSeg + REP * kSeg + kThreads * MVW) * 4;
-    if (int rc = allow_lds(attention_scores_kernel<REP, SVW>, lds1)) return rc;
+    const bool fresh = !q; // a few new tokens, not prepared
+    const size_t lds1 = ((size_t)REP * p.dim + REP * kSeg + (fresh ? p.S * p.dim : 0)) * 4;
+    const size_t lds2 = (size_t)mix_floats(REP, slots, MVW) * 4;
+    if (int rc = fresh ? allow_lds(attention_scores_kernel<REP, SVW, true>, lds1) : allow_lds(attention_scores_kernel<REP, SVW, false>, lds1)) return rc;
     if (int rc = allow_lds(attention_mix_kernel<REP, MVW>, lds2)) return rc;
     const dim3 grid(nseg, p.kv_heads * groups, rows);
-    hipLaunchKernelGGL((attention_scores_kernel<REP, SVW>), grid, dim3(kThreads), lds1, be->stream, p, q, row0, nseg, scores, stats);
+    if (fresh) hipLaunchKernelGGL((attention_scores_kernel<REP, SVW, true>), grid, dim3(kThreads), lds1, be->stream, p, q, row0, nseg, scores, stats);
+    else hipLaunchKernelGGL((attention_scores_kernel<REP, SVW, false>), grid, dim3(kThreads), lds1, be->stream, p, q, row0, nseg, scores, stats);
     hipLaunchKernelGGL((attention_mix_kernel<REP, MVW>), grid, dim3(kThreads), lds2, be->stream, p, row0, nseg, scores, stats, nseg > 1 ? parts : p.out, nseg > 1);
     if (nseg > 1) {
         const uint32_t n = p.heads * p.vdim;
@@ -285,16 +356,21 @@ int rows_kernels(cg_backend *be, const AttentionPlan &p, const float *q, uint32_
 
 int launch_attention(cg_backend *be, const AttentionPlan &p) {
     const uint32_t rows = p.B * p.S, all = p.cached + p.S;
+    const bool fresh = p.S <= kFewRows && p.dim <= 512;
     Scratch qbuf(be);
-    if (int rc = qbuf.get((size_t)rows * p.heads * p.dim * 4)) return rc;
-    float *q = static_cast<float *>(qbuf.p);
-    hipLaunchKernelGGL(attention_prepare_kernel, dim3(rows), dim3(kThreads), 0, be->stream, p, q);
-    if (int rc = launched("attention_prepare")) return rc;
+    float *q = nullptr;
+    if (!fresh) {
+        if (int rc = qbuf.get((size_t)rows * p.heads * p.dim * 4)) return rc;
+        q = static_cast<float *>(qbuf.p);
+        hipLaunchKernelGGL(attention_prepare_kernel, dim3(rows), dim3(kThreads), 0, be->stream, p, q);
+        if (int rc = launched("attention_prepare")) return rc;
+    }
     const uint32_t most = p.window ? std::min(p.window, all) : all, nseg = (most + kSeg - 1) / kSeg, rep = p.heads / p.kv_heads;
     double pairs = 0.0; // visible (query, key) pairs
     for (uint32_t s = 0; s < p.S; s++) pairs += (double)std::min(p.window ? p.window : ~0u, p.cached + s + 1);
     ProfScope prof(be, CG_K_ATTENTION, pairs * p.B * p.heads * (2.0 * p.dim + 2.0 * p.vdim + (p.talk ? 2.0 * p.heads : 0.0)));
-    if (int rc = launch_attention_tiles(be, p, q); rc != kDeclined) return rc;
+    if (!fresh)
+        if (int rc = launch_attention_tiles(be, p, q); rc != kDeclined) return rc;
     // rows in parts that keep the scores within 64 MB
     const size_t per_row = (size_t)p.heads * nseg * (kSeg * 4 + sizeof(float2)) + (nseg > 1 ? (size_t)nseg * p.heads * p.vdim * 4 : 0);
     const uint32_t part = (uint32_t)std::max<size_t>(1, std::min<size_t>(std::min<size_t>(rows, 65535), (64u << 20) / per_row));

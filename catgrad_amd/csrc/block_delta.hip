@@ -356,6 +356,7 @@ __device__ __forceinline__ float step_sum(float v, float *red) { // over the wor
 __device__ __forceinline__ float quad_dot(const float *__restrict__ w, const float *__restrict__ x, uint32_t n, uint32_t sub) {
     float s = 0.0f;
     if (n % 4 == 0 && (reinterpret_cast<uintptr_t>(w) & 15) == 0 && (reinterpret_cast<uintptr_t>(x) & 15) == 0) {
+#pragma unroll 4
         for (uint32_t i = sub; i < n / 4; i += 4) {
             const float4 a = reinterpret_cast<const float4 *>(w)[i], c = reinterpret_cast<const float4 *>(x)[i];
             s = fmaf(a.x, c.x, fmaf(a.y, c.y, fmaf(a.z, c.z, fmaf(a.w, c.w, s))));
@@ -368,8 +369,33 @@ __device__ __forceinline__ float quad_dot(const float *__restrict__ w, const flo
     return s;
 }
 
+// conv_silu with the inputs and taps asked for together when there are TAPS of them
+template <int TAPS> __device__ __forceinline__ float conv_step(const DeltaPlan &p, uint32_t b, int t, uint32_t c) {
+    if constexpr (TAPS == 0) {
+        return conv_silu(p, b, t, c);
+    } else {
+        const uint32_t kc = p.kv_heads * p.dim, C = 2 * kc + p.heads * p.vdim;
+        const bool is_q = c < kc, is_k = !is_q && c < 2 * kc;
+        const uint32_t e = is_q ? c : is_k ? c - kc : c - 2 * kc;
+        const float *w = (is_q ? p.conv_q : is_k ? p.conv_k : p.conv_v) + (int64_t)e * TAPS;
+        const Rows &src = is_q ? p.q : is_k ? p.k : p.v;
+        const float *now = src.p + ((int64_t)b * p.S + t) * src.pitch + e;
+        const float *kept = p.conv_state ? p.conv_state + ((int64_t)b * (TAPS - 1) + t + TAPS - 1) * C + c : now;
+        float x[TAPS], tap[TAPS], s = 0.0f;
+#pragma unroll
+        for (int i = 0; i < TAPS; i++) {
+            const int back = TAPS - 1 - i; // tokens before t
+            tap[i] = w[i];
+            x[i] = back <= t ? now[-(int64_t)back * src.pitch] : p.conv_state ? kept[-(int64_t)back * C] : 0.0f;
+        }
+#pragma unroll
+        for (int i = 0; i < TAPS; i++) s = fmaf(x[i], tap[i], s);
+        return s * sigmoid(s);
+    }
+}
+
 // Thread (c, group) holds rows group, group + groups, ... (at most R) of column c of the head's state.
-template <int R> __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(const DeltaPlan p, const uint32_t lanes) {
+template <int R, int TAPS> __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(const DeltaPlan p, const uint32_t lanes) {
     __shared__ float q[256], k[256], g[256], v[kStepThreads], gate[kStepThreads], part[kStepThreads], red[kStepThreads / 64];
     const uint32_t h = blockIdx.x, b = blockIdx.y, rep = p.heads / p.kv_heads, kh = h / rep, D = p.dim, V = p.vdim, kc = p.kv_heads * D;
     const uint32_t tid = threadIdx.x, c = tid & (lanes - 1), group = tid / lanes, groups = kStepThreads / lanes;
@@ -380,23 +406,23 @@ template <int R> __global__ __launch_bounds__(kStepThreads) void delta_step_kern
         const uint32_t d = group + i * groups;
         S[i] = p.state && d < D && c < V ? p.state[sb + (int64_t)d * V + c] : 0.0f;
     }
-    keep_inputs(p, b, h);
     for (uint32_t t = 0; t < p.S; t++) {
         const int64_t r = (int64_t)b * p.S + t;
         float sq = 0.0f, sk = 0.0f;
         for (uint32_t u = tid; u < 2 * D + V; u += kStepThreads) {
             if (u < D) {
-                const float x = conv_silu(p, b, (int)t, kh * D + u);
+                const float x = conv_step<TAPS>(p, b, (int)t, kh * D + u);
                 q[u] = x;
                 sq = fmaf(x, x, sq);
             } else if (u < 2 * D) {
-                const float x = conv_silu(p, b, (int)t, kc + kh * D + (u - D));
+                const float x = conv_step<TAPS>(p, b, (int)t, kc + kh * D + (u - D));
                 k[u - D] = x;
                 sk = fmaf(x, x, sk);
             } else {
-                v[u - 2 * D] = conv_silu(p, b, (int)t, 2 * kc + h * V + (u - 2 * D));
+                v[u - 2 * D] = conv_step<TAPS>(p, b, (int)t, 2 * kc + h * V + (u - 2 * D));
             }
         }
+#pragma unroll 2
         for (uint32_t u = tid / 4; u < D + V; u += kStepThreads / 4) { // the two factored projections
             if (u < D) {
                 const float a = quad_dot(p.decay_w + ((int64_t)h * D + u) * p.decay_rank, p.decay.p + r * p.decay.pitch, p.decay_rank, tid & 3);
@@ -441,6 +467,7 @@ template <int R> __global__ __launch_bounds__(kStepThreads) void delta_step_kern
         if (group == 0 && c < V) p.out[r * p.heads * V + h * V + c] = y * f * p.norm[c] * gate[c];
         __syncthreads(); // the next token overwrites what this one reads
     }
+    keep_inputs(p, b, h);
 #pragma unroll
     for (int i = 0; i < R; i++) {
         const uint32_t d = group + i * groups;
@@ -558,10 +585,14 @@ int launch_channel_delta(cg_backend *be, const DeltaPlan &p) {
     if (step_shape(p, &lanes, &held)) {
         ProfScope prof(be, CG_K_RECURRENCE, flop * rows);
         const dim3 grid(p.heads, p.B);
-        if (held <= 4) hipLaunchKernelGGL((delta_step_kernel<4>), grid, dim3(kStepThreads), 0, be->stream, p, lanes);
-        else if (held <= 16) hipLaunchKernelGGL((delta_step_kernel<16>), grid, dim3(kStepThreads), 0, be->stream, p, lanes);
-        else if (held <= 32) hipLaunchKernelGGL((delta_step_kernel<32>), grid, dim3(kStepThreads), 0, be->stream, p, lanes);
-        else hipLaunchKernelGGL((delta_step_kernel<64>), grid, dim3(kStepThreads), 0, be->stream, p, lanes);
+#define CG_STEP(R)                                                                                                          \
+    if (p.taps == 4) hipLaunchKernelGGL((delta_step_kernel<R, 4>), grid, dim3(kStepThreads), 0, be->stream, p, lanes);      \
+    else hipLaunchKernelGGL((delta_step_kernel<R, 0>), grid, dim3(kStepThreads), 0, be->stream, p, lanes)
+        if (held <= 4) { CG_STEP(4); }
+        else if (held <= 16) { CG_STEP(16); }
+        else if (held <= 32) { CG_STEP(32); }
+        else { CG_STEP(64); }
+#undef CG_STEP
         return launched("channel_delta step");
     }
     Scratch mem(be);
