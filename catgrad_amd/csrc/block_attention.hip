@@ -207,7 +207,7 @@ __global__ __launch_bounds__(kThreads) void attention_mix_kernel(const Attention
     uint32_t lo, hi;
     visible(p, s, &lo, &hi);
     const uint32_t j0 = lo + seg * kSeg, keys = j0 < hi ? min(kSeg, hi - j0) : 0;
-    const float *Vp = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)j0 * p.vdim;
+    const float *Vp = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)min(j0, hi - 1) * p.vdim;
     uint32_t lanes = 1; // lanes side by side along vdim; the others take keys in turn
     while (lanes < kThreads && lanes * VW < p.vdim) lanes *= 2;
     const uint32_t across = threadIdx.x & (lanes - 1), turn = threadIdx.x / lanes, turns = kThreads / lanes;
@@ -215,12 +215,13 @@ __global__ __launch_bounds__(kThreads) void attention_mix_kernel(const Attention
     constexpr int AHEAD = 16;
     float v[AHEAD][VW];
     auto load = [&](uint32_t d, uint32_t k, float(&t)[VW]) {
-        const bool there = d < p.vdim && k < keys;
+        // (clamped, not tested: what is not there is not used)
+        const float *x = Vp + (int64_t)min(k, max(keys, 1u) - 1) * p.vdim + min(d, p.vdim - VW);
         if constexpr (VW == 4) {
-            const float4 x = there ? *reinterpret_cast<const float4 *>(Vp + (int64_t)k * p.vdim + d) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
-            t[0] = x.x, t[1] = x.y, t[2] = x.z, t[3] = x.w;
+            const float4 f = *reinterpret_cast<const float4 *>(x);
+            t[0] = f.x, t[1] = f.y, t[2] = f.z, t[3] = f.w;
         } else {
-            t[0] = there ? Vp[(int64_t)k * p.vdim + d] : 0.0f;
+            t[0] = *x;
         }
     };
 #pragma unroll

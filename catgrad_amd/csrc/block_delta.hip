@@ -89,9 +89,14 @@ template <int TAPS> __device__ __forceinline__ void conv_chunk(const DeltaPlan &
 #pragma unroll
         for (int i = 0; i < TAPS; i++) wt[i] = w[i];
 #pragma unroll
-        for (int i = 0; i < TAPS - 1; i++) in[i] = conv_input(p, b, (int)t0 + i - (TAPS - 1), c);
+        for (uint32_t t = 0; t < kChunk; t++) in[t + TAPS - 1] = x[(int64_t)min(t, n - 1) * src.pitch]; // (clamped, not tested: no load waits)
+        if (t0 >= TAPS - 1) {
 #pragma unroll
-        for (uint32_t t = 0; t < kChunk; t++) in[t + TAPS - 1] = t < n ? x[(int64_t)t * src.pitch] : 0.0f;
+            for (int i = 0; i < TAPS - 1; i++) in[i] = x[(int64_t)(i - (TAPS - 1)) * src.pitch];
+        } else {
+#pragma unroll
+            for (int i = 0; i < TAPS - 1; i++) in[i] = conv_input(p, b, (int)t0 + i - (TAPS - 1), c);
+        }
 #pragma unroll
         for (uint32_t t = 0; t < kChunk; t++) {
             float s = 0.0f;
@@ -123,10 +128,13 @@ template <int TAPS> __global__ __launch_bounds__(kThreads, 4) void delta_chunk_k
             conv_chunk<TAPS>(p, b, t0, n, which * kc + g * D + d, y);
         } else {
             const float *a = decay + ((int64_t)b * p.S + t0) * p.heads * D + h * D + d;
+            const float rate = -expf(p.a_log[h]) * kLog2e, bias = p.dt_bias[h * D + d];
             float sum = 0.0f;
 #pragma unroll
+            for (uint32_t t = 0; t < kChunk; t++) y[t] = a[(int64_t)min(t, n - 1) * p.heads * D];
+#pragma unroll
             for (uint32_t t = 0; t < kChunk; t++) {
-                if (t < n) sum += log2_decay(p, a[(int64_t)t * p.heads * D], h, d);
+                sum += t < n ? rate * softplus(y[t] + bias) : 0.0f;
                 y[t] = sum;
             }
         }
@@ -386,7 +394,8 @@ template <int TAPS> __device__ __forceinline__ float conv_step(const DeltaPlan &
         for (int i = 0; i < TAPS; i++) {
             const int back = TAPS - 1 - i; // tokens before t
             tap[i] = w[i];
-            x[i] = back <= t ? now[-(int64_t)back * src.pitch] : p.conv_state ? kept[-(int64_t)back * C] : 0.0f;
+            const float *at = back <= t ? now - (int64_t)back * src.pitch : kept - (int64_t)back * C; // (one load, whichever it is)
+            x[i] = back <= t || p.conv_state ? *at : 0.0f;
         }
 #pragma unroll
         for (int i = 0; i < TAPS; i++) s = fmaf(x[i], tap[i], s);
@@ -396,7 +405,7 @@ template <int TAPS> __device__ __forceinline__ float conv_step(const DeltaPlan &
 
 // Thread (c, group) holds rows group, group + groups, ... (at most R) of column c of the head's state.
 template <int R, int TAPS> __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(const DeltaPlan p, const uint32_t lanes) {
-    __shared__ float q[256], k[256], g[256], v[kStepThreads], gate[kStepThreads], part[kStepThreads], red[kStepThreads / 64];
+    __shared__ float q[257], k[257], g[257], v[kStepThreads], gate[kStepThreads], part[kStepThreads], red[kStepThreads / 64];
     const uint32_t h = blockIdx.x, b = blockIdx.y, rep = p.heads / p.kv_heads, kh = h / rep, D = p.dim, V = p.vdim, kc = p.kv_heads * D;
     const uint32_t tid = threadIdx.x, c = tid & (lanes - 1), group = tid / lanes, groups = kStepThreads / lanes;
     const int64_t sb = ((int64_t)b * p.heads + h) * D * V;
@@ -404,8 +413,10 @@ template <int R, int TAPS> __global__ __launch_bounds__(kStepThreads) void delta
 #pragma unroll
     for (int i = 0; i < R; i++) {
         const uint32_t d = group + i * groups;
-        S[i] = p.state && d < D && c < V ? p.state[sb + (int64_t)d * V + c] : 0.0f;
+        const float x = p.state ? p.state[sb + (int64_t)min(d, D - 1) * V + min(c, V - 1)] : 0.0f; // (clamped, not tested: no load waits)
+        S[i] = d < D ? x : 0.0f;
     }
+    if (tid == 0) q[D] = k[D] = g[D] = 0.0f; // what the rows behind the last one read
     for (uint32_t t = 0; t < p.S; t++) {
         const int64_t r = (int64_t)b * p.S + t;
         float sq = 0.0f, sk = 0.0f;
@@ -437,11 +448,9 @@ template <int R, int TAPS> __global__ __launch_bounds__(kStepThreads) void delta
         float read = 0.0f; // (the sums above end behind a barrier: q, k, v, g and gate are there)
 #pragma unroll
         for (int i = 0; i < R; i++) {
-            const uint32_t d = group + i * groups;
-            if (d < D) {
-                S[i] *= g[d];
-                read = fmaf(S[i], k[d] * fk, read);
-            }
+            const uint32_t d = min(group + i * groups, D);
+            S[i] *= g[d];
+            read = fmaf(S[i], k[d] * fk, read);
         }
         part[tid] = read;
         __syncthreads();
@@ -451,11 +460,9 @@ template <int R, int TAPS> __global__ __launch_bounds__(kStepThreads) void delta
         float y = 0.0f;
 #pragma unroll
         for (int i = 0; i < R; i++) {
-            const uint32_t d = group + i * groups;
-            if (d < D) {
-                S[i] = fmaf(k[d] * fk, u, S[i]);
-                y = fmaf(S[i], q[d] * fq, y);
-            }
+            const uint32_t d = min(group + i * groups, D);
+            S[i] = fmaf(k[d] * fk, u, S[i]);
+            y = fmaf(S[i], q[d] * fq, y);
         }
         __syncthreads();
         part[tid] = y;

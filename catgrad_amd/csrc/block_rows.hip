@@ -261,8 +261,8 @@ template <bool BF16> struct Frag { // a lane's weights, or its activations in th
 template <bool BF16> __device__ __forceinline__ Frag<BF16> load_weights(const Weight &w, uint32_t n, uint32_t k) {
     typedef uint32_t u4 __attribute__((ext_vector_type(4)));
     Frag<BF16> f;
-    u4 t = {0, 0, 0, 0};
-    if (k < w.k) t = __builtin_nontemporal_load(reinterpret_cast<const u4 *>(static_cast<const char *>(w.p) + ((int64_t)n * w.pitch + k) * (BF16 ? 2 : 4)));
+    k = min(k, w.k - Frag<BF16>::W); // (behind the last column the activations are zero: no load waits for a test)
+    const u4 t = __builtin_nontemporal_load(reinterpret_cast<const u4 *>(static_cast<const char *>(w.p) + ((int64_t)n * w.pitch + k) * (BF16 ? 2 : 4)));
 #pragma unroll
     for (int i = 0; i < 4; i++) f.v[i] = t[i];
     return f;
@@ -299,12 +299,12 @@ template <bool BF16> __device__ __forceinline__ f32x4 multiply(const Frag<BF16> 
 template <bool BF16> __device__ __forceinline__ void load_input(const ProductInput &in, uint32_t r, bool there, uint32_t k, float (&x)[Frag<BF16>::W]) {
 #pragma unroll
     for (uint32_t i = 0; i < Frag<BF16>::W; i += 4) {
-        f32x4 t = {0.0f, 0.0f, 0.0f, 0.0f};
-        if (there && k + i < in.k)
-            t = k + i < in.k1 ? *reinterpret_cast<const f32x4 *>(in.x.p + (int64_t)r * in.x.pitch + k + i)
-                              : *reinterpret_cast<const f32x4 *>(in.x2.p + (int64_t)r * in.x2.pitch + (k + i - in.k1));
+        const uint32_t at = min(k + i, in.k - 4);
+        const float *first = in.x.p + (int64_t)r * in.x.pitch + at, *second = in.x2.p + (int64_t)r * in.x2.pitch + at - in.k1;
+        const f32x4 t = *reinterpret_cast<const f32x4 *>(at < in.k1 ? first : second);
+        const bool in_row = there && k + i < in.k;
 #pragma unroll
-        for (int j = 0; j < 4; j++) x[i + j] = t[j];
+        for (int j = 0; j < 4; j++) x[i + j] = in_row ? t[j] : 0.0f;
     }
 }
 // over the 16 lanes that share j
@@ -336,12 +336,12 @@ __global__ __launch_bounds__(WAVES * 64) void four_rows_linear_kernel(const Prod
     for (int s = 0; s < STEPS; s++) {
         const uint32_t k = k0 + s * WAVES * SPAN;
         float z[W];
-        load_input<BF16>(in, j, j < rows, k, z);
+        load_input<BF16>(in, min(j, rows - 1), j < rows, k, z);
         if (in.gamma) {
 #pragma unroll
             for (uint32_t i = 0; i < W; i++) {
                 ss = fmaf(z[i], z[i], ss);
-                z[i] = k + i < in.k ? z[i] * in.gamma[k + i] : 0.0f;
+                z[i] *= in.gamma[min(k + i, in.k - 1)];
             }
         }
         x[s] = pack<BF16>(z);
@@ -403,7 +403,7 @@ __device__ __forceinline__ void walk_branch(const ResidualBranch &b, uint32_t ro
 #pragma unroll
             for (int g = 0; g < NG; g++) wt[a][g] = load_weights<BF16>(b.w, n[g], k0 + a * STEP);
 #pragma unroll
-        for (int a = 0; a < AHEAD; a++) load_input<BF16>(b.in, j, j < rows, k0 + a * STEP, z[a]);
+        for (int a = 0; a < AHEAD; a++) load_input<BF16>(b.in, min(j, rows - 1), j < rows, k0 + a * STEP, z[a]);
 #pragma unroll
         for (int a = 0; a < AHEAD; a++) {
             Frag<BF16> x = pack<BF16>(z[a]);
@@ -426,7 +426,9 @@ __device__ __forceinline__ void walk_branch(const ResidualBranch &b, uint32_t ro
 #pragma unroll
                 for (int g = 0; g < NG; g++) o.acc[g][2] = multiply<BF16>(wt[a][g], x, o.acc[g][2]);
 #pragma unroll
-                for (int g = 0; g < NG; g++) o.acc[g][3] = multiply<BF16>(wt[a][g], ones, o.acc[g][3]);
+                for (int i = 0; i < 4; i++) x.v[i] = k0 + a * STEP < b.w.k ? ones.v[i] : 0;
+#pragma unroll
+                for (int g = 0; g < NG; g++) o.acc[g][3] = multiply<BF16>(wt[a][g], x, o.acc[g][3]);
             }
         }
     }
