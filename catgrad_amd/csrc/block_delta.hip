@@ -29,24 +29,41 @@ __device__ __forceinline__ float wave_sum(float v) {
     for (int d = 32; d > 0; d >>= 1) v += __shfl_xor(v, d, 64);
     return v;
 }
-__device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// on the hardware's exp2, log2 and reciprocal (about one unit in the last place each)
+__device__ __forceinline__ float sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * -1.44269504088896341f)); }
+// max(z, 0) + ln(1 + e^-|z|), by its series where 1 + e^-|z| would lose what a slow decay lives on
+__device__ __forceinline__ float softplus(float z) {
+    const float t = __builtin_amdgcn_exp2f(-fabsf(z) * 1.44269504088896341f);
+    const float l = t < 0.01f ? t * fmaf(t, fmaf(t, 0.33333333f, -0.5f), 1.0f) : __builtin_amdgcn_logf(1.0f + t) * 0.69314718055994531f;
+    return fmaxf(z, 0.0f) + l;
+}
 
-// Channel c of the three projections side by side, at time t of sequence b (t < 0: what the state kept).
-__device__ __forceinline__ float conv_input(const DeltaPlan &p, uint32_t b, int t, uint32_t c) {
-    const uint32_t kc = p.kv_heads * p.dim, vc = p.heads * p.vdim;
-    if (t < 0) return p.conv_state ? p.conv_state[((int64_t)b * (p.taps - 1) + (t + (int)p.taps - 1)) * (2 * kc + vc) + c] : 0.0f;
-    const int64_t r = (int64_t)b * p.S + t;
-    return c < kc ? p.q.p[r * p.q.pitch + c] : c < 2 * kc ? p.k.p[r * p.k.pitch + c - kc] : p.v.p[r * p.v.pitch + c - 2 * kc];
+// Channel c of the three projections side by side: where its column of tokens begins (at sequence b, token 0), and its taps.
+// (Values are selected, not references: a reference into the arguments would have them fetched lane by lane.)
+struct Channel {
+    const float *x, *taps;
+    int64_t pitch;
+};
+__device__ __forceinline__ Channel channel(const DeltaPlan &p, uint32_t b, uint32_t c) {
+    const uint32_t kc = p.kv_heads * p.dim;
+    const bool is_q = c < kc, is_k = c < 2 * kc;
+    const uint32_t e = is_q ? c : is_k ? c - kc : c - 2 * kc;
+    const float *x = is_q ? p.q.p : is_k ? p.k.p : p.v.p, *w = is_q ? p.conv_q : is_k ? p.conv_k : p.conv_v;
+    const int64_t pitch = is_q ? p.q.pitch : is_k ? p.k.pitch : p.v.pitch;
+    return {x + (int64_t)b * p.S * pitch + e, w + (int64_t)e * p.taps, pitch};
+}
+// its input at time t (t < 0: what the state kept)
+__device__ __forceinline__ float conv_input(const DeltaPlan &p, const Channel &ch, uint32_t b, int t, uint32_t c) {
+    if (t >= 0) return ch.x[(int64_t)t * ch.pitch];
+    const uint32_t C = 2 * p.kv_heads * p.dim + p.heads * p.vdim;
+    return p.conv_state ? p.conv_state[((int64_t)b * (p.taps - 1) + (t + (int)p.taps - 1)) * C + c] : 0.0f;
 }
 __device__ __forceinline__ float conv_silu(const DeltaPlan &p, uint32_t b, int t, uint32_t c) {
-    const uint32_t kc = p.kv_heads * p.dim;
-    const float *w = c < kc ? p.conv_q + (int64_t)c * p.taps : c < 2 * kc ? p.conv_k + (int64_t)(c - kc) * p.taps : p.conv_v + (int64_t)(c - 2 * kc) * p.taps;
+    const Channel ch = channel(p, b, c);
     float s = 0.0f;
-    for (uint32_t i = 0; i < p.taps; i++) s = fmaf(conv_input(p, b, t - (int)(p.taps - 1 - i), c), w[i], s);
+    for (uint32_t i = 0; i < p.taps; i++) s = fmaf(conv_input(p, ch, b, t - (int)(p.taps - 1 - i), c), ch.taps[i], s);
     return s * sigmoid(s);
 }
-
 
 constexpr float kLog2e = 1.44269504088896341f;
 constexpr uint32_t kChunk = 16;
@@ -64,7 +81,7 @@ __device__ void keep_inputs(const DeltaPlan &p, uint32_t b, uint32_t h) {
     for (uint32_t i = threadIdx.x; i < past * n; i += blockDim.x) {
         const uint32_t j = i / n, e = i - j * n;
         const uint32_t c = e < nq ? (h / rep) * p.dim + e : e < 2 * nq ? kc + (h / rep) * p.dim + (e - nq) : 2 * kc + h * p.vdim + (e - 2 * nq);
-        p.conv_out[((int64_t)b * past + j) * C + c] = conv_input(p, b, (int)(p.S + j) - (int)past, c);
+        p.conv_out[((int64_t)b * past + j) * C + c] = conv_input(p, channel(p, b, c), b, (int)(p.S + j) - (int)past, c);
     }
 }
 
@@ -81,21 +98,19 @@ __device__ __host__ constexpr uint32_t chunk_floats(uint32_t dp) { return 48 * d
 // Outputs of the convolution of channel c (of 16 tokens from t0; n of them are there), silu applied.  TAPS 0: any count.
 template <int TAPS> __device__ __forceinline__ void conv_chunk(const DeltaPlan &p, uint32_t b, uint32_t t0, uint32_t n, uint32_t c, float (&y)[kChunk]) {
     if constexpr (TAPS > 0) {
-        const uint32_t kc = p.kv_heads * p.dim;
-        const float *w = c < kc ? p.conv_q + (int64_t)c * TAPS : c < 2 * kc ? p.conv_k + (int64_t)(c - kc) * TAPS : p.conv_v + (int64_t)(c - 2 * kc) * TAPS;
-        const Rows &src = c < kc ? p.q : c < 2 * kc ? p.k : p.v;
-        const float *x = src.p + ((int64_t)b * p.S + t0) * src.pitch + (c < kc ? c : c < 2 * kc ? c - kc : c - 2 * kc);
+        const Channel ch = channel(p, b, c);
+        const float *x = ch.x + (int64_t)t0 * ch.pitch;
         float in[kChunk + TAPS - 1], wt[TAPS];
 #pragma unroll
-        for (int i = 0; i < TAPS; i++) wt[i] = w[i];
+        for (uint32_t t = 0; t < kChunk; t++) in[t + TAPS - 1] = x[(int64_t)min(t, n - 1) * ch.pitch]; // (clamped, not tested: no load waits)
 #pragma unroll
-        for (uint32_t t = 0; t < kChunk; t++) in[t + TAPS - 1] = x[(int64_t)min(t, n - 1) * src.pitch]; // (clamped, not tested: no load waits)
+        for (int i = 0; i < TAPS; i++) wt[i] = ch.taps[i];
         if (t0 >= TAPS - 1) {
 #pragma unroll
-            for (int i = 0; i < TAPS - 1; i++) in[i] = x[(int64_t)(i - (TAPS - 1)) * src.pitch];
+            for (int i = 0; i < TAPS - 1; i++) in[i] = x[(int64_t)(i - (TAPS - 1)) * ch.pitch];
         } else {
 #pragma unroll
-            for (int i = 0; i < TAPS - 1; i++) in[i] = conv_input(p, b, (int)t0 + i - (TAPS - 1), c);
+            for (int i = 0; i < TAPS - 1; i++) in[i] = conv_input(p, ch, b, (int)t0 + i - (TAPS - 1), c);
         }
 #pragma unroll
         for (uint32_t t = 0; t < kChunk; t++) {
@@ -110,7 +125,7 @@ template <int TAPS> __device__ __forceinline__ void conv_chunk(const DeltaPlan &
     }
 }
 
-template <int TAPS> __global__ __launch_bounds__(kThreads, 4) void delta_chunk_kernel(const DeltaPlan p, const ChunkArrays o, const float *__restrict__ decay) {
+template <int TAPS> __global__ __launch_bounds__(kThreads, 3) void delta_chunk_kernel(const DeltaPlan p, const ChunkArrays o, const float *__restrict__ decay) {
     extern __shared__ float lds[]; // q, k, G: [16][pitch] each
     __shared__ float beta[kChunk], lower[kChunk][kChunk + 4], tb[kChunk][kChunk + 4]; // tb[s][t] = T[t][s]
     const uint32_t chunk = blockIdx.x, h = blockIdx.y, b = blockIdx.z, rep = p.heads / p.kv_heads, g = h / rep;
@@ -153,23 +168,40 @@ template <int TAPS> __global__ __launch_bounds__(kThreads, 4) void delta_chunk_k
     __syncthreads();
     float *mats = o.mats + (((int64_t)b * p.heads + h) * o.chunks + chunk) * chunk_floats(dp);
     float *W = mats, *Q = W + kChunk * dp, *K = Q + kChunk * dp, *A = K + kChunk * dp, *E = A + kChunk * kChunk;
-    {
-        const uint32_t t = tid / kChunk, s = tid % kChunk;
+    // the 120 pairs s < t, two lanes each (the key channels' quads in turn); the other 16 threads take A's diagonal
+    if (tid < kChunk * (kChunk - 1)) {
+        const uint32_t pair = tid >> 1;
+        uint32_t t = (uint32_t)((1.0f + sqrtf(8.0f * (float)pair + 1.0f)) * 0.5f); // row of the pair-th entry below the diagonal
+        t -= t * (t - 1) / 2 > pair ? 1 : 0;
+        t += t * (t + 1) / 2 <= pair ? 1 : 0;
+        const uint32_t s = pair - t * (t - 1) / 2;
         float m = 0.0f, a = 0.0f;
-        if (s <= t)
-            for (uint32_t d = 0; d < D; d += 4) { // (zeros behind the last channel)
-                const float4 gt = *reinterpret_cast<const float4 *>(G + t * pitch + d), gs = *reinterpret_cast<const float4 *>(G + s * pitch + d);
-                const float4 kt = *reinterpret_cast<const float4 *>(k + t * pitch + d), qt = *reinterpret_cast<const float4 *>(q + t * pitch + d);
-                float4 ks = *reinterpret_cast<const float4 *>(k + s * pitch + d);
-                ks.x *= exp2_of(gt.x - gs.x);
-                ks.y *= exp2_of(gt.y - gs.y);
-                ks.z *= exp2_of(gt.z - gs.z);
-                ks.w *= exp2_of(gt.w - gs.w);
-                m = fmaf(kt.x, ks.x, fmaf(kt.y, ks.y, fmaf(kt.z, ks.z, fmaf(kt.w, ks.w, m))));
-                a = fmaf(qt.x, ks.x, fmaf(qt.y, ks.y, fmaf(qt.z, ks.z, fmaf(qt.w, ks.w, a))));
-            }
-        lower[t][s] = s < t ? beta[t] * m : 0.0f;
-        A[t * kChunk + s] = a;
+        for (uint32_t d = (tid & 1) * 4; d < dp; d += 8) { // (zeros behind the last channel)
+            const float4 gt = *reinterpret_cast<const float4 *>(G + t * pitch + d), gs = *reinterpret_cast<const float4 *>(G + s * pitch + d);
+            const float4 kt = *reinterpret_cast<const float4 *>(k + t * pitch + d), qt = *reinterpret_cast<const float4 *>(q + t * pitch + d);
+            float4 ks = *reinterpret_cast<const float4 *>(k + s * pitch + d);
+            ks.x *= exp2_of(gt.x - gs.x);
+            ks.y *= exp2_of(gt.y - gs.y);
+            ks.z *= exp2_of(gt.z - gs.z);
+            ks.w *= exp2_of(gt.w - gs.w);
+            m = fmaf(kt.x, ks.x, fmaf(kt.y, ks.y, fmaf(kt.z, ks.z, fmaf(kt.w, ks.w, m))));
+            a = fmaf(qt.x, ks.x, fmaf(qt.y, ks.y, fmaf(qt.z, ks.z, fmaf(qt.w, ks.w, a))));
+        }
+        m += __shfl_xor(m, 1, 64);
+        a += __shfl_xor(a, 1, 64);
+        if ((tid & 1) == 0) {
+            lower[t][s] = beta[t] * m;
+            A[t * kChunk + s] = a;
+            A[s * kChunk + t] = 0.0f;
+        }
+    } else {
+        const uint32_t t = tid - kChunk * (kChunk - 1);
+        float a = 0.0f;
+        for (uint32_t d = 0; d < dp; d += 4) {
+            const float4 kt = *reinterpret_cast<const float4 *>(k + t * pitch + d), qt = *reinterpret_cast<const float4 *>(q + t * pitch + d);
+            a = fmaf(qt.x, kt.x, fmaf(qt.y, kt.y, fmaf(qt.z, kt.z, fmaf(qt.w, kt.w, a))));
+        }
+        A[t * kChunk + t] = a;
     }
     __syncthreads();
     if (wave == 0) { // T: forward substitution, a lane per column
@@ -363,11 +395,21 @@ __device__ __forceinline__ float step_sum(float v, float *red) { // over the wor
 // w[row, :] . x, four lanes of a quad together
 __device__ __forceinline__ float quad_dot(const float *__restrict__ w, const float *__restrict__ x, uint32_t n, uint32_t sub) {
     float s = 0.0f;
-    if (n % 4 == 0 && (reinterpret_cast<uintptr_t>(w) & 15) == 0 && (reinterpret_cast<uintptr_t>(x) & 15) == 0) {
-#pragma unroll 4
-        for (uint32_t i = sub; i < n / 4; i += 4) {
-            const float4 a = reinterpret_cast<const float4 *>(w)[i], c = reinterpret_cast<const float4 *>(x)[i];
-            s = fmaf(a.x, c.x, fmaf(a.y, c.y, fmaf(a.z, c.z, fmaf(a.w, c.w, s))));
+    if (n % 4 == 0 && ((reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(x)) & 15) == 0) { // (the same for every lane)
+        constexpr int AHEAD = 4;
+        const uint32_t quads = n / 4;
+        for (uint32_t i0 = sub; i0 < quads; i0 += 4 * AHEAD) {
+            float4 a[AHEAD], c[AHEAD];
+#pragma unroll
+            for (int j = 0; j < AHEAD; j++) {
+                a[j] = reinterpret_cast<const float4 *>(w)[min(i0 + 4 * j, quads - 1)];
+                c[j] = reinterpret_cast<const float4 *>(x)[min(i0 + 4 * j, quads - 1)];
+            }
+#pragma unroll
+            for (int j = 0; j < AHEAD; j++) {
+                const float t = fmaf(a[j].x, c[j].x, fmaf(a[j].y, c[j].y, fmaf(a[j].z, c[j].z, a[j].w * c[j].w)));
+                s += i0 + 4 * j < quads ? t : 0.0f;
+            }
         }
     } else {
         for (uint32_t i = sub; i < n; i += 4) s = fmaf(w[i], x[i], s);
@@ -382,21 +424,20 @@ template <int TAPS> __device__ __forceinline__ float conv_step(const DeltaPlan &
     if constexpr (TAPS == 0) {
         return conv_silu(p, b, t, c);
     } else {
-        const uint32_t kc = p.kv_heads * p.dim, C = 2 * kc + p.heads * p.vdim;
-        const bool is_q = c < kc, is_k = !is_q && c < 2 * kc;
-        const uint32_t e = is_q ? c : is_k ? c - kc : c - 2 * kc;
-        const float *w = (is_q ? p.conv_q : is_k ? p.conv_k : p.conv_v) + (int64_t)e * TAPS;
-        const Rows &src = is_q ? p.q : is_k ? p.k : p.v;
-        const float *now = src.p + ((int64_t)b * p.S + t) * src.pitch + e;
+        const uint32_t C = 2 * p.kv_heads * p.dim + p.heads * p.vdim;
+        const Channel ch = channel(p, b, c);
+        const float *now = ch.x + (int64_t)t * ch.pitch;
         const float *kept = p.conv_state ? p.conv_state + ((int64_t)b * (TAPS - 1) + t + TAPS - 1) * C + c : now;
+        const int64_t kept_pitch = p.conv_state ? C : 0;
         float x[TAPS], tap[TAPS], s = 0.0f;
 #pragma unroll
         for (int i = 0; i < TAPS; i++) {
             const int back = TAPS - 1 - i; // tokens before t
-            tap[i] = w[i];
-            const float *at = back <= t ? now - (int64_t)back * src.pitch : kept - (int64_t)back * C; // (one load, whichever it is)
-            x[i] = back <= t || p.conv_state ? *at : 0.0f;
+            tap[i] = ch.taps[i];
+            x[i] = *(back <= t ? now - (int64_t)back * ch.pitch : kept - (int64_t)back * kept_pitch); // (one load, whichever it is)
         }
+#pragma unroll
+        for (int i = 0; i < TAPS; i++) x[i] = TAPS - 1 - i <= t || p.conv_state ? x[i] : 0.0f;
 #pragma unroll
         for (int i = 0; i < TAPS; i++) s = fmaf(x[i], tap[i], s);
         return s * sigmoid(s);
@@ -410,37 +451,36 @@ template <int R, int TAPS> __global__ __launch_bounds__(kStepThreads) void delta
     const uint32_t tid = threadIdx.x, c = tid & (lanes - 1), group = tid / lanes, groups = kStepThreads / lanes;
     const int64_t sb = ((int64_t)b * p.heads + h) * D * V;
     float S[R];
+    if (p.state) { // (clamped, not tested: no load waits)
+        const float *src = p.state + sb + min(c, V - 1);
 #pragma unroll
-    for (int i = 0; i < R; i++) {
-        const uint32_t d = group + i * groups;
-        const float x = p.state ? p.state[sb + (int64_t)min(d, D - 1) * V + min(c, V - 1)] : 0.0f; // (clamped, not tested: no load waits)
-        S[i] = d < D ? x : 0.0f;
+        for (int i = 0; i < R; i++) S[i] = src[(int64_t)min(group + i * groups, D - 1) * V];
+#pragma unroll
+        for (int i = 0; i < R; i++) S[i] = group + i * groups < D ? S[i] : 0.0f;
+    } else {
+#pragma unroll
+        for (int i = 0; i < R; i++) S[i] = 0.0f;
     }
     if (tid == 0) q[D] = k[D] = g[D] = 0.0f; // what the rows behind the last one read
     for (uint32_t t = 0; t < p.S; t++) {
         const int64_t r = (int64_t)b * p.S + t;
         float sq = 0.0f, sk = 0.0f;
         for (uint32_t u = tid; u < 2 * D + V; u += kStepThreads) {
-            if (u < D) {
-                const float x = conv_step<TAPS>(p, b, (int)t, kh * D + u);
-                q[u] = x;
-                sq = fmaf(x, x, sq);
-            } else if (u < 2 * D) {
-                const float x = conv_step<TAPS>(p, b, (int)t, kc + kh * D + (u - D));
-                k[u - D] = x;
-                sk = fmaf(x, x, sk);
-            } else {
-                v[u - 2 * D] = conv_step<TAPS>(p, b, (int)t, 2 * kc + h * V + (u - 2 * D));
-            }
+            const bool is_q = u < D, is_k = !is_q && u < 2 * D;
+            const uint32_t e = is_q ? u : is_k ? u - D : u - 2 * D;
+            const float x = conv_step<TAPS>(p, b, (int)t, (is_q ? kh * D : is_k ? kc + kh * D : 2 * kc + h * V) + e);
+            sq = is_q ? fmaf(x, x, sq) : sq;
+            sk = is_k ? fmaf(x, x, sk) : sk;
+            (is_q ? q : is_k ? k : v)[e] = x;
         }
-#pragma unroll 2
         for (uint32_t u = tid / 4; u < D + V; u += kStepThreads / 4) { // the two factored projections
-            if (u < D) {
-                const float a = quad_dot(p.decay_w + ((int64_t)h * D + u) * p.decay_rank, p.decay.p + r * p.decay.pitch, p.decay_rank, tid & 3);
-                if ((tid & 3) == 0) g[u] = exp2_of(log2_decay(p, a, h, u));
-            } else {
-                const float a = quad_dot(p.gate_w + ((int64_t)h * V + (u - D)) * p.gate_rank, p.gate.p + r * p.gate.pitch, p.gate_rank, tid & 3);
-                if ((tid & 3) == 0) gate[u - D] = sigmoid(a);
+            const bool is_g = u < D;
+            const uint32_t e = is_g ? u : u - D;
+            const float a = quad_dot(is_g ? p.decay_w + ((int64_t)h * D + e) * p.decay_rank : p.gate_w + ((int64_t)h * V + e) * p.gate_rank,
+                                     is_g ? p.decay.p + r * p.decay.pitch : p.gate.p + r * p.gate.pitch, is_g ? p.decay_rank : p.gate_rank, tid & 3);
+            if ((tid & 3) == 0) {
+                if (is_g) g[e] = exp2_of(log2_decay(p, a, h, e));
+                else gate[e] = sigmoid(a);
             }
         }
         const float fq = 1.0f / sqrtf(step_sum(sq, red) + 1e-6f) * (1.0f / sqrtf((float)D)), fk = 1.0f / sqrtf(step_sum(sk, red) + 1e-6f);

@@ -23,7 +23,9 @@ __device__ __forceinline__ float block_sum(float v, float *red) {
     __syncthreads();
     return (red[0] + red[1]) + (red[2] + red[3]);
 }
-__device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float sigmoid(float z) { // on the hardware's exp2 and reciprocal
+    return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * -1.44269504088896341f));
+}
 __device__ __forceinline__ float bf16_lo(uint32_t w) { return asf(w << 16); }
 __device__ __forceinline__ float bf16_hi(uint32_t w) { return asf(w & 0xFFFF0000u); }
 
