@@ -125,7 +125,7 @@ template <int TAPS> __device__ __forceinline__ void conv_chunk(const DeltaPlan &
     }
 }
 
-template <int TAPS> __global__ __launch_bounds__(kThreads, 3) void delta_chunk_kernel(const DeltaPlan p, const ChunkArrays o, const float *__restrict__ decay) {
+template <int TAPS> __global__ __launch_bounds__(kThreads, 2) void delta_chunk_kernel(const DeltaPlan p, const ChunkArrays o, const float *__restrict__ decay) {
     extern __shared__ float lds[]; // q, k, G: [16][pitch] each
     __shared__ float beta[kChunk], lower[kChunk][kChunk + 4], tb[kChunk][kChunk + 4]; // tb[s][t] = T[t][s]
     const uint32_t chunk = blockIdx.x, h = blockIdx.y, b = blockIdx.z, rep = p.heads / p.kv_heads, g = h / rep;
