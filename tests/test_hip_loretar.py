@@ -1,0 +1,96 @@
+"""The Loretar model on the GPU: prompts, portions, decoding, requests and generation against loretar_reference.py."""
+import numpy as np
+import pytest
+
+import loretar_cases as C
+import loretar_reference as R
+from block_cases import bf16
+from catgrad_amd.loretar import attention_layer, config_of, delta_layer, random_params
+from catgrad_amd.runner import Session
+
+pytestmark = pytest.mark.gpu
+
+
+@pytest.fixture(scope="module")
+def session():
+    return Session()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("how", list(C.PORTIONS))
+@pytest.mark.parametrize("name", list(C.CONFIGS))
+def test_portions(session, name, how, dtype):
+    C.check_portions(session, name, how, dtype)
+
+
+@pytest.mark.parametrize("name", list(C.CONFIGS))
+def test_one_token(session, name):
+    C.check_one_token(session, name)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", ["mixed", "wider", "odd_sizes"])
+def test_interleaved_requests(session, name, dtype):
+    C.check_interleaved(session, name, dtype)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", ["mixed", "wider"])
+def test_long_decode(session, name, dtype):
+    C.check_long_decode(session, name, 260, dtype)
+
+
+@pytest.mark.parametrize("name", ["mixed", "attention_only", "recurrence_only", "odd_sizes", "wider"])
+def test_generate(session, name):
+    C.check_generate(session, name)
+
+
+@pytest.mark.parametrize("name", ["mixed", "odd_sizes", "wider"])
+def test_batch_logits(session, name):
+    C.check_batch_logits(session, name)
+
+
+def test_recorded_schedules(session):
+    C.load(session, "mixed")
+    t = C.tokens_of("mixed", 30)
+    want = C.run(session, t, [20, 1, 9])
+    try:
+        for schedule in (1, 2):
+            session.set_schedule(schedule)
+            np.testing.assert_allclose(C.run(session, t, [20, 1, 9]), want, rtol=1e-5, atol=1e-5)
+    finally:
+        session.set_schedule(0)
+
+
+def test_ended_requests_give_their_memory_back(session):
+    C.load(session, "wider")
+    t = C.tokens_of("wider", 120)
+
+    def once():
+        for r in range(4):
+            C.run(session, t, [90] + [1] * 30, request=r, end=False)
+        held = session.pool_stats()[0]
+        for r in range(4):
+            session.end(r)
+        session.sync()
+        return held, session.pool_stats()[0]
+
+    first = once()
+    assert first[0] > first[1]
+    assert once()[1] == first[1]
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_layers_of_a_larger_model(session, dtype):
+    """One layer of each kind at widths that take the big product tiles, prompts longer than the window, cut and decoded."""
+    c = config_of([delta_layer(8, 4, 64, 128, 1536), attention_layer(16, 4, 64, 64, 200, 1536, every=100)], 1024, 1024,
+                  loop={"start": 0, "stop": 2, "times": 2})
+    p = {n: bf16(w) for n, w in random_params(c, 5, low_rank=32)}
+    session.clear_params()
+    session.load_config(c, dtype)
+    for n, w in p.items():
+        session.set_param(n, w)
+    t = np.random.default_rng(6).integers(0, 1024, size=330)
+    want = R.logits(c, p, t)
+    for portions in ([330], [300] + [1] * 30, [3, 2, 130, 4, 1, 150, 12, 28]):
+        C.close(C.run(session, t, portions), want, {"float32": 1e-4, "bfloat16": 4e-2}[dtype], f"portions {portions[:4]}, {dtype}")

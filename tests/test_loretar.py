@@ -1,0 +1,197 @@
+"""The Loretar model of the host driver on the CPU oracle: configuration, weights, request states, generation and the trace
+runner against the plain statement in loretar_reference.py."""
+import copy
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+from safetensors.torch import save_file
+
+import loretar_cases as C
+import loretar_reference as R
+from catgrad_amd.loretar import param_shapes
+from catgrad_amd.runner import Session, random_params
+from model_cases import TINY
+from oracle_loader import ORACLE_LIB, oracle_library
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+
+@pytest.fixture(scope="module")
+def session():
+    oracle_library()
+    return Session(ORACLE_LIB)
+
+
+@pytest.mark.parametrize("name", list(C.CONFIGS))
+def test_whole_prompt(session, name):
+    C.check_portions(session, name, "whole")
+
+
+@pytest.mark.parametrize("how", [h for h in C.PORTIONS if h != "whole"])
+@pytest.mark.parametrize("name", ["mixed", "odd_sizes", "a_window_of_one"])
+def test_portions(session, name, how):
+    C.check_portions(session, name, how)
+
+
+@pytest.mark.parametrize("name", ["mixed", "recurrence_only", "one_head_each"])
+def test_bfloat16_weights(session, name):
+    C.check_portions(session, name, "prompt_then_decode", "bfloat16")
+
+
+def test_one_token(session):
+    C.check_one_token(session, "mixed")
+
+
+def test_interleaved_requests(session):
+    C.check_interleaved(session, "mixed")
+
+
+def test_long_decode(session):
+    C.check_long_decode(session, "no_loop")
+
+
+@pytest.mark.parametrize("name", ["mixed", "attention_only"])
+def test_generate(session, name):
+    C.check_generate(session, name, steps=6)
+
+
+def test_batch_logits(session):
+    C.check_batch_logits(session, "mixed")
+
+
+def test_recorded_schedules(session):
+    """The layered and the recorded evaluation orders run the same operations."""
+    C.load(session, "mixed")
+    t = C.tokens_of("mixed", 30)
+    want = C.run(session, t, [20, 1, 9])
+    try:
+        for schedule in (1, 2):
+            session.set_schedule(schedule)
+            np.testing.assert_array_equal(C.run(session, t, [20, 1, 9]), want)
+    finally:
+        session.set_schedule(0)
+
+
+def test_a_parameter_set_again_is_used(session):
+    p = C.load(session, "mixed")
+    t = C.tokens_of("mixed", 12)
+    C.run(session, t, [12])
+    p["l1.mix.k"] = p["l1.mix.k"] * np.float32(-0.5)
+    session.set_param("l1.mix.k", p["l1.mix.k"])
+    C.close(C.run(session, t, [12]), R.logits(C.CONFIGS["mixed"], p, t), 5e-5, "after a parameter was set again")
+
+
+def write_model(folder, name, seed=0):
+    p = C.params_of(name, seed)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(C.CONFIGS[name], f)
+    save_file({n: torch.from_numpy(np.ascontiguousarray(w)).to(torch.bfloat16) for n, w in p.items()}, os.path.join(folder, "model.safetensors"))
+    return p
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_a_model_folder(session, tmp_path, dtype):
+    p = write_model(tmp_path, "everything_looped")
+    stats = session.load_pretrained(tmp_path, dtype)
+    assert stats["tensors"] == len(p)
+    t = C.tokens_of("everything_looped", 30)
+    C.close(C.run(session, t, [20, 1, 9]), R.logits(C.CONFIGS["everything_looped"], p, t), C.TOLERANCE[dtype], f"model folder, {dtype}")
+
+
+def test_trace_run(tmp_path):
+    """Two requests step by step through the program: wanted places, steps without any, ends, and a name used again."""
+    model, out = tmp_path / "model", tmp_path / "out"
+    model.mkdir(), out.mkdir()
+    p = write_model(model, "mixed")
+    c = C.CONFIGS["mixed"]
+    a, b = C.tokens_of("mixed", 26, 1), C.tokens_of("mixed", 9, 2)
+    steps = [{"step": 0, "entries": [{"id": "x", "tokens": a[:20].tolist(), "want": [0, 19]}], "end": []},
+             {"step": 1, "entries": [{"id": "y", "tokens": b[:7].tolist(), "want": []}], "end": []},
+             {"step": 2, "entries": [{"id": "x", "tokens": a[20:].tolist(), "want": [5, 2]}], "end": ["x"]},
+             {"step": 3, "entries": [{"id": "x", "tokens": b.tolist(), "want": [8]}], "end": []},
+             {"step": 5, "entries": [{"id": "y", "tokens": b[7:].tolist(), "want": [1]}, {"id": "x", "tokens": [3], "want": [0]}], "end": ["x", "y"]}]
+    r = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", str(model), "--dtype", "float32", "--out", str(out),
+                        "--max-tokens", "64", "--backend-library", ORACLE_LIB], input="".join(json.dumps(s) + "\n" for s in steps), text=True,
+                       stdout=subprocess.PIPE, timeout=120)
+    assert r.returncode == 0
+    assert [l for l in r.stdout.splitlines() if l.startswith("done")] == [f"done {s['step']}" for s in steps]
+    assert sorted(os.listdir(out)) == ["0.f32", "2.f32", "3.f32", "5.f32"]
+    la, lb = R.logits(c, p, a), R.logits(c, p, list(b) + [3])
+    for step, want in ((0, la[[0, 19]]), (2, la[[25, 22]]), (3, lb[[8]]), (5, lb[[8, 9]])):
+        got = np.fromfile(out / f"{step}.f32", "<f4").reshape(len(want), c["vocab"])
+        C.close(got, want, 5e-5, f"step {step}")
+    bad = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", str(tmp_path), "--dtype", "float32", "--out", str(out),
+                          "--max-tokens", "64", "--backend-library", ORACLE_LIB], input="", text=True, stderr=subprocess.PIPE, timeout=120)
+    assert bad.returncode != 0
+
+
+def changed(name, edit):
+    c = copy.deepcopy(C.CONFIGS[name])
+    edit(c)
+    return c
+
+
+@pytest.mark.parametrize("edit", [
+    lambda c: c["layers"][0].update(type="convolution"), lambda c: c["layers"][0]["mixer"].update(kv_heads=3),
+    lambda c: c["layers"][0]["mlp"].update(kind="sparse"), lambda c: c["loop"].update(stop=9), lambda c: c["loop"].update(times=0),
+    lambda c: c["layers"][0]["mixer"]["mask"].update(size=0), lambda c: c["layers"][0]["mixer"]["q_temp"].update(every=0),
+    lambda c: c["layers"][1]["mixer"].update(conv=0), lambda c: c.pop("width"), lambda c: c["layers"][0]["mixer"].update(heads=2.5),
+    lambda c: c.update(architecture="Nothing")], ids=range(11))
+def test_configurations_that_do_not_fit(session, edit):
+    with pytest.raises(RuntimeError):
+        session.load_config(changed("mixed", edit))
+    with pytest.raises(RuntimeError):
+        session.load_config("{\"architecture\": \"Loretar\"")
+
+
+def test_parameters_that_do_not_fit(session):
+    p = C.load(session, "mixed")
+    t = C.tokens_of("mixed", 4)
+    session.set_param("l0.mix.talk", np.eye(3, dtype=np.float32))
+    with pytest.raises(RuntimeError, match="l0.mix.talk"):
+        session.step(1, t)
+    session.set_param("l0.mix.talk", p["l0.mix.talk"])
+    session.step(1, t)
+    with pytest.raises(RuntimeError):
+        session.step(1, t, rows=[4])
+    with pytest.raises(RuntimeError):
+        session.step(1, [])
+    session.end(1)
+    session.clear_params()
+    with pytest.raises(RuntimeError, match="MissingParameter"):
+        session.step(1, t)
+    session.end(1)
+    assert session.requests_in_progress() == 0
+
+
+def test_the_shapes_of_a_configuration():
+    for name, c in C.CONFIGS.items():
+        names = [n for n, _ in param_shapes(c)]
+        assert len(names) == len(set(names))
+        assert ("loop.in" in names) == bool(c["loop"]), name
+        for i, l in enumerate(c["layers"]):
+            assert (f"l{i}.rg2" in names) == (f"l{i}.mlp.up" in names) == bool(l["mlp"])
+
+
+def test_other_architectures_by_configuration(session):
+    """A Llama and a Qwen3 configuration through the registry: the same model as through its fields, and request steps."""
+    for name in ("tiny_llama", "tiny_qwen3"):
+        cfg = TINY[name]
+        params = list(random_params(cfg, 3))
+        session.load_model(cfg, params=params)
+        t = np.random.default_rng(4).integers(0, cfg.vocab_size, size=(1, 14), dtype=np.uint32)
+        _, want = session.forward(t, max_positions=32)
+        session.load_config({"model_type": cfg.arch, "hidden_size": cfg.hidden_size, "num_hidden_layers": cfg.num_hidden_layers,
+                             "num_attention_heads": cfg.num_attention_heads, "num_key_value_heads": cfg.num_key_value_heads, "head_dim": cfg.hd,
+                             "intermediate_size": cfg.intermediate_size, "vocab_size": cfg.vocab_size, "rms_norm_eps": cfg.rms_norm_eps,
+                             "rope_theta": cfg.rope_theta, "tie_word_embeddings": cfg.tie_word_embeddings})
+        got = np.concatenate([session.step(1, t[0, :9], range(9), max_positions=32), session.step(1, t[0, 9:], range(5), max_positions=32)])
+        session.end(1)
+        np.testing.assert_allclose(got, want[0], rtol=1e-4, atol=1e-5)
+    with pytest.raises(RuntimeError):
+        session.load_config({"model_type": "llama"}, "bfloat16")
