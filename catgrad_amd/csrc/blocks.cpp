@@ -119,7 +119,7 @@ int check_sizes(int64_t rows, int64_t a, int64_t b) {
 
 // in[rows, k] . w^T -> y [rows, n] (dense f32) for any number of rows: the operand in memory in the form the weights ask
 // for, then the general product.
-int general_product(cg_backend *be, Held &h, const ProductInput &in, uint32_t rows, cg_tensor *w, float *y) {
+int general_product(cg_backend *be, Held &h, const ProductInput &in, uint32_t rows, const Weight &weight, cg_tensor *w, float *y) {
     const bool bf16 = w->dt == CG_BF16;
     const int64_t K = in.k, N = w->dims[0];
     cg_tensor wt; // w^T, on the stack; its buffer is borrowed
@@ -167,17 +167,23 @@ int general_product(cg_backend *be, Held &h, const ProductInput &in, uint32_t ro
     } else {
         // patterns when the product reads them as they lie, else words that hold rounded values
         int fmt = kFmtWords;
-        if (bf16 && rows >= 256 && K % 8 == 0) {
+        bool tiles = false; // the product is for the 128-wide tiles: it does not fill the device with the others
+        if (bf16 && K % 8 == 0 && (rows >= 256 || takes_bf16_tiles(rows, weight))) {
             rc = new_dense(be, CG_BF16, xd, 2, &x, 0, kFmtBF16);
-            if (!rc && launch_matmul(be, x, &wt, nullptr) == CG_OK) fmt = kFmtBF16;
+            tiles = !rc && (rows < 256 || launch_matmul(be, x, &wt, nullptr) != CG_OK);
+            if (!rc && (!tiles || takes_bf16_tiles(rows, weight))) fmt = kFmtBF16;
             else if (!rc) {
+                tiles = false;
                 release(x);
                 x = nullptr;
             }
         }
         if (!rc && !x) rc = new_dense(be, w->dt, xd, 2, &x);
         if (!rc) rc = launch_product_input(be, in, rows, x->buf->ptr, bf16, fmt);
-        if (!rc) rc = launch_matmul(be, x, &wt, &out);
+        if (!rc) {
+            const int trc = tiles ? launch_bf16_tiles(be, x->buf->ptr, rows, weight, y) : kDeclined;
+            rc = trc == kDeclined ? launch_matmul(be, x, &wt, &out) : trc;
+        }
         h.add(x);
     }
     wt.buf = nullptr;
@@ -321,7 +327,7 @@ int cg_block_linear(cg_backend *b, const cg_linear_args *a, cg_tensor **out) {
         if (few_rows_slots((uint64_t)rows, (uint64_t)staged_pitch((uint32_t)K) * 4)) {
             rc = launch_few_rows_linear(b, in, (uint32_t)rows, w, bias, a->scale, y);
         } else {
-            rc = general_product(b, h, in, (uint32_t)rows, wv, y);
+            rc = general_product(b, h, in, (uint32_t)rows, w, wv, y);
             if (!rc && (bias || a->scale != 1.0f)) rc = launch_affine_rows(b, y, (uint32_t)rows, w.n, bias, a->scale);
         }
     }
@@ -376,7 +382,7 @@ int cg_block_residual(cg_backend *b, cg_tensor *x, const cg_branch *br, size_t n
             for (size_t i = 0; i < n && !rc; i++) {
                 void *p = nullptr;
                 rc = tmp.get((size_t)rows * width * 4, &p);
-                if (!rc) rc = general_product(b, h, r[i].in, (uint32_t)rows, wv[i], static_cast<float *>(p));
+                if (!rc) rc = general_product(b, h, r[i].in, (uint32_t)rows, r[i].w, wv[i], static_cast<float *>(p));
                 t[i].y = static_cast<const float *>(p);
                 t[i].gate = r[i].gate;
                 t[i].gate_bias = r[i].gate_bias;

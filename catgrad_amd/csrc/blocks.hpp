@@ -51,6 +51,10 @@ struct ResidualBranch {
 bool takes_few_rows_residual(const ResidualBranch *br, int n, uint32_t rows);
 int launch_few_rows_residual(cg_backend *be, const Rows &x, const ResidualBranch *br, int n, uint32_t rows, uint32_t width, float *out);
 
+// y[rows, w.n] = x . w^T of dense bfloat16 patterns x [rows, w.k] on 128-wide tiles; kDeclined: operands it does not take.
+int launch_bf16_tiles(cg_backend *be, const void *x, uint32_t rows, const Weight &w, float *y);
+bool takes_bf16_tiles(uint32_t rows, const Weight &w);
+
 // dst[r, 0 .. k) = the product input of row r, as 32-bit words (bf16: rounded to it first) or bfloat16 patterns
 int launch_product_input(cg_backend *be, const ProductInput &in, uint32_t rows, void *dst, bool round_bf16, int fmt);
 // y[r, n] = y[r, n] * scale + bias[n] in place
