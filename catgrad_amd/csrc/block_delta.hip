@@ -1,4 +1,4 @@
-// Gated delta rule with a decay per key channel (cg_block_channel_delta).
+// The delta rule with a state that decays channel by channel (cg_block_channel_delta).
 //
 // A few new tokens (a decode step): delta_step_kernel, a workgroup per (sequence, head) that does everything from the
 // convolutions to the gated norm, the state in registers from the first token to the last.

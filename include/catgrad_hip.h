@@ -268,21 +268,21 @@ typedef struct cg_linear_args {
 int cg_block_linear(cg_backend *b, const cg_linear_args *a, cg_tensor **out);
 
 /* out = x + sum_i sigmoid(gate_i + gate_bias_i) * (act_i(y_i) . w_i^T): the residual stream after up to two sublayers that
- * read the same input.  act is the identity, or with poly = [a, b, c, e] the polynomial norm
- * a N(z) + b N(z^2) + c N(z^3) + e, where N divides a row by its root mean square (eps inside the root). */
+ * read the same input.  act is the identity, or with poly = [p1, p2, p3, p0] the row-normed cubic
+ * p0 + sum_{n=1..3} pn y^n / sqrt(mean(y^(2n)) + eps), the mean over the row. */
 typedef struct cg_branch {
     cg_tensor *y, *w, *gate, *gate_bias, *poly; /* gate (with gate_bias) and poly: may be null */
 } cg_branch;
 int cg_block_residual(cg_backend *b, cg_tensor *x, const cg_branch *branches, size_t n, float eps, cg_tensor **out);
 
 /* Causal attention of S new tokens (positions position .. position + S - 1) behind a cache.
- *  q [B, S, heads * dim], k [B, S, kv_heads * dim], v [B, S, kv_heads * vdim]; query head h reads key / value head
- *  h / (heads / kv_heads).
- *  q_norm / k_norm: RMS norm over a token's whole projection (all heads at once).
- *  temp_every > 0: the query at position p is multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1).
- *  score(i, j) = scale * q_i . k_j, minus 2^(-8 (h + 1) / heads) * (i - j) with distance_bias.
- *  window > 0: position i sees 0 <= i - j < window; window == 0: every j <= i.
- *  talk [heads, heads]: after the soft-max, weight_h <- sum_g talk[h, g] weight_g.
+ *  q [B, S, heads * dim], k [B, S, kv_heads * dim], v [B, S, kv_heads * vdim]: consecutive runs of heads / kv_heads
+ *  query heads share a key / value head.
+ *  q_norm / k_norm [heads * dim] / [kv_heads * dim]: RMS norms over a token's query / key row, all its heads together.
+ *  temp_every > 0: a query at position p grows by the factor 1 + temp_coef * log1p((p + 1) div temp_every).
+ *  The score of key j for query i and head number n = 1 .. heads is scale * <q_i, k_j>, and with distance_bias also
+ *  - (i - j) / 2^(8 n / heads); a window hides the keys j <= i - window (window == 0: none).
+ *  talk [heads, heads]: the soft-max weights W [heads, S * keys] become talk . W.
  *  k_cache [B, kv_heads, T, dim], v_cache [B, kv_heads, T, vdim]: the keys (as they enter the scores) and values of the T
  *  positions before `position`, at least min(position, window - 1) of them.  The results k_out / v_out hold the last
  *  min(T + S, window - 1) positions (all of them without a window) and are appended in place when they end at the
@@ -295,15 +295,14 @@ typedef struct cg_attention_args {
 } cg_attention_args;
 int cg_block_attention(cg_backend *b, const cg_attention_args *a, cg_tensor **out, cg_tensor **k_out, cg_tensor **v_out);
 
-/* Gated delta rule with a decay per key channel.
- *  q, k [B, S, kv_heads * dim], v [B, S, heads * vdim]: each through a causal convolution over time per channel
- *  (conv_* [channels, taps], last column = the current token) and silu; q and k are then unit vectors per head,
- *  x / sqrt(sum(x^2) + 1e-6), and q is multiplied by dim^(-1/2); head h uses q / k head h / (heads / kv_heads).
- *  beta [B, S, heads]: through a sigmoid.  decay [B, S, r] . decay_w^T [heads * dim, r] = a, and the factor on the state's
- *  row (h, d) is exp(-exp(a_log[h]) * softplus(a + dt_bias)).
- *  Per head: S <- g * S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.
- *  o is divided by its root mean square over vdim (eps inside the root), times norm [vdim], times
- *  sigmoid(gate [B, S, r2] . gate_w^T [heads * vdim, r2]).
+/* Delta rule whose state decays channel by channel, with an output gate.
+ *  q, k [B, S, kv_heads * dim], v [B, S, heads * vdim] (consecutive runs of heads / kv_heads heads share a q / k head) go
+ *  through conv_* [channels, taps], a causal filter over time with its taps in time order, and x sigmoid(x).  Then
+ *  k^ = k / sqrt(|k|^2 + 10^-6) and q^ = q / sqrt(dim (|q|^2 + 10^-6)) per head.
+ *  With b = sigmoid(beta [B, S, heads]) and D = diag(exp(-exp(a_log) log(1 + exp(decay . decay_w^T + dt_bias)))), where
+ *  decay is [B, S, r], decay_w [heads * dim, r], a_log [heads] and dt_bias [heads * dim], a head's state is
+ *      M_t = D_t M_{t-1} + b_t k^_t (v_t - (D_t M_{t-1})^T k^_t)^T,     and it reads y_t = M_t^T q^_t.
+ *  out = RMS norm of y over vdim with the weights norm [vdim], times sigmoid(gate [B, S, r2] . gate_w [heads * vdim, r2]^T).
  *  state [B, heads, dim, vdim] f32, conv_state [B, taps - 1, channels of q, k, v]: the convolutions' last inputs. */
 typedef struct cg_channel_delta_args {
     cg_tensor *q, *k, *v, *conv_q, *conv_k, *conv_v, *beta, *decay, *decay_w, *a_log, *dt_bias, *gate, *gate_w, *norm, *state,

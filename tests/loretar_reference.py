@@ -19,7 +19,7 @@ def softplus(x):
 
 
 def rms(x, eps):
-    """x divided by its root mean square over the last axis."""
+    """x at a mean square of one along the last axis."""
     return x / np.sqrt((x * x).mean(-1, keepdims=True) + eps)
 
 
@@ -77,7 +77,7 @@ def attention_mixer(h, W, p, m, eps):
 
 
 def short_conv(x, taps):
-    """Causal convolution per channel: x [S, C], taps [C, n], the last column is the current token's."""
+    """Causal convolution per channel: x [S, C], taps [C, n] in time order."""
     S, C = x.shape
     n = taps.shape[1]
     padded = np.concatenate([np.zeros((n - 1, C)), x])
