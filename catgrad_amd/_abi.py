@@ -30,9 +30,31 @@ _SZP = C.POINTER(C.c_size_t)
 _I = C.c_int
 
 
-# cg_linear_args, cg_branch, cg_attention_args, cg_channel_delta_args
+# cg_linear_args, cg_pair_embedding_args, cg_conv_input, cg_conv_linear_args, cg_experts, cg_branch, cg_token_side_args,
+# cg_attention_args, cg_channel_delta_args
 class LinearArgs(C.Structure):
-    _fields_ = [(n, _P) for n in ("x", "x2", "gamma", "w", "bias")] + [("eps", C.c_float), ("scale", C.c_float)]
+    _fields_ = [(n, _P) for n in ("x", "x2", "gamma", "w", "bias")] + [("eps", C.c_float), ("scale", C.c_float), ("groups", _SZ)]
+
+
+class PairEmbeddingArgs(C.Structure):
+    _fields_ = [(n, _P) for n in ("ids", "previous", "table", "pairs")] + [("mul_prev", _SZ), ("mul_cur", _SZ)]
+
+
+class ConvInput(C.Structure):
+    _fields_ = [(n, _P) for n in ("gamma", "conv", "w")] + [("keep", _I), ("keep_bf16", _I)]
+
+
+class ConvLinearArgs(C.Structure):
+    _fields_ = [("x", _P), ("state", _P), ("in_", ConvInput * 2), ("n", _SZ), ("groups", _SZ), ("eps", C.c_float)]
+
+
+class Experts(C.Structure):
+    _fields_ = ([(n, _P) for n in ("h", "logits", "correction", "gate_up", "down")] + [(n, _SZ) for n in ("top", "groups", "keep")]
+                + [("limit", C.c_float), ("slope", C.c_float)])
+
+
+class TokenSideArgs(C.Structure):
+    _fields_ = ([(n, _P) for n in ("x", "ids", "table", "gate", "proj", "norm")] + [("first", _SZ), ("eps", C.c_float), ("scale", C.c_float)])
 
 
 class Branch(C.Structure):
@@ -42,7 +64,8 @@ class Branch(C.Structure):
 class AttentionArgs(C.Structure):
     _fields_ = ([(n, _P) for n in ("q", "k", "v", "q_norm", "k_norm", "talk", "k_cache", "v_cache")]
                 + [(n, _SZ) for n in ("heads", "kv_heads", "dim", "vdim", "position", "window", "temp_every")]
-                + [("scale", C.c_float), ("norm_eps", C.c_float), ("temp_coef", C.c_float), ("distance_bias", C.c_int)])
+                + [("scale", C.c_float), ("norm_eps", C.c_float), ("temp_coef", C.c_float), ("distance_bias", _I), ("rot_dims", _SZ),
+                   ("rot_base", C.c_double), ("unit_heads", _I), ("mix_scores", _I), ("zero_sink", _I)])
 
 
 class ChannelDeltaArgs(C.Structure):
@@ -97,7 +120,10 @@ SIGNATURES = {
     "cg_concat": (_I, [_P, _P, _P, _SZ, _PP]),
     "cg_index": (_I, [_P, _P, _SZ, _P, _PP]),
     "cg_block_linear": (_I, [_P, C.POINTER(LinearArgs), _PP]),
-    "cg_block_residual": (_I, [_P, _P, C.POINTER(Branch), _SZ, C.c_float, _PP]),
+    "cg_block_pair_embedding": (_I, [_P, C.POINTER(PairEmbeddingArgs), _PP, _PP]),
+    "cg_block_conv_linear": (_I, [_P, C.POINTER(ConvLinearArgs), _PP, _PP, _PP]),
+    "cg_block_residual": (_I, [_P, _P, C.POINTER(Branch), _SZ, C.c_float, C.c_float, C.POINTER(Experts), _PP]),
+    "cg_block_token_side": (_I, [_P, C.POINTER(TokenSideArgs), _PP]),
     "cg_block_attention": (_I, [_P, C.POINTER(AttentionArgs), _PP, _PP, _PP]),
     "cg_block_channel_delta": (_I, [_P, C.POINTER(ChannelDeltaArgs), _PP, _PP, _PP]),
 }

@@ -331,14 +331,40 @@ class Backend:
                 setattr(a, name, self._take(t))
         return a
 
-    def block_linear(self, x, w, x2=None, gamma=None, bias=None, eps=0.0, scale=1.0) -> Tensor:
-        a = self._block(A.LinearArgs, dict(x=x, w=w, x2=x2, gamma=gamma, bias=bias), dict(eps=eps, scale=scale))
+    def block_linear(self, x, w, x2=None, gamma=None, bias=None, eps=0.0, scale=1.0, groups=0) -> Tensor:
+        a = self._block(A.LinearArgs, dict(x=x, w=w, x2=x2, gamma=gamma, bias=bias), dict(eps=eps, scale=scale, groups=groups))
         return self._op(lambda b, o: self._lib.cg_block_linear(b, C.byref(a), o))
 
-    def block_residual(self, x, branches, eps=0.0) -> Tensor:
-        """branches: dictionaries with y, w and optionally gate, gate_bias, poly."""
+    def block_pair_embedding(self, tensors: dict, **options):
+        """-> (rows, last tokens); tensors: ids, previous, table, pairs."""
+        a = self._block(A.PairEmbeddingArgs, tensors, options)
+        o = [C.c_void_p() for _ in range(2)]
+        self._check(self._lib.cg_block_pair_embedding(self._b, C.byref(a), *[C.byref(p) for p in o]))
+        return tuple(Tensor(self, p.value) for p in o)
+
+    def block_conv_linear(self, x, state, inputs, groups=1, eps=0.0):
+        """inputs: up to two dictionaries with gamma, conv, w and optionally keep, keep_bf16.  -> (products, normed and
+        filtered inputs (None where not kept), state)"""
+        a = A.ConvLinearArgs(n=len(inputs), groups=groups, eps=eps)
+        a.x, a.state = self._take(x), self._take(state)
+        for i, d in enumerate(inputs):
+            flags = {k: int(d[k]) for k in ("keep", "keep_bf16") if k in d}
+            a.in_[i] = self._block(A.ConvInput, {k: v for k, v in d.items() if k not in flags}, flags)
+        y, h, s = (C.c_void_p * 2)(), (C.c_void_p * 2)(), C.c_void_p()
+        self._check(self._lib.cg_block_conv_linear(self._b, C.byref(a), y, h, C.byref(s)))
+        return ([Tensor(self, y[i]) for i in range(len(inputs))], [Tensor(self, h[i]) if h[i] else None for i in range(len(inputs))],
+                Tensor(self, s.value))
+
+    def block_residual(self, x, branches, eps=0.0, scale=1.0, experts=None, **expert_options) -> Tensor:
+        """branches: dictionaries with y, w and optionally gate, gate_bias, poly; experts: a dictionary with h, logits,
+        gate_up, down and optionally correction."""
         br = (A.Branch * max(len(branches), 1))(*[self._block(A.Branch, d, {}) for d in branches])
-        return self._op(lambda b, o: self._lib.cg_block_residual(b, self._take(x), br, len(branches), eps, o))
+        ex = C.byref(self._block(A.Experts, experts, expert_options)) if experts else None
+        return self._op(lambda b, o: self._lib.cg_block_residual(b, self._take(x), br, len(branches), eps, scale, ex, o))
+
+    def block_token_side(self, tensors: dict, **options) -> Tensor:
+        a = self._block(A.TokenSideArgs, tensors, options)
+        return self._op(lambda b, o: self._lib.cg_block_token_side(b, C.byref(a), o))
 
     def _three(self, fn, a):
         o = [C.c_void_p() for _ in range(3)]

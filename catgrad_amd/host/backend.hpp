@@ -42,7 +42,7 @@ struct Abi {
     CGH_FN(cg_binary) CGH_FN(cg_where) CGH_FN(cg_matmul) CGH_FN(cg_sum) CGH_FN(cg_max) CGH_FN(cg_argmax)
     CGH_FN(cg_topk) CGH_FN(cg_broadcast) CGH_FN(cg_reshape) CGH_FN(cg_transpose) CGH_FN(cg_slice)
     CGH_FN(cg_concat) CGH_FN(cg_index) CGH_FN(cg_profile_enable) CGH_FN(cg_profile_read)
-    CGH_FN(cg_block_linear) CGH_FN(cg_block_residual) CGH_FN(cg_block_attention) CGH_FN(cg_block_channel_delta)
+    CGH_FN(cg_block_linear) CGH_FN(cg_block_pair_embedding) CGH_FN(cg_block_conv_linear) CGH_FN(cg_block_residual) CGH_FN(cg_block_token_side) CGH_FN(cg_block_attention) CGH_FN(cg_block_channel_delta)
 #undef CGH_FN
     void *handle = nullptr;
 
@@ -61,7 +61,7 @@ struct Abi {
         CGH_LOAD(cg_max) CGH_LOAD(cg_argmax) CGH_LOAD(cg_topk) CGH_LOAD(cg_broadcast) CGH_LOAD(cg_reshape)
         CGH_LOAD(cg_transpose) CGH_LOAD(cg_slice) CGH_LOAD(cg_concat) CGH_LOAD(cg_index)
         CGH_LOAD(cg_profile_enable) CGH_LOAD(cg_profile_read)
-        CGH_LOAD(cg_block_linear) CGH_LOAD(cg_block_residual) CGH_LOAD(cg_block_attention) CGH_LOAD(cg_block_channel_delta)
+        CGH_LOAD(cg_block_linear) CGH_LOAD(cg_block_pair_embedding) CGH_LOAD(cg_block_conv_linear) CGH_LOAD(cg_block_residual) CGH_LOAD(cg_block_token_side) CGH_LOAD(cg_block_attention) CGH_LOAD(cg_block_channel_delta)
 #undef CGH_LOAD
     }
     Abi(const Abi &) = delete;
@@ -265,14 +265,25 @@ class Backend {
     Tensor block_linear(const cg_linear_args &a) {
         return out([&](cg_tensor **o) { return abi_.cg_block_linear(b_, &a, o); });
     }
-    Tensor block_residual(Tensor x, const std::vector<cg_branch> &br, float eps) {
-        return out([&](cg_tensor **o) { return abi_.cg_block_residual(b_, x.into_raw(), br.data(), br.size(), eps, o); });
+    // -> rows, last tokens
+    std::vector<Tensor> block_pair_embedding(const cg_pair_embedding_args &a) {
+        return outs<2>([&](cg_tensor **o) { return abi_.cg_block_pair_embedding(b_, &a, &o[0], &o[1]); });
+    }
+    // -> products, kept inputs, state
+    std::vector<Tensor> block_conv_linear(const cg_conv_linear_args &a) {
+        return outs<5>([&](cg_tensor **o) { return abi_.cg_block_conv_linear(b_, &a, &o[0], &o[2], &o[4]); });
+    }
+    Tensor block_residual(Tensor x, const std::vector<cg_branch> &br, float eps, float scale, const cg_experts *experts) {
+        return out([&](cg_tensor **o) { return abi_.cg_block_residual(b_, x.into_raw(), br.data(), br.size(), eps, scale, experts, o); });
+    }
+    Tensor block_token_side(const cg_token_side_args &a) {
+        return out([&](cg_tensor **o) { return abi_.cg_block_token_side(b_, &a, o); });
     }
     std::vector<Tensor> block_attention(const cg_attention_args &a) {
-        return out3([&](cg_tensor **o) { return abi_.cg_block_attention(b_, &a, &o[0], &o[1], &o[2]); });
+        return outs<3>([&](cg_tensor **o) { return abi_.cg_block_attention(b_, &a, &o[0], &o[1], &o[2]); });
     }
     std::vector<Tensor> block_channel_delta(const cg_channel_delta_args &a) {
-        return out3([&](cg_tensor **o) { return abi_.cg_block_channel_delta(b_, &a, &o[0], &o[1], &o[2]); });
+        return outs<3>([&](cg_tensor **o) { return abi_.cg_block_channel_delta(b_, &a, &o[0], &o[1], &o[2]); });
     }
     bool to_bool(const Tensor &x) {
         calls++;
@@ -331,15 +342,17 @@ class Backend {
         }
         return Tensor(&abi_, o);
     }
-    template <class F> std::vector<Tensor> out3(F &&f) {
+    // a call of up to N results, without those that it has left out
+    template <size_t N, class F> std::vector<Tensor> outs(F &&f) {
         calls++;
-        cg_tensor *o[3] = {nullptr, nullptr, nullptr};
+        cg_tensor *o[N] = {};
         const auto t0 = std::chrono::steady_clock::now();
         const int rc = f(o);
         if (time_calls) seconds_in_backend += std::chrono::duration<double>(std::chrono::steady_clock::now() - t0).count();
         check(rc);
         std::vector<Tensor> r;
-        for (cg_tensor *t : o) r.emplace_back(&abi_, t);
+        for (cg_tensor *t : o)
+            if (t) r.emplace_back(&abi_, t);
         return r;
     }
     Tensor from_vec(cg_dtype dt, const void *data, size_t len, const Shape &shape) {

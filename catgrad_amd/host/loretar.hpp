@@ -8,10 +8,7 @@
 // same input are kept as one matrix; a parameter that went into it stays available under its name as a view.
 #pragma once
 
-#include "blocks.hpp"
-#include "json.hpp"
-#include "model.hpp"
-#include "nn.hpp"
+#include "layers.hpp"
 
 namespace cgh {
 
@@ -27,7 +24,7 @@ struct LoretarLayer {
 struct LoretarConfig {
     std::vector<LoretarLayer> layers;
     size_t vocab = 0, width = 0;
-    size_t loop_start = 0, loop_stop = 0, loop_times = 0; // times 0: no layer runs more than once
+    LayerLoop loop;
     float eps = 0.0f, logit_scale = 1.0f;
 
     static LoretarConfig read(const Json &j) {
@@ -75,39 +72,16 @@ struct LoretarConfig {
             }
             c.layers.push_back(o);
         }
-        if (const Json *lp = j.find("loop")) {
-            c.loop_start = lp->at("start").nat();
-            c.loop_stop = lp->at("stop").nat();
-            c.loop_times = lp->at("times").nat();
-            if (c.loop_start >= c.loop_stop || c.loop_stop > c.layers.size() || !c.loop_times) throw ConfigError("config: the loop does not fit the layers");
-        }
+        c.loop = LayerLoop::read(j, c.layers.size());
         if (!c.vocab || !c.width) throw ConfigError("config: sizes must be positive");
         return c;
     }
-
-    // One evaluation of a layer; `begins`: the pass of the loop that starts with it, or -1.
-    struct LayerRun {
-        size_t layer;
-        int begins;
-    };
-    std::vector<LayerRun> runs() const {
-        std::vector<LayerRun> r;
-        const size_t from = loop_times ? loop_start : layers.size(), to = loop_times ? loop_stop : layers.size();
-        for (size_t l = 0; l < from; l++) r.push_back({l, -1});
-        for (size_t t = 0; t < loop_times; t++)
-            for (size_t l = from; l < to; l++) r.push_back({l, l == from ? (int)t : -1});
-        for (size_t l = to; l < layers.size(); l++) r.push_back({l, -1});
-        return r;
-    }
 };
 
-class LoretarModel : public Model {
+class LoretarModel : public LayeredModel {
   public:
-    // weights: CG_F32, or CG_BF16 for matrices held and multiplied at bfloat16 precision
-    LoretarModel(Interpreter &i, const LoretarConfig &c, cg_dtype weights) : Model(i), c_(c), weights_(weights), runs_(c.runs()) {}
+    LoretarModel(Interpreter &i, const LoretarConfig &c, cg_dtype weights) : LayeredModel(i, weights), c_(c), runs_(c.loop.runs(c.layers.size())) {}
     size_t vocab_size() const override { return c_.vocab; }
-    bool selects_rows() const override { return true; }
-    void parameters_changed() override { prepared_ = false; }
 
     State empty_state(size_t B) override {
         State s;
@@ -135,13 +109,13 @@ class LoretarModel : public Model {
         x = cast(i, index(i, 0, std::move(x), i.param("embed")), CG_F32);
         x = reshape(i, Shape{B, S, W}, std::move(x));
         Tensor x0;
-        if (c_.loop_times) x0 = x;
+        if (c_.loop.times) x0 = x;
         Parts p;
         for (size_t r = 0; r < runs_.size(); r++) {
             const int begins = runs_[r].begins;
             if (begins >= 0) { // x <- loop.in [x; x0] + loop.step[pass]
                 Tensor step = reshape(i, Shape{W}, slice(i, 0, (size_t)begins, 1, i.param("loop.step")));
-                Tensor again = begins + 1 == (int)c_.loop_times ? std::move(x0) : x0;
+                Tensor again = begins + 1 == (int)c_.loop.times ? std::move(x0) : x0;
                 x = blocks::linear(i, std::move(x), std::move(again), Tensor(), i.param("loop.in"), std::move(step), {});
             }
             Tensor s0 = std::move(state[2 * r]), s1 = std::move(state[2 * r + 1]);
@@ -150,36 +124,26 @@ class LoretarModel : public Model {
             p.state.push_back(std::move(s1));
         }
         if (!want.tokens && !want.logits) return p;
-        if (want.rows) {
-            x = reshape(i, Shape{B * S, W}, std::move(x));
-            Tensor rows = i.backend.ndarray_from_vec_u32(want.rows->data(), want.rows->size(), Shape{want.rows->size()});
-            x = nn::unsqueeze(i, 0, index(i, 0, std::move(rows), std::move(x)));
-        }
         blocks::LinearOptions opt;
         opt.eps = c_.eps;
         opt.scale = c_.logit_scale;
-        x = blocks::linear(i, std::move(x), Tensor(), i.param("final.norm"), i.param("head"), Tensor(), opt);
-        if (want.logits) p.out.logits = x;
-        if (want.tokens) p.out.tokens = argmax(i, std::move(x));
+        p.out = head(std::move(x), want, opt);
         return p;
     }
 
     // The weight matrices that read a layer's normed input become one, everything that is multiplied takes the form it is
     // multiplied in, and the shapes are checked against the configuration.
-    void prepare() override {
-        if (prepared_) return;
-        Interpreter &i = i_;
+    void prepare_weights() override {
         expect("embed", {c_.vocab, c_.width});
         expect("head", {c_.vocab, c_.width});
         expect("final.norm", {c_.width});
         store("embed");
         store("head");
-        if (c_.loop_times) {
+        if (c_.loop.times) {
             expect("loop.in", {c_.width, 2 * c_.width});
-            expect("loop.step", {c_.loop_times, c_.width});
+            expect("loop.step", {c_.loop.times, c_.width});
             store("loop.in");
         }
-        in_.clear();
         for (size_t l = 0; l < c_.layers.size(); l++) {
             const LoretarLayer &c = c_.layers[l];
             const std::string p = "l" + std::to_string(l), m = p + ".mix";
@@ -229,50 +193,11 @@ class LoretarModel : public Model {
                 rows(p + ".rg2", c_.width);
                 expect(p + ".rg2.b", {c_.width});
             }
-            pack(p, parts);
+            stack(p + ".in", parts);
         }
-        i.backend.sync();
-        prepared_ = true;
     }
 
   private:
-    struct Part { // columns of the product that reads a layer's normed input
-        size_t at, n;
-    };
-
-    Shape dims(const std::string &name) {
-        auto it = i_.parameters.find(name);
-        if (it == i_.parameters.end()) throw InterpreterError("MissingParameter: " + name);
-        Shape s = it->second.shape();
-        if (s.empty()) throw InterpreterError("parameter " + name + " has no extents");
-        return s;
-    }
-    void expect(const std::string &name, const Shape &s) {
-        if (dims(name) != s) throw InterpreterError("parameter " + name + " does not have the shape the configuration asks for");
-    }
-    void store(const std::string &name) { i_.parameters[name] = i_.backend.cast(std::move(i_.parameters[name]), weights_); }
-
-    // One matrix of all `parts`, each beginning at a multiple of 8 rows; the parts' own names become views of it.
-    void pack(const std::string &p, const std::vector<std::string> &parts) {
-        Backend &be = i_.backend;
-        std::map<std::string, Part> where;
-        Tensor all;
-        size_t at = 0;
-        auto append = [&](Tensor t) { all = all ? be.concat(std::move(all), std::move(t), 0) : std::move(t); };
-        for (const std::string &name : parts) {
-            Tensor t = be.cast(std::move(i_.parameters[name]), CG_F32);
-            const size_t n = t.shape()[0], pad = (8 - n % 8) % 8;
-            append(std::move(t));
-            if (pad) append(be.zeros(Shape{pad, c_.width}, CG_F32));
-            where[name] = {at, n};
-            at += n + pad;
-        }
-        all = be.cast(std::move(all), weights_);
-        for (const std::string &name : parts) i_.parameters[name] = be.slice(all, 0, where[name].at, where[name].n);
-        i_.parameters[p + ".in"] = std::move(all);
-        in_[p] = std::move(where);
-    }
-
     Tensor layer(size_t l, size_t position, Tensor x, Tensor *s0, Tensor *s1) {
         using namespace ops;
         I &i = i_;
@@ -281,11 +206,7 @@ class LoretarModel : public Model {
         blocks::LinearOptions opt;
         opt.eps = c_.eps;
         Tensor h = blocks::linear(i, x, Tensor(), i.param(p + ".norm1"), i.param(p + ".in"), Tensor(), opt);
-        const std::map<std::string, Part> &where = in_.at(p);
-        auto part = [&](const std::string &name) {
-            const Part &w = where.at(name);
-            return slice(i, 2, w.at, w.n, h);
-        };
+        auto part = [&](const std::string &name) { return part_of(h, p + ".in", name); };
         std::vector<Tensor> r;
         if (c.mixer == LoretarLayer::ATTENTION) {
             blocks::AttentionTensors t{part(m + ".q"),          part(m + ".k"),          part(m + ".v"), i.param(m + ".q.norm"),
@@ -307,10 +228,7 @@ class LoretarModel : public Model {
     }
 
     LoretarConfig c_;
-    cg_dtype weights_;
-    std::vector<LoretarConfig::LayerRun> runs_;
-    std::map<std::string, std::map<std::string, Part>> in_;
-    bool prepared_ = false;
+    std::vector<LayerLoop::Run> runs_;
 };
 
 } // namespace cgh

@@ -5,6 +5,7 @@
 #include <memory>
 
 #include "loretar.hpp"
+#include "lufatar.hpp"
 #include "models.hpp"
 
 namespace cgh {
@@ -36,6 +37,7 @@ inline std::unique_ptr<Model> make_model(Interpreter &i, const Json &config, cg_
     else if (const Json *l = config.find("architectures"))
         if (!l->list().empty()) name = l->list()[0].str();
     if (name == "Loretar") return std::make_unique<LoretarModel>(i, LoretarConfig::read(config), weights);
+    if (name == "Lufatar") return std::make_unique<LufatarModel>(i, LufatarConfig::read(config), weights);
     int arch = name == "llama" || name == "LlamaForCausalLM" ? 0 : name == "qwen3" || name == "Qwen3ForCausalLM" ? 1 : -1;
     if (arch < 0) throw ConfigError("config: unknown architecture '" + name + "'");
     if (weights != CG_F32) throw ConfigError("config: this architecture runs in f32 only");

@@ -260,20 +260,75 @@ int cg_index(cg_backend *b, cg_tensor *x, size_t dim, cg_tensor *indices, cg_ten
  * product are taken at bfloat16 precision, or better, and the sums are f32.  Everything else is computed in f32. */
 
 /* out[.., n] = scale * sum_k norm(x | x2)[.., k] * w[n, k] + bias[n], where (x | x2) is x, followed by x2 along the last
- * axis when given, and norm is the RMS norm v / sqrt(mean(v^2) + eps) * gamma when gamma is given. */
+ * axis when given, and norm is the RMS norm v / sqrt(mean(v^2) + eps) * gamma when gamma is given.  groups > 1: the mean is
+ * taken in each of so many equal runs of v on its own (x2 absent then). */
 typedef struct cg_linear_args {
     cg_tensor *x, *x2, *gamma, *w, *bias; /* x2, gamma, bias: may be null */
     float eps, scale;
+    size_t groups; /* 0 or 1: one mean for all of v */
 } cg_linear_args;
 int cg_block_linear(cg_backend *b, const cg_linear_args *a, cg_tensor **out);
 
-/* out = x + sum_i sigmoid(gate_i + gate_bias_i) * (act_i(y_i) . w_i^T): the residual stream after up to two sublayers that
- * read the same input.  act is the identity, or with poly = [p1, p2, p3, p0] the row-normed cubic
- * p0 + sum_{n=1..3} pn y^n / sqrt(mean(y^(2n)) + eps), the mean over the row. */
+/* Rows of an embedding table, plus rows of a second one chosen by pairs of neighbouring tokens:
+ *   out[b, s] = table[ids[b, s]] + pairs[(ids[b, s - 1] * mul_prev + ids[b, s] * mul_cur) mod buckets]     (f32)
+ * in exact integer arithmetic, with pairs [buckets + 1, width], whose last row stands for the pair of a sequence's first
+ * token.  ids u32 [B, S]; previous u32 [B, n]: tokens in front of them, of which the last counts (n == 0: a sequence
+ * begins).  previous_out [B, 1]: the last of the new tokens. */
+typedef struct cg_pair_embedding_args {
+    cg_tensor *ids, *previous, *table, *pairs;
+    size_t mul_prev, mul_cur;
+} cg_pair_embedding_args;
+int cg_block_pair_embedding(cg_backend *b, const cg_pair_embedding_args *a, cg_tensor **out, cg_tensor **previous_out);
+
+/* Up to two products that read the same rows, each through a norm and a short filter over time of its own:
+ *   z_t = x_t with every one of `groups` equal runs divided by sqrt(its mean square + eps),
+ *   h_t = u_t + sum_{j < taps} conv[:, j] * u_{t - taps + 1 + j},  u = z * gamma  (zero before the sequence's start),
+ *   y = h . w^T.
+ * x [B, S, width]; state [B, taps - 1, width] f32: z of the last tokens before these, state_out of the last up to now.
+ * keep: h itself is a result too, f32, or with keep_bf16 CG_BF16. */
+typedef struct cg_conv_input {
+    cg_tensor *gamma, *conv, *w; /* conv: [width, taps], the same taps for all inputs */
+    int keep, keep_bf16;
+} cg_conv_input;
+typedef struct cg_conv_linear_args {
+    cg_tensor *x, *state;
+    cg_conv_input in[2];
+    size_t n, groups;
+    float eps;
+} cg_conv_linear_args;
+/* y [n]; h [n], untouched where an input has no `keep` */
+int cg_block_conv_linear(cg_backend *b, const cg_conv_linear_args *a, cg_tensor **y, cg_tensor **h, cg_tensor **state_out);
+
+/* A mixture of small gated feed-forward layers, of which every token uses `top`:
+ *   s = sigmoid(logits); choice = s + correction (correction may be null);
+ * the experts form `groups` equal runs, of which the `keep` with the largest sums of their two largest choices count; among
+ * their members the `top` with the largest choices are used (equal ones: the first), each weighted by its s:
+ *   sum_e s_e W2_e (g sigmoid(slope g) (u + 1)),  g = min(W1_e h, limit), u = clamp(W1'_e h, -limit, limit).
+ * h [B, S, width] f32 or CG_BF16; logits [B, S, experts]; gate_up [experts, 2, ff, width]: W1_e, then W1'_e;
+ * down [experts, width, ff]. */
+typedef struct cg_experts {
+    cg_tensor *h, *logits, *correction, *gate_up, *down;
+    size_t top, groups, keep;
+    float limit, slope;
+} cg_experts;
+
+/* out = x + scale * (sum_i sigmoid(gate_i + gate_bias_i) * (act_i(y_i) . w_i^T) + experts): the residual stream after up to
+ * two sublayers that read the same input and, when `experts` is given, a mixture of experts.  act is the identity, or with
+ * poly = [p1, p2, p3, p0] the row-normed cubic p0 + sum_{n=1..3} pn y^n / sqrt(mean(y^(2n)) + eps), the mean over the row. */
 typedef struct cg_branch {
     cg_tensor *y, *w, *gate, *gate_bias, *poly; /* gate (with gate_bias) and poly: may be null */
 } cg_branch;
-int cg_block_residual(cg_backend *b, cg_tensor *x, const cg_branch *branches, size_t n, float eps, cg_tensor **out);
+int cg_block_residual(cg_backend *b, cg_tensor *x, const cg_branch *branches, size_t n, float eps, float scale, const cg_experts *experts, cg_tensor **out);
+
+/* What a token's own vector adds to its row: out = x + scale * y / sqrt(mean(y^2) + eps) * norm with
+ * y = (gelu(x . gate^T) * e) . proj^T, gelu the tanh form and e = table[ids, first .. first + dim).
+ * x [B, S, width], ids u32 [B, S], gate [dim, width], proj [width, dim], norm [width]. */
+typedef struct cg_token_side_args {
+    cg_tensor *x, *ids, *table, *gate, *proj, *norm;
+    size_t first;
+    float eps, scale;
+} cg_token_side_args;
+int cg_block_token_side(cg_backend *b, const cg_token_side_args *a, cg_tensor **out);
 
 /* Causal attention of S new tokens (positions position .. position + S - 1) behind a cache.
  *  q [B, S, heads * dim], k [B, S, kv_heads * dim], v [B, S, kv_heads * vdim]: consecutive runs of heads / kv_heads
@@ -282,7 +337,12 @@ int cg_block_residual(cg_backend *b, cg_tensor *x, const cg_branch *branches, si
  *  temp_every > 0: a query at position p grows by the factor 1 + temp_coef * log1p((p + 1) div temp_every).
  *  The score of key j for query i and head number n = 1 .. heads is scale * <q_i, k_j>, and with distance_bias also
  *  - (i - j) / 2^(8 n / heads); a window hides the keys j <= i - window (window == 0: none).
- *  talk [heads, heads]: the soft-max weights W [heads, S * keys] become talk . W.
+ *  talk [heads, heads]: the soft-max weights W [heads, S * keys] become talk . W; with mix_scores it is the scores, before
+ *  keys are hidden and before the soft-max, that become talk . scores.
+ *  rot_dims > 0 (even): the pairs (2 i, 2 i + 1) among the first rot_dims values of every query and key head are turned by
+ *  the angle position * rot_base^(-2 i / rot_dims); unit_heads: every query and key head, turned already, is divided by
+ *  sqrt(its mean square + norm_eps).  Both after q_norm / k_norm.
+ *  zero_sink: the soft-max's sum has exp(0) added.
  *  k_cache [B, kv_heads, T, dim], v_cache [B, kv_heads, T, vdim]: the keys (as they enter the scores) and values of the T
  *  positions before `position`, at least min(position, window - 1) of them.  The results k_out / v_out hold the last
  *  min(T + S, window - 1) positions (all of them without a window) and are appended in place when they end at the
@@ -292,6 +352,9 @@ typedef struct cg_attention_args {
     size_t heads, kv_heads, dim, vdim, position, window, temp_every;
     float scale, norm_eps, temp_coef;
     int distance_bias;
+    size_t rot_dims;
+    double rot_base;
+    int unit_heads, mix_scores, zero_sink;
 } cg_attention_args;
 int cg_block_attention(cg_backend *b, const cg_attention_args *a, cg_tensor **out, cg_tensor **k_out, cg_tensor **v_out);
 

@@ -1398,6 +1398,14 @@ double mean_square(const double *x, size_t n) {
     return s / (double)n;
 }
 
+// every run of n values divided by the root of its mean square
+void unit_runs(std::vector<double> &x, size_t n, double eps) {
+    for (size_t at = 0; at < x.size(); at += n) {
+        const double d = std::sqrt(mean_square(&x[at], n) + eps);
+        for (size_t i = 0; i < n; i++) x[at + i] /= d;
+    }
+}
+
 // y[rows, n] = x[rows, k] . w[n, k]^T
 std::vector<double> product(const std::vector<double> &x, size_t rows, size_t k, const cg_tensor *w) {
     const size_t n = w->dims[0];
@@ -1442,10 +1450,10 @@ int cg_block_linear(cg_backend *, const cg_linear_args *a, cg_tensor **out) {
     }
     if (a->gamma) {
         std::vector<double> g = wide(a->gamma);
-        for (size_t r = 0; r < rows; r++) {
-            const double d = std::sqrt(mean_square(&x[r * k], k) + a->eps);
-            for (size_t i = 0; i < k; i++) x[r * k + i] = x[r * k + i] / d * g[i];
-        }
+        const size_t groups = std::max<size_t>(1, a->groups);
+        if (k % groups) return fail(CG_ERR_SHAPE, "block_linear: the groups do not divide the row");
+        unit_runs(x, k / groups, a->eps);
+        for (size_t i = 0; i < x.size(); i++) x[i] *= g[i % k];
     }
     std::vector<double> y = product(x, rows, k, a->w);
     std::vector<double> bias = a->bias ? wide(a->bias) : std::vector<double>(n, 0.0);
@@ -1457,12 +1465,170 @@ int cg_block_linear(cg_backend *, const cg_linear_args *a, cg_tensor **out) {
     return CG_OK;
 }
 
-int cg_block_residual(cg_backend *, cg_tensor *x, const cg_branch *br, size_t n, float eps, cg_tensor **out) {
+int cg_block_pair_embedding(cg_backend *, const cg_pair_embedding_args *a, cg_tensor **out, cg_tensor **previous_out) {
+    if (!a) return fail(CG_ERR_ARG, "null argument");
+    Owned own{{a->ids, a->previous, a->table, a->pairs}};
+    if (!a->ids || !a->previous || !a->table || !a->pairs || !out || !previous_out) return fail(CG_ERR_ARG, "null argument");
+    const size_t B = a->ids->dims[0], S = a->ids->dims[1], W = a->table->dims[1], V = a->table->dims[0], buckets = a->pairs->dims[0] - 1, P = a->previous->dims[1];
+    if (a->ids->rank != 2 || a->pairs->dims[1] != W || a->previous->dims[0] != B || !buckets) return fail(CG_ERR_SHAPE, "block_pair_embedding: incompatible shapes");
+    Vec<uint32_t> ids = dense<uint32_t>(a->ids), prev = dense<uint32_t>(a->previous);
+    std::vector<double> t = wide(a->table), h = wide(a->pairs), o(B * S * W);
+    cg_tensor *last = nullptr;
+    for (size_t b = 0; b < B; b++)
+        for (size_t s = 0; s < S; s++) {
+            const size_t id = ids[b * S + s];
+            if (id >= V) return fail(CG_ERR_RANGE, "block_pair_embedding: a token outside the table");
+            size_t row = buckets;
+            if (s || P) {
+                const unsigned __int128 before = s ? ids[b * S + s - 1] : prev[b * P + P - 1];
+                row = (size_t)((before * a->mul_prev + (unsigned __int128)id * a->mul_cur) % buckets);
+            }
+            for (size_t i = 0; i < W; i++) o[(b * S + s) * W + i] = t[id * W + i] + h[row * W + i];
+        }
+    const size_t ld[2] = {B, 1};
+    last = new_tensor(CG_U32, ld, 2);
+    for (size_t b = 0; b < B; b++) data_of<uint32_t>(last)[b] = ids[b * S + S - 1];
+    *out = result(o, {B, S, W});
+    *previous_out = last;
+    return CG_OK;
+}
+
+int cg_block_conv_linear(cg_backend *, const cg_conv_linear_args *a, cg_tensor **y, cg_tensor **h, cg_tensor **state_out) {
+    if (!a) return fail(CG_ERR_ARG, "null argument");
+    Owned own{{a->x, a->state}};
+    for (size_t i = 0; i < a->n && i < 2; i++) own.t.insert(own.t.end(), {a->in[i].gamma, a->in[i].conv, a->in[i].w});
+    for (const cg_tensor *t : own.t)
+        if (!t) return fail(CG_ERR_ARG, "null argument");
+    if (a->n < 1 || a->n > 2 || !y || !h || !state_out) return fail(CG_ERR_ARG, "block_conv_linear: bad argument");
+    const size_t B = a->x->dims[0], S = a->x->dims[1], W = a->x->dims[2], taps = a->in[0].conv->dims[1], past = taps - 1, groups = std::max<size_t>(1, a->groups);
+    if (a->x->rank != 3 || !taps || W % groups || numel(a->state) != B * past * W) return fail(CG_ERR_SHAPE, "block_conv_linear: incompatible shapes");
+    std::vector<double> x = wide(a->x), st = wide(a->state), z(B * (past + S) * W), keep(B * past * W);
+    unit_runs(x, W / groups, a->eps);
+    for (size_t b = 0; b < B; b++)
+        for (size_t t = 0; t < past + S; t++)
+            for (size_t i = 0; i < W; i++) z[(b * (past + S) + t) * W + i] = t < past ? st[(b * past + t) * W + i] : x[(b * S + t - past) * W + i];
+    for (size_t k = 0; k < a->n; k++) {
+        const cg_conv_input &in = a->in[k];
+        if (numel(in.gamma) != W || numel(in.conv) != W * taps || in.w->rank != 2 || in.w->dims[1] != W) return fail(CG_ERR_SHAPE, "block_conv_linear: incompatible shapes");
+        std::vector<double> g = wide(in.gamma), c = wide(in.conv), f(B * S * W);
+        for (size_t b = 0; b < B; b++)
+            for (size_t t = 0; t < S; t++)
+                for (size_t i = 0; i < W; i++) {
+                    double v = z[(b * (past + S) + past + t) * W + i] * g[i];
+                    for (size_t j = 0; j < taps; j++) v += c[i * taps + j] * z[(b * (past + S) + t + j) * W + i] * g[i];
+                    f[(b * S + t) * W + i] = v;
+                }
+        if (in.keep) {
+            const size_t d[3] = {B, S, W};
+            h[k] = new_tensor(in.keep_bf16 ? CG_BF16 : CG_F32, d, 3);
+            for (size_t i = 0; i < f.size(); i++) data_of<float>(h[k])[i] = (float)f[i];
+            round_tensor(h[k]);
+            f = wide(h[k]);
+        }
+        y[k] = result(product(f, B * S, W, in.w), {B, S, in.w->dims[0]});
+    }
+    for (size_t b = 0; b < B; b++)
+        for (size_t t = 0; t < past; t++)
+            for (size_t i = 0; i < W; i++) keep[(b * past + t) * W + i] = z[(b * (past + S) + S + t) * W + i];
+    *state_out = result(keep, {B, past, W});
+    return CG_OK;
+}
+
+// the experts that a token uses, by their choice scores
+static std::vector<size_t> choose(const std::vector<double> &choice, size_t top, size_t groups, size_t keep) {
+    const double none = -std::numeric_limits<double>::infinity();
+    const size_t size = choice.size() / groups;
+    std::vector<double> worth(groups), left(choice.size(), none);
+    for (size_t g = 0; g < groups; g++) {
+        std::vector<double> m(choice.begin() + g * size, choice.begin() + (g + 1) * size);
+        std::sort(m.rbegin(), m.rend());
+        worth[g] = m[0] + (size > 1 ? m[1] : 0.0);
+    }
+    auto take = [&](std::vector<double> &v) {
+        const size_t i = (size_t)(std::max_element(v.begin(), v.end()) - v.begin());
+        v[i] = none;
+        return i;
+    };
+    for (size_t k = 0; k < keep; k++) {
+        const size_t g = take(worth);
+        for (size_t i = g * size; i < (g + 1) * size; i++) left[i] = choice[i];
+    }
+    std::vector<size_t> r;
+    for (size_t k = 0; k < top; k++) r.push_back(take(left));
+    return r;
+}
+
+static int add_experts(const cg_experts &e, size_t rows, size_t width, float scale, std::vector<double> &o) {
+    if (e.gate_up->rank != 4 || e.down->rank != 3) return fail(CG_ERR_SHAPE, "experts: bad ranks");
+    const size_t E = e.gate_up->dims[0], F = e.gate_up->dims[2], groups = std::max<size_t>(1, e.groups), kept = e.groups ? e.keep : 1;
+    if (e.gate_up->dims[1] != 2 || e.gate_up->dims[3] != width || e.down->dims[0] != E || e.down->dims[1] != width || e.down->dims[2] != F ||
+        numel(e.h) != rows * width || numel(e.logits) != rows * E || (e.correction && numel(e.correction) != E))
+        return fail(CG_ERR_SHAPE, "experts: incompatible shapes");
+    if (E % groups || kept < 1 || kept > groups || e.top < 1 || e.top > kept * (E / groups)) return fail(CG_ERR_ARG, "experts: bad counts");
+    std::vector<double> h = wide(e.h), z = wide(e.logits), c(E, 0.0), w1 = wide(e.gate_up), w2 = wide(e.down);
+    if (e.correction) c = wide(e.correction);
+    for (double &v : h) v = operand(v, e.gate_up);
+    for (size_t r = 0; r < rows; r++) {
+        std::vector<double> choice(E), y(F);
+        for (size_t i = 0; i < E; i++) choice[i] = sigmoid(z[r * E + i]) + c[i];
+        for (size_t i : choose(choice, e.top, groups, kept)) {
+            for (size_t f = 0; f < F; f++) {
+                double g = 0, u = 0;
+                for (size_t k = 0; k < width; k++) {
+                    g += h[r * width + k] * w1[((i * 2) * F + f) * width + k];
+                    u += h[r * width + k] * w1[((i * 2 + 1) * F + f) * width + k];
+                }
+                g = std::min(g, (double)e.limit);
+                u = std::min(std::max(u, -(double)e.limit), (double)e.limit);
+                y[f] = operand(g * sigmoid(e.slope * g) * (u + 1.0), e.down);
+            }
+            for (size_t k = 0; k < width; k++) {
+                double v = 0;
+                for (size_t f = 0; f < F; f++) v += y[f] * w2[(i * width + k) * F + f];
+                o[r * width + k] += scale * sigmoid(z[r * E + i]) * v;
+            }
+        }
+    }
+    return CG_OK;
+}
+
+int cg_block_token_side(cg_backend *, const cg_token_side_args *a, cg_tensor **out) {
+    if (!a) return fail(CG_ERR_ARG, "null argument");
+    Owned own{{a->x, a->ids, a->table, a->gate, a->proj, a->norm}};
+    for (const cg_tensor *t : own.t)
+        if (!t) return fail(CG_ERR_ARG, "null argument");
+    if (!out) return fail(CG_ERR_ARG, "null argument");
+    const size_t width = a->x->dims[a->x->rank - 1], rows = numel(a->x) / width, dim = a->gate->dims[0], cols = a->table->dims[1];
+    if (a->gate->rank != 2 || a->gate->dims[1] != width || a->proj->rank != 2 || a->proj->dims[0] != width || a->proj->dims[1] != dim || numel(a->norm) != width ||
+        numel(a->ids) != rows || a->first + dim > cols)
+        return fail(CG_ERR_SHAPE, "block_token_side: incompatible shapes");
+    Vec<uint32_t> ids = dense<uint32_t>(a->ids);
+    std::vector<double> x = wide(a->x), t = wide(a->table), norm = wide(a->norm), g = product(x, rows, width, a->gate);
+    for (size_t r = 0; r < rows; r++) {
+        if (ids[r] >= a->table->dims[0]) return fail(CG_ERR_RANGE, "block_token_side: a token outside the table");
+        for (size_t i = 0; i < dim; i++) {
+            const double v = g[r * dim + i];
+            g[r * dim + i] = 0.5 * v * (1.0 + std::tanh(std::sqrt(2.0 / M_PI) * (v + 0.044715 * v * v * v))) * t[ids[r] * cols + a->first + i];
+        }
+    }
+    std::vector<double> y = product(g, rows, dim, a->proj);
+    unit_runs(y, width, a->eps);
+    for (size_t i = 0; i < x.size(); i++) x[i] += (double)a->scale * y[i] * norm[i % width];
+    *out = result(x, dims_of(a->x));
+    return CG_OK;
+}
+
+int cg_block_residual(cg_backend *, cg_tensor *x, const cg_branch *br, size_t n, float eps, float scale, const cg_experts *experts, cg_tensor **out) {
     Owned own{{x}};
     for (size_t i = 0; i < n; i++) own.t.insert(own.t.end(), {br[i].y, br[i].w, br[i].gate, br[i].gate_bias, br[i].poly});
+    if (experts) own.t.insert(own.t.end(), {experts->h, experts->logits, experts->correction, experts->gate_up, experts->down});
     if (!x || !out || n > 2) return fail(CG_ERR_ARG, "bad argument");
     const size_t width = x->dims[x->rank - 1], rows = numel(x) / width;
     std::vector<double> o = wide(x);
+    if (experts) {
+        if (!experts->h || !experts->logits || !experts->gate_up || !experts->down) return fail(CG_ERR_ARG, "null argument");
+        if (int rc = add_experts(*experts, rows, width, scale, o)) return rc;
+    }
     for (size_t i = 0; i < n; i++) {
         const cg_branch &b = br[i];
         const size_t k = b.y->dims[b.y->rank - 1];
@@ -1484,7 +1650,7 @@ int cg_block_residual(cg_backend *, cg_tensor *x, const cg_branch *br, size_t n,
         if (b.gate_bias) gb = wide(b.gate_bias);
         for (size_t r = 0; r < rows; r++)
             for (size_t j = 0; j < width; j++)
-                o[r * width + j] += p[r * width + j] * (b.gate ? sigmoid(g[r * width + j] + (b.gate_bias ? gb[j] : 0.0)) : 1.0);
+                o[r * width + j] += scale * p[r * width + j] * (b.gate ? sigmoid(g[r * width + j] + (b.gate_bias ? gb[j] : 0.0)) : 1.0);
     }
     *out = result(o, dims_of(x));
     return CG_OK;
@@ -1511,6 +1677,20 @@ int cg_block_attention(cg_backend *, const cg_attention_args *a, cg_tensor **out
     };
     norm(q, H * D, a->q_norm);
     norm(k, G * D, a->k_norm);
+    if (a->rot_dims > D || a->rot_dims % 2) return fail(CG_ERR_ARG, "block_attention: bad rotation");
+    for (auto *x : {&q, &k}) {
+        const size_t heads = x == &q ? H : G;
+        for (size_t r = 0; r < B * S; r++)
+            for (size_t i = 0; i < a->rot_dims / 2; i++) {
+                const double t = (double)(a->position + r % S) * std::pow(a->rot_base, -2.0 * (double)i / (double)a->rot_dims), co = std::cos(t), si = std::sin(t);
+                for (size_t g = 0; g < heads; g++) {
+                    double *p = &(*x)[(r * heads + g) * D + 2 * i], u = p[0], w = p[1];
+                    p[0] = u * co - w * si;
+                    p[1] = w * co + u * si;
+                }
+            }
+        if (a->unit_heads) unit_runs(*x, D, a->norm_eps);
+    }
     std::vector<double> talk;
     if (a->talk) talk = wide(a->talk);
     const size_t all = T + S, keep = a->window ? std::min(all, a->window - 1) : all, first = a->position - T;
@@ -1529,27 +1709,34 @@ int cg_block_attention(cg_backend *, const cg_attention_args *a, cg_tensor **out
             const size_t p = a->position + s, lo = a->window && p + 1 > a->window ? p + 1 - a->window : 0;
             const size_t j0 = lo > first ? lo - first : 0, j1 = T + s + 1;
             const double temp = a->temp_every ? 1.0 + a->temp_coef * std::log(std::floor((double)(p + 1) / (double)a->temp_every) + 1.0) : 1.0;
+            auto mix = [&](size_t j) { // talk over the column of key j
+                if (!a->talk) return;
+                for (size_t h = 0; h < H; h++) {
+                    mixed[h] = 0.0;
+                    for (size_t g = 0; g < H; g++) mixed[h] += talk[h * H + g] * w[g * all + j];
+                }
+                for (size_t h = 0; h < H; h++) w[h * all + j] = mixed[h];
+            };
             for (size_t h = 0; h < H; h++) {
                 const double slope = a->distance_bias ? std::pow(2.0, -8.0 * (double)(h + 1) / (double)H) : 0.0;
-                double m = -std::numeric_limits<double>::infinity(), sum = 0;
                 for (size_t j = j0; j < j1; j++) {
                     double x = 0;
                     for (size_t d = 0; d < D; d++) x += q[((b * S + s) * H + h) * D + d] * K[((b * G + h / rep) * all + j) * D + d];
-                    x = x * temp * a->scale - slope * (double)(p - (first + j));
-                    w[h * all + j] = x;
-                    m = std::max(m, x);
+                    w[h * all + j] = x * temp * a->scale - slope * (double)(p - (first + j));
                 }
+            }
+            for (size_t j = j0; j < j1 && a->mix_scores; j++) mix(j);
+            for (size_t h = 0; h < H; h++) {
+                double m = a->zero_sink ? 0.0 : -std::numeric_limits<double>::infinity(), sum = 0;
+                for (size_t j = j0; j < j1; j++) m = std::max(m, w[h * all + j]);
+                if (a->zero_sink) sum = std::exp(-m);
                 for (size_t j = j0; j < j1; j++) sum += w[h * all + j] = std::exp(w[h * all + j] - m);
                 for (size_t j = j0; j < j1; j++) w[h * all + j] /= sum;
             }
             for (size_t j = j0; j < j1; j++) {
-                for (size_t h = 0; h < H; h++) {
-                    mixed[h] = a->talk ? 0.0 : w[h * all + j];
-                    if (a->talk)
-                        for (size_t g = 0; g < H; g++) mixed[h] += talk[h * H + g] * w[g * all + j];
-                }
+                if (!a->mix_scores) mix(j);
                 for (size_t h = 0; h < H; h++)
-                    for (size_t d = 0; d < V; d++) o[((b * S + s) * H + h) * V + d] += mixed[h] * Vv[((b * G + h / rep) * all + j) * V + d];
+                    for (size_t d = 0; d < V; d++) o[((b * S + s) * H + h) * V + d] += w[h * all + j] * Vv[((b * G + h / rep) * all + j) * V + d];
             }
         }
     auto tail = [&](const std::vector<double> &x, size_t n) {
