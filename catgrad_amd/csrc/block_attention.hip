@@ -73,6 +73,61 @@ __global__ __launch_bounds__(kThreads) void attention_prepare_kernel(const Atten
     }
 }
 
+// The same with every head turned by its token's angles and brought to a mean square of one, a wave per head.
+__global__ __launch_bounds__(kThreads) void attention_turn_kernel(const AttentionPlan p, float *__restrict__ q) {
+    extern __shared__ float2 turn[]; // {cos, sin} per pair
+    __shared__ float red[kWaves];
+    const uint32_t r = blockIdx.x, b = r / p.S, s = r - b * p.S, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const uint32_t nq = p.heads * p.dim, nk = p.kv_heads * p.dim, nv = p.kv_heads * p.vdim;
+    const float *qr = p.q.p + (int64_t)r * p.q.pitch, *kr = p.k.p + (int64_t)r * p.k.pitch, *vr = p.v.p + (int64_t)r * p.v.pitch;
+    for (uint32_t i = threadIdx.x; i < p.rot_dims / 2; i += kThreads) {
+        double a = (double)(p.position + s) * exp2(-2.0 * (double)i / (double)p.rot_dims * p.rot_log2);
+        a -= 6.283185307179586 * rint(a * 0.15915494309189535);
+        float sn, cs;
+        sincosf((float)a, &sn, &cs);
+        turn[i] = make_float2(cs, sn);
+    }
+    float mq = 0.0f, mk = 0.0f;
+    if (p.q_norm)
+        for (uint32_t i = threadIdx.x; i < nq; i += kThreads) mq = fmaf(qr[i], qr[i], mq);
+    if (p.k_norm)
+        for (uint32_t i = threadIdx.x; i < nk; i += kThreads) mk = fmaf(kr[i], kr[i], mk);
+    float fq = 1.0f, fk = 1.0f;
+    if (p.q_norm) fq = 1.0f / sqrtf(block_sum(mq, red) / (float)nq + p.eps);
+    if (p.k_norm) fk = 1.0f / sqrtf(block_sum(mk, red) / (float)nk + p.eps);
+    float temp = p.scale;
+    if (p.temp_every) temp *= 1.0f + p.temp_coef * logf((float)((p.position + s + 1) / p.temp_every + 1));
+    __syncthreads();
+    for (uint32_t h = wave; h < p.heads + p.kv_heads; h += kWaves) {
+        const bool key = h >= p.heads;
+        const uint32_t g = h - p.heads;
+        const float *src = key ? kr + g * p.dim : qr + h * p.dim, *w = key ? p.k_norm : p.q_norm;
+        if (w) w += (key ? g : h) * p.dim;
+        float *dst = key ? p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)(p.cached + s) * p.dim : q + (int64_t)r * nq + h * p.dim;
+        const float f = key ? fk : fq;
+        auto plain = [&](uint32_t d) { return w ? src[d] * f * w[d] : src[d]; };
+        auto value = [&](uint32_t d) {
+            const float v = plain(d);
+            if (d >= p.rot_dims) return v;
+            const float2 cs = turn[d / 2];
+            return d & 1 ? fmaf(v, cs.x, plain(d - 1) * cs.y) : fmaf(v, cs.x, -plain(d + 1) * cs.y);
+        };
+        const float v0 = lane < p.dim ? value(lane) : 0.0f, v1 = lane + 64 < p.dim ? value(lane + 64) : 0.0f;
+        float m = fmaf(v0, v0, v1 * v1), c = key ? 1.0f : temp;
+        for (uint32_t d = lane + 128; d < p.dim; d += 64) {
+            const float v = value(d);
+            m = fmaf(v, v, m);
+        }
+        if (p.unit_heads) c /= sqrtf(wave_sum(m) / (float)p.dim + p.eps);
+        for (uint32_t d = lane; d < p.dim; d += 64) dst[d] = (d == lane ? v0 : d == lane + 64 ? v1 : value(d)) * c;
+    }
+    float *vc = p.values + (int64_t)b * p.kv_heads * p.v_block + (int64_t)(p.cached + s) * p.vdim;
+    for (uint32_t i = threadIdx.x; i < nv; i += kThreads) {
+        const uint32_t g = i / p.vdim, d = i - g * p.vdim;
+        vc[(int64_t)g * p.v_block + d] = vr[i];
+    }
+}
+
 // n consecutive floats of a row, 16 bytes at a time where they lie so
 __device__ __forceinline__ float row_squares(const float *__restrict__ x, uint32_t n) {
     float m = 0.0f;
@@ -230,7 +285,7 @@ __global__ __launch_bounds__(kThreads) void attention_mix_kernel(const Attention
     for (uint32_t h = threadIdx.x / kSeg; h < nm; h += kThreads / kSeg) ex[h * kSeg + key] = scores[(((int64_t)blockIdx.z * p.heads + first + h) * nseg + seg) * kSeg + key];
     for (uint32_t h = threadIdx.x; h < nm; h += kThreads) {
         const float2 *st = stats + ((int64_t)blockIdx.z * p.heads + first + h) * nseg;
-        float m = -INFINITY, l = 0.0f;
+        float m = p.zero_sink ? 0.0f : -INFINITY, l = p.zero_sink ? 1.0f : 0.0f;
 #pragma unroll 4
         for (uint32_t i = 0; i < nseg; i++) { // the running pair: one walk along the segments
             const float2 t = st[i];
@@ -331,10 +386,12 @@ int rows_kernels(cg_backend *be, const AttentionPlan &p, const float *q, uint32_
     const size_t lds1 = ((size_t)REP * p.dim + REP * kSeg + (fresh ? p.S * p.dim : 0)) * 4;
     const size_t lds2 = (size_t)mix_floats(REP, slots, MVW) * 4;
     if (int rc = fresh ? allow_lds(attention_scores_kernel<REP, SVW, true>, lds1) : allow_lds(attention_scores_kernel<REP, SVW, false>, lds1)) return rc;
-    if (int rc = allow_lds(attention_mix_kernel<REP, MVW>, lds2)) return rc;
+    if (!p.mix_scores)
+        if (int rc = allow_lds(attention_mix_kernel<REP, MVW>, lds2)) return rc;
     const dim3 grid(nseg, p.kv_heads * groups, rows);
     if (fresh) hipLaunchKernelGGL((attention_scores_kernel<REP, SVW, true>), grid, dim3(kThreads), lds1, be->stream, p, q, row0, nseg, scores, stats);
     else hipLaunchKernelGGL((attention_scores_kernel<REP, SVW, false>), grid, dim3(kThreads), lds1, be->stream, p, q, row0, nseg, scores, stats);
+    if (p.mix_scores) return launch_mixed_rows(be, p, row0, rows, nseg, scores, parts, reinterpret_cast<float2 *>(parts + (size_t)rows * nseg * p.heads * p.vdim));
     hipLaunchKernelGGL((attention_mix_kernel<REP, MVW>), grid, dim3(kThreads), lds2, be->stream, p, row0, nseg, scores, stats, nseg > 1 ? parts : p.out, nseg > 1);
     if (nseg > 1) {
         const uint32_t n = p.heads * p.vdim;
@@ -357,23 +414,25 @@ int rows_kernels(cg_backend *be, const AttentionPlan &p, const float *q, uint32_
 
 int launch_attention(cg_backend *be, const AttentionPlan &p) {
     const uint32_t rows = p.B * p.S, all = p.cached + p.S;
-    const bool fresh = p.S <= kFewRows && p.dim <= 512;
+    const bool turned = p.rot_dims || p.unit_heads, fresh = p.S <= kFewRows && p.dim <= 512 && !turned;
+    const uint32_t most = p.window ? std::min(p.window, all) : all, nseg = (most + kSeg - 1) / kSeg, rep = p.heads / p.kv_heads;
+    double pairs = 0.0; // visible (query, key) pairs
+    for (uint32_t s = 0; s < p.S; s++) pairs += (double)std::min(p.window ? p.window : ~0u, p.cached + s + 1);
+    ProfScope prof(be, CG_K_ATTENTION, pairs * p.B * p.heads * (2.0 * p.dim + 2.0 * p.vdim + (p.talk ? 2.0 * p.heads : 0.0)));
+    if (p.mix_scores)
+        if (int rc = launch_mixed_step(be, p); rc != kDeclined) return rc;
     Scratch qbuf(be);
     float *q = nullptr;
     if (!fresh) {
         if (int rc = qbuf.get((size_t)rows * p.heads * p.dim * 4)) return rc;
         q = static_cast<float *>(qbuf.p);
-        hipLaunchKernelGGL(attention_prepare_kernel, dim3(rows), dim3(kThreads), 0, be->stream, p, q);
+        if (turned) hipLaunchKernelGGL(attention_turn_kernel, dim3(rows), dim3(kThreads), (size_t)(p.rot_dims / 2) * sizeof(float2), be->stream, p, q);
+        else hipLaunchKernelGGL(attention_prepare_kernel, dim3(rows), dim3(kThreads), 0, be->stream, p, q);
         if (int rc = launched("attention_prepare")) return rc;
+        if (int rc = p.mix_scores ? launch_mixed_tiles(be, p, q) : launch_attention_tiles(be, p, q); rc != kDeclined) return rc;
     }
-    const uint32_t most = p.window ? std::min(p.window, all) : all, nseg = (most + kSeg - 1) / kSeg, rep = p.heads / p.kv_heads;
-    double pairs = 0.0; // visible (query, key) pairs
-    for (uint32_t s = 0; s < p.S; s++) pairs += (double)std::min(p.window ? p.window : ~0u, p.cached + s + 1);
-    ProfScope prof(be, CG_K_ATTENTION, pairs * p.B * p.heads * (2.0 * p.dim + 2.0 * p.vdim + (p.talk ? 2.0 * p.heads : 0.0)));
-    if (!fresh)
-        if (int rc = launch_attention_tiles(be, p, q); rc != kDeclined) return rc;
     // rows in parts that keep the scores within 64 MB
-    const size_t per_row = (size_t)p.heads * nseg * (kSeg * 4 + sizeof(float2)) + (nseg > 1 ? (size_t)nseg * p.heads * p.vdim * 4 : 0);
+    const size_t per_row = (size_t)p.heads * nseg * (kSeg * 4 + sizeof(float2)) + (nseg > 1 || p.mix_scores ? (size_t)nseg * p.heads * (p.vdim * 4 + (p.mix_scores ? sizeof(float2) : 0)) : 0);
     const uint32_t part = (uint32_t)std::max<size_t>(1, std::min<size_t>(std::min<size_t>(rows, 65535), (64u << 20) / per_row));
     Scratch mem(be);
     if (int rc = mem.get((size_t)part * per_row)) return rc;

@@ -1,0 +1,632 @@
+// cg_block_attention when the scores are mixed over the heads before the soft-max.  A query's mixed scores need every head's
+// score for the same key, but no other key's: the soft-max runs along, its results unfinished until the largest score and the
+// sum are known.
+//
+//   attention_mixed_step_kernel   a few new tokens: a workgroup per (token, segment of keys) for all heads, from the projections
+//                                 as they are to the segment's weighted values
+//   attention_mixed_tiles_kernel  prompts: 16 query rows of all heads against 16 keys at a time on v_mfma_f32_16x16x4; scores,
+//                                 mixing (the product talk . scores, a column per (query, key)) and soft-max with values run a
+//                                 key tile apart on three buffers, one barrier per tile
+//   attention_mixed_rows_kernel   other sizes: behind attention_scores_kernel, a workgroup per (token, kv head, 128 keys)
+//   attention_merge_kernel        the segments' unfinished results, each with its largest score and sum, become one
+//
+// Unfinished results carry {top, sum}: weights are 2^(score log2 e - top), `top` in units of log2.
+#include "blocks.hpp"
+#include "device_utils.hpp"
+
+#include <algorithm>
+
+namespace cg {
+namespace {
+
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+constexpr int kThreads = 256;
+constexpr uint32_t kSeg = 128; // keys of a segment of attention_scores_kernel
+constexpr float kLog2e = 1.44269504088896341f, kNone = -1e30f;
+
+__device__ __forceinline__ float wave_sum(float v) {
+#pragma unroll
+    for (int d = 32; d > 0; d >>= 1) v += __shfl_xor(v, d, 64);
+    return v;
+}
+__device__ __forceinline__ float wave_max(float v) {
+#pragma unroll
+    for (int d = 32; d > 0; d >>= 1) v = fmaxf(v, __shfl_xor(v, d, 64));
+    return v;
+}
+__device__ __forceinline__ float slope_of(uint32_t h, uint32_t heads) { return exp2f(-8.0f * (float)(h + 1) / (float)heads); }
+__device__ __forceinline__ uint32_t first_visible(const AttentionPlan &p, uint32_t i) { return p.window && i + 1 > p.window ? i + 1 - p.window : 0; }
+
+// out = the segments' results together; result i of a row: head i / vdim.  parts at row * row_pitch + segment * seg_pitch,
+// stats the same in heads.
+__global__ __launch_bounds__(kThreads) void attention_merge_kernel(const float *__restrict__ parts, const float2 *__restrict__ stats, const uint32_t segs, const uint64_t row_pitch,
+                                                                   const uint64_t seg_pitch, const uint32_t heads, const uint32_t vdim, const bool sink, float *__restrict__ out) {
+    const uint32_t n = heads * vdim, i = blockIdx.x * kThreads + threadIdx.x;
+    if (i >= n) return;
+    const uint64_t row = blockIdx.y;
+    const float *p = parts + row * row_pitch * vdim + i;
+    const float2 *st = stats + row * row_pitch + i / vdim;
+    float m = sink ? 0.0f : kNone;
+#pragma unroll 8
+    for (uint32_t k = 0; k < segs; k++) m = fmaxf(m, st[k * seg_pitch].x);
+    float l = sink ? __builtin_amdgcn_exp2f(-m) : 0.0f, o = 0.0f;
+#pragma unroll 8
+    for (uint32_t k = 0; k < segs; k++) {
+        const float2 t = st[k * seg_pitch];
+        const float f = __builtin_amdgcn_exp2f(t.x - m);
+        l = fmaf(t.y, f, l);
+        o = fmaf(p[k * seg_pitch * vdim], f, o);
+    }
+    out[row * n + i] = o / l;
+}
+
+// ---- other sizes -----------------------------------------------------------------------------------------------------
+__host__ __device__ constexpr uint32_t mixed_floats(uint32_t rep, uint32_t slots, uint32_t vw) { return slots * kSeg + rep * kSeg + rep * vw * kThreads; }
+
+template <int REP, int VW>
+__global__ __launch_bounds__(kThreads) void attention_mixed_rows_kernel(const AttentionPlan p, const uint32_t row0, const uint32_t nseg, const float *__restrict__ scores,
+                                                                        float *__restrict__ parts, float2 *__restrict__ stats) {
+    extern __shared__ float lds[];
+    const uint32_t rep = p.heads / p.kv_heads, groups = (rep + REP - 1) / REP;
+    const uint32_t g = blockIdx.y / groups, h0 = g * rep + (blockIdx.y - g * groups) * REP, nh = min((uint32_t)REP, (g + 1) * rep - h0);
+    const uint32_t r = row0 + blockIdx.z, b = r / p.S, s = r - b * p.S, seg = blockIdx.x;
+    const uint32_t first = p.talk ? 0 : h0, nm = p.talk ? p.heads : nh, slots = p.talk ? p.heads : REP;
+    float *raw = lds, *wt = raw + slots * kSeg, *red = wt + REP * kSeg;
+    const uint32_t hi = p.cached + s + 1, j0 = first_visible(p, p.cached + s) + seg * kSeg, keys = j0 < hi ? min(kSeg, hi - j0) : 0;
+    const uint32_t key = threadIdx.x % kSeg; // two threads share a key's column of scores
+    for (uint32_t h = threadIdx.x / kSeg; h < nm; h += kThreads / kSeg)
+        raw[h * kSeg + key] = key < keys ? scores[(((int64_t)blockIdx.z * p.heads + first + h) * nseg + seg) * kSeg + key] : 0.0f;
+    __syncthreads();
+    for (uint32_t o = threadIdx.x / kSeg; o < nh; o += kThreads / kSeg) {
+        float w = 0.0f;
+        if (p.talk) {
+            for (uint32_t h = 0; h < nm; h++) w = fmaf(p.talk[(int64_t)(h0 + o) * p.heads + h], raw[h * kSeg + key], w);
+        } else {
+            w = raw[o * kSeg + key];
+        }
+        wt[o * kSeg + key] = key < keys ? w * kLog2e : -INFINITY;
+    }
+    __syncthreads();
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    for (uint32_t o = wave; o < nh; o += kThreads / 64) {
+        const float a = wt[o * kSeg + lane], c = wt[o * kSeg + 64 + lane];
+        const float m = fmaxf(kNone, wave_max(fmaxf(a, c)));
+        const float ea = __builtin_amdgcn_exp2f(a - m), ec = __builtin_amdgcn_exp2f(c - m), l = wave_sum(ea + ec);
+        wt[o * kSeg + lane] = ea;
+        wt[o * kSeg + 64 + lane] = ec;
+        if (lane == 0) stats[((int64_t)blockIdx.z * nseg + seg) * p.heads + h0 + o] = make_float2(m, l);
+    }
+    __syncthreads();
+    const float *V = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)min(j0, hi - 1) * p.vdim;
+    uint32_t lanes = 1; // lanes side by side along vdim; the others take keys in turn
+    while (lanes < kThreads && lanes * VW < p.vdim) lanes *= 2;
+    const uint32_t across = threadIdx.x & (lanes - 1), turn = threadIdx.x / lanes, turns = kThreads / lanes;
+    for (uint32_t d0 = 0; d0 < p.vdim; d0 += lanes * VW) {
+        const uint32_t d = min(d0 + across * VW, p.vdim - VW);
+        float acc[REP][VW] = {};
+#pragma unroll 8
+        for (uint32_t k = turn; k < keys; k += turns) {
+            float v[VW];
+            if constexpr (VW == 4) {
+                const float4 f = *reinterpret_cast<const float4 *>(V + (int64_t)k * p.vdim + d);
+                v[0] = f.x, v[1] = f.y, v[2] = f.z, v[3] = f.w;
+            } else {
+                v[0] = V[(int64_t)k * p.vdim + d];
+            }
+#pragma unroll
+            for (int o = 0; o < REP; o++) {
+                if (o >= (int)nh) break;
+                const float w = wt[o * kSeg + k];
+#pragma unroll
+                for (int e = 0; e < VW; e++) acc[o][e] = fmaf(w, v[e], acc[o][e]);
+            }
+        }
+#pragma unroll
+        for (int o = 0; o < REP; o++)
+#pragma unroll
+            for (int e = 0; e < VW; e++) red[(o * VW + e) * kThreads + threadIdx.x] = acc[o][e];
+        __syncthreads();
+        const uint32_t cols = min(lanes * VW, p.vdim - d0);
+        for (uint32_t i = threadIdx.x; i < nh * cols; i += kThreads) {
+            const uint32_t o = i / cols, c = i - o * cols;
+            float sum = 0.0f;
+            for (uint32_t t = 0; t < turns; t++) sum += red[(o * VW + c % VW) * kThreads + t * lanes + c / VW];
+            parts[(((int64_t)blockIdx.z * nseg + seg) * p.heads + h0 + o) * p.vdim + d0 + c] = sum;
+        }
+        __syncthreads();
+    }
+}
+
+// ---- prompts ---------------------------------------------------------------------------------------------------------
+// The 16x16x4 instruction takes A[i = lane % 16][k = lane / 16], B[k = lane / 16][j = lane % 16] and leaves
+// C[4 (lane / 16) + r][lane % 16] in register r.  The order of k inside a product is free: lane group g supplies
+// k = 16 c + 4 g + t to the t-th of four instructions, for A and B alike.
+constexpr int kTileWaves = 8;
+constexpr uint32_t kRowsT = 16, kKeysT = 16;
+constexpr uint32_t kRowPitch = kKeysT + 4;                // floats; 16-byte reads of 16 rows cover all banks
+constexpr uint32_t kHeadPitch = kRowsT * kRowPitch + 4;   // heads four apart lie 16 banks apart
+constexpr float kSlack = 24.0f;                           // a row's `top` moves when a score exceeds it by more
+
+__device__ __forceinline__ f32x4 mfma(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+// Workgroup ids go to the eight XCDs in turn: the last rows, which see the most keys, go first.
+template <int DT> __device__ __forceinline__ void load_q(const AttentionPlan &p, const float *q, uint32_t b, uint32_t s0, uint32_t li, uint32_t lg, uint32_t h, f32x4 (&f)[DT]) {
+    const uint32_t s = min(s0 + li, p.S - 1);
+    const float *row = q + (((int64_t)b * p.S + s) * p.heads + h) * p.dim;
+#pragma unroll
+    for (int c = 0; c < DT; c++) {
+        const uint32_t d = 16 * c + 4 * lg;
+        f[c] = d < p.dim ? *reinterpret_cast<const f32x4 *>(row + d) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    }
+}
+template <int DT> __device__ __forceinline__ f32x4 scores(const f32x4 (&q)[DT], const f32x4 (&k)[DT]) {
+    f32x4 a = {0.0f, 0.0f, 0.0f, 0.0f}, b = a;
+#pragma unroll
+    for (int c = 0; c < DT; c += 2) { // two chains
+#pragma unroll
+        for (int t = 0; t < 4; t++) {
+            a = mfma(q[c][t], k[c][t], a);
+            if (c + 1 < DT) b = mfma(q[c + 1][t], k[c + 1][t], b);
+        }
+    }
+    return a + b;
+}
+
+// DT / VT: 16-wide pieces of a key / a value row.  QREG: the queries stay in registers; else they are read for every key tile.
+template <int HPW, int DT, int VT, bool QREG>
+__global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(const AttentionPlan p, const float *__restrict__ q, const uint32_t tiles, const uint32_t splits,
+                                                                                float *__restrict__ dst, float2 *__restrict__ stats) {
+    extern __shared__ float lds[]; // three buffers of scores [heads rounded up to 16][16][16], talk [heads rounded up][the same + 4]
+    constexpr int RT = (HPW * kTileWaves + 15) / 16; // row tiles of the mixing product
+    const uint32_t wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, li = lane & 15, lg = lane >> 4;
+    const uint32_t tile = tiles - 1 - blockIdx.x / splits, split = blockIdx.x % splits, b = blockIdx.y, s0 = tile * kRowsT;
+    const uint32_t h0 = wave * HPW, rep = p.heads / p.kv_heads, tiles16 = (p.heads + 15) / 16, buffer = tiles16 * 16 * kHeadPitch;
+    const bool shared = min(h0 + HPW - 1, p.heads - 1) / rep == min(h0, p.heads - 1) / rep; // one kv head for all of this wave's heads
+    const uint32_t first_row = p.cached + s0, last_row = p.cached + min(s0 + kRowsT, p.S) - 1, last = p.cached + p.S - 1;
+    uint32_t lo = first_visible(p, first_row);
+    const uint32_t ntiles = (last_row + 1 - lo + kKeysT - 1) / kKeysT, per = (ntiles + splits - 1) / splits;
+    const uint32_t from = min(ntiles, split * per), n = min(ntiles, from + per) - from;
+    lo += from * kKeysT;
+
+    f32x4 qf[QREG ? HPW : 1][DT], out[HPW][VT];
+    float slope[HPW], top[HPW], l[HPW]; // of row li, l of this lane's keys
+    const uint32_t talk_pitch = tiles16 * 16 + 4;
+    float *talk = lds + 3 * buffer;
+#pragma unroll
+    for (int i = 0; i < HPW; i++) {
+        const uint32_t h = min(h0 + i, p.heads - 1);
+        if constexpr (QREG) load_q<DT>(p, q, b, s0, li, lg, h, qf[i]);
+        slope[i] = p.bias ? slope_of(h, p.heads) : 0.0f;
+        top[i] = p.zero_sink ? 0.0f : kNone;
+        l[i] = 0.0f;
+#pragma unroll
+        for (int c = 0; c < VT; c++) out[i][c] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    }
+    for (uint32_t i = threadIdx.x; i < tiles16 * 16 * tiles16 * 16; i += kTileWaves * 64) {
+        const uint32_t h = i / (tiles16 * 16), g = i % (tiles16 * 16);
+        talk[h * talk_pitch + g] = h < p.heads && g < p.heads ? p.talk[(int64_t)h * p.heads + g] : 0.0f;
+    }
+    for (uint32_t i = p.heads * kHeadPitch + threadIdx.x; i < buffer; i += kTileWaves * 64) // heads that are not there
+        lds[i] = lds[buffer + i] = lds[2 * buffer + i] = 0.0f;
+    __syncthreads();
+    auto load_k = [&](uint32_t g, uint32_t key, f32x4(&f)[DT]) {
+        const float *base = p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)key * p.dim; // (the same for the whole wave)
+        const uint32_t row = min(li, last - key) * p.dim + 4 * lg;
+#pragma unroll
+        for (int c = 0; c < DT; c++) f[c] = 16 * c + 4 * lg < p.dim ? *reinterpret_cast<const f32x4 *>(base + (row + 16 * c)) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    };
+    uint32_t b0 = 0, b1 = 2, b2 = 1; // buffers of this iteration's scores, mixing, values
+    for (uint32_t it = 0; it < n + 2; it++) {
+        const bool do_s = it < n && h0 < p.heads, do_v = it >= 2 && h0 < p.heads;
+        const uint32_t js = lo + it * kKeysT, jv = lo + (it - 2) * kKeysT;
+        f32x4 k[DT];
+        float v[4][VT];
+        auto load_v = [&](uint32_t g) {
+            const float *base = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)jv * p.vdim;
+#pragma unroll
+            for (int t = 0; t < 4; t++) {
+                const uint32_t row = min(4 * lg + t, last - jv) * p.vdim + li;
+#pragma unroll
+                for (int c = 0; c < VT; c++) v[t][c] = 16 * c + li < p.vdim ? base[row + 16 * c] : 0.0f;
+            }
+        };
+        if (do_s) load_k(h0 / rep, js, k);
+        if (do_v) load_v(h0 / rep);
+        if (it >= 1 && it < n + 1) {
+            // talk [heads, heads] . scores [heads, 256 columns]: a wave owns whole columns and writes them back in place
+#pragma unroll
+            for (uint32_t e = 0; e < kRowsT / kTileWaves; e++) {
+                float *w = lds + b1 * buffer + (wave * (kRowsT / kTileWaves) + e) * kRowPitch + li;
+                f32x4 acc[RT];
+#pragma unroll
+                for (int a = 0; a < RT; a++) acc[a] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+                for (int c = 0; c < RT; c++) {
+                    if (c >= (int)tiles16) break;
+                    f32x4 f[RT];
+#pragma unroll
+                    for (int a = 0; a < RT; a++) f[a] = *reinterpret_cast<const f32x4 *>(talk + min(16 * a + li, tiles16 * 16 - 1) * talk_pitch + 16 * c + 4 * lg);
+#pragma unroll
+                    for (int t = 0; t < 4; t++) {
+                        const float x = w[(16 * c + 4 * lg + t) * kHeadPitch];
+#pragma unroll
+                        for (int a = 0; a < RT; a++) acc[a] = mfma(f[a][t], x, acc[a]);
+                    }
+                }
+#pragma unroll
+                for (int a = 0; a < RT; a++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const uint32_t h = 16 * a + 4 * lg + r;
+                        if (h < p.heads) w[h * kHeadPitch] = acc[a][r];
+                    }
+            }
+        }
+        if (do_s) { // scores of this wave's heads (of keys that a row does not see as well)
+#pragma unroll
+            for (int i = 0; i < HPW; i++) {
+                const uint32_t h = h0 + i;
+                if (h >= p.heads) break;
+                if (i > 0 && !shared) load_k(h / rep, js, k);
+                if constexpr (!QREG) load_q<DT>(p, q, b, s0, li, lg, h, qf[0]);
+                const f32x4 a = scores<DT>(qf[QREG ? i : 0], k);
+                float *w = lds + b0 * buffer + h * kHeadPitch + li;
+                const float d = (float)(int)(first_row + 4 * lg - js - li);
+#pragma unroll
+                for (int r = 0; r < 4; r++) w[(4 * lg + r) * kRowPitch] = fmaf(-slope[i], d + (float)r, a[r]);
+            }
+        }
+        if (do_v) { // mixed scores -> weights . values; a lane has four keys of row li
+            const bool whole = jv + kKeysT - 1 <= first_row && (!p.window || last_row - jv < p.window);
+#pragma unroll
+            for (int i = 0; i < HPW; i++) {
+                const uint32_t h = h0 + i;
+                if (h >= p.heads) break;
+                if (i > 0 && !shared) load_v(h / rep);
+                f32x4 x = *reinterpret_cast<const f32x4 *>(lds + b2 * buffer + h * kHeadPitch + li * kRowPitch + 4 * lg);
+                bool moves = false;
+#pragma unroll
+                for (int t = 0; t < 4; t++) {
+                    const int32_t d = (int32_t)(first_row + li) - (int32_t)(jv + 4 * lg + t);
+                    x[t] = whole || (d >= 0 && (!p.window || (uint32_t)d < p.window)) ? x[t] * kLog2e : -INFINITY;
+                    moves = moves || x[t] - top[i] > kSlack;
+                }
+                if (__any(moves)) {
+                    float up = fmaxf(fmaxf(x[0], x[1]), fmaxf(x[2], x[3]));
+                    up = fmaxf(up, __shfl_xor(up, 16, 64));
+                    up = fmaxf(top[i], fmaxf(up, __shfl_xor(up, 32, 64)));
+                    const float f = __builtin_amdgcn_exp2f(top[i] - up);
+                    top[i] = up;
+                    l[i] *= f;
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const float fr = __shfl(f, 4 * lg + r, 64);
+#pragma unroll
+                        for (int c = 0; c < VT; c++) out[i][c][r] *= fr;
+                    }
+                }
+#pragma unroll
+                for (int t = 0; t < 4; t++) x[t] = __builtin_amdgcn_exp2f(x[t] - top[i]);
+                l[i] += (x[0] + x[1]) + (x[2] + x[3]);
+#pragma unroll
+                for (int t = 0; t < 4; t++)
+#pragma unroll
+                    for (int c = 0; c < VT; c++) out[i][c] = mfma(x[t], v[t][c], out[i][c]);
+            }
+        }
+        __syncthreads();
+        const uint32_t t = b2;
+        b2 = b1;
+        b1 = b0;
+        b0 = t;
+    }
+    const uint64_t rows = (uint64_t)p.B * p.S;
+#pragma unroll
+    for (int i = 0; i < HPW; i++) {
+        const uint32_t h = h0 + i;
+        if (h >= p.heads) break;
+        float sum = l[i];
+        sum += __shfl_xor(sum, 16, 64);
+        sum += __shfl_xor(sum, 32, 64);
+        if (splits > 1) {
+            if (lg == 0 && s0 + li < p.S) stats[(split * rows + (uint64_t)b * p.S + s0 + li) * p.heads + h] = make_float2(top[i], sum);
+            sum = 1.0f;
+        } else if (p.zero_sink) {
+            sum += __builtin_amdgcn_exp2f(-top[i]);
+        }
+        const float inv = 1.0f / sum;
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            const float f = __shfl(inv, 4 * lg + r, 64);
+            const uint32_t s = s0 + 4 * lg + r;
+            if (s >= p.S) continue;
+            float *row = dst + ((split * rows + (uint64_t)b * p.S + s) * p.heads + h) * p.vdim + li;
+#pragma unroll
+            for (int c = 0; c < VT; c++)
+                if (16 * c + li < p.vdim) row[16 * c] = out[i][c][r] * f;
+        }
+    }
+}
+
+// ---- a few new tokens ------------------------------------------------------------------------------------------------
+constexpr uint32_t kMaxStepKeys = 64;
+struct StepLds { // floats
+    uint32_t turn, q, fresh, talk, raw, mixed, total;
+};
+__host__ __device__ inline StepLds step_lds(uint32_t S, uint32_t heads, uint32_t kv_heads, uint32_t dim, uint32_t rot, uint32_t keys) {
+    StepLds o{};
+    uint32_t at = 0;
+    auto take = [&](uint32_t n) {
+        const uint32_t r = at;
+        at += (n + 3) / 4 * 4;
+        return r;
+    };
+    o.turn = take(rot * S);                      // {cos, sin} per pair and new token
+    o.q = take(heads * dim);
+    o.fresh = take(kv_heads * dim * S);          // new keys
+    o.talk = take(heads * heads);
+    o.raw = take(heads * (keys + 1));
+    o.mixed = take(heads * (keys + 1));
+    o.total = at;
+    return o;
+}
+
+template <int REP>
+__global__ __launch_bounds__(kThreads) void attention_mixed_step_kernel(const AttentionPlan p, const uint32_t seg_keys, float *__restrict__ parts, float2 *__restrict__ stats) {
+    extern __shared__ float lds[];
+    const uint32_t rep = p.heads / p.kv_heads, seg = blockIdx.x, nseg = gridDim.x, r = blockIdx.y, b = r / p.S, s = r - b * p.S;
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, pitch = seg_keys + 1;
+    const StepLds at = step_lds(p.S, p.heads, p.kv_heads, p.dim, p.rot_dims, seg_keys);
+    const uint32_t j0 = first_visible(p, p.cached + s) + seg * seg_keys, hi = p.cached + s + 1, keys = j0 < hi ? min(seg_keys, hi - j0) : 0;
+    // the angles of this token and of those new ones in front of it whose keys this workgroup scores
+    const uint32_t t0 = j0 > p.cached ? j0 - p.cached : 0, t1 = j0 + keys > p.cached ? j0 + keys - p.cached : 0; // new keys [t0, t1)
+    const uint32_t pairs = p.rot_dims / 2;
+    float2 *turn = reinterpret_cast<float2 *>(lds + at.turn);
+    for (uint32_t i = threadIdx.x; i < pairs * p.S; i += kThreads) {
+        const uint32_t t = i / pairs, k = i - t * pairs;
+        if (t != s && (t < t0 || t >= t1)) continue;
+        double a = (double)(p.position + t) * exp2(-2.0 * (double)k / (double)p.rot_dims * p.rot_log2);
+        a -= 6.283185307179586 * rint(a * 0.15915494309189535);
+        float sn, cs;
+        sincosf((float)a, &sn, &cs);
+        turn[i] = make_float2(cs, sn);
+    }
+    for (uint32_t i = threadIdx.x; i < p.heads * p.heads; i += kThreads) lds[at.talk + i] = p.talk ? p.talk[i] : i / p.heads == i % p.heads ? 1.0f : 0.0f;
+    __syncthreads();
+    // a head of new token t: turned, at a mean square of one, times f; a wave per head
+    auto head = [&](const float *src, uint32_t t, float f, float *dst, float *also) {
+        auto value = [&](uint32_t d) {
+            const float v = src[d];
+            if (d >= p.rot_dims) return v;
+            const float2 cs = turn[t * pairs + d / 2];
+            return d & 1 ? fmaf(v, cs.x, src[d - 1] * cs.y) : fmaf(v, cs.x, -src[d + 1] * cs.y);
+        };
+        float m = 0.0f;
+        const float v0 = lane < p.dim ? value(lane) : 0.0f, v1 = lane + 64 < p.dim ? value(lane + 64) : 0.0f;
+        m = fmaf(v0, v0, v1 * v1);
+        for (uint32_t d = lane + 128; d < p.dim; d += 64) {
+            const float v = value(d);
+            m = fmaf(v, v, m);
+        }
+        float g = f;
+        if (p.unit_heads) g /= sqrtf(wave_sum(m) / (float)p.dim + p.eps);
+        for (uint32_t d = lane; d < p.dim; d += 64) {
+            const float v = (d == lane ? v0 : d == lane + 64 ? v1 : value(d)) * g;
+            dst[d] = v;
+            if (also) also[d] = v;
+        }
+    };
+    float temp = p.scale;
+    if (p.temp_every) temp *= 1.0f + p.temp_coef * logf((float)((p.position + s + 1) / p.temp_every + 1));
+    for (uint32_t h = wave; h < p.heads; h += kThreads / 64) head(p.q.p + (int64_t)r * p.q.pitch + h * p.dim, s, temp, lds + at.q + h * p.dim, nullptr);
+    for (uint32_t i = wave; i < (t1 - min(t0, t1)) * p.kv_heads; i += kThreads / 64) {
+        const uint32_t t = t0 + i / p.kv_heads, g = i % p.kv_heads;
+        float *cache = t == s ? p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)(p.cached + t) * p.dim : nullptr; // its own workgroup's
+        head(p.k.p + ((int64_t)b * p.S + t) * p.k.pitch + g * p.dim, t, 1.0f, lds + at.fresh + (t * p.kv_heads + g) * p.dim, cache);
+    }
+    if (t1 == s + 1 && t0 <= s) // the last segment: this token's values
+        for (uint32_t i = threadIdx.x; i < p.kv_heads * p.vdim; i += kThreads) {
+            const uint32_t g = i / p.vdim, d = i - g * p.vdim;
+            p.values[((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)(p.cached + s) * p.vdim + d] = p.v.p[(int64_t)r * p.v.pitch + i];
+        }
+    __syncthreads();
+    // scores: four lanes share a key of a kv head
+    const uint32_t sub = threadIdx.x & 3;
+    for (uint32_t i = threadIdx.x >> 2; i < seg_keys * p.kv_heads; i += kThreads / 4) {
+        const uint32_t g = i / seg_keys, key = i - g * seg_keys, j = j0 + min(key, max(keys, 1u) - 1);
+        const bool fresh = keys && j >= p.cached;
+        const float *kp = fresh ? lds + at.fresh + ((j - p.cached) * p.kv_heads + g) * p.dim
+                                : p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)min(j, p.cached ? p.cached - 1 : 0) * p.dim;
+        for (uint32_t h0 = 0; h0 < rep; h0 += REP) {
+            float acc[REP] = {};
+            const float *qh = lds + at.q + (g * rep + h0) * p.dim;
+#pragma unroll 8
+            for (uint32_t d = sub * 4; d < p.dim; d += 16) {
+                const float4 kv = *reinterpret_cast<const float4 *>(kp + d);
+#pragma unroll
+                for (int h = 0; h < REP; h++) {
+                    if (h0 + h >= rep) break;
+                    const float4 qv = *reinterpret_cast<const float4 *>(qh + h * p.dim + d);
+                    acc[h] = fmaf(kv.x, qv.x, fmaf(kv.y, qv.y, fmaf(kv.z, qv.z, fmaf(kv.w, qv.w, acc[h]))));
+                }
+            }
+#pragma unroll
+            for (int h = 0; h < REP; h++) {
+                float v = acc[h];
+                v += __shfl_xor(v, 1, 64);
+                v += __shfl_xor(v, 2, 64);
+                if (sub == 0 && h0 + h < rep) {
+                    const uint32_t hh = g * rep + h0 + h;
+                    if (p.bias) v -= slope_of(hh, p.heads) * (float)(int)(p.cached + s - j);
+                    lds[at.raw + hh * pitch + key] = v;
+                }
+            }
+        }
+    }
+    __syncthreads();
+    for (uint32_t i = threadIdx.x; i < p.heads * seg_keys; i += kThreads) {
+        const uint32_t h = i / seg_keys, key = i - h * seg_keys;
+        float w = 0.0f;
+#pragma unroll 4
+        for (uint32_t g = 0; g < p.heads; g++) w = fmaf(lds[at.talk + h * p.heads + g], lds[at.raw + g * pitch + key], w);
+        lds[at.mixed + h * pitch + key] = key < keys ? w * kLog2e : -INFINITY;
+    }
+    __syncthreads();
+    for (uint32_t h = wave; h < p.heads; h += kThreads / 64) {
+        const float x = lane < seg_keys ? lds[at.mixed + h * pitch + lane] : -INFINITY;
+        const float m = fmaxf(kNone, wave_max(x)), e = __builtin_amdgcn_exp2f(x - m), l = wave_sum(e);
+        if (lane < seg_keys) lds[at.mixed + h * pitch + lane] = e;
+        if (lane == 0) stats[((int64_t)r * nseg + seg) * p.heads + h] = make_float2(m, l);
+    }
+    __syncthreads();
+    // values: a thread per four columns of a kv head's values, for its query heads
+    const uint32_t vec = p.vdim / 4;
+    for (uint32_t i = threadIdx.x; i < p.kv_heads * vec; i += kThreads) {
+        const uint32_t g = i / vec, d = (i - g * vec) * 4;
+        const float *V = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + d;
+        for (uint32_t h0 = 0; h0 < rep; h0 += REP) {
+            f32x4 acc[REP] = {};
+            auto add = [&](const f32x4 v, uint32_t k) {
+#pragma unroll
+                for (int h = 0; h < REP; h++) {
+                    if (h0 + h >= rep) break;
+                    const float w = lds[at.mixed + (g * rep + h0 + h) * pitch + k];
+#pragma unroll
+                    for (int e = 0; e < 4; e++) acc[h][e] = fmaf(w, v[e], acc[h][e]);
+                }
+            };
+            const uint32_t old = j0 >= p.cached ? 0 : min(keys, p.cached - j0); // the new ones come from the projections
+#pragma unroll 8
+            for (uint32_t k = 0; k < old; k++) add(*reinterpret_cast<const f32x4 *>(V + (int64_t)(j0 + k) * p.vdim), k);
+            for (uint32_t k = old; k < keys; k++) {
+                const float *src = p.v.p + ((int64_t)b * p.S + (j0 + k - p.cached)) * p.v.pitch + g * p.vdim + d;
+                add(f32x4{src[0], src[1], src[2], src[3]}, k);
+            }
+#pragma unroll
+            for (int h = 0; h < REP; h++) {
+                if (h0 + h >= rep) break;
+                *reinterpret_cast<f32x4 *>(parts + (((int64_t)r * nseg + seg) * p.heads + g * rep + h0 + h) * p.vdim + d) = acc[h];
+            }
+        }
+    }
+}
+
+int launched(const char *what) {
+    const hipError_t e = hipGetLastError();
+    return e == hipSuccess ? CG_OK : hip_fail(e, what);
+}
+constexpr size_t kMaxLds = 160 << 10;
+int allow_lds(const void *kernel, size_t bytes) {
+    if (bytes > kMaxLds) return fail(CG_ERR_UNSUPPORTED, "block_attention: heads or sizes beyond what the kernels hold");
+    if (bytes <= (64 << 10)) return CG_OK;
+    const hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
+    return e == hipSuccess ? CG_OK : hip_fail(e, "hipFuncSetAttribute");
+}
+
+struct Scratch {
+    cg_backend *be;
+    void *p = nullptr;
+    size_t cls = 0;
+    explicit Scratch(cg_backend *b) : be(b) {}
+    int get(size_t bytes) { return be->pool.alloc(bytes ? bytes : 4, &p, &cls); }
+    ~Scratch() {
+        if (p) be->pool.free(p, cls);
+    }
+};
+
+void merge(cg_backend *be, const AttentionPlan &p, const float *parts, const float2 *stats, uint32_t segs, uint64_t row_pitch, uint64_t seg_pitch, uint32_t rows, float *out) {
+    const uint32_t n = p.heads * p.vdim;
+    for (uint32_t r0 = 0; r0 < rows; r0 += 65535) {
+        const uint32_t nr = std::min(rows - r0, 65535u);
+        hipLaunchKernelGGL(attention_merge_kernel, dim3((n + kThreads - 1) / kThreads, nr), dim3(kThreads), 0, be->stream, parts + (uint64_t)r0 * row_pitch * p.vdim,
+                           stats + (uint64_t)r0 * row_pitch, segs, row_pitch, seg_pitch, p.heads, p.vdim, p.zero_sink, out + (uint64_t)r0 * n);
+    }
+}
+
+template <int REP, int VW>
+int mixed_rows(cg_backend *be, const AttentionPlan &p, uint32_t row0, uint32_t rows, uint32_t nseg, const float *scores, float *parts, float2 *stats) {
+    const uint32_t rep = p.heads / p.kv_heads, groups = (rep + REP - 1) / REP, slots = p.talk ? p.heads : REP;
+    const size_t lds = (size_t)mixed_floats(REP, slots, VW) * 4;
+    if (int rc = allow_lds(reinterpret_cast<const void *>(&attention_mixed_rows_kernel<REP, VW>), lds)) return rc;
+    hipLaunchKernelGGL((attention_mixed_rows_kernel<REP, VW>), dim3(nseg, p.kv_heads * groups, rows), dim3(kThreads), lds, be->stream, p, row0, nseg, scores, parts, stats);
+    merge(be, p, parts, stats, nseg, (uint64_t)nseg * p.heads, p.heads, rows, p.out + (uint64_t)row0 * p.heads * p.vdim);
+    return launched("attention_mixed_rows");
+}
+
+template <int HPW, int DT, int VT, bool QREG> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t splits, float *dst, float2 *stats) {
+    const uint32_t tiles = (p.S + kRowsT - 1) / kRowsT;
+    const size_t h16 = (p.heads + 15) / 16 * 16, lds = (3 * h16 * kHeadPitch + h16 * (h16 + 4)) * 4;
+    if (int rc = allow_lds(reinterpret_cast<const void *>(&attention_mixed_tiles_kernel<HPW, DT, VT, QREG>), lds)) return rc;
+    hipLaunchKernelGGL((attention_mixed_tiles_kernel<HPW, DT, VT, QREG>), dim3(tiles * splits, p.B), dim3(kTileWaves * 64), lds, be->stream, p, q, tiles, splits, dst, stats);
+    return CG_OK;
+}
+template <int HPW> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t splits, float *dst, float2 *stats) {
+    const uint32_t d = p.dim, v = p.vdim;
+    if (d <= 32 && v <= 32) return run_tiles<HPW, 2, 2, true>(be, p, q, splits, dst, stats);
+    if (d <= 64 && v <= 64) return run_tiles<HPW, 4, 4, true>(be, p, q, splits, dst, stats);
+    if (d <= 64 && v <= 96) return run_tiles<HPW, 4, 6, true>(be, p, q, splits, dst, stats);
+    if (d <= 96 && v <= 96) return run_tiles<HPW, 6, 6, (HPW < 4)>(be, p, q, splits, dst, stats);
+    return run_tiles<HPW, 8, 8, (HPW < 4)>(be, p, q, splits, dst, stats);
+}
+
+} // namespace
+
+int launch_mixed_rows(cg_backend *be, const AttentionPlan &p, uint32_t row0, uint32_t rows, uint32_t nseg, const float *scores, float *parts, float2 *part_stats) {
+    const uint32_t rep = p.heads / p.kv_heads;
+    const bool vec = p.vdim % 4 == 0; // (cache rows begin at multiples of their length: 16-byte loads then)
+#define CG_ROWS(R) (vec ? mixed_rows<R, 4>(be, p, row0, rows, nseg, scores, parts, part_stats) : mixed_rows<R, 1>(be, p, row0, rows, nseg, scores, parts, part_stats))
+    return rep <= 1 ? CG_ROWS(1) : rep <= 2 ? CG_ROWS(2) : rep <= 4 ? CG_ROWS(4) : CG_ROWS(8);
+#undef CG_ROWS
+}
+
+int launch_mixed_tiles(cg_backend *be, const AttentionPlan &p, const float *q) {
+    if (p.S <= kFewRows || p.heads > 32 || p.dim % 4 || p.dim > 128 || p.vdim > 128 || p.B > 65535 || !p.talk) return kDeclined;
+    const uint64_t n = (uint64_t)p.B * p.S * p.heads * p.vdim;
+    const uint32_t tiles = (p.S + kRowsT - 1) / kRowsT, keys = p.cached + p.S, most = p.window ? std::min(p.window + kRowsT, keys) : keys;
+    // too few row tiles for the device: their keys are cut over up to 4 workgroups, each with at least 8 key tiles
+    const uint32_t want = (uint32_t)(2 * be->compute_units) / std::max(1u, tiles * p.B);
+    const uint32_t splits = std::max(1u, std::min(std::min(4u, want), most / (8 * kKeysT)));
+    Scratch parts(be), stats(be);
+    if (splits > 1) {
+        if (int rc = parts.get((size_t)n * splits * 4)) return rc;
+        if (int rc = stats.get((size_t)p.B * p.S * p.heads * splits * sizeof(float2))) return rc;
+    }
+    float *dst = splits > 1 ? static_cast<float *>(parts.p) : p.out;
+    float2 *st = static_cast<float2 *>(stats.p);
+    const int rc = p.heads <= 8    ? run_tiles<1>(be, p, q, splits, dst, st)
+                   : p.heads <= 16 ? run_tiles<2>(be, p, q, splits, dst, st)
+                                   : run_tiles<4>(be, p, q, splits, dst, st);
+    if (rc) return rc;
+    if (splits > 1) merge(be, p, dst, st, splits, p.heads, (uint64_t)p.B * p.S * p.heads, p.B * p.S, p.out);
+    return launched("attention_mixed_tiles");
+}
+
+int launch_mixed_step(cg_backend *be, const AttentionPlan &p) {
+    const uint32_t rows = p.B * p.S, keys = p.cached + p.S, most = p.window ? std::min(p.window, keys) : keys, rep = p.heads / p.kv_heads;
+    if (p.S > kFewRows || p.dim % 4 || p.vdim % 4 || rows > 65535 || p.q_norm || p.k_norm) return kDeclined;
+    // segments that fill the device, of 8 to 64 keys
+    uint32_t seg = 8;
+    while (seg < kMaxStepKeys && (uint64_t)rows * ((most + seg - 1) / seg) > be->compute_units) seg *= 2;
+    const size_t lds = (size_t)step_lds(p.S, p.heads, p.kv_heads, p.dim, p.rot_dims, seg).total * 4;
+    if (lds > kMaxLds / 2) return kDeclined;
+    const uint32_t nseg = (most + seg - 1) / seg;
+    Scratch mem(be);
+    const size_t n = (size_t)rows * nseg * p.heads;
+    if (int rc = mem.get(n * p.vdim * 4 + n * sizeof(float2))) return rc;
+    float *parts = static_cast<float *>(mem.p);
+    float2 *stats = reinterpret_cast<float2 *>(parts + n * p.vdim);
+    const dim3 grid(nseg, rows);
+#define CG_STEP(R)                                                                                                                   \
+    {                                                                                                                                \
+        if (int rc = allow_lds(reinterpret_cast<const void *>(&attention_mixed_step_kernel<R>), lds)) return rc;                     \
+        hipLaunchKernelGGL((attention_mixed_step_kernel<R>), grid, dim3(kThreads), lds, be->stream, p, seg, parts, stats);            \
+    }
+    if (rep <= 1) CG_STEP(1)
+    else if (rep <= 2) CG_STEP(2)
+    else CG_STEP(4)
+#undef CG_STEP
+    merge(be, p, parts, stats, nseg, (uint64_t)nseg * p.heads, p.heads, rows, p.out);
+    return launched("attention_mixed_step");
+}
+
+} // namespace cg

@@ -118,7 +118,7 @@ __global__ __launch_bounds__(kStatWaves * 64) void attention_row_stats_kernel(co
         slope[i] = p.bias ? slope_of(h, p.heads) : 0.0f;
 #pragma unroll
         for (int r = 0; r < 4; r++) {
-            top[i][r] = -1e30f; // (finite: a masked score against it weighs nothing)
+            top[i][r] = p.zero_sink ? 0.0f : -1e30f; // (finite: a masked score against it weighs nothing)
             l[i][r] = 0.0f;
         }
     }
@@ -167,6 +167,7 @@ __global__ __launch_bounds__(kStatWaves * 64) void attention_row_stats_kernel(co
             float sum = l[i][r];
 #pragma unroll
             for (int d = 1; d < 16; d <<= 1) sum += __shfl_xor(sum, d, 64);
+            if (p.zero_sink) sum += __builtin_amdgcn_exp2f(-top[i][r]);
             const uint32_t s = at.s0 + 4 * at.lg + r;
             if (at.li == 0 && s < p.S && h0 + i < p.heads) stats[((int64_t)at.b * p.S + s) * p.heads + h0 + i] = make_float2(top[i][r], 1.0f / sum);
         }

@@ -607,6 +607,9 @@ struct GatedSumArgs {
     GatedTerm t[2];
     int n;
     uint32_t width;
+    float scale;
+    const float *extra; // [rows, slots, width]
+    uint32_t slots;
 };
 template <int VW> __global__ __launch_bounds__(kThreads) void gated_sum_kernel(const GatedSumArgs a, float *__restrict__ out) {
     const uint32_t k = (blockIdx.x * kThreads + threadIdx.x) * VW, r = blockIdx.y;
@@ -630,8 +633,16 @@ template <int VW> __global__ __launch_bounds__(kThreads) void gated_sum_kernel(c
         for (int j = 0; j < VW; j++)
             s[j] += a.t[i].gate.p ? sigmoid(g[j] + (a.t[i].gate_bias ? a.t[i].gate_bias[k + j] : 0.0f)) * y[j] : y[j];
     }
+    if (a.extra) {
+#pragma unroll 4
+        for (uint32_t i = 0; i < a.slots; i++) {
+            load(a.extra + ((int64_t)r * a.slots + i) * a.width + k, y);
 #pragma unroll
-    for (int j = 0; j < VW; j++) x[j] += s[j];
+            for (int j = 0; j < VW; j++) s[j] += y[j];
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < VW; j++) x[j] += a.scale * s[j];
     float *o = out + (int64_t)r * a.width + k;
     if constexpr (VW == 4) *reinterpret_cast<float4 *>(o) = make_float4(x[0], x[1], x[2], x[3]);
     else *o = x[0];
@@ -834,16 +845,20 @@ int launch_affine_rows(cg_backend *be, float *y, uint32_t rows, uint32_t n, cons
     return launched("affine_rows");
 }
 
-int launch_gated_sum(cg_backend *be, const Rows &x, const GatedTerm *t, int n, uint32_t rows, uint32_t width, float *out) {
-    bool vec = width % 4 == 0 && x.pitch % 4 == 0 && aligned16(x.p) && aligned16(out);
+int launch_gated_sum(cg_backend *be, const Rows &x, const GatedTerm *t, int n, uint32_t rows, uint32_t width, float *out, float scale, const float *extra,
+                     uint32_t slots) {
+    bool vec = width % 4 == 0 && x.pitch % 4 == 0 && aligned16(x.p) && aligned16(out) && aligned16(extra);
     for (int i = 0; i < n; i++) vec = vec && (!t[i].gate.p || (t[i].gate.pitch % 4 == 0 && aligned16(t[i].gate.p))) && aligned16(t[i].y);
     for (uint32_t r0 = 0; r0 < rows; r0 += 65535) {
         const uint32_t nr = rows - r0 < 65535 ? rows - r0 : 65535;
-        ProfScope prof(be, CG_K_ELEMENTWISE, (2.0 + 2.0 * n) * 4.0 * nr * width);
+        ProfScope prof(be, CG_K_ELEMENTWISE, (2.0 + 2.0 * n + (extra ? slots : 0)) * 4.0 * nr * width);
         GatedSumArgs a{};
         a.x = {x.p + (int64_t)r0 * x.pitch, x.pitch};
         a.n = n;
         a.width = width;
+        a.scale = scale;
+        a.extra = extra ? extra + (int64_t)r0 * slots * width : nullptr;
+        a.slots = slots;
         for (int i = 0; i < n; i++) {
             a.t[i] = t[i];
             a.t[i].y += (int64_t)r0 * width;

@@ -65,7 +65,70 @@ struct GatedTerm {
     Rows gate;
     const float *gate_bias = nullptr;
 };
-int launch_gated_sum(cg_backend *be, const Rows &x, const GatedTerm *t, int n, uint32_t rows, uint32_t width, float *out);
+// extra: [rows, slots, width] more terms, added up (null: none); out = x + scale * (all terms)
+int launch_gated_sum(cg_backend *be, const Rows &x, const GatedTerm *t, int n, uint32_t rows, uint32_t width, float *out, float scale = 1.0f,
+                     const float *extra = nullptr, uint32_t slots = 0);
+
+// ---- embeddings, grouped norms with filters, the tokens' own vectors ---------------------------------------------------
+// A table's rows in 32-bit words or bfloat16 patterns.
+struct Table {
+    const void *p = nullptr;
+    int64_t pitch = 0; // elements
+    int fmt = kFmtWords;
+};
+// Token ids in memory, or one id.
+struct Tokens {
+    const uint32_t *p = nullptr;
+    uint32_t value = 0;
+};
+struct PairEmbeddingPlan {
+    uint32_t B, S, width, vocab;
+    uint64_t buckets, mul_prev, mul_cur; // multipliers below `buckets`
+    Tokens ids, previous;
+    uint32_t previous_n;                 // tokens of `previous` per sequence
+    Table table, pairs;
+    float *out;
+    uint32_t *previous_out;
+};
+int launch_pair_embedding(cg_backend *be, const PairEmbeddingPlan &p);
+
+constexpr uint32_t kMaxTaps = 16;
+struct ConvRowsPlan {
+    uint32_t B, S, width, groups, taps, run;
+    float eps;
+    Rows x;
+    const float *state; // null: zeros
+    float *state_out;   // null with one tap
+    int n;
+    struct {
+        const float *gamma, *conv; // conv null: the norm alone
+        void *dst;
+        int fmt;    // words or bfloat16 patterns
+        bool round; // words: rounded to bfloat16
+    } out[2];
+};
+int launch_conv_rows(cg_backend *be, ConvRowsPlan p);
+
+int launch_side_gate(cg_backend *be, float *g, const Tokens &ids, const Table &table, uint32_t vocab, uint32_t first, uint32_t dim, uint32_t rows);
+int launch_side_sum(cg_backend *be, const Rows &x, const float *y, const float *norm, uint32_t rows, uint32_t width, float eps, float scale, float *out);
+
+// ---- mixtures of experts ---------------------------------------------------------------------------------------------
+struct ExpertsPlan {
+    uint32_t rows, width, ff, experts, top, groups, keep;
+    float limit, slope;
+    const void *h;   // [rows, width], words or bfloat16 patterns
+    int h_fmt;
+    const float *logits, *correction; // correction may be null
+    const void *gate_up, *down;       // [experts, 2, ff, width], [experts, width, ff], dense
+    int fmt;                          // of the weights
+};
+// y[r, slot, 0 .. width) = weight * expert of row r's slot-th choice, for any number of rows
+int launch_experts(cg_backend *be, const ExpertsPlan &p, float *y);
+// A few rows: hidden[r, slot, 0 .. ff) (weights applied) and the chosen experts' numbers.
+int launch_experts_first(cg_backend *be, const ExpertsPlan &p, float *hidden, uint32_t *chosen);
+// out[r] = x[r] + scale * (y[r] . w^T + sum_slot hidden[r, slot] . down[chosen[r, slot]]^T), rows <= kFewRows
+int launch_experts_second(cg_backend *be, const ExpertsPlan &p, const float *hidden, const uint32_t *chosen, const Rows &x, const Rows &y, const Weight *w, float scale,
+                          float *out);
 
 // ---- attention -------------------------------------------------------------------------------------------------------
 struct AttentionPlan {
@@ -75,7 +138,9 @@ struct AttentionPlan {
     uint64_t position;  // of the first new token
     uint64_t temp_every;
     float temp_coef, scale, eps;
-    bool bias;
+    bool bias, unit_heads, mix_scores, zero_sink;
+    uint32_t rot_dims;          // 0: no rotation
+    double rot_log2;            // log2 of its base
     Rows q, k, v;
     const float *q_norm, *k_norm, *talk;
     float *keys, *values;       // row 0 of the cached rows of (b 0, kv head 0); the new rows follow the cached ones
@@ -85,6 +150,11 @@ struct AttentionPlan {
 int launch_attention(cg_backend *be, const AttentionPlan &p);
 // More than a few new tokens, on the matrix instructions (q: the prepared queries); kDeclined: sizes it does not take.
 int launch_attention_tiles(cg_backend *be, const AttentionPlan &p, const float *q);
+// Soft-max over mixed scores (block_attention_mixed.hip).  `scores`: the scores' segments as attention_scores_kernel leaves
+// them, of the rows row0 .. row0 + rows - 1; parts / part_stats: memory of nseg results per (row, head).
+int launch_mixed_rows(cg_backend *be, const AttentionPlan &p, uint32_t row0, uint32_t rows, uint32_t nseg, const float *scores, float *parts, float2 *part_stats);
+int launch_mixed_tiles(cg_backend *be, const AttentionPlan &p, const float *q);
+int launch_mixed_step(cg_backend *be, const AttentionPlan &p);
 
 // ---- gated delta rule ------------------------------------------------------------------------------------------------
 struct DeltaPlan {
