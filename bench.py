@@ -357,25 +357,42 @@ def loretar_config(size):
     return config_of(layers, vocab, width, loop={"start": once, "stop": once + twice, "times": 2})
 
 
-def measure_loretar(size, dtype, steps, warmup, seed=0):
-    """Prefill + greedy decode of Loretar at the size of a BASELINE configuration: the whole job, then the kernel classes of
-    one more pass (event records around every launch, untimed)."""
-    from catgrad_amd import _abi as A
-    from catgrad_amd.loretar import random_params
+# Lufatar at the same sizes: every layer run attends (no window), the feed-forward is 8 of 32 experts that are together as
+# wide as the closest model's, and the middle half of the layers runs twice.
+def lufatar_config(size):
+    from catgrad_amd.lufatar import attention_layer, config_of, experts
+
+    if size == 5:
+        width, ff, vocab, runs, at, rot, base = 2048, 1024, 128256, 16, (32, 8, 64, 64), 64, 500000.0
+    else:
+        width, ff, vocab, runs, at, rot, base = 1024, 384, 151936, 28, (16, 8, 128, 128), 64, 1000000.0
+    once = runs // 4
+    twice = (runs - 2 * once) // 2
+    layers = [attention_layer(*at, experts(32, 8, ff, groups=4, keep=2, limit=7.0), rot=rot, base=base) for _ in range(2 * once + twice)]
+    return config_of(layers, vocab, width, loop={"start": once, "stop": once + twice, "times": 2}, groups=4, mult=0.5, taps=4, side=64,
+                     buckets=65521, mul_prev=7919, mul_cur=104729)
+
+
+def measure_blocks(design, size, dtype, steps, warmup, seed=0):
+    """Prefill + greedy decode of a model of decoder blocks ("loretar" or "lufatar") at the size of a BASELINE configuration:
+    the whole job, then the kernel classes of one more pass (event records around every launch, untimed)."""
+    from catgrad_amd import _abi as A, loretar, lufatar
     from catgrad_amd.runner import Session
 
     B, S, T, _ = CONFIGS[size]
-    config = loretar_config(size)
+    config = loretar_config(size) if design == "loretar" else lufatar_config(size)
+    params = loretar.random_params(config, seed, low_rank=64) if design == "loretar" else lufatar.random_params(config, seed)
     sess = Session()
     sess.load_config(config, dtype)
     weights = 0
     lp = config["loop"]
-    for name, w in random_params(config, seed, low_rank=64):
+    for name, w in params:  # weights: matrix elements that a token is multiplied with, experts at the share that it uses
         sess.set_param(name, w)
-        if w.ndim == 2 and not name.startswith(("embed", "loop.step")) and not name.endswith((".conv", ".talk")):
+        if w.ndim == 2 and not name.startswith(("embed", "bigram", "side.embed", "loop.step")) and not name.endswith((".conv", ".talk", ".canon1", ".canon2")):
             i = int(name[1:].split(".")[0]) if name[0] == "l" and name[1].isdigit() else None
             n = lp["times"] if name == "loop.in" or (i is not None and lp["start"] <= i < lp["stop"]) else 1
-            weights += n * w.size
+            router = config["layers"][i]["mlp"]["router"] if ".mlp.e" in name else None
+            weights += n * w.size * (router["top"] / router["experts"] if router else 1)
     prompt = np.random.default_rng(seed).integers(0, config["vocab"], size=(B, S), dtype=np.uint32)
     for _ in range(max(warmup, 1)):
         sess.generate(prompt, steps=T, max_positions=S + T)
@@ -407,15 +424,16 @@ def measure_loretar(size, dtype, steps, warmup, seed=0):
     sess.close()
     wb = 2 if dtype == "bfloat16" else 4
     at = [l["mixer"] for l in config["layers"] if l["type"] == "attention"]
+    window = at[0]["mask"]["size"] if "mask" in at[0] else None
     linear_flop = 2.0 * B * S * (weights - config["vocab"] * config["width"])
     out = {
-        "workload": f"Loretar, {dtype}, batch {B}, prefill {S} + {T} decode steps, sizes of BASELINE config {size}",
+        "workload": f"{design.capitalize()}, {dtype}, batch {B}, prefill {S} + {T} decode steps, sizes of BASELINE config {size}",
         "tok_s": round(B * (S + T) / (pp + tg), 1), "prefill_ms": round(pp * 1e3, 3), "prefill_tok_s": round(B * S / pp, 1),
         "decode_ms_per_step": round(tg / T * 1e3, 4), "decode_tok_s": round(B * T / tg, 1),
         "weight_bytes_per_step": int(weights * wb), "decode_hbm_frac_weights": round(weights * wb / (tg / T) / HBM_PEAK, 4),
         "prefill_linear_flop": linear_flop,
         "prefill_linear_peak_frac": round(linear_flop / pp / (2.5e15 if dtype == "bfloat16" else MFMA_F32_PEAK), 4),
-        "window": at[0]["mask"]["size"], "kernel_classes": per_class, "first_tokens": tokens[:2].tolist(),
+        "window": window, "kernel_classes": per_class, "first_tokens": tokens[:2].tolist(),
     }
     return out
 
@@ -442,6 +460,8 @@ def main():
     ap.add_argument("--loretar", choices=["float32", "bfloat16", "both"], default=None,
                     help="only the Loretar model at the size of --config 5 or 4, beside that configuration's own model "
                          "(one JSON line of their own)")
+    ap.add_argument("--lufatar", choices=["float32", "bfloat16", "both"], default=None, help="the same for the Lufatar model")
+    ap.add_argument("--no-closest", action="store_true", help="with --loretar / --lufatar: without the configuration's own model")
     ap.add_argument("--micro-only", action="store_true", help="only the op micro-benchmarks (one JSON line of their own)")
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="only run a strided copy of known size (268435456 B read + 268435456 B written per launch), "
@@ -468,15 +488,19 @@ def main():
         print(json.dumps({"micro": micro_bench()}))
         return
 
-    if args.loretar:
+    for design, which in (("loretar", args.loretar), ("lufatar", args.lufatar)):
+        if not which:
+            continue
         if args.config == 3:
-            ap.error("--loretar takes --config 5 or 4")
+            ap.error(f"--{design} takes --config 5 or 4")
         line = {}
-        for dt in ("float32", "bfloat16") if args.loretar == "both" else (args.loretar,):
-            line[f"loretar_{dt}"] = measure_loretar(args.config, dt, args.steps, args.warmup, args.seed)
-            print(f"loretar {dt} measured", file=sys.stderr, flush=True)
-        line["closest_model"] = other_config_line(args.config, args.steps, args.warmup)
-        print(json.dumps({"loretar": line}))
+        for dt in ("float32", "bfloat16") if which == "both" else (which,):
+            line[f"{design}_{dt}"] = measure_blocks(design, args.config, dt, args.steps, args.warmup, args.seed)
+            print(f"{design} {dt} measured", file=sys.stderr, flush=True)
+        if not args.no_closest:
+            line["closest_model"] = other_config_line(args.config, args.steps, args.warmup)
+        print(json.dumps({design: line}))
+    if args.loretar or args.lufatar:
         return
 
     import torch  # device-wide synchronisation around the timed region

@@ -42,7 +42,7 @@ struct Abi {
     CGH_FN(cg_binary) CGH_FN(cg_where) CGH_FN(cg_matmul) CGH_FN(cg_sum) CGH_FN(cg_max) CGH_FN(cg_argmax)
     CGH_FN(cg_topk) CGH_FN(cg_broadcast) CGH_FN(cg_reshape) CGH_FN(cg_transpose) CGH_FN(cg_slice)
     CGH_FN(cg_concat) CGH_FN(cg_index) CGH_FN(cg_profile_enable) CGH_FN(cg_profile_read)
-    CGH_FN(cg_block_linear) CGH_FN(cg_block_pair_embedding) CGH_FN(cg_block_conv_linear) CGH_FN(cg_block_residual) CGH_FN(cg_block_token_side) CGH_FN(cg_block_attention) CGH_FN(cg_block_channel_delta)
+    CGH_FN(cg_realize) CGH_FN(cg_block_linear) CGH_FN(cg_block_pair_embedding) CGH_FN(cg_block_conv_linear) CGH_FN(cg_block_residual) CGH_FN(cg_block_token_side) CGH_FN(cg_block_attention) CGH_FN(cg_block_channel_delta)
 #undef CGH_FN
     void *handle = nullptr;
 
@@ -61,7 +61,7 @@ struct Abi {
         CGH_LOAD(cg_max) CGH_LOAD(cg_argmax) CGH_LOAD(cg_topk) CGH_LOAD(cg_broadcast) CGH_LOAD(cg_reshape)
         CGH_LOAD(cg_transpose) CGH_LOAD(cg_slice) CGH_LOAD(cg_concat) CGH_LOAD(cg_index)
         CGH_LOAD(cg_profile_enable) CGH_LOAD(cg_profile_read)
-        CGH_LOAD(cg_block_linear) CGH_LOAD(cg_block_pair_embedding) CGH_LOAD(cg_block_conv_linear) CGH_LOAD(cg_block_residual) CGH_LOAD(cg_block_token_side) CGH_LOAD(cg_block_attention) CGH_LOAD(cg_block_channel_delta)
+        CGH_LOAD(cg_realize) CGH_LOAD(cg_block_linear) CGH_LOAD(cg_block_pair_embedding) CGH_LOAD(cg_block_conv_linear) CGH_LOAD(cg_block_residual) CGH_LOAD(cg_block_token_side) CGH_LOAD(cg_block_attention) CGH_LOAD(cg_block_channel_delta)
 #undef CGH_LOAD
     }
     Abi(const Abi &) = delete;
@@ -261,6 +261,8 @@ class Backend {
     }
     // A tensor that takes over a reference given up with into_raw.
     Tensor adopt(cg_tensor *h) { return Tensor(&abi_, h); }
+    // A deferred result is computed now, for all handles that share it from here on.
+    void realize(const Tensor &x) { check(abi_.cg_realize(b_, x.get())); }
     // Decoder blocks (include/catgrad_hip.h): the argument structures hold raw references, which the call consumes.
     Tensor block_linear(const cg_linear_args &a) {
         return out([&](cg_tensor **o) { return abi_.cg_block_linear(b_, &a, o); });

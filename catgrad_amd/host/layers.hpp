@@ -69,7 +69,13 @@ class LayeredModel : public Model {
     void expect(const std::string &name, const Shape &s) {
         if (dims(name) != s) throw InterpreterError("parameter " + name + " does not have the shape the configuration asks for");
     }
-    void store(const std::string &name) { i_.parameters[name] = i_.backend.cast(std::move(i_.parameters[name]), weights_); }
+    // (computed at once: a view of a deferred tensor would compute it again for itself)
+    Tensor stored_form(Tensor t) {
+        t = i_.backend.cast(std::move(t), weights_);
+        i_.backend.realize(t);
+        return t;
+    }
+    void store(const std::string &name) { i_.parameters[name] = stored_form(std::move(i_.parameters[name])); }
 
     // The matrices `parts` [.., cols] one below the other as parameter `name`, each beginning at a multiple of `align`
     // rows; the parts' own names become views of it.
@@ -88,7 +94,7 @@ class LayeredModel : public Model {
             where[part] = {at, n};
             at += n + pad;
         }
-        all = be.cast(std::move(all), weights_);
+        all = stored_form(std::move(all));
         for (const std::string &part : parts) i_.parameters[part] = be.slice(all, 0, where[part].at, where[part].n);
         i_.parameters[name] = std::move(all);
         in_[name] = std::move(where);
