@@ -281,7 +281,18 @@ int experts_of(cg_backend *be, Held &h, const cg_experts &e, int64_t rows, int64
     int f2;
     if (int rc = dense_weights(be, h, e.gate_up, &p->gate_up, &p->fmt, "experts gate_up")) return rc;
     if (int rc = dense_weights(be, h, e.down, &p->down, &f2, "experts down")) return rc;
-    if (f2 != p->fmt) return fail(CG_ERR_DTYPE, "experts: the weights lie in different forms");
+    if (f2 != p->fmt) { // one of them small enough to lie in words: both as words
+        p->fmt = kFmtWords;
+        for (auto &w : {std::make_pair(e.gate_up, &p->gate_up), std::make_pair(e.down, &p->down)}) {
+            cg_tensor *t = w.first;
+            if (t->uniform || !is_contiguous(t)) {
+                cg_tensor *m = nullptr;
+                if (int rc = materialize(be, t, &m)) return rc;
+                t = h.add(m);
+            }
+            if (int rc = device_ptr(t, w.second)) return rc;
+        }
+    }
     return CG_OK;
 }
 
@@ -548,6 +559,11 @@ int cg_block_conv_linear(cg_backend *b, const cg_conv_linear_args *a, cg_tensor 
         const int64_t xd[2] = {rows, W};
         if (few) rc = new_dense(b, c.keep && c.keep_bf16 ? CG_BF16 : CG_F32, xd, 2, &in[i].x);
         else rc = product_operand(b, rows, in[i].w, in[i].wv, &in[i].x, &in[i].tiles);
+        if (!rc && !few && c.keep && c.keep_bf16 && W % 8 == 0 && in[i].x->buf->fmt == kFmtWords) { // (who reads the kept rows takes patterns)
+            release(in[i].x);
+            in[i].x = nullptr;
+            rc = new_dense(b, CG_BF16, xd, 2, &in[i].x, 0, kFmtBF16);
+        }
         h.add(in[i].x);
         if (rc) return rc;
         if (c.keep && !c.keep_bf16 && in[i].x->dt != CG_F32) return fail(CG_ERR_DTYPE, "block_conv_linear: rows kept in f32 go through f32 weights");

@@ -1,8 +1,6 @@
-"""Small Loretar models shared by the CPU and GPU tests, and what is checked on them: the package's request steps, batches
-and greedy generation against the whole-sequence statement in loretar_reference.py."""
-import numpy as np
-
+"""Small Loretar models shared by the CPU and GPU tests (what is checked on them: design_cases.py)."""
 import loretar_reference as R
+from design_cases import Design
 from catgrad_amd.loretar import attention_layer, config_of, delta_layer, random_params
 
 
@@ -27,132 +25,4 @@ CONFIGS = {
                        loop={"start": 0, "stop": 2, "times": 2}),
 }
 
-
-def params_of(name, seed=0, bf16=True):
-    """Weights as a dictionary; bf16: rounded to bfloat16, as a model file holds them."""
-    from block_cases import bf16 as rounded
-
-    p = dict(random_params(CONFIGS[name], seed, low_rank=5 if name == "odd_sizes" else 8))
-    return {n: rounded(w) for n, w in p.items()} if bf16 else p
-
-
-def load(session, name, seed=0, dtype="float32"):
-    p = params_of(name, seed)
-    session.clear_params()
-    session.load_config(CONFIGS[name], dtype)
-    for n, w in p.items():
-        session.set_param(n, w)
-    return p
-
-
-def tokens_of(name, n, seed=1):
-    return np.random.default_rng(seed).integers(0, CONFIGS[name]["vocab"], size=n)
-
-
-def run(session, tokens, portions, request=1, end=True):
-    """Logits [len(tokens), vocab] of a request in these portions."""
-    at, out = 0, []
-    for n in portions:
-        out.append(session.step(request, tokens[at:at + n], range(n)))
-        at += n
-    assert at == len(tokens)
-    if end:
-        session.end(request)
-    return np.concatenate(out)
-
-
-def close(got, want, tol, what):
-    """Per position: root mean square of the difference over the vocabulary, over the scale of all of them."""
-    scale = np.sqrt(((want - want.mean(-1, keepdims=True)) ** 2).mean())
-    d = got - want
-    err = np.sqrt(((d - d.mean(-1, keepdims=True)) ** 2).mean(-1)) / scale
-    assert err.max() <= tol, f"{what}: {err.max():.3g} of the logits' scale at position {int(err.argmax())}, allowed {tol:.3g}"
-
-
-TOLERANCE = {"float32": 5e-5, "bfloat16": 4e-2}
-PORTIONS = {"whole": [50], "token_by_token": [1] * 50, "halves": [25, 25], "twos_and_threes": [2, 3] * 10, "prompt_then_decode": [38] + [1] * 12,
-            "uneven": [17, 2, 1, 9, 1, 1, 16, 3], "sixteens": [16, 16, 16, 2]}
-
-
-def check_portions(session, name, how, dtype="float32"):
-    p = load(session, name, dtype=dtype)
-    t = tokens_of(name, 50)
-    close(run(session, t, PORTIONS[how]), R.logits(CONFIGS[name], p, t), TOLERANCE[dtype], f"{name}, {how}, {dtype}")
-
-
-def check_one_token(session, name):
-    p = load(session, name)
-    for seed in range(3):
-        t = tokens_of(name, 1, seed)
-        close(run(session, t, [1]), R.logits(CONFIGS[name], p, t), TOLERANCE["float32"], f"{name}, one token")
-
-
-def check_interleaved(session, name, dtype="float32"):
-    """Requests of unequal length, a step of each in turn, ended and begun again under the same numbers."""
-    p = load(session, name, dtype=dtype)
-    rng = np.random.default_rng(3)
-    for round_ in range(2):
-        reqs = {r: tokens_of(name, n, seed=10 * round_ + r) for r, n in ((1, 44), (2, 7), (3, 29), (4, 1))}
-        at, got = dict.fromkeys(reqs, 0), {r: [] for r in reqs}
-        while at:
-            for r in list(at):
-                n = int(min(rng.integers(1, 12), len(reqs[r]) - at[r]))
-                got[r].append(session.step(r, reqs[r][at[r]:at[r] + n], range(n)))
-                at[r] += n
-                if at[r] == len(reqs[r]):
-                    session.end(r)
-                    del at[r]
-        assert session.requests_in_progress() == 0
-        for r, t in reqs.items():
-            close(np.concatenate(got[r]), R.logits(CONFIGS[name], p, t), TOLERANCE[dtype], f"{name}, request {r} among others")
-
-
-def check_long_decode(session, name, n=150, dtype="float32"):
-    p = load(session, name, dtype=dtype)
-    t = tokens_of(name, n)
-    close(run(session, t, [5] + [1] * (n - 5)), R.logits(CONFIGS[name], p, t), TOLERANCE[dtype], f"{name}, decoding from token 5 to {n}")
-
-
-def greedy(config, p, prompt, steps):
-    toks, out, gaps = list(prompt), [], []
-    for _ in range(steps + 1):
-        lg = R.logits(config, p, toks)[-1]
-        top = np.sort(lg)
-        out.append(int(lg.argmax()))
-        gaps.append((top[-1] - top[-2]) / lg.std())
-        toks.append(out[-1])
-    return out, gaps
-
-
-def check_generate(session, name, steps=12):
-    """Two prompts of equal length as a batch through the generate loop; a prompt through request steps that ask for the
-    next token; both against recomputing the whole sequence for every token."""
-    p = load(session, name)
-    prompts = np.stack([tokens_of(name, 21, seed=s) for s in (5, 6)])
-    got, _ = session.generate(prompts, steps)
-    for b in range(2):
-        want, gaps = greedy(CONFIGS[name], p, prompts[b], steps)
-        same = [int(x) for x in got[:, b]]
-        for i, (a, w) in enumerate(zip(same, want)):
-            if a != w:
-                assert gaps[i] < 1e-3, f"{name}: token {i} of sequence {b} is {a}, not {w}"
-                break
-        toks, nxt = prompts[b], []
-        for _ in range(steps + 1):
-            _, t = session.step(9, toks, (), want_next=True)
-            nxt.append(t)
-            toks = [t]
-        session.end(9)
-        assert nxt == same
-
-
-def check_batch_logits(session, name):
-    """The logits of a batch's prompts in one run against each alone."""
-    p = load(session, name)
-    prompts = np.stack([tokens_of(name, 23, seed=s) for s in (7, 8, 9)])
-    _, lg = session.forward(prompts)
-    for b in range(3):
-        close(lg[b], R.logits(CONFIGS[name], p, prompts[b]), TOLERANCE["float32"], f"{name}, sequence {b} of a batch")
-    rows = [4, 23 + 22, 2 * 23]
-    _, picked = session.forward_rows(prompts, rows)
-    np.testing.assert_allclose(picked, lg.reshape(-1, lg.shape[-1])[rows], rtol=1e-6, atol=1e-6)
+LORETAR = Design(CONFIGS, R, lambda config, seed, name, dtype: random_params(config, seed, low_rank=5 if name == "odd_sizes" else 8), {"float32": 5e-5, "bfloat16": 4e-2})

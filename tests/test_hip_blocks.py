@@ -1,4 +1,4 @@
-"""The decoder blocks on the GPU against the plain statements of loretar_reference.py."""
+"""The decoder blocks on the GPU against the plain statements of loretar_reference.py and lufatar_reference.py."""
 import numpy as np
 import pytest
 
@@ -35,6 +35,56 @@ def test_attention_tile_shapes(hip, heads, kv_heads, dim):
     for vdim, talk in ((dim, True), (max(8, dim - 12), False)):
         o = C.options(heads, kv_heads, dim, vdim, 37)
         C.check_attention(hip, C.attention_case(rng, 1, 90, o, True, talk), o, [41, 49])
+
+
+@pytest.mark.parametrize("name", list(C.MIXED))
+def test_mixed_scores(hip, name):
+    C.run_mixed_case(hip, name)
+
+
+@pytest.mark.parametrize("portions", [[20, 1, 2, 17], [80, 1, 1, 2, 70], [140, 1, 3, 9, 1]], ids=str)
+def test_mixed_scores_needles(hip, portions):
+    C.run_mixed_needles(hip, C.turned(4, 2, 16, 16, 0), portions)
+
+
+@pytest.mark.parametrize("dim,vdim", [(16, 16), (32, 20), (48, 96), (64, 64), (64, 80), (96, 48), (128, 128)])
+@pytest.mark.parametrize("heads,kv_heads", [(4, 2), (8, 8), (12, 3), (16, 2), (20, 5), (32, 8), (32, 4)])
+def test_mixed_scores_shapes(hip, heads, kv_heads, dim, vdim):
+    """Every instantiation of the tiled and the step kernels: heads per wave, query heads per key head, widths."""
+    rng = np.random.default_rng(heads * dim + vdim)
+    o = C.turned(heads, kv_heads, dim, vdim, dim // 2 // 2 * 2)
+    C.check_attention(hip, C.attention_case(rng, 1, 94, o, False, True), o, [41, 49, 1, 1, 2], tol=6e-5)
+
+
+@pytest.mark.parametrize("dtype", ["f32", "bf16"])
+def test_pair_embedding(hip, dtype):
+    C.run_pair_embedding(hip, dtype)
+    C.run_pair_embedding(hip, dtype, B=1, vocab=5000, buckets=4099, width=512, mul_prev=2 ** 40 + 9, mul_cur=2 ** 31 + 11)
+
+
+@pytest.mark.parametrize("case", C.CONV, ids=str)
+def test_conv_linear(hip, case):
+    C.run_conv_linear(hip, case)
+
+
+@pytest.mark.parametrize("case", [(3, 40, 5, 7, "f32"), (1, 2048, 4, 5000, "bf16"), (4, 1024, 8, 300, "f32"), (50, 96, 3, 130, "bf16"), (50, 30, 3, 13, "f32")], ids=str)
+def test_grouped_linear(hip, case):
+    C.run_grouped_linear(hip, *case)
+
+
+@pytest.mark.parametrize("case", C.EXPERTS, ids=str)
+def test_experts(hip, case):
+    C.run_experts(hip, case)
+
+
+@pytest.mark.parametrize("rows", [1, 5, 20, 300])
+def test_expert_choices(hip, rows):
+    C.run_expert_choices(hip, rows)
+
+
+@pytest.mark.parametrize("case", C.SIDE, ids=str)
+def test_token_side(hip, case):
+    C.run_side(hip, case)
 
 
 @pytest.mark.parametrize("name", list(C.DELTA))
@@ -80,6 +130,13 @@ def test_blocks_give_their_memory_back(hip):
         C.run_delta(hip, u, d, [40, 1, 1, 18])
         C.run_linear(hip, C.LINEAR[2])
         C.run_residual(hip, C.RESIDUAL[2])
+        C.run_mixed_case(hip, "twos_and_threes")
+        for case in (C.CONV[2], C.CONV[9]):
+            C.run_conv_linear(hip, case)
+        for case in (C.EXPERTS[2], C.EXPERTS[10], C.EXPERTS[13]):
+            C.run_experts(hip, case)
+        for case in (C.SIDE[1], C.SIDE[5]):
+            C.run_side(hip, case)
 
     once()
     hip.sync()
@@ -106,3 +163,16 @@ def test_misfits_are_errors(hip):
         hip.block_linear(x, hip.from_numpy(np.ones((4, 9), np.float32)))
     with pytest.raises(BackendPanic):
         hip.block_residual(x, [{"y": x, "w": hip.from_numpy(np.ones((9, 8), np.float32))}])
+    ones = lambda *s: hip.from_numpy(np.ones(s, np.float32))
+    ex = dict(h=x, logits=ones(1, 2, 4), gate_up=ones(4, 2, 6, 8), down=ones(4, 8, 6))
+    for bad in (dict(top=5, groups=1, keep=1), dict(top=3, groups=2, keep=1), dict(top=2, groups=3, keep=1), dict(top=0, groups=1, keep=1), dict(top=2, groups=2, keep=3)):
+        with pytest.raises(BackendPanic):
+            hip.block_residual(x, [], experts=ex, **bad)
+    with pytest.raises(BackendPanic):
+        hip.block_residual(x, [], experts={**ex, "down": ones(4, 8, 5)}, top=2, groups=1, keep=1)
+    with pytest.raises(BackendPanic):   # groups that do not divide the row
+        hip.block_conv_linear(x, hip.zeros((1, 1, 8), 0), [{"gamma": ones(8), "conv": ones(8, 2), "w": ones(3, 8)}], groups=3)
+    with pytest.raises(BackendPanic):
+        hip.block_conv_linear(x, hip.zeros((1, 2, 8), 0), [{"gamma": ones(8), "conv": ones(8, 2), "w": ones(3, 8)}])
+    with pytest.raises(BackendPanic):   # the table ends before the part
+        hip.block_token_side(dict(x=x, ids=hip.from_numpy(np.zeros((1, 2), np.uint32)), table=ones(5, 8), gate=ones(4, 8), proj=ones(8, 4), norm=ones(8)), first=6)

@@ -2,9 +2,10 @@
 import numpy as np
 import pytest
 
-import loretar_cases as C
+import design_cases as C
 import loretar_reference as R
 from block_cases import bf16
+from loretar_cases import LORETAR as D
 from catgrad_amd.loretar import attention_layer, config_of, delta_layer, random_params
 from catgrad_amd.runner import Session
 
@@ -18,41 +19,41 @@ def session():
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("how", list(C.PORTIONS))
-@pytest.mark.parametrize("name", list(C.CONFIGS))
+@pytest.mark.parametrize("name", list(D.configs))
 def test_portions(session, name, how, dtype):
-    C.check_portions(session, name, how, dtype)
+    C.check_portions(D, session, name, how, dtype)
 
 
-@pytest.mark.parametrize("name", list(C.CONFIGS))
+@pytest.mark.parametrize("name", list(D.configs))
 def test_one_token(session, name):
-    C.check_one_token(session, name)
+    C.check_one_token(D, session, name)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("name", ["mixed", "wider", "odd_sizes"])
 def test_interleaved_requests(session, name, dtype):
-    C.check_interleaved(session, name, dtype)
+    C.check_interleaved(D, session, name, dtype)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("name", ["mixed", "wider"])
 def test_long_decode(session, name, dtype):
-    C.check_long_decode(session, name, 260, dtype)
+    C.check_long_decode(D, session, name, 260, dtype)
 
 
 @pytest.mark.parametrize("name", ["mixed", "attention_only", "recurrence_only", "odd_sizes", "wider"])
 def test_generate(session, name):
-    C.check_generate(session, name)
+    C.check_generate(D, session, name)
 
 
 @pytest.mark.parametrize("name", ["mixed", "odd_sizes", "wider"])
 def test_batch_logits(session, name):
-    C.check_batch_logits(session, name)
+    C.check_batch_logits(D, session, name)
 
 
 def test_recorded_schedules(session):
-    C.load(session, "mixed")
-    t = C.tokens_of("mixed", 30)
+    C.load(D, session, "mixed")
+    t = C.tokens_of(D, "mixed", 30)
     want = C.run(session, t, [20, 1, 9])
     try:
         for schedule in (1, 2):
@@ -63,8 +64,8 @@ def test_recorded_schedules(session):
 
 
 def test_ended_requests_give_their_memory_back(session):
-    C.load(session, "wider")
-    t = C.tokens_of("wider", 120)
+    C.load(D, session, "wider")
+    t = C.tokens_of(D, "wider", 120)
 
     def once():
         for r in range(4):

@@ -8,11 +8,10 @@ import sys
 
 import numpy as np
 import pytest
-import torch
-from safetensors.torch import save_file
 
-import loretar_cases as C
+import design_cases as C
 import loretar_reference as R
+from loretar_cases import LORETAR as D
 from catgrad_amd.loretar import param_shapes
 from catgrad_amd.runner import Session, random_params
 from model_cases import TINY
@@ -27,47 +26,47 @@ def session():
     return Session(ORACLE_LIB)
 
 
-@pytest.mark.parametrize("name", list(C.CONFIGS))
+@pytest.mark.parametrize("name", list(D.configs))
 def test_whole_prompt(session, name):
-    C.check_portions(session, name, "whole")
+    C.check_portions(D, session, name, "whole")
 
 
 @pytest.mark.parametrize("how", [h for h in C.PORTIONS if h != "whole"])
 @pytest.mark.parametrize("name", ["mixed", "odd_sizes", "a_window_of_one"])
 def test_portions(session, name, how):
-    C.check_portions(session, name, how)
+    C.check_portions(D, session, name, how)
 
 
 @pytest.mark.parametrize("name", ["mixed", "recurrence_only", "one_head_each"])
 def test_bfloat16_weights(session, name):
-    C.check_portions(session, name, "prompt_then_decode", "bfloat16")
+    C.check_portions(D, session, name, "prompt_then_decode", "bfloat16")
 
 
 def test_one_token(session):
-    C.check_one_token(session, "mixed")
+    C.check_one_token(D, session, "mixed")
 
 
 def test_interleaved_requests(session):
-    C.check_interleaved(session, "mixed")
+    C.check_interleaved(D, session, "mixed")
 
 
 def test_long_decode(session):
-    C.check_long_decode(session, "no_loop")
+    C.check_long_decode(D, session, "no_loop")
 
 
 @pytest.mark.parametrize("name", ["mixed", "attention_only"])
 def test_generate(session, name):
-    C.check_generate(session, name, steps=6)
+    C.check_generate(D, session, name, steps=6)
 
 
 def test_batch_logits(session):
-    C.check_batch_logits(session, "mixed")
+    C.check_batch_logits(D, session, "mixed")
 
 
 def test_recorded_schedules(session):
     """The layered and the recorded evaluation orders run the same operations."""
-    C.load(session, "mixed")
-    t = C.tokens_of("mixed", 30)
+    C.load(D, session, "mixed")
+    t = C.tokens_of(D, "mixed", 30)
     want = C.run(session, t, [20, 1, 9])
     try:
         for schedule in (1, 2):
@@ -78,38 +77,30 @@ def test_recorded_schedules(session):
 
 
 def test_a_parameter_set_again_is_used(session):
-    p = C.load(session, "mixed")
-    t = C.tokens_of("mixed", 12)
+    p = C.load(D, session, "mixed")
+    t = C.tokens_of(D, "mixed", 12)
     C.run(session, t, [12])
     p["l1.mix.k"] = p["l1.mix.k"] * np.float32(-0.5)
     session.set_param("l1.mix.k", p["l1.mix.k"])
-    C.close(C.run(session, t, [12]), R.logits(C.CONFIGS["mixed"], p, t), 5e-5, "after a parameter was set again")
-
-
-def write_model(folder, name, seed=0):
-    p = C.params_of(name, seed)
-    with open(os.path.join(folder, "config.json"), "w") as f:
-        json.dump(C.CONFIGS[name], f)
-    save_file({n: torch.from_numpy(np.ascontiguousarray(w)).to(torch.bfloat16) for n, w in p.items()}, os.path.join(folder, "model.safetensors"))
-    return p
+    C.close(C.run(session, t, [12]), R.logits(D.configs["mixed"], p, t), 5e-5, "after a parameter was set again")
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_a_model_folder(session, tmp_path, dtype):
-    p = write_model(tmp_path, "everything_looped")
+    p = C.write_model(D, tmp_path, "everything_looped", dtype=dtype)
     stats = session.load_pretrained(tmp_path, dtype)
     assert stats["tensors"] == len(p)
-    t = C.tokens_of("everything_looped", 30)
-    C.close(C.run(session, t, [20, 1, 9]), R.logits(C.CONFIGS["everything_looped"], p, t), C.TOLERANCE[dtype], f"model folder, {dtype}")
+    t = C.tokens_of(D, "everything_looped", 30)
+    C.close(C.run(session, t, [20, 1, 9]), R.logits(D.configs["everything_looped"], p, t), D.tolerance[dtype], f"model folder, {dtype}")
 
 
 def test_trace_run(tmp_path):
     """Two requests step by step through the program: wanted places, steps without any, ends, and a name used again."""
     model, out = tmp_path / "model", tmp_path / "out"
     model.mkdir(), out.mkdir()
-    p = write_model(model, "mixed")
-    c = C.CONFIGS["mixed"]
-    a, b = C.tokens_of("mixed", 26, 1), C.tokens_of("mixed", 9, 2)
+    p = C.write_model(D, model, "mixed")
+    c = D.configs["mixed"]
+    a, b = C.tokens_of(D, "mixed", 26, 1), C.tokens_of(D, "mixed", 9, 2)
     steps = [{"step": 0, "entries": [{"id": "x", "tokens": a[:20].tolist(), "want": [0, 19]}], "end": []},
              {"step": 1, "entries": [{"id": "y", "tokens": b[:7].tolist(), "want": []}], "end": []},
              {"step": 2, "entries": [{"id": "x", "tokens": a[20:].tolist(), "want": [5, 2]}], "end": ["x"]},
@@ -131,7 +122,7 @@ def test_trace_run(tmp_path):
 
 
 def changed(name, edit):
-    c = copy.deepcopy(C.CONFIGS[name])
+    c = copy.deepcopy(D.configs[name])
     edit(c)
     return c
 
@@ -150,8 +141,8 @@ def test_configurations_that_do_not_fit(session, edit):
 
 
 def test_parameters_that_do_not_fit(session):
-    p = C.load(session, "mixed")
-    t = C.tokens_of("mixed", 4)
+    p = C.load(D, session, "mixed")
+    t = C.tokens_of(D, "mixed", 4)
     session.set_param("l0.mix.talk", np.eye(3, dtype=np.float32))
     with pytest.raises(RuntimeError, match="l0.mix.talk"):
         session.step(1, t)
@@ -170,7 +161,7 @@ def test_parameters_that_do_not_fit(session):
 
 
 def test_the_shapes_of_a_configuration():
-    for name, c in C.CONFIGS.items():
+    for name, c in D.configs.items():
         names = [n for n, _ in param_shapes(c)]
         assert len(names) == len(set(names))
         assert ("loop.in" in names) == bool(c["loop"]), name
