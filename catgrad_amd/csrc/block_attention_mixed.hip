@@ -38,26 +38,60 @@ __device__ __forceinline__ float slope_of(uint32_t h, uint32_t heads) { return e
 __device__ __forceinline__ uint32_t first_visible(const AttentionPlan &p, uint32_t i) { return p.window && i + 1 > p.window ? i + 1 - p.window : 0; }
 
 // out = the segments' results together; result i of a row: head i / vdim.  parts at row * row_pitch + segment * seg_pitch,
-// stats the same in heads.
-__global__ __launch_bounds__(kThreads) void attention_merge_kernel(const float *__restrict__ parts, const float2 *__restrict__ stats, const uint32_t segs, const uint64_t row_pitch,
-                                                                   const uint64_t seg_pitch, const uint32_t heads, const uint32_t vdim, const bool sink, float *__restrict__ out) {
-    const uint32_t n = heads * vdim, i = blockIdx.x * kThreads + threadIdx.x;
-    if (i >= n) return;
+// stats the same in heads.  A workgroup per 64 results, its waves a run of segments each.
+constexpr int kMergeWaves = 8;
+__global__ __launch_bounds__(kMergeWaves * 64) void attention_merge_kernel(const float *__restrict__ parts, const float2 *__restrict__ stats, const uint32_t segs,
+                                                                           const uint64_t row_pitch, const uint64_t seg_pitch, const uint32_t heads, const uint32_t vdim,
+                                                                           const bool sink, float *__restrict__ out) {
+    __shared__ float sums[3][kMergeWaves][64];
+    const uint32_t n = heads * vdim, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, i = min(blockIdx.x * 64 + lane, n - 1);
     const uint64_t row = blockIdx.y;
     const float *p = parts + row * row_pitch * vdim + i;
     const float2 *st = stats + row * row_pitch + i / vdim;
-    float m = sink ? 0.0f : kNone;
-#pragma unroll 8
-    for (uint32_t k = 0; k < segs; k++) m = fmaxf(m, st[k * seg_pitch].x);
-    float l = sink ? __builtin_amdgcn_exp2f(-m) : 0.0f, o = 0.0f;
-#pragma unroll 8
-    for (uint32_t k = 0; k < segs; k++) {
-        const float2 t = st[k * seg_pitch];
-        const float f = __builtin_amdgcn_exp2f(t.x - m);
-        l = fmaf(t.y, f, l);
-        o = fmaf(p[k * seg_pitch * vdim], f, o);
+    const uint32_t per = (segs + kMergeWaves - 1) / kMergeWaves, k0 = min(segs, wave * per), k1 = min(segs, k0 + per);
+    float m = kNone, l = 0.0f, o = 0.0f;
+    constexpr int AHEAD = 8;
+    for (uint32_t k = k0; k < k1; k += AHEAD) {
+        float2 t[AHEAD];
+        float v[AHEAD];
+#pragma unroll
+        for (int e = 0; e < AHEAD; e++) { // (clamped: a segment behind the last weighs nothing)
+            const uint64_t at = (uint64_t)min(k + e, k1 - 1) * seg_pitch;
+            t[e] = st[at];
+            v[e] = p[at * vdim];
+            if (k + e >= k1) t[e] = make_float2(kNone, 0.0f);
+        }
+        float up = m;
+#pragma unroll
+        for (int e = 0; e < AHEAD; e++) up = fmaxf(up, t[e].x);
+        const float f = __builtin_amdgcn_exp2f(m - up);
+        l *= f;
+        o *= f;
+        m = up;
+#pragma unroll
+        for (int e = 0; e < AHEAD; e++) {
+            const float w = k + e < k1 ? __builtin_amdgcn_exp2f(t[e].x - m) : 0.0f;
+            l = fmaf(t[e].y, w, l);
+            o = fmaf(v[e], w, o);
+        }
     }
-    out[row * n + i] = o / l;
+    sums[0][wave][lane] = m;
+    sums[1][wave][lane] = l;
+    sums[2][wave][lane] = o;
+    __syncthreads();
+    if (wave) return;
+    m = sink ? 0.0f : kNone;
+#pragma unroll
+    for (int w = 0; w < kMergeWaves; w++) m = fmaxf(m, sums[0][w][lane]);
+    l = sink ? __builtin_amdgcn_exp2f(-m) : 0.0f;
+    o = 0.0f;
+#pragma unroll
+    for (int w = 0; w < kMergeWaves; w++) {
+        const float f = __builtin_amdgcn_exp2f(sums[0][w][lane] - m);
+        l = fmaf(sums[1][w][lane], f, l);
+        o = fmaf(sums[2][w][lane], f, o);
+    }
+    if (blockIdx.x * 64 + lane < n) out[row * n + i] = o / l;
 }
 
 // ---- other sizes -----------------------------------------------------------------------------------------------------
@@ -349,11 +383,14 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
 }
 
 // ---- a few new tokens ------------------------------------------------------------------------------------------------
-constexpr uint32_t kMaxStepKeys = 64;
+// Keys are taken in chunks of `chunk`, a workgroup takes `chunks` of them.  Their keys and values are asked for first and
+// arrive while the queries are prepared: four lanes share a key of a kv head (PI such keys per four lanes, DQ 16-byte pieces
+// per lane), a thread has four columns of a kv head's values (for every turns-th key of the chunk).
+constexpr uint32_t kMaxChunk = 64, kValuesAhead = 8;
 struct StepLds { // floats
-    uint32_t turn, q, fresh, talk, raw, mixed, total;
+    uint32_t turn, q, fresh, talk, raw, mixed, state, total;
 };
-__host__ __device__ inline StepLds step_lds(uint32_t S, uint32_t heads, uint32_t kv_heads, uint32_t dim, uint32_t rot, uint32_t keys) {
+__host__ __device__ inline StepLds step_lds(uint32_t S, uint32_t heads, uint32_t kv_heads, uint32_t dim, uint32_t rot, uint32_t chunk, uint32_t vdim) {
     StepLds o{};
     uint32_t at = 0;
     auto take = [&](uint32_t n) {
@@ -361,63 +398,105 @@ __host__ __device__ inline StepLds step_lds(uint32_t S, uint32_t heads, uint32_t
         at += (n + 3) / 4 * 4;
         return r;
     };
-    o.turn = take(rot * S);                      // {cos, sin} per pair and new token
+    o.turn = take(rot * S);             // {cos, sin} per pair and new token
     o.q = take(heads * dim);
-    o.fresh = take(kv_heads * dim * S);          // new keys
+    o.fresh = take(kv_heads * dim * S); // new keys
     o.talk = take(heads * heads);
-    o.raw = take(heads * (keys + 1));
-    o.mixed = take(heads * (keys + 1));
+    o.raw = take(heads * (chunk + 1));
+    o.mixed = take(heads * (chunk + 1));
+    o.state = take(3 * heads);          // top, sum, what the results so far are multiplied by
+    if (o.q + heads * vdim > at) at = o.q + heads * vdim; // (at the end the results of turns meet from `q` on)
     o.total = at;
     return o;
 }
 
-template <int REP>
-__global__ __launch_bounds__(kThreads) void attention_mixed_step_kernel(const AttentionPlan p, const uint32_t seg_keys, float *__restrict__ parts, float2 *__restrict__ stats) {
+template <int REP, int DQ, int PI>
+__global__ __launch_bounds__(kThreads) void attention_mixed_step_kernel(const AttentionPlan p, const uint32_t chunk, const uint32_t chunks, float *__restrict__ parts,
+                                                                        float2 *__restrict__ stats) {
     extern __shared__ float lds[];
     const uint32_t rep = p.heads / p.kv_heads, seg = blockIdx.x, nseg = gridDim.x, r = blockIdx.y, b = r / p.S, s = r - b * p.S;
-    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, pitch = seg_keys + 1;
-    const StepLds at = step_lds(p.S, p.heads, p.kv_heads, p.dim, p.rot_dims, seg_keys);
-    const uint32_t j0 = first_visible(p, p.cached + s) + seg * seg_keys, hi = p.cached + s + 1, keys = j0 < hi ? min(seg_keys, hi - j0) : 0;
-    // the angles of this token and of those new ones in front of it whose keys this workgroup scores
-    const uint32_t t0 = j0 > p.cached ? j0 - p.cached : 0, t1 = j0 + keys > p.cached ? j0 + keys - p.cached : 0; // new keys [t0, t1)
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, pitch = chunk + 1, sub = threadIdx.x & 3;
+    const StepLds at = step_lds(p.S, p.heads, p.kv_heads, p.dim, p.rot_dims, chunk, p.vdim);
+    const uint32_t first = first_visible(p, p.cached + s) + seg * chunk * chunks, hi = p.cached + s + 1, end = min(hi, first + chunk * chunks);
+    const uint32_t vec = p.vdim / 4, cols = p.kv_heads * vec, turns = max(1u, kThreads / cols);
+    const uint32_t mine = threadIdx.x % cols, my_turn = threadIdx.x / cols; // (more columns than threads: turns 1, a second round)
+    const bool has_values = cols > kThreads || my_turn < turns;
+    f32x4 k[PI][DQ], v[kValuesAhead];
+    auto key_of = [&](uint32_t j0, int i, uint32_t *g, uint32_t *key) {
+        const uint32_t pair = (threadIdx.x >> 2) + i * (kThreads / 4);
+        *g = min(pair / chunk, p.kv_heads - 1);
+        *key = pair - pair / chunk * chunk;
+        return pair < chunk * p.kv_heads;
+    };
+    // (rows that are not there or not in the cache are clamped into it: what they hold is replaced or hidden)
+    auto ask_keys = [&](uint32_t j0) {
+#pragma unroll
+        for (int i = 0; i < PI; i++) {
+            uint32_t g, key;
+            key_of(j0, i, &g, &key);
+            const float *src = p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)min(j0 + key, p.cached ? p.cached - 1 : 0) * p.dim;
+#pragma unroll
+            for (int d = 0; d < DQ; d++) k[i][d] = *reinterpret_cast<const f32x4 *>(src + min((uint32_t)(d * 16 + sub * 4), p.dim - 4));
+        }
+    };
+    auto value_row = [&](uint32_t j, uint32_t g) { // new ones come from the projections
+        return j < p.cached ? p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)j * p.vdim
+                            : p.v.p + ((int64_t)b * p.S + (min(j, hi - 1) - p.cached)) * p.v.pitch + g * p.vdim;
+    };
+    auto ask_values = [&](uint32_t j0, uint32_t c) {
+        const uint32_t g = min(c / vec, p.kv_heads - 1), d = (c - c / vec * vec) * 4;
+#pragma unroll
+        for (uint32_t e = 0; e < kValuesAhead; e++)
+            if (e * turns < chunk) v[e] = *reinterpret_cast<const f32x4 *>(value_row(min(j0 + my_turn % turns + e * turns, hi - 1), g) + d);
+    };
+    ask_keys(first);
+    ask_values(first, mine);
+
+    // the angles of this token and of those new ones whose keys this workgroup scores
+    const uint32_t t0 = first > p.cached ? first - p.cached : 0, t1 = end > p.cached && end > first ? end - p.cached : 0; // new keys [t0, t1)
     const uint32_t pairs = p.rot_dims / 2;
     float2 *turn = reinterpret_cast<float2 *>(lds + at.turn);
     for (uint32_t i = threadIdx.x; i < pairs * p.S; i += kThreads) {
-        const uint32_t t = i / pairs, k = i - t * pairs;
+        const uint32_t t = i / pairs, n = i - t * pairs;
         if (t != s && (t < t0 || t >= t1)) continue;
-        double a = (double)(p.position + t) * exp2(-2.0 * (double)k / (double)p.rot_dims * p.rot_log2);
+        double a = (double)(p.position + t) * exp2(-2.0 * (double)n / (double)p.rot_dims * p.rot_log2);
         a -= 6.283185307179586 * rint(a * 0.15915494309189535);
         float sn, cs;
         sincosf((float)a, &sn, &cs);
         turn[i] = make_float2(cs, sn);
     }
     for (uint32_t i = threadIdx.x; i < p.heads * p.heads; i += kThreads) lds[at.talk + i] = p.talk ? p.talk[i] : i / p.heads == i % p.heads ? 1.0f : 0.0f;
+    for (uint32_t h = threadIdx.x; h < p.heads; h += kThreads) {
+        lds[at.state + h] = kNone;
+        lds[at.state + p.heads + h] = 0.0f;
+    }
     __syncthreads();
     // a head of new token t: turned, at a mean square of one, times f; a wave per head
     auto head = [&](const float *src, uint32_t t, float f, float *dst, float *also) {
         auto value = [&](uint32_t d) {
-            const float v = src[d];
-            if (d >= p.rot_dims) return v;
+            const float x = src[d];
+            if (d >= p.rot_dims) return x;
             const float2 cs = turn[t * pairs + d / 2];
-            return d & 1 ? fmaf(v, cs.x, src[d - 1] * cs.y) : fmaf(v, cs.x, -src[d + 1] * cs.y);
+            return d & 1 ? fmaf(x, cs.x, src[d - 1] * cs.y) : fmaf(x, cs.x, -src[d + 1] * cs.y);
         };
         float m = 0.0f;
         const float v0 = lane < p.dim ? value(lane) : 0.0f, v1 = lane + 64 < p.dim ? value(lane + 64) : 0.0f;
         m = fmaf(v0, v0, v1 * v1);
         for (uint32_t d = lane + 128; d < p.dim; d += 64) {
-            const float v = value(d);
-            m = fmaf(v, v, m);
+            const float x = value(d);
+            m = fmaf(x, x, m);
         }
         float g = f;
         if (p.unit_heads) g /= sqrtf(wave_sum(m) / (float)p.dim + p.eps);
         for (uint32_t d = lane; d < p.dim; d += 64) {
-            const float v = (d == lane ? v0 : d == lane + 64 ? v1 : value(d)) * g;
-            dst[d] = v;
-            if (also) also[d] = v;
+            const float x = (d == lane ? v0 : d == lane + 64 ? v1 : value(d)) * g;
+            dst[d] = x;
+            if (also) also[d] = x;
         }
     };
     float temp = p.scale;
     if (p.temp_every) temp *= 1.0f + p.temp_coef * logf((float)((p.position + s + 1) / p.temp_every + 1));
+#pragma unroll 4
     for (uint32_t h = wave; h < p.heads; h += kThreads / 64) head(p.q.p + (int64_t)r * p.q.pitch + h * p.dim, s, temp, lds + at.q + h * p.dim, nullptr);
     for (uint32_t i = wave; i < (t1 - min(t0, t1)) * p.kv_heads; i += kThreads / 64) {
         const uint32_t t = t0 + i / p.kv_heads, g = i % p.kv_heads;
@@ -430,84 +509,121 @@ __global__ __launch_bounds__(kThreads) void attention_mixed_step_kernel(const At
             p.values[((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)(p.cached + s) * p.vdim + d] = p.v.p[(int64_t)r * p.v.pitch + i];
         }
     __syncthreads();
-    // scores: four lanes share a key of a kv head
-    const uint32_t sub = threadIdx.x & 3;
-    for (uint32_t i = threadIdx.x >> 2; i < seg_keys * p.kv_heads; i += kThreads / 4) {
-        const uint32_t g = i / seg_keys, key = i - g * seg_keys, j = j0 + min(key, max(keys, 1u) - 1);
-        const bool fresh = keys && j >= p.cached;
-        const float *kp = fresh ? lds + at.fresh + ((j - p.cached) * p.kv_heads + g) * p.dim
-                                : p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)min(j, p.cached ? p.cached - 1 : 0) * p.dim;
-        for (uint32_t h0 = 0; h0 < rep; h0 += REP) {
-            float acc[REP] = {};
-            const float *qh = lds + at.q + (g * rep + h0) * p.dim;
-#pragma unroll 8
-            for (uint32_t d = sub * 4; d < p.dim; d += 16) {
-                const float4 kv = *reinterpret_cast<const float4 *>(kp + d);
+    f32x4 acc[REP] = {};
+    for (uint32_t j0 = first; j0 < end; j0 += chunk) {
+        const uint32_t keys = min(chunk, end - j0);
+#pragma unroll
+        for (int i = 0; i < PI; i++) {
+            uint32_t g, key;
+            const bool there = key_of(j0, i, &g, &key);
+            const uint32_t j = j0 + key;
+            if (there && key < keys && j >= p.cached) {
+#pragma unroll
+                for (int d = 0; d < DQ; d++)
+                    k[i][d] = *reinterpret_cast<const f32x4 *>(lds + at.fresh + ((j - p.cached) * p.kv_heads + g) * p.dim + min((uint32_t)(d * 16 + sub * 4), p.dim - 4));
+            }
+            for (uint32_t h0 = 0; h0 < rep; h0 += REP) {
 #pragma unroll
                 for (int h = 0; h < REP; h++) {
-                    if (h0 + h >= rep) break;
-                    const float4 qv = *reinterpret_cast<const float4 *>(qh + h * p.dim + d);
-                    acc[h] = fmaf(kv.x, qv.x, fmaf(kv.y, qv.y, fmaf(kv.z, qv.z, fmaf(kv.w, qv.w, acc[h]))));
-                }
-            }
+                    const uint32_t hh = g * rep + min(h0 + h, rep - 1);
+                    const float *qh = lds + at.q + hh * p.dim;
+                    float x = 0.0f;
 #pragma unroll
-            for (int h = 0; h < REP; h++) {
-                float v = acc[h];
-                v += __shfl_xor(v, 1, 64);
-                v += __shfl_xor(v, 2, 64);
-                if (sub == 0 && h0 + h < rep) {
-                    const uint32_t hh = g * rep + h0 + h;
-                    if (p.bias) v -= slope_of(hh, p.heads) * (float)(int)(p.cached + s - j);
-                    lds[at.raw + hh * pitch + key] = v;
+                    for (int d = 0; d < DQ; d++) {
+                        const uint32_t e = d * 16 + sub * 4;
+                        const f32x4 qv = *reinterpret_cast<const f32x4 *>(qh + min(e, p.dim - 4));
+                        const float y = fmaf(k[i][d][0], qv[0], fmaf(k[i][d][1], qv[1], fmaf(k[i][d][2], qv[2], k[i][d][3] * qv[3])));
+                        x += e < p.dim ? y : 0.0f;
+                    }
+                    x += __shfl_xor(x, 1, 64);
+                    x += __shfl_xor(x, 2, 64);
+                    if (sub == 0 && there && h0 + h < rep) {
+                        if (p.bias) x -= slope_of(hh, p.heads) * (float)(int)(p.cached + s - j);
+                        lds[at.raw + hh * pitch + key] = key < keys ? x : 0.0f;
+                    }
                 }
             }
         }
-    }
-    __syncthreads();
-    for (uint32_t i = threadIdx.x; i < p.heads * seg_keys; i += kThreads) {
-        const uint32_t h = i / seg_keys, key = i - h * seg_keys;
-        float w = 0.0f;
-#pragma unroll 4
-        for (uint32_t g = 0; g < p.heads; g++) w = fmaf(lds[at.talk + h * p.heads + g], lds[at.raw + g * pitch + key], w);
-        lds[at.mixed + h * pitch + key] = key < keys ? w * kLog2e : -INFINITY;
-    }
-    __syncthreads();
-    for (uint32_t h = wave; h < p.heads; h += kThreads / 64) {
-        const float x = lane < seg_keys ? lds[at.mixed + h * pitch + lane] : -INFINITY;
-        const float m = fmaxf(kNone, wave_max(x)), e = __builtin_amdgcn_exp2f(x - m), l = wave_sum(e);
-        if (lane < seg_keys) lds[at.mixed + h * pitch + lane] = e;
-        if (lane == 0) stats[((int64_t)r * nseg + seg) * p.heads + h] = make_float2(m, l);
-    }
-    __syncthreads();
-    // values: a thread per four columns of a kv head's values, for its query heads
-    const uint32_t vec = p.vdim / 4;
-    for (uint32_t i = threadIdx.x; i < p.kv_heads * vec; i += kThreads) {
-        const uint32_t g = i / vec, d = (i - g * vec) * 4;
-        const float *V = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + d;
-        for (uint32_t h0 = 0; h0 < rep; h0 += REP) {
-            f32x4 acc[REP] = {};
-            auto add = [&](const f32x4 v, uint32_t k) {
-#pragma unroll
-                for (int h = 0; h < REP; h++) {
-                    if (h0 + h >= rep) break;
-                    const float w = lds[at.mixed + (g * rep + h0 + h) * pitch + k];
-#pragma unroll
-                    for (int e = 0; e < 4; e++) acc[h][e] = fmaf(w, v[e], acc[h][e]);
-                }
-            };
-            const uint32_t old = j0 >= p.cached ? 0 : min(keys, p.cached - j0); // the new ones come from the projections
+        if (j0 + chunk < end) ask_keys(j0 + chunk); // on their way meanwhile
+        __syncthreads();
+        for (uint32_t i = threadIdx.x; i < p.heads * chunk; i += kThreads) {
+            const uint32_t h = i / chunk, key = i - h * chunk;
+            float w = 0.0f;
 #pragma unroll 8
-            for (uint32_t k = 0; k < old; k++) add(*reinterpret_cast<const f32x4 *>(V + (int64_t)(j0 + k) * p.vdim), k);
-            for (uint32_t k = old; k < keys; k++) {
-                const float *src = p.v.p + ((int64_t)b * p.S + (j0 + k - p.cached)) * p.v.pitch + g * p.vdim + d;
-                add(f32x4{src[0], src[1], src[2], src[3]}, k);
+            for (uint32_t g = 0; g < p.heads; g++) w = fmaf(lds[at.talk + h * p.heads + g], lds[at.raw + g * pitch + key], w);
+            lds[at.mixed + h * pitch + key] = key < keys ? w * kLog2e : -INFINITY;
+        }
+        __syncthreads();
+        // (lanes side by side take a head each, a run of the chunk's keys every one)
+        for (uint32_t i = threadIdx.x; i < p.heads * 4; i += kThreads) {
+            const uint32_t h = i / 4;
+            float *x = lds + at.mixed + h * pitch;
+            const float top = lds[at.state + h];
+            float m = top, l = 0.0f;
+            for (uint32_t key = i % 4; key < chunk; key += 4) m = fmaxf(m, x[key]);
+            m = fmaxf(m, __shfl_xor(m, 1, 64));
+            m = fmaxf(m, __shfl_xor(m, 2, 64));
+            for (uint32_t key = i % 4; key < chunk; key += 4) {
+                const float e = __builtin_amdgcn_exp2f(x[key] - m);
+                x[key] = e;
+                l += e;
             }
-#pragma unroll
-            for (int h = 0; h < REP; h++) {
-                if (h0 + h >= rep) break;
-                *reinterpret_cast<f32x4 *>(parts + (((int64_t)r * nseg + seg) * p.heads + g * rep + h0 + h) * p.vdim + d) = acc[h];
+            l += __shfl_xor(l, 1, 64);
+            l += __shfl_xor(l, 2, 64);
+            if (i % 4 == 0) {
+                const float f = __builtin_amdgcn_exp2f(top - m);
+                lds[at.state + h] = m;
+                lds[at.state + p.heads + h] = fmaf(lds[at.state + p.heads + h], f, l);
+                lds[at.state + 2 * p.heads + h] = f;
             }
         }
+        __syncthreads();
+        // a thread's columns: results of this chunk for one kv head's query heads, REP at a time
+        auto weigh = [&](uint32_t c, uint32_t h0, f32x4(&o)[REP]) {
+            const uint32_t g = c / vec;
+#pragma unroll
+            for (uint32_t e = 0; e < kValuesAhead; e++) {
+                const uint32_t key = my_turn % turns + e * turns;
+                if (key >= keys) break;
+#pragma unroll
+                for (int h = 0; h < REP; h++) {
+                    const float w = lds[at.mixed + (g * rep + min(h0 + h, rep - 1)) * pitch + key];
+#pragma unroll
+                    for (int d = 0; d < 4; d++) o[h][d] = fmaf(w, v[e][d], o[h][d]);
+                }
+            }
+        };
+        if (has_values) {
+#pragma unroll
+            for (int h = 0; h < REP; h++) acc[h] *= lds[at.state + 2 * p.heads + (mine / vec) * rep + min((uint32_t)h, rep - 1)];
+            weigh(mine, 0, acc);
+        }
+        if (j0 + chunk < end) {
+            ask_values(j0 + chunk, mine);
+            __syncthreads();
+        }
+    }
+    __syncthreads();
+    for (uint32_t h = threadIdx.x; h < p.heads; h += kThreads) stats[((int64_t)r * nseg + seg) * p.heads + h] = make_float2(lds[at.state + h], lds[at.state + p.heads + h]);
+    float *dst = parts + ((int64_t)r * nseg + seg) * p.heads * p.vdim;
+    if (turns > 1) { // the turns' results meet in LDS, from the queries' place on, one turn after the other
+        for (uint32_t t = 0; t < turns; t++) {
+            __syncthreads();
+            if (my_turn == t) {
+#pragma unroll
+                for (int h = 0; h < REP; h++) {
+                    if (h >= (int)rep) break;
+                    f32x4 *o = reinterpret_cast<f32x4 *>(lds + at.q + ((mine / vec) * rep + h) * p.vdim + (mine % vec) * 4);
+                    *o = t ? *o + acc[h] : acc[h];
+                }
+            }
+        }
+        __syncthreads();
+        for (uint32_t i = threadIdx.x; i < p.heads * vec; i += kThreads) *reinterpret_cast<f32x4 *>(dst + 4 * i) = *reinterpret_cast<const f32x4 *>(lds + at.q + 4 * i);
+    } else if (has_values) {
+#pragma unroll
+        for (int h = 0; h < REP; h++)
+            if (h < (int)rep) *reinterpret_cast<f32x4 *>(dst + ((mine / vec) * rep + h) * p.vdim + (mine % vec) * 4) = acc[h];
     }
 }
 
@@ -538,7 +654,7 @@ void merge(cg_backend *be, const AttentionPlan &p, const float *parts, const flo
     const uint32_t n = p.heads * p.vdim;
     for (uint32_t r0 = 0; r0 < rows; r0 += 65535) {
         const uint32_t nr = std::min(rows - r0, 65535u);
-        hipLaunchKernelGGL(attention_merge_kernel, dim3((n + kThreads - 1) / kThreads, nr), dim3(kThreads), 0, be->stream, parts + (uint64_t)r0 * row_pitch * p.vdim,
+        hipLaunchKernelGGL(attention_merge_kernel, dim3((n + 63) / 64, nr), dim3(kMergeWaves * 64), 0, be->stream, parts + (uint64_t)r0 * row_pitch * p.vdim,
                            stats + (uint64_t)r0 * row_pitch, segs, row_pitch, seg_pitch, p.heads, p.vdim, p.zero_sink, out + (uint64_t)r0 * n);
     }
 }
@@ -564,7 +680,7 @@ template <int HPW> int run_tiles(cg_backend *be, const AttentionPlan &p, const f
     const uint32_t d = p.dim, v = p.vdim;
     if (d <= 32 && v <= 32) return run_tiles<HPW, 2, 2, true>(be, p, q, splits, dst, stats);
     if (d <= 64 && v <= 64) return run_tiles<HPW, 4, 4, true>(be, p, q, splits, dst, stats);
-    if (d <= 64 && v <= 96) return run_tiles<HPW, 4, 6, true>(be, p, q, splits, dst, stats);
+    if (d <= 64 && v <= 96) return run_tiles<HPW, 4, 6, (HPW < 4)>(be, p, q, splits, dst, stats);
     if (d <= 96 && v <= 96) return run_tiles<HPW, 6, 6, (HPW < 4)>(be, p, q, splits, dst, stats);
     return run_tiles<HPW, 8, 8, (HPW < 4)>(be, p, q, splits, dst, stats);
 }
@@ -601,30 +717,44 @@ int launch_mixed_tiles(cg_backend *be, const AttentionPlan &p, const float *q) {
     return launched("attention_mixed_tiles");
 }
 
+template <int REP, int DQ>
+static int step_kernels(cg_backend *be, const AttentionPlan &p, uint32_t chunk, uint32_t chunks, dim3 grid, size_t lds, float *parts, float2 *stats) {
+    constexpr int PI = 8 / DQ; // keys of four lanes: 8 pieces per lane
+    if (int rc = allow_lds(reinterpret_cast<const void *>(&attention_mixed_step_kernel<REP, DQ, PI>), lds)) return rc;
+    hipLaunchKernelGGL((attention_mixed_step_kernel<REP, DQ, PI>), grid, dim3(kThreads), lds, be->stream, p, chunk, chunks, parts, stats);
+    return CG_OK;
+}
+
 int launch_mixed_step(cg_backend *be, const AttentionPlan &p) {
-    const uint32_t rows = p.B * p.S, keys = p.cached + p.S, most = p.window ? std::min(p.window, keys) : keys, rep = p.heads / p.kv_heads;
-    if (p.S > kFewRows || p.dim % 4 || p.vdim % 4 || rows > 65535 || p.q_norm || p.k_norm) return kDeclined;
-    // segments that fill the device, of 8 to 64 keys
-    uint32_t seg = 8;
-    while (seg < kMaxStepKeys && (uint64_t)rows * ((most + seg - 1) / seg) > be->compute_units) seg *= 2;
-    const size_t lds = (size_t)step_lds(p.S, p.heads, p.kv_heads, p.dim, p.rot_dims, seg).total * 4;
+    const uint32_t rows = p.B * p.S, keys = p.cached + p.S, most = p.window ? std::min(p.window, keys) : keys, rep = p.heads / p.kv_heads, cols = p.kv_heads * p.vdim / 4;
+    auto aligned = [](const Rows &x) { return x.pitch % 4 == 0 && (reinterpret_cast<uintptr_t>(x.p) & 15) == 0; };
+    if (p.S > kFewRows || p.dim % 4 || p.vdim % 4 || rows > 65535 || p.q_norm || p.k_norm || rep > 8 || p.dim > 128 || cols > kThreads || !aligned(p.v)) return kDeclined;
+    // chunks whose keys and values a workgroup holds in registers
+    const uint32_t turns = std::max(1u, (uint32_t)kThreads / cols), dq = p.dim <= 32 ? 2 : p.dim <= 64 ? 4 : 8, pairs = kThreads / 4 * (8 / dq);
+    if (p.kv_heads > pairs) return kDeclined;
+    uint32_t chunk = kMaxChunk;
+    while (chunk * p.kv_heads > pairs || chunk > turns * kValuesAhead) chunk /= 2;
+    const size_t lds = (size_t)step_lds(p.S, p.heads, p.kv_heads, p.dim, p.rot_dims, chunk, p.vdim).total * 4;
     if (lds > kMaxLds / 2) return kDeclined;
-    const uint32_t nseg = (most + seg - 1) / seg;
+    // up to four workgroups per compute unit
+    const uint32_t all = (most + chunk - 1) / chunk;
+    const uint32_t chunks = (uint32_t)(((uint64_t)rows * all + 4 * be->compute_units - 1) / (4 * be->compute_units)), nseg = (all + chunks - 1) / chunks;
     Scratch mem(be);
     const size_t n = (size_t)rows * nseg * p.heads;
     if (int rc = mem.get(n * p.vdim * 4 + n * sizeof(float2))) return rc;
     float *parts = static_cast<float *>(mem.p);
     float2 *stats = reinterpret_cast<float2 *>(parts + n * p.vdim);
     const dim3 grid(nseg, rows);
-#define CG_STEP(R)                                                                                                                   \
-    {                                                                                                                                \
-        if (int rc = allow_lds(reinterpret_cast<const void *>(&attention_mixed_step_kernel<R>), lds)) return rc;                     \
-        hipLaunchKernelGGL((attention_mixed_step_kernel<R>), grid, dim3(kThreads), lds, be->stream, p, seg, parts, stats);            \
-    }
-    if (rep <= 1) CG_STEP(1)
-    else if (rep <= 2) CG_STEP(2)
-    else CG_STEP(4)
+    int rc;
+#define CG_STEP(R) (p.dim <= 32 ? step_kernels<R, 2>(be, p, chunk, chunks, grid, lds, parts, stats) \
+                    : p.dim <= 64 ? step_kernels<R, 4>(be, p, chunk, chunks, grid, lds, parts, stats) \
+                                  : step_kernels<R, 8>(be, p, chunk, chunks, grid, lds, parts, stats))
+    if (rep <= 1) rc = CG_STEP(1);
+    else if (rep <= 2) rc = CG_STEP(2);
+    else if (rep <= 4) rc = CG_STEP(4);
+    else rc = CG_STEP(8);
 #undef CG_STEP
+    if (rc) return rc;
     merge(be, p, parts, stats, nseg, (uint64_t)nseg * p.heads, p.heads, rows, p.out);
     return launched("attention_mixed_step");
 }

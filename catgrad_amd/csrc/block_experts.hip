@@ -36,16 +36,16 @@ __device__ __forceinline__ float activation(float g, float u, float limit, float
 
 // ---- the choice ------------------------------------------------------------------------------------------------------
 // Every score is ranked against those it competes with: first a group's members, then the groups, then the members of the
-// groups that count.  LDS: route_floats(experts, groups) floats.  N threads, all of them; `chosen` and `weight` (LDS) are
-// there after the last barrier.
+// groups that count.  LDS: route_floats(experts, groups) floats.  Thread t of N; `chosen` and `weight` (LDS) are there after
+// the last barrier, which is the whole workgroup's.
 __host__ __device__ constexpr uint32_t route_floats(uint32_t experts, uint32_t groups) { return 2 * experts + 3 * groups; }
 __device__ __forceinline__ bool beats(float a, uint32_t i, float b, uint32_t j) { return a > b || (a == b && i < j); }
 
 template <int N>
-__device__ void choose_experts(const ExpertsPlan &p, uint32_t row, float *lds, uint32_t *chosen, float *weight) {
+__device__ void choose_experts(const ExpertsPlan &p, uint32_t row, float *lds, uint32_t *chosen, float *weight, const uint32_t t) {
     float *choice = lds, *own = lds + p.experts, *worth = own + p.experts; // worth: [groups][2], then [groups] whether it counts
     float *counts = worth + 2 * p.groups;
-    const uint32_t size = p.experts / p.groups, t = threadIdx.x;
+    const uint32_t size = p.experts / p.groups;
     for (uint32_t e = t; e < p.experts; e += N) {
         const float s = sigmoid(p.logits[(int64_t)row * p.experts + e]);
         own[e] = s;
@@ -159,7 +159,7 @@ __global__ __launch_bounds__(kThreads) void expert_first_kernel(const ExpertsPla
     };
 #pragma unroll
     for (int s = 0; s < STEPS; s++) take(s * SPAN + lane * W, x[s]);
-    choose_experts<kThreads>(p, row, lds, chosen, weight);
+    choose_experts<kThreads>(p, row, lds, chosen, weight, threadIdx.x);
     const uint32_t e = chosen[slot];
     const float weigh = weight[slot];
     if (blockIdx.x == 0 && threadIdx.x == 0) chosen_out[blockIdx.y] = e;
@@ -198,42 +198,52 @@ __global__ __launch_bounds__(kThreads) void expert_first_kernel(const ExpertsPla
     }
 }
 
-// A wave per output column and row block: out = x + scale * (y . w^T + sum over the choices), or without w the choices' sum alone per slot.
-template <bool BF16, bool VEC>
+// A wave per NC output columns of a row: out = x + scale * (y . w^T + sum over the choices).  The choices' rows and w's are
+// walked as one run of pieces (64 lanes' worth), AHEAD of them in flight.
+template <bool BF16, bool VEC, int NC>
 __global__ __launch_bounds__(kThreads) void expert_second_kernel(const ExpertsPlan p, const float *__restrict__ hidden, const uint32_t *__restrict__ chosen, const Rows x,
                                                                  const Rows y, const Weight w, const float scale, float *__restrict__ out) {
     typedef Streamed<BF16, VEC> St;
     constexpr uint32_t W = St::W, SPAN = 64 * W, EB = BF16 ? 2 : 4;
-    const uint32_t lane = threadIdx.x & 63, n = blockIdx.x * kWaves + (threadIdx.x >> 6), row = blockIdx.y;
-    if (n >= p.width) return;
-    const float xs = x.p[(int64_t)row * x.pitch + n];
-    float a = 0.0f;
-    for (uint32_t slot = 0; slot < p.top; slot++) {
-        const uint64_t at = (uint64_t)row * p.top + slot;
-        const char *d = static_cast<const char *>(p.down) + ((uint64_t)chosen[at] * p.width + n) * p.ff * EB;
-#pragma unroll 2
-        for (uint32_t k = lane * W; k < p.ff; k += SPAN) {
-            St s;
-            s.load(d, k);
-            float v[W];
-            St::input(hidden + at * p.ff, k, v);
-            a = s.dot(v, a);
-        }
+    constexpr int AHEAD = 4;
+    const uint32_t lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), row = blockIdx.y;
+    const uint32_t n0 = (blockIdx.x * kWaves + wave) * NC;
+    if (n0 >= p.width) return;
+    const uint32_t steps = (p.ff + SPAN - 1) / SPAN, wsteps = w.p ? (w.k + SPAN - 1) / SPAN : 0, total = p.top * steps + wsteps;
+    float xs[NC], a[NC];
+#pragma unroll
+    for (int c = 0; c < NC; c++) {
+        xs[c] = x.p[(int64_t)row * x.pitch + min(n0 + c, p.width - 1)];
+        a[c] = 0.0f;
     }
-    if (w.p) {
-        const char *d = static_cast<const char *>(w.p) + (uint64_t)n * w.pitch * EB;
-        const float *yr = y.p + (int64_t)row * y.pitch;
-#pragma unroll 4
-        for (uint32_t k = lane * W; k < w.k; k += SPAN) {
-            St s;
-            s.load(d, k);
-            float v[W];
-            St::input(yr, k, v);
-            a = s.dot(v, a);
+    const float *yr = y.p + (int64_t)row * y.pitch, *hr = hidden + (uint64_t)row * p.top * p.ff;
+    for (uint32_t i0 = 0; i0 < total; i0 += AHEAD) {
+        St s[AHEAD][NC];
+        float v[AHEAD][W];
+#pragma unroll
+        for (int e = 0; e < AHEAD; e++) { // (pieces behind the last, and lanes behind a row's end: clamped, and times zero)
+            const uint32_t i = min(i0 + e, total - 1), slot = i / steps;
+            const bool first = i < p.top * steps;
+            const uint32_t k0 = (first ? i - slot * steps : i - p.top * steps) * SPAN + lane * W, K = first ? p.ff : w.k, k = min(k0, K - W);
+            const char *d = first ? static_cast<const char *>(p.down) + (uint64_t)chosen[(uint64_t)row * p.top + slot] * p.width * p.ff * EB : static_cast<const char *>(w.p);
+            const uint64_t pitch = first ? p.ff : (uint64_t)w.pitch;
+#pragma unroll
+            for (int c = 0; c < NC; c++) s[e][c].load(d + min(n0 + c, p.width - 1) * pitch * EB, k);
+            St::input(first ? hr + slot * p.ff : yr, k, v[e]);
+            const bool there = i0 + e < total && k0 < K;
+#pragma unroll
+            for (uint32_t j = 0; j < W; j++) v[e][j] = there ? v[e][j] : 0.0f;
         }
+#pragma unroll
+        for (int e = 0; e < AHEAD; e++)
+#pragma unroll
+            for (int c = 0; c < NC; c++) a[c] = s[e][c].dot(v[e], a[c]);
     }
-    a = wave_sum(a);
-    if (lane == 0) out[(uint64_t)row * p.width + n] = xs + scale * a;
+#pragma unroll
+    for (int c = 0; c < NC; c++) {
+        const float sum = wave_sum(a[c]);
+        if (lane == 0 && n0 + c < p.width) out[(uint64_t)row * p.width + n0 + c] = fmaf(scale, sum, xs[c]);
+    }
 }
 
 // the same for one (row, choice) at a time, of any number: y[row * top + slot, n]
@@ -263,16 +273,34 @@ __global__ __launch_bounds__(kThreads) void expert_second_slots_kernel(const Exp
 struct Routed {
     uint32_t expert, place;
 };
-__global__ __launch_bounds__(64) void route_kernel(const ExpertsPlan p, Routed *__restrict__ routed, float *__restrict__ weights, uint32_t *__restrict__ count) {
+// A workgroup takes kRouteRows tokens, a wave one at a time, and its places in the experts' lists in one go.
+constexpr uint32_t kRouteRows = 32;
+__host__ __device__ constexpr uint32_t route_wave_floats(const ExpertsPlan &p) { return route_floats(p.experts, p.groups) + 2 * p.top; }
+__global__ __launch_bounds__(kThreads) void route_kernel(const ExpertsPlan p, Routed *__restrict__ routed, float *__restrict__ weights, uint32_t *__restrict__ count) {
     extern __shared__ float lds[];
-    uint32_t *chosen = reinterpret_cast<uint32_t *>(lds + route_floats(p.experts, p.groups));
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r0 = blockIdx.x * kRouteRows, n = min(kRouteRows, p.rows - r0);
+    float *mine = lds + wave * route_wave_floats(p);
+    uint32_t *chosen = reinterpret_cast<uint32_t *>(mine + route_floats(p.experts, p.groups));
     float *weight = reinterpret_cast<float *>(chosen + p.top);
-    choose_experts<64>(p, blockIdx.x, lds, chosen, weight);
-    for (uint32_t i = threadIdx.x; i < p.top; i += 64) {
-        const uint64_t at = (uint64_t)blockIdx.x * p.top + i;
-        const uint32_t e = chosen[i];
-        routed[at] = {e, atomicAdd(count + e, 1u)};
-        weights[at] = weight[i];
+    uint32_t *seen = reinterpret_cast<uint32_t *>(lds + kWaves * route_wave_floats(p)), *base = seen + p.experts, *place = base + p.experts, *whose = place + kRouteRows * p.top; // [kRouteRows][top]
+    for (uint32_t e = threadIdx.x; e < p.experts; e += kThreads) seen[e] = 0;
+    __syncthreads();
+    for (uint32_t i = wave; i < kRouteRows; i += kWaves) { // (the same trips for every wave: the choice has barriers)
+        const uint32_t row = r0 + min(i, n - 1);
+        choose_experts<64>(p, row, mine, chosen, weight, lane);
+        if (i < n)
+            for (uint32_t t = lane; t < p.top; t += 64) {
+                const uint64_t at = (uint64_t)row * p.top + t;
+                weights[at] = weight[t];
+                whose[i * p.top + t] = chosen[t];
+                place[i * p.top + t] = atomicAdd(seen + chosen[t], 1u);
+            }
+        __syncthreads();
+    }
+    for (uint32_t e = threadIdx.x; e < p.experts; e += kThreads) base[e] = seen[e] ? atomicAdd(count + e, seen[e]) : 0;
+    __syncthreads();
+    for (uint32_t i = threadIdx.x; i < n * p.top; i += kThreads) {
+        routed[(uint64_t)r0 * p.top + i] = {whose[i], base[whose[i]] + place[i]};
     }
 }
 __global__ __launch_bounds__(kThreads) void clear_kernel(uint32_t *p, uint32_t n) {
@@ -312,7 +340,7 @@ __global__ __launch_bounds__(kThreads) void route_lists_kernel(const uint32_t ex
     }
 }
 
-constexpr uint32_t kTileN = 128, kStages = 4;
+constexpr uint32_t kTileN = 128, kStages = 4, kXcds = 8, kGroupM = 8;
 typedef float float16v __attribute__((ext_vector_type(16)));
 typedef float float4v __attribute__((ext_vector_type(4)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -323,7 +351,7 @@ struct ExpertTileArgs {
     const uint32_t *list;
     const uint4 *tiles;
     const float *weights;     // FIRST: per choice
-    void *out;                // FIRST: hidden [place in the list, ff], in the form of x; else f32 [choice, N]
+    void *out;                // FIRST: hidden [place in the list, ff], else [choice, N]; in the form of x
     uint32_t N, K;            // FIRST: N = ff
     uint32_t top, tiles_n;
     float limit, slope;
@@ -340,7 +368,11 @@ template <bool BF16, bool FIRST, int MT> __global__ __launch_bounds__(kThreads) 
     extern __shared__ float lds_dyn[];
     typedef __attribute__((address_space(3))) char lds_char;
     lds_char *const lds = (lds_char *)lds_dyn;
-    const uint32_t tile = blockIdx.x / a.tiles_n, n0 = (blockIdx.x - tile * a.tiles_n) * OUT_N;
+    // a run of tiles per XCD, down a column of kGroupM row tiles (mostly one expert's) first
+    const uint32_t ntiles = gridDim.x, xcd = blockIdx.x % kXcds, q8 = ntiles / kXcds, r8 = ntiles % kXcds, tiles_m = ntiles / a.tiles_n;
+    const uint32_t lin = xcd * q8 + min(xcd, r8) + blockIdx.x / kXcds, group = lin / (kGroupM * a.tiles_n), in_group = lin % (kGroupM * a.tiles_n);
+    const uint32_t gsize = min(tiles_m - group * kGroupM, kGroupM);
+    const uint32_t tile = group * kGroupM + in_group % gsize, n0 = in_group / gsize * OUT_N;
     const uint4 job = a.tiles[tile];
     const uint32_t m = job.z, nk = (a.K + STAGE_K - 1) / STAGE_K;
     if (m == 0) return;
@@ -435,7 +467,9 @@ template <bool BF16, bool FIRST, int MT> __global__ __launch_bounds__(kThreads) 
 #pragma unroll
                 for (int j = 0; j < 2; j++) {
                     const uint32_t n = n0 + wn + j * 32 + li;
-                    if (n < a.N) static_cast<float *>(a.out)[(uint64_t)choice * a.N + n] = acc[i][j][v];
+                    if (n >= a.N) continue;
+                    if constexpr (BF16) static_cast<uint16_t *>(a.out)[(uint64_t)choice * a.N + n] = (uint16_t)(round_bf16(acc[i][j][v]) >> 16);
+                    else static_cast<float *>(a.out)[(uint64_t)choice * a.N + n] = acc[i][j][v];
                 }
             }
         }
@@ -459,6 +493,7 @@ struct Scratch {
 };
 
 size_t route_bytes(const ExpertsPlan &p) { return (route_floats(p.experts, p.groups) + 2 * (size_t)p.top) * 4; }
+size_t many_route_bytes(const ExpertsPlan &p) { return (kWaves * (size_t)route_wave_floats(p) + 2 * (size_t)p.experts + 2 * (size_t)kRouteRows * p.top) * 4; }
 bool vector_rows(const ExpertsPlan &p) {
     const uint32_t vw = p.fmt == kFmtBF16 ? 8 : 4;
     return p.width % vw == 0 && p.ff % vw == 0 && aligned16(p.gate_up) && aligned16(p.down) && aligned16(p.h);
@@ -520,21 +555,28 @@ int launch_experts_second(cg_backend *be, const ExpertsPlan &p, const float *hid
         vec = vec && w->k % vw == 0 && w->pitch % vw == 0 && aligned16(w->p) && y.pitch % 4 == 0 && aligned16(y.p);
     }
     ProfScope prof(be, CG_K_GEMM_SKINNY, first_bytes(p, p.rows * p.top) / 2 + (w ? (double)w->n * w->k * (bf16 ? 2.0 : 4.0) : 0.0));
-    const dim3 grid((p.width + kWaves - 1) / kWaves, p.rows);
-#define CG_SECOND(BF, VE) hipLaunchKernelGGL((expert_second_kernel<BF, VE>), grid, dim3(kThreads), 0, be->stream, p, hidden, chosen, x, y, w ? *w : none, scale, out)
-    if (bf16 && vec) CG_SECOND(true, true);
-    else if (bf16) CG_SECOND(true, false);
-    else if (vec) CG_SECOND(false, true);
-    else CG_SECOND(false, false);
+    const bool two = vec && (uint64_t)p.rows * p.width >= 16ull * be->compute_units; // columns of a wave
+    const uint32_t per = kWaves * (two ? 2 : 1);
+    const dim3 grid((p.width + per - 1) / per, p.rows);
+#define CG_SECOND(BF, VE)                                                                                                                                            \
+    {                                                                                                                                                                \
+        if (two) hipLaunchKernelGGL((expert_second_kernel<BF, VE, VE ? 2 : 1>), grid, dim3(kThreads), 0, be->stream, p, hidden, chosen, x, y, w ? *w : none, scale, out); \
+        else hipLaunchKernelGGL((expert_second_kernel<BF, VE, 1>), grid, dim3(kThreads), 0, be->stream, p, hidden, chosen, x, y, w ? *w : none, scale, out);           \
+    }
+    if (bf16 && vec) CG_SECOND(true, true)
+    else if (bf16) CG_SECOND(true, false)
+    else if (vec) CG_SECOND(false, true)
+    else CG_SECOND(false, false)
 #undef CG_SECOND
     return launched("expert_second");
 }
 
-int launch_experts(cg_backend *be, const ExpertsPlan &p, float *y) {
+int launch_experts(cg_backend *be, const ExpertsPlan &p, float *y, int *y_fmt) {
+    *y_fmt = kFmtWords;
     const bool bf16 = p.fmt == kFmtBF16, vec = vector_rows(p);
     const uint64_t n = (uint64_t)p.rows * p.top;
-    if (n > 0x7FFFFFFFull || p.experts > 4096 || route_bytes(p) > (64u << 10)) return fail(CG_ERR_UNSUPPORTED, "experts: more than the kernels hold");
-    const bool tiled = vec && (p.h_fmt == kFmtBF16) == bf16 && aligned16(p.h);
+    if (n > 0x7FFFFFFFull || p.experts > 4096) return fail(CG_ERR_UNSUPPORTED, "experts: more than the kernels hold");
+    const bool tiled = vec && many_route_bytes(p) <= (64u << 10) && (p.h_fmt == kFmtBF16) == bf16 && aligned16(p.h);
     if (!tiled) { // shapes that do not lie in 16-byte pieces: every choice on its own
         Scratch hid(be), ch(be);
         if (int rc = hid.get(n * p.ff * 4)) return rc;
@@ -554,6 +596,7 @@ int launch_experts(cg_backend *be, const ExpertsPlan &p, float *y) {
         }
         return launched("expert_slots");
     }
+    *y_fmt = bf16 ? kFmtBF16 : kFmtWords;
     // lists
     const bool low = n <= 64ull * p.experts; // few rows per expert: short tiles
     const uint32_t tm = low ? 64 : 128, max_tiles = (uint32_t)(n / tm + std::min<uint64_t>(p.experts, n));
@@ -568,7 +611,7 @@ int launch_experts(cg_backend *be, const ExpertsPlan &p, float *y) {
     {
         ProfScope prof(be, CG_K_GATHER, 4.0 * p.rows * p.experts + 20.0 * n);
         hipLaunchKernelGGL(clear_kernel, dim3((p.experts + kThreads - 1) / kThreads), dim3(kThreads), 0, be->stream, count, p.experts);
-        hipLaunchKernelGGL(route_kernel, dim3(p.rows), dim3(64), route_bytes(p), be->stream, p, routed, weights, count);
+        hipLaunchKernelGGL(route_kernel, dim3((p.rows + kRouteRows - 1) / kRouteRows), dim3(kThreads), many_route_bytes(p), be->stream, p, routed, weights, count);
         hipLaunchKernelGGL(route_lists_kernel, dim3((uint32_t)((n + kThreads - 1) / kThreads)), dim3(kThreads), (size_t)(p.experts + 1) * 8, be->stream, p.experts, (uint32_t)n, tm,
                            max_tiles, routed, count, list, tiles);
         if (int rc = launched("route")) return rc;

@@ -608,8 +608,9 @@ struct GatedSumArgs {
     int n;
     uint32_t width;
     float scale;
-    const float *extra; // [rows, slots, width]
+    const void *extra; // [rows, slots, width]
     uint32_t slots;
+    int extra_fmt;
 };
 template <int VW> __global__ __launch_bounds__(kThreads) void gated_sum_kernel(const GatedSumArgs a, float *__restrict__ out) {
     const uint32_t k = (blockIdx.x * kThreads + threadIdx.x) * VW, r = blockIdx.y;
@@ -636,7 +637,18 @@ template <int VW> __global__ __launch_bounds__(kThreads) void gated_sum_kernel(c
     if (a.extra) {
 #pragma unroll 4
         for (uint32_t i = 0; i < a.slots; i++) {
-            load(a.extra + ((int64_t)r * a.slots + i) * a.width + k, y);
+            const int64_t at = ((int64_t)r * a.slots + i) * a.width + k;
+            if (a.extra_fmt == kFmtBF16) {
+                const uint16_t *e = static_cast<const uint16_t *>(a.extra) + at;
+                if constexpr (VW == 4) {
+                    const uint2 t = *reinterpret_cast<const uint2 *>(e);
+                    y[0] = bf16_lo(t.x), y[1] = bf16_hi(t.x), y[2] = bf16_lo(t.y), y[3] = bf16_hi(t.y);
+                } else {
+                    y[0] = asf((uint32_t)*e << 16);
+                }
+            } else {
+                load(static_cast<const float *>(a.extra) + at, y);
+            }
 #pragma unroll
             for (int j = 0; j < VW; j++) s[j] += y[j];
         }
@@ -845,20 +857,21 @@ int launch_affine_rows(cg_backend *be, float *y, uint32_t rows, uint32_t n, cons
     return launched("affine_rows");
 }
 
-int launch_gated_sum(cg_backend *be, const Rows &x, const GatedTerm *t, int n, uint32_t rows, uint32_t width, float *out, float scale, const float *extra,
-                     uint32_t slots) {
+int launch_gated_sum(cg_backend *be, const Rows &x, const GatedTerm *t, int n, uint32_t rows, uint32_t width, float *out, float scale, const void *extra,
+                     uint32_t slots, int extra_fmt) {
     bool vec = width % 4 == 0 && x.pitch % 4 == 0 && aligned16(x.p) && aligned16(out) && aligned16(extra);
     for (int i = 0; i < n; i++) vec = vec && (!t[i].gate.p || (t[i].gate.pitch % 4 == 0 && aligned16(t[i].gate.p))) && aligned16(t[i].y);
     for (uint32_t r0 = 0; r0 < rows; r0 += 65535) {
         const uint32_t nr = rows - r0 < 65535 ? rows - r0 : 65535;
-        ProfScope prof(be, CG_K_ELEMENTWISE, (2.0 + 2.0 * n + (extra ? slots : 0)) * 4.0 * nr * width);
+        ProfScope prof(be, CG_K_ELEMENTWISE, (2.0 + 2.0 * n + (extra ? (extra_fmt == kFmtBF16 ? 0.5 : 1.0) * slots : 0.0)) * 4.0 * nr * width);
         GatedSumArgs a{};
         a.x = {x.p + (int64_t)r0 * x.pitch, x.pitch};
         a.n = n;
         a.width = width;
         a.scale = scale;
-        a.extra = extra ? extra + (int64_t)r0 * slots * width : nullptr;
+        a.extra = extra ? static_cast<const char *>(extra) + (int64_t)r0 * slots * width * (extra_fmt == kFmtBF16 ? 2 : 4) : nullptr;
         a.slots = slots;
+        a.extra_fmt = extra_fmt;
         for (int i = 0; i < n; i++) {
             a.t[i] = t[i];
             a.t[i].y += (int64_t)r0 * width;

@@ -728,11 +728,12 @@ int cg_block_residual(cg_backend *b, cg_tensor *x, const cg_branch *br, size_t n
                 t[i].gate_bias = r[i].gate_bias;
             }
             void *p = nullptr;
+            int fmt = kFmtWords;
             if (experts && !rc) {
                 rc = tmp.get((size_t)rows * ep.top * width * 4, &p);
-                if (!rc) rc = launch_experts(b, ep, static_cast<float *>(p));
+                if (!rc) rc = launch_experts(b, ep, static_cast<float *>(p), &fmt);
             }
-            if (!rc) rc = launch_gated_sum(b, xr, t, (int)n, (uint32_t)rows, (uint32_t)width, y, scale, static_cast<const float *>(p), ep.top);
+            if (!rc) rc = launch_gated_sum(b, xr, t, (int)n, (uint32_t)rows, (uint32_t)width, y, scale, p, ep.top, fmt);
         }
     }
     if (rc) {

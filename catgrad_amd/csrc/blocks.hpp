@@ -65,9 +65,9 @@ struct GatedTerm {
     Rows gate;
     const float *gate_bias = nullptr;
 };
-// extra: [rows, slots, width] more terms, added up (null: none); out = x + scale * (all terms)
+// extra: [rows, slots, width] more terms in words or bfloat16 patterns, added up (null: none); out = x + scale * (all terms)
 int launch_gated_sum(cg_backend *be, const Rows &x, const GatedTerm *t, int n, uint32_t rows, uint32_t width, float *out, float scale = 1.0f,
-                     const float *extra = nullptr, uint32_t slots = 0);
+                     const void *extra = nullptr, uint32_t slots = 0, int extra_fmt = kFmtWords);
 
 // ---- embeddings, grouped norms with filters, the tokens' own vectors ---------------------------------------------------
 // A table's rows in 32-bit words or bfloat16 patterns.
@@ -122,8 +122,8 @@ struct ExpertsPlan {
     const void *gate_up, *down;       // [experts, 2, ff, width], [experts, width, ff], dense
     int fmt;                          // of the weights
 };
-// y[r, slot, 0 .. width) = weight * expert of row r's slot-th choice, for any number of rows
-int launch_experts(cg_backend *be, const ExpertsPlan &p, float *y);
+// y[r, slot, 0 .. width) = weight * expert of row r's slot-th choice, for any number of rows; words or bfloat16 patterns
+int launch_experts(cg_backend *be, const ExpertsPlan &p, float *y, int *y_fmt);
 // A few rows: hidden[r, slot, 0 .. ff) (weights applied) and the chosen experts' numbers.
 int launch_experts_first(cg_backend *be, const ExpertsPlan &p, float *hidden, uint32_t *chosen);
 // out[r] = x[r] + scale * (y[r] . w^T + sum_slot hidden[r, slot] . down[chosen[r, slot]]^T), rows <= kFewRows
