@@ -73,6 +73,15 @@ __global__ __launch_bounds__(kThreads) void attention_prepare_kernel(const Atten
     }
 }
 
+// Rows of a rotation's table: {cos, sin} of the positions first, first + step, ...
+__global__ __launch_bounds__(kThreads) void rotation_table_kernel(float2 *__restrict__ t, const uint32_t rows, const uint32_t step, const uint32_t dims, const double log2_base) {
+    const uint32_t i = blockIdx.x * kThreads + threadIdx.x, pairs = dims / 2;
+    if (i >= rows * pairs) return;
+    double a = (double)((uint64_t)(i / pairs) * step) * exp2(-2.0 * (double)(i % pairs) / (double)dims * log2_base);
+    a -= 6.283185307179586 * rint(a * 0.15915494309189535);
+    t[i] = make_float2((float)cos(a), (float)sin(a));
+}
+
 // The same with every head turned by its token's angles and brought to a mean square of one, a wave per head.
 __global__ __launch_bounds__(kThreads) void attention_turn_kernel(const AttentionPlan p, float *__restrict__ q) {
     extern __shared__ float2 turn[]; // {cos, sin} per pair
@@ -80,13 +89,7 @@ __global__ __launch_bounds__(kThreads) void attention_turn_kernel(const Attentio
     const uint32_t r = blockIdx.x, b = r / p.S, s = r - b * p.S, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const uint32_t nq = p.heads * p.dim, nk = p.kv_heads * p.dim, nv = p.kv_heads * p.vdim;
     const float *qr = p.q.p + (int64_t)r * p.q.pitch, *kr = p.k.p + (int64_t)r * p.k.pitch, *vr = p.v.p + (int64_t)r * p.v.pitch;
-    for (uint32_t i = threadIdx.x; i < p.rot_dims / 2; i += kThreads) {
-        double a = (double)(p.position + s) * exp2(-2.0 * (double)i / (double)p.rot_dims * p.rot_log2);
-        a -= 6.283185307179586 * rint(a * 0.15915494309189535);
-        float sn, cs;
-        sincosf((float)a, &sn, &cs);
-        turn[i] = make_float2(cs, sn);
-    }
+    for (uint32_t i = threadIdx.x; i < p.rot_dims / 2; i += kThreads) turn[i] = rotation_at(p, p.position + s, i);
     float mq = 0.0f, mk = 0.0f;
     if (p.q_norm)
         for (uint32_t i = threadIdx.x; i < nq; i += kThreads) mq = fmaf(qr[i], qr[i], mq);
@@ -125,6 +128,49 @@ __global__ __launch_bounds__(kThreads) void attention_turn_kernel(const Attentio
     for (uint32_t i = threadIdx.x; i < nv; i += kThreads) {
         const uint32_t g = i / p.vdim, d = i - g * p.vdim;
         vc[(int64_t)g * p.v_block + d] = vr[i];
+    }
+}
+
+// The same for heads of 4 * LANES values or fewer (a multiple of 4) without norms over whole projections: LANES lanes share a
+// head, 64 / LANES heads a wave at a time, all of a workgroup's tokens' heads in turn.
+template <int LANES> __global__ __launch_bounds__(kThreads) void attention_turn_heads_kernel(const AttentionPlan p, float *__restrict__ q) {
+    const uint32_t sub = threadIdx.x % LANES, r = blockIdx.x, b = r / p.S, s = r - b * p.S, d = min(sub * 4, p.dim - 4);
+    const bool there = sub * 4 < p.dim;
+    float2 t0 = make_float2(1.0f, 0.0f), t1 = t0;
+    if (sub * 4 < p.rot_dims) t0 = rotation_at(p, p.position + s, sub * 2);
+    if (sub * 4 + 2 < p.rot_dims) t1 = rotation_at(p, p.position + s, sub * 2 + 1);
+    float temp = p.scale;
+    if (p.temp_every) temp *= 1.0f + p.temp_coef * logf((float)((p.position + s + 1) / p.temp_every + 1));
+    const uint32_t heads = p.heads + p.kv_heads;
+#pragma unroll 2
+    for (uint32_t h0 = 0; h0 < heads; h0 += kThreads / LANES) { // (the same trips for every lane: the sums are over lanes)
+        const uint32_t h = min(h0 + threadIdx.x / LANES, heads - 1), g = h - p.heads;
+        const bool key = h >= p.heads;
+        const float4 v = *reinterpret_cast<const float4 *>((key ? p.k.p + (int64_t)r * p.k.pitch + g * p.dim : p.q.p + (int64_t)r * p.q.pitch + h * p.dim) + d);
+        float4 x = make_float4(fmaf(v.x, t0.x, -v.y * t0.y), fmaf(v.y, t0.x, v.x * t0.y), fmaf(v.z, t1.x, -v.w * t1.y), fmaf(v.w, t1.x, v.z * t1.y));
+        float c = key ? 1.0f : temp;
+        if (p.unit_heads) {
+            float m = there ? fmaf(x.x, x.x, fmaf(x.y, x.y, fmaf(x.z, x.z, x.w * x.w))) : 0.0f;
+#pragma unroll
+            for (int e = 1; e < LANES; e <<= 1) m += __shfl_xor(m, e, 64);
+            c /= sqrtf(m / (float)p.dim + p.eps);
+        }
+        if (!there || h0 + threadIdx.x / LANES >= heads) continue;
+        float *dst = key ? p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)(p.cached + s) * p.dim : q + ((int64_t)r * p.heads + h) * p.dim;
+        *reinterpret_cast<float4 *>(dst + d) = make_float4(x.x * c, x.y * c, x.z * c, x.w * c);
+    }
+    float *vc = p.values + (int64_t)b * p.kv_heads * p.v_block + (int64_t)(p.cached + s) * p.vdim;
+    const float *vr = p.v.p + (int64_t)r * p.v.pitch;
+    if (p.vdim % 4 == 0 && p.v.pitch % 4 == 0 && (reinterpret_cast<uintptr_t>(p.v.p) & 15) == 0) {
+        for (uint32_t i = threadIdx.x; i < p.kv_heads * p.vdim / 4; i += kThreads) {
+            const uint32_t g = i * 4 / p.vdim, e = i * 4 - g * p.vdim;
+            *reinterpret_cast<float4 *>(vc + (int64_t)g * p.v_block + e) = *reinterpret_cast<const float4 *>(vr + 4 * i);
+        }
+    } else {
+        for (uint32_t i = threadIdx.x; i < p.kv_heads * p.vdim; i += kThreads) {
+            const uint32_t g = i / p.vdim, e = i - g * p.vdim;
+            vc[(int64_t)g * p.v_block + e] = vr[i];
+        }
     }
 }
 
@@ -412,7 +458,58 @@ int rows_kernels(cg_backend *be, const AttentionPlan &p, const float *q, uint32_
 
 } // namespace
 
-int launch_attention(cg_backend *be, const AttentionPlan &p) {
+// The tables of a plan's rotation, for the positions before `end`: made when a model first asks for them, the coarse one in
+// powers of two.
+static int rotation_tables(cg_backend *be, AttentionPlan &p, uint64_t end) {
+    const uint32_t pairs = p.rot_dims / 2;
+    RotTable *t = nullptr;
+    for (RotTable &r : be->rot_tables)
+        if (r.dims == p.rot_dims && r.log2_base == p.rot_log2) t = &r;
+    auto fill = [&](uint32_t rows, uint32_t step, Buffer **out) {
+        Buffer *b = new Buffer;
+        b->be = be;
+        b->elems = (int64_t)rows * pairs * 2;
+        if (int rc = be->pool.alloc((size_t)b->elems * 4, &b->ptr, &b->cls)) {
+            delete b;
+            return rc;
+        }
+        hipLaunchKernelGGL(rotation_table_kernel, dim3((rows * pairs + kThreads - 1) / kThreads), dim3(kThreads), 0, be->stream, static_cast<float2 *>(b->ptr), rows, step,
+                           p.rot_dims, p.rot_log2);
+        *out = b;
+        return launched("rotation_table");
+    };
+    const uint64_t need = (end + kRotFine - 1) / kRotFine;
+    if (need > (1u << 24) / std::max(1u, pairs)) return fail(CG_ERR_UNSUPPORTED, "block_attention: a position beyond the rotation's tables");
+    if (!t) {
+        RotTable r{p.rot_dims, p.rot_log2, nullptr, nullptr, 0};
+        if (int rc = fill(kRotFine, 1, &r.fine)) return rc;
+        uint32_t n = 16;
+        while (n < need) n *= 2;
+        if (int rc = fill(n, kRotFine, &r.coarse)) {
+            buffer_release(r.fine);
+            return rc;
+        }
+        r.coarse_n = n;
+        be->rot_tables.push_back(r);
+        t = &be->rot_tables.back();
+    } else if (need > t->coarse_n) {
+        uint32_t n = t->coarse_n;
+        while (n < need) n *= 2;
+        Buffer *b = nullptr;
+        if (int rc = fill(n, kRotFine, &b)) return rc;
+        buffer_release(t->coarse); // (stream-ordered)
+        t->coarse = b;
+        t->coarse_n = n;
+    }
+    p.rot_fine = static_cast<const float2 *>(t->fine->ptr);
+    p.rot_coarse = static_cast<const float2 *>(t->coarse->ptr);
+    return CG_OK;
+}
+
+int launch_attention(cg_backend *be, const AttentionPlan &plan) {
+    AttentionPlan p = plan;
+    if (p.rot_dims)
+        if (int rc = rotation_tables(be, p, p.position + p.S)) return rc;
     const uint32_t rows = p.B * p.S, all = p.cached + p.S;
     const bool turned = p.rot_dims || p.unit_heads, fresh = p.S <= kFewRows && p.dim <= 512 && !turned;
     const uint32_t most = p.window ? std::min(p.window, all) : all, nseg = (most + kSeg - 1) / kSeg, rep = p.heads / p.kv_heads;
@@ -426,7 +523,13 @@ int launch_attention(cg_backend *be, const AttentionPlan &p) {
     if (!fresh) {
         if (int rc = qbuf.get((size_t)rows * p.heads * p.dim * 4)) return rc;
         q = static_cast<float *>(qbuf.p);
-        if (turned) hipLaunchKernelGGL(attention_turn_kernel, dim3(rows), dim3(kThreads), (size_t)(p.rot_dims / 2) * sizeof(float2), be->stream, p, q);
+        auto aligned = [](const Rows &x) { return x.pitch % 4 == 0 && (reinterpret_cast<uintptr_t>(x.p) & 15) == 0; };
+        const bool pieces = turned && !p.q_norm && !p.k_norm && p.dim % 4 == 0 && p.dim <= 256 && aligned(p.q) && aligned(p.k);
+        if (pieces && p.dim <= 32) hipLaunchKernelGGL((attention_turn_heads_kernel<8>), dim3(rows), dim3(kThreads), 0, be->stream, p, q);
+        else if (pieces && p.dim <= 64) hipLaunchKernelGGL((attention_turn_heads_kernel<16>), dim3(rows), dim3(kThreads), 0, be->stream, p, q);
+        else if (pieces && p.dim <= 128) hipLaunchKernelGGL((attention_turn_heads_kernel<32>), dim3(rows), dim3(kThreads), 0, be->stream, p, q);
+        else if (pieces) hipLaunchKernelGGL((attention_turn_heads_kernel<64>), dim3(rows), dim3(kThreads), 0, be->stream, p, q);
+        else if (turned) hipLaunchKernelGGL(attention_turn_kernel, dim3(rows), dim3(kThreads), (size_t)(p.rot_dims / 2) * sizeof(float2), be->stream, p, q);
         else hipLaunchKernelGGL(attention_prepare_kernel, dim3(rows), dim3(kThreads), 0, be->stream, p, q);
         if (int rc = launched("attention_prepare")) return rc;
         if (int rc = p.mix_scores ? launch_mixed_tiles(be, p, q) : launch_attention_tiles(be, p, q); rc != kDeclined) return rc;

@@ -24,11 +24,6 @@ constexpr int kThreads = 256;
 constexpr uint32_t kSeg = 128; // keys of a segment of attention_scores_kernel
 constexpr float kLog2e = 1.44269504088896341f, kNone = -1e30f;
 
-__device__ __forceinline__ float wave_sum(float v) {
-#pragma unroll
-    for (int d = 32; d > 0; d >>= 1) v += __shfl_xor(v, d, 64);
-    return v;
-}
 __device__ __forceinline__ float wave_max(float v) {
 #pragma unroll
     for (int d = 32; d > 0; d >>= 1) v = fmaxf(v, __shfl_xor(v, d, 64));
@@ -125,7 +120,7 @@ __global__ __launch_bounds__(kThreads) void attention_mixed_rows_kernel(const At
     for (uint32_t o = wave; o < nh; o += kThreads / 64) {
         const float a = wt[o * kSeg + lane], c = wt[o * kSeg + 64 + lane];
         const float m = fmaxf(kNone, wave_max(fmaxf(a, c)));
-        const float ea = __builtin_amdgcn_exp2f(a - m), ec = __builtin_amdgcn_exp2f(c - m), l = wave_sum(ea + ec);
+        const float ea = __builtin_amdgcn_exp2f(a - m), ec = __builtin_amdgcn_exp2f(c - m), l = wave_total(ea + ec);
         wt[o * kSeg + lane] = ea;
         wt[o * kSeg + 64 + lane] = ec;
         if (lane == 0) stats[((int64_t)blockIdx.z * nseg + seg) * p.heads + h0 + o] = make_float2(m, l);
@@ -190,7 +185,9 @@ template <int DT> __device__ __forceinline__ void load_q(const AttentionPlan &p,
 #pragma unroll
     for (int c = 0; c < DT; c++) {
         const uint32_t d = 16 * c + 4 * lg;
-        f[c] = d < p.dim ? *reinterpret_cast<const f32x4 *>(row + d) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+        f[c] = *reinterpret_cast<const f32x4 *>(row + min(d, p.dim - 4));
+#pragma unroll
+        for (int t = 0; t < 4; t++) f[c][t] = d < p.dim ? f[c][t] : 0.0f;
     }
 }
 template <int DT> __device__ __forceinline__ f32x4 scores(const f32x4 (&q)[DT], const f32x4 (&k)[DT]) {
@@ -206,15 +203,16 @@ template <int DT> __device__ __forceinline__ f32x4 scores(const f32x4 (&q)[DT], 
     return a + b;
 }
 
-// DT / VT: 16-wide pieces of a key / a value row.  QREG: the queries stay in registers; else they are read for every key tile.
-template <int HPW, int DT, int VT, bool QREG>
+// DT / VT: 16-wide pieces of a key / a value row (EXACT: without a rest).  QREG: the queries stay in registers; else they are read for every key tile.
+template <int HPW, int DT, int VT, bool QREG, bool EXACT>
 __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(const AttentionPlan p, const float *__restrict__ q, const uint32_t tiles, const uint32_t splits,
                                                                                 float *__restrict__ dst, float2 *__restrict__ stats) {
     extern __shared__ float lds[]; // three buffers of scores [heads rounded up to 16][16][16], talk [heads rounded up][the same + 4]
-    constexpr int RT = (HPW * kTileWaves + 15) / 16; // row tiles of the mixing product
+    constexpr int RT = (HPW * kTileWaves + 15) / 16; // row tiles of the mixing product: the heads rounded up to 16
+    constexpr bool EARLY_K = HPW * VT + (QREG ? HPW * DT : 0) + DT + VT <= 40, EARLY_V = EARLY_K; // registers for what is asked for at a tile's start
     const uint32_t wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, li = lane & 15, lg = lane >> 4;
     const uint32_t tile = tiles - 1 - blockIdx.x / splits, split = blockIdx.x % splits, b = blockIdx.y, s0 = tile * kRowsT;
-    const uint32_t h0 = wave * HPW, rep = p.heads / p.kv_heads, tiles16 = (p.heads + 15) / 16, buffer = tiles16 * 16 * kHeadPitch;
+    const uint32_t h0 = wave * HPW, rep = p.heads / p.kv_heads, tiles16 = RT, buffer = tiles16 * 16 * kHeadPitch;
     const bool shared = min(h0 + HPW - 1, p.heads - 1) / rep == min(h0, p.heads - 1) / rep; // one kv head for all of this wave's heads
     const uint32_t first_row = p.cached + s0, last_row = p.cached + min(s0 + kRowsT, p.S) - 1, last = p.cached + p.S - 1;
     uint32_t lo = first_visible(p, first_row);
@@ -245,9 +243,9 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
     __syncthreads();
     auto load_k = [&](uint32_t g, uint32_t key, f32x4(&f)[DT]) {
         const float *base = p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)key * p.dim; // (the same for the whole wave)
-        const uint32_t row = min(li, last - key) * p.dim + 4 * lg;
+        const uint32_t row = min(li, last - key) * p.dim;
 #pragma unroll
-        for (int c = 0; c < DT; c++) f[c] = 16 * c + 4 * lg < p.dim ? *reinterpret_cast<const f32x4 *>(base + (row + 16 * c)) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+        for (int c = 0; c < DT; c++) f[c] = *reinterpret_cast<const f32x4 *>(base + (row + (EXACT ? 16 * c + 4 * lg : min(16 * c + 4 * lg, p.dim - 4)))); // (clamped: the query is zero there)
     };
     uint32_t b0 = 0, b1 = 2, b2 = 1; // buffers of this iteration's scores, mixing, values
     for (uint32_t it = 0; it < n + 2; it++) {
@@ -259,13 +257,13 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
             const float *base = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)jv * p.vdim;
 #pragma unroll
             for (int t = 0; t < 4; t++) {
-                const uint32_t row = min(4 * lg + t, last - jv) * p.vdim + li;
+                const uint32_t row = min(4 * lg + t, last - jv) * p.vdim;
 #pragma unroll
-                for (int c = 0; c < VT; c++) v[t][c] = 16 * c + li < p.vdim ? base[row + 16 * c] : 0.0f;
+                for (int c = 0; c < VT; c++) v[t][c] = base[row + (EXACT ? 16 * c + li : min(16 * c + li, p.vdim - 1))]; // (clamped: columns that nobody stores)
             }
         };
-        if (do_s) load_k(h0 / rep, js, k);
-        if (do_v) load_v(h0 / rep);
+        if (do_s && EARLY_K) load_k(h0 / rep, js, k);
+        if (do_v && EARLY_V) load_v(h0 / rep);
         if (it >= 1 && it < n + 1) {
             // talk [heads, heads] . scores [heads, 256 columns]: a wave owns whole columns and writes them back in place
 #pragma unroll
@@ -276,10 +274,9 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
                 for (int a = 0; a < RT; a++) acc[a] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
                 for (int c = 0; c < RT; c++) {
-                    if (c >= (int)tiles16) break;
                     f32x4 f[RT];
 #pragma unroll
-                    for (int a = 0; a < RT; a++) f[a] = *reinterpret_cast<const f32x4 *>(talk + min(16 * a + li, tiles16 * 16 - 1) * talk_pitch + 16 * c + 4 * lg);
+                    for (int a = 0; a < RT; a++) f[a] = *reinterpret_cast<const f32x4 *>(talk + (16 * a + li) * talk_pitch + 16 * c + 4 * lg);
 #pragma unroll
                     for (int t = 0; t < 4; t++) {
                         const float x = w[(16 * c + 4 * lg + t) * kHeadPitch];
@@ -291,8 +288,7 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
                 for (int a = 0; a < RT; a++)
 #pragma unroll
                     for (int r = 0; r < 4; r++) {
-                        const uint32_t h = 16 * a + 4 * lg + r;
-                        if (h < p.heads) w[h * kHeadPitch] = acc[a][r];
+                        w[(16 * a + 4 * lg + r) * kHeadPitch] = acc[a][r]; // (heads that are not there: zero)
                     }
             }
         }
@@ -301,7 +297,7 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
             for (int i = 0; i < HPW; i++) {
                 const uint32_t h = h0 + i;
                 if (h >= p.heads) break;
-                if (i > 0 && !shared) load_k(h / rep, js, k);
+                if (i > 0 ? !shared : !EARLY_K) load_k(h / rep, js, k);
                 if constexpr (!QREG) load_q<DT>(p, q, b, s0, li, lg, h, qf[0]);
                 const f32x4 a = scores<DT>(qf[QREG ? i : 0], k);
                 float *w = lds + b0 * buffer + h * kHeadPitch + li;
@@ -316,7 +312,7 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
             for (int i = 0; i < HPW; i++) {
                 const uint32_t h = h0 + i;
                 if (h >= p.heads) break;
-                if (i > 0 && !shared) load_v(h / rep);
+                if (i > 0 ? !shared : !EARLY_V) load_v(h / rep);
                 f32x4 x = *reinterpret_cast<const f32x4 *>(lds + b2 * buffer + h * kHeadPitch + li * kRowPitch + 4 * lg);
                 bool moves = false;
 #pragma unroll
@@ -377,7 +373,7 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
             float *row = dst + ((split * rows + (uint64_t)b * p.S + s) * p.heads + h) * p.vdim + li;
 #pragma unroll
             for (int c = 0; c < VT; c++)
-                if (16 * c + li < p.vdim) row[16 * c] = out[i][c][r] * f;
+                if (EXACT || 16 * c + li < p.vdim) row[16 * c] = out[i][c][r] * f;
         }
     }
 }
@@ -388,9 +384,9 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
 // per lane), a thread has four columns of a kv head's values (for every turns-th key of the chunk).
 constexpr uint32_t kMaxChunk = 64, kValuesAhead = 8;
 struct StepLds { // floats
-    uint32_t turn, q, fresh, talk, raw, mixed, state, total;
+    uint32_t q, fresh, talk, raw, mixed, state, total;
 };
-__host__ __device__ inline StepLds step_lds(uint32_t S, uint32_t heads, uint32_t kv_heads, uint32_t dim, uint32_t rot, uint32_t chunk, uint32_t vdim) {
+__host__ __device__ inline StepLds step_lds(uint32_t S, uint32_t heads, uint32_t kv_heads, uint32_t dim, uint32_t chunk, uint32_t vdim) {
     StepLds o{};
     uint32_t at = 0;
     auto take = [&](uint32_t n) {
@@ -398,7 +394,6 @@ __host__ __device__ inline StepLds step_lds(uint32_t S, uint32_t heads, uint32_t
         at += (n + 3) / 4 * 4;
         return r;
     };
-    o.turn = take(rot * S);             // {cos, sin} per pair and new token
     o.q = take(heads * dim);
     o.fresh = take(kv_heads * dim * S); // new keys
     o.talk = take(heads * heads);
@@ -411,12 +406,12 @@ __host__ __device__ inline StepLds step_lds(uint32_t S, uint32_t heads, uint32_t
 }
 
 template <int REP, int DQ, int PI>
-__global__ __launch_bounds__(kThreads) void attention_mixed_step_kernel(const AttentionPlan p, const uint32_t chunk, const uint32_t chunks, float *__restrict__ parts,
+__global__ __launch_bounds__(kThreads, REP <= 4 ? 3 : 2) void attention_mixed_step_kernel(const AttentionPlan p, const uint32_t chunk, const uint32_t chunks, float *__restrict__ parts,
                                                                         float2 *__restrict__ stats) {
     extern __shared__ float lds[];
     const uint32_t rep = p.heads / p.kv_heads, seg = blockIdx.x, nseg = gridDim.x, r = blockIdx.y, b = r / p.S, s = r - b * p.S;
     const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, pitch = chunk + 1, sub = threadIdx.x & 3;
-    const StepLds at = step_lds(p.S, p.heads, p.kv_heads, p.dim, p.rot_dims, chunk, p.vdim);
+    const StepLds at = step_lds(p.S, p.heads, p.kv_heads, p.dim, chunk, p.vdim);
     const uint32_t first = first_visible(p, p.cached + s) + seg * chunk * chunks, hi = p.cached + s + 1, end = min(hi, first + chunk * chunks);
     const uint32_t vec = p.vdim / 4, cols = p.kv_heads * vec, turns = max(1u, kThreads / cols);
     const uint32_t mine = threadIdx.x % cols, my_turn = threadIdx.x / cols; // (more columns than threads: turns 1, a second round)
@@ -449,59 +444,77 @@ __global__ __launch_bounds__(kThreads) void attention_mixed_step_kernel(const At
         for (uint32_t e = 0; e < kValuesAhead; e++)
             if (e * turns < chunk) v[e] = *reinterpret_cast<const f32x4 *>(value_row(min(j0 + my_turn % turns + e * turns, hi - 1), g) + d);
     };
+    // a wave's heads: values lane and lane + 64 of each (one of a kind where a head is shorter)
+    constexpr int QH = 4, QV = DQ > 4 ? 2 : 1;
+    constexpr uint32_t kWaves = kThreads / 64;
+    float qv[QH][QV];
+    const uint32_t d0 = min(lane, p.dim - 1), d1 = min(lane + 64, p.dim - 1);
+    auto ask_heads = [&](const float *src, uint32_t h0, uint32_t n) {
+#pragma unroll
+        for (int i = 0; i < QH; i++) {
+            const float *x = src + min(h0 + i * kWaves + wave, n - 1) * p.dim;
+            qv[i][0] = x[d0];
+            if (QV > 1) qv[i][QV - 1] = x[d1];
+        }
+    };
+    float2 turn[QV];
+    auto ask_turn = [&](uint32_t t) {
+#pragma unroll
+        for (int v = 0; v < QV; v++) {
+            const uint32_t d = lane + 64 * v;
+            turn[v] = make_float2(1.0f, 0.0f);
+            if (d < p.rot_dims) turn[v] = rotation_at(p, p.position + t, d / 2);
+            if (!(d & 1)) turn[v].y = -turn[v].y;
+        }
+    };
+    ask_heads(p.q.p + (int64_t)r * p.q.pitch, 0, p.heads);
+    ask_turn(s);
     ask_keys(first);
     ask_values(first, mine);
 
-    // the angles of this token and of those new ones whose keys this workgroup scores
     const uint32_t t0 = first > p.cached ? first - p.cached : 0, t1 = end > p.cached && end > first ? end - p.cached : 0; // new keys [t0, t1)
-    const uint32_t pairs = p.rot_dims / 2;
-    float2 *turn = reinterpret_cast<float2 *>(lds + at.turn);
-    for (uint32_t i = threadIdx.x; i < pairs * p.S; i += kThreads) {
-        const uint32_t t = i / pairs, n = i - t * pairs;
-        if (t != s && (t < t0 || t >= t1)) continue;
-        double a = (double)(p.position + t) * exp2(-2.0 * (double)n / (double)p.rot_dims * p.rot_log2);
-        a -= 6.283185307179586 * rint(a * 0.15915494309189535);
-        float sn, cs;
-        sincosf((float)a, &sn, &cs);
-        turn[i] = make_float2(cs, sn);
+    for (uint32_t i = threadIdx.x; i < p.heads * p.heads; i += kThreads) { // (transposed: lanes side by side read other heads' columns)
+        const uint32_t h = i / p.heads, g = i - h * p.heads;
+        lds[at.talk + g * p.heads + h] = p.talk ? p.talk[i] : h == g ? 1.0f : 0.0f;
     }
-    for (uint32_t i = threadIdx.x; i < p.heads * p.heads; i += kThreads) lds[at.talk + i] = p.talk ? p.talk[i] : i / p.heads == i % p.heads ? 1.0f : 0.0f;
     for (uint32_t h = threadIdx.x; h < p.heads; h += kThreads) {
         lds[at.state + h] = kNone;
         lds[at.state + p.heads + h] = 0.0f;
     }
-    __syncthreads();
-    // a head of new token t: turned, at a mean square of one, times f; a wave per head
-    auto head = [&](const float *src, uint32_t t, float f, float *dst, float *also) {
-        auto value = [&](uint32_t d) {
-            const float x = src[d];
-            if (d >= p.rot_dims) return x;
-            const float2 cs = turn[t * pairs + d / 2];
-            return d & 1 ? fmaf(x, cs.x, src[d - 1] * cs.y) : fmaf(x, cs.x, -src[d + 1] * cs.y);
-        };
-        float m = 0.0f;
-        const float v0 = lane < p.dim ? value(lane) : 0.0f, v1 = lane + 64 < p.dim ? value(lane + 64) : 0.0f;
-        m = fmaf(v0, v0, v1 * v1);
-        for (uint32_t d = lane + 128; d < p.dim; d += 64) {
-            const float x = value(d);
-            m = fmaf(x, x, m);
-        }
-        float g = f;
-        if (p.unit_heads) g /= sqrtf(wave_sum(m) / (float)p.dim + p.eps);
-        for (uint32_t d = lane; d < p.dim; d += 64) {
-            const float x = (d == lane ? v0 : d == lane + 64 ? v1 : value(d)) * g;
-            dst[d] = x;
-            if (also) also[d] = x;
+    // the heads of a token: turned, at a mean square of one, times f
+    auto put_heads = [&](uint32_t h0, uint32_t n, float f, float *dst, float *cache, int64_t cache_pitch) {
+#pragma unroll
+        for (int i = 0; i < QH; i++) {
+            const uint32_t h = h0 + i * kWaves + wave;
+            float x[QV], m = 0.0f;
+#pragma unroll
+            for (int v = 0; v < QV; v++) {
+                x[v] = fmaf(qv[i][v], turn[v].x, __shfl_xor(qv[i][v], 1, 64) * turn[v].y);
+                if (lane + 64 * v < p.dim) m = fmaf(x[v], x[v], m);
+            }
+            float g = f;
+            if (p.unit_heads) g /= sqrtf(wave_total(m) / (float)p.dim + p.eps);
+#pragma unroll
+            for (int v = 0; v < QV; v++)
+                if (h < n && lane + 64 * v < p.dim) {
+                    dst[h * p.dim + lane + 64 * v] = x[v] * g;
+                    if (cache) cache[h * cache_pitch + lane + 64 * v] = x[v] * g;
+                }
         }
     };
     float temp = p.scale;
     if (p.temp_every) temp *= 1.0f + p.temp_coef * logf((float)((p.position + s + 1) / p.temp_every + 1));
-#pragma unroll 4
-    for (uint32_t h = wave; h < p.heads; h += kThreads / 64) head(p.q.p + (int64_t)r * p.q.pitch + h * p.dim, s, temp, lds + at.q + h * p.dim, nullptr);
-    for (uint32_t i = wave; i < (t1 - min(t0, t1)) * p.kv_heads; i += kThreads / 64) {
-        const uint32_t t = t0 + i / p.kv_heads, g = i % p.kv_heads;
-        float *cache = t == s ? p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)(p.cached + t) * p.dim : nullptr; // its own workgroup's
-        head(p.k.p + ((int64_t)b * p.S + t) * p.k.pitch + g * p.dim, t, 1.0f, lds + at.fresh + (t * p.kv_heads + g) * p.dim, cache);
+    for (uint32_t h0 = 0; h0 < p.heads; h0 += QH * kWaves) {
+        if (h0) ask_heads(p.q.p + (int64_t)r * p.q.pitch, h0, p.heads);
+        put_heads(h0, p.heads, temp, lds + at.q, nullptr, 0);
+    }
+    for (uint32_t t = t0; t < t1; t++) {
+        if (t != s || t > t0) ask_turn(t);
+        float *cache = t == s ? p.keys + (int64_t)b * p.kv_heads * p.k_block + (int64_t)(p.cached + t) * p.dim : nullptr; // its own workgroup's
+        for (uint32_t h0 = 0; h0 < p.kv_heads; h0 += QH * kWaves) {
+            ask_heads(p.k.p + ((int64_t)b * p.S + t) * p.k.pitch, h0, p.kv_heads);
+            put_heads(h0, p.kv_heads, 1.0f, lds + at.fresh + t * p.kv_heads * p.dim, cache, p.k_block);
+        }
     }
     if (t1 == s + 1 && t0 <= s) // the last segment: this token's values
         for (uint32_t i = threadIdx.x; i < p.kv_heads * p.vdim; i += kThreads) {
@@ -547,10 +560,10 @@ __global__ __launch_bounds__(kThreads) void attention_mixed_step_kernel(const At
         if (j0 + chunk < end) ask_keys(j0 + chunk); // on their way meanwhile
         __syncthreads();
         for (uint32_t i = threadIdx.x; i < p.heads * chunk; i += kThreads) {
-            const uint32_t h = i / chunk, key = i - h * chunk;
+            const uint32_t key = i / p.heads, h = i - key * p.heads;
             float w = 0.0f;
 #pragma unroll 8
-            for (uint32_t g = 0; g < p.heads; g++) w = fmaf(lds[at.talk + h * p.heads + g], lds[at.raw + g * pitch + key], w);
+            for (uint32_t g = 0; g < p.heads; g++) w = fmaf(lds[at.talk + g * p.heads + h], lds[at.raw + g * pitch + key], w);
             lds[at.mixed + h * pitch + key] = key < keys ? w * kLog2e : -INFINITY;
         }
         __syncthreads();
@@ -650,8 +663,49 @@ struct Scratch {
     }
 };
 
+// few segments of many rows: a thread per four results (vdim a multiple of 4) or one
+template <int VW>
+__global__ __launch_bounds__(kThreads) void attention_merge_rows_kernel(const float *__restrict__ parts, const float2 *__restrict__ stats, const uint32_t segs,
+                                                                        const uint64_t row_pitch, const uint64_t seg_pitch, const uint32_t heads, const uint32_t vdim,
+                                                                        const bool sink, const uint64_t total, float *__restrict__ out) {
+    const uint64_t i = ((uint64_t)blockIdx.x * kThreads + threadIdx.x) * VW;
+    if (i >= total) return;
+    const uint32_t n = heads * vdim;
+    const uint64_t row = i / n;
+    const uint32_t c = (uint32_t)(i - row * n);
+    const float *p = parts + row * row_pitch * vdim + c;
+    const float2 *st = stats + row * row_pitch + c / vdim;
+    float m = sink ? 0.0f : kNone, l = 0.0f, o[VW] = {};
+    for (uint32_t k = 0; k < segs; k++) m = fmaxf(m, st[k * seg_pitch].x);
+    if (sink) l = __builtin_amdgcn_exp2f(-m);
+    for (uint32_t k = 0; k < segs; k++) {
+        const float2 t = st[k * seg_pitch];
+        const float f = __builtin_amdgcn_exp2f(t.x - m);
+        l = fmaf(t.y, f, l);
+        if constexpr (VW == 4) {
+            const float4 v = *reinterpret_cast<const float4 *>(p + k * seg_pitch * vdim);
+            o[0] = fmaf(v.x, f, o[0]), o[1] = fmaf(v.y, f, o[1]), o[2] = fmaf(v.z, f, o[2]), o[3] = fmaf(v.w, f, o[3]);
+        } else {
+            o[0] = fmaf(p[k * seg_pitch * vdim], f, o[0]);
+        }
+    }
+    const float inv = 1.0f / l;
+    if constexpr (VW == 4) *reinterpret_cast<float4 *>(out + i) = make_float4(o[0] * inv, o[1] * inv, o[2] * inv, o[3] * inv);
+    else out[i] = o[0] * inv;
+}
+
 void merge(cg_backend *be, const AttentionPlan &p, const float *parts, const float2 *stats, uint32_t segs, uint64_t row_pitch, uint64_t seg_pitch, uint32_t rows, float *out) {
     const uint32_t n = p.heads * p.vdim;
+    if (segs <= 8) {
+        const uint64_t total = (uint64_t)rows * n;
+        if (p.vdim % 4 == 0)
+            hipLaunchKernelGGL((attention_merge_rows_kernel<4>), dim3((uint32_t)((total / 4 + kThreads - 1) / kThreads)), dim3(kThreads), 0, be->stream, parts, stats, segs, row_pitch,
+                               seg_pitch, p.heads, p.vdim, p.zero_sink, total, out);
+        else
+            hipLaunchKernelGGL((attention_merge_rows_kernel<1>), dim3((uint32_t)((total + kThreads - 1) / kThreads)), dim3(kThreads), 0, be->stream, parts, stats, segs, row_pitch,
+                               seg_pitch, p.heads, p.vdim, p.zero_sink, total, out);
+        return;
+    }
     for (uint32_t r0 = 0; r0 < rows; r0 += 65535) {
         const uint32_t nr = std::min(rows - r0, 65535u);
         hipLaunchKernelGGL(attention_merge_kernel, dim3((n + 63) / 64, nr), dim3(kMergeWaves * 64), 0, be->stream, parts + (uint64_t)r0 * row_pitch * p.vdim,
@@ -669,15 +723,17 @@ int mixed_rows(cg_backend *be, const AttentionPlan &p, uint32_t row0, uint32_t r
     return launched("attention_mixed_rows");
 }
 
-template <int HPW, int DT, int VT, bool QREG> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t splits, float *dst, float2 *stats) {
+template <int HPW, int DT, int VT, bool QREG, bool EXACT = false> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t splits, float *dst, float2 *stats) {
     const uint32_t tiles = (p.S + kRowsT - 1) / kRowsT;
-    const size_t h16 = (p.heads + 15) / 16 * 16, lds = (3 * h16 * kHeadPitch + h16 * (h16 + 4)) * 4;
-    if (int rc = allow_lds(reinterpret_cast<const void *>(&attention_mixed_tiles_kernel<HPW, DT, VT, QREG>), lds)) return rc;
-    hipLaunchKernelGGL((attention_mixed_tiles_kernel<HPW, DT, VT, QREG>), dim3(tiles * splits, p.B), dim3(kTileWaves * 64), lds, be->stream, p, q, tiles, splits, dst, stats);
+    const size_t h16 = (HPW * kTileWaves + 15) / 16 * 16, lds = (3 * h16 * kHeadPitch + h16 * (h16 + 4)) * 4;
+    if (int rc = allow_lds(reinterpret_cast<const void *>(&attention_mixed_tiles_kernel<HPW, DT, VT, QREG, EXACT>), lds)) return rc;
+    hipLaunchKernelGGL((attention_mixed_tiles_kernel<HPW, DT, VT, QREG, EXACT>), dim3(tiles * splits, p.B), dim3(kTileWaves * 64), lds, be->stream, p, q, tiles, splits, dst, stats);
     return CG_OK;
 }
 template <int HPW> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t splits, float *dst, float2 *stats) {
     const uint32_t d = p.dim, v = p.vdim;
+    if (d == 64 && v == 64) return run_tiles<HPW, 4, 4, true, true>(be, p, q, splits, dst, stats);
+    if (d == 128 && v == 128) return run_tiles<HPW, 8, 8, (HPW < 4), true>(be, p, q, splits, dst, stats);
     if (d <= 32 && v <= 32) return run_tiles<HPW, 2, 2, true>(be, p, q, splits, dst, stats);
     if (d <= 64 && v <= 64) return run_tiles<HPW, 4, 4, true>(be, p, q, splits, dst, stats);
     if (d <= 64 && v <= 96) return run_tiles<HPW, 4, 6, (HPW < 4)>(be, p, q, splits, dst, stats);
@@ -734,11 +790,11 @@ int launch_mixed_step(cg_backend *be, const AttentionPlan &p) {
     if (p.kv_heads > pairs) return kDeclined;
     uint32_t chunk = kMaxChunk;
     while (chunk * p.kv_heads > pairs || chunk > turns * kValuesAhead) chunk /= 2;
-    const size_t lds = (size_t)step_lds(p.S, p.heads, p.kv_heads, p.dim, p.rot_dims, chunk, p.vdim).total * 4;
+    const size_t lds = (size_t)step_lds(p.S, p.heads, p.kv_heads, p.dim, chunk, p.vdim).total * 4;
     if (lds > kMaxLds / 2) return kDeclined;
-    // up to four workgroups per compute unit
+    // as many workgroups as run at a time
     const uint32_t all = (most + chunk - 1) / chunk;
-    const uint32_t chunks = (uint32_t)(((uint64_t)rows * all + 4 * be->compute_units - 1) / (4 * be->compute_units)), nseg = (all + chunks - 1) / chunks;
+    const uint32_t resident = (rep <= 4 ? 3 : 2) * be->compute_units, chunks = (uint32_t)(((uint64_t)rows * all + resident - 1) / resident), nseg = (all + chunks - 1) / chunks;
     Scratch mem(be);
     const size_t n = (size_t)rows * nseg * p.heads;
     if (int rc = mem.get(n * p.vdim * 4 + n * sizeof(float2))) return rc;

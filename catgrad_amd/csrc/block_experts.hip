@@ -19,11 +19,6 @@ namespace {
 
 constexpr int kThreads = 256, kWaves = 4;
 
-__device__ __forceinline__ float wave_sum(float v) {
-#pragma unroll
-    for (int d = 32; d > 0; d >>= 1) v += __shfl_xor(v, d, 64);
-    return v;
-}
 __device__ __forceinline__ float bf16_lo(uint32_t w) { return asf(w << 16); }
 __device__ __forceinline__ float bf16_hi(uint32_t w) { return asf(w & 0xFFFF0000u); }
 __device__ __forceinline__ uint32_t round_bf16(float v) { return asu(v) + 0x7FFFu + ((asu(v) >> 16) & 1u); } // (bits above 15 hold the pattern)
@@ -192,8 +187,8 @@ __global__ __launch_bounds__(kThreads) void expert_first_kernel(const ExpertsPla
                 b = wu.dot(v, b);
             }
         }
-        a = wave_sum(a);
-        b = wave_sum(b);
+        a = wave_total(a);
+        b = wave_total(b);
         if (lane == 0) hidden[(uint64_t)blockIdx.y * p.ff + f] = weigh * activation(a, b, p.limit, p.slope);
     }
 }
@@ -241,7 +236,7 @@ __global__ __launch_bounds__(kThreads) void expert_second_kernel(const ExpertsPl
     }
 #pragma unroll
     for (int c = 0; c < NC; c++) {
-        const float sum = wave_sum(a[c]);
+        const float sum = wave_total(a[c]);
         if (lane == 0 && n0 + c < p.width) out[(uint64_t)row * p.width + n0 + c] = fmaf(scale, sum, xs[c]);
     }
 }
@@ -264,7 +259,7 @@ __global__ __launch_bounds__(kThreads) void expert_second_slots_kernel(const Exp
         St::input(hidden + at * p.ff, k, v);
         a = s.dot(v, a);
     }
-    a = wave_sum(a);
+    a = wave_total(a);
     if (lane == 0) y[at * p.width + n] = a;
 }
 
@@ -273,19 +268,18 @@ __global__ __launch_bounds__(kThreads) void expert_second_slots_kernel(const Exp
 struct Routed {
     uint32_t expert, place;
 };
-// A workgroup takes kRouteRows tokens, a wave one at a time, and its places in the experts' lists in one go.
-constexpr uint32_t kRouteRows = 32;
+// A workgroup takes `run` tokens, a wave one at a time, and its places in the experts' lists in one go.
 __host__ __device__ constexpr uint32_t route_wave_floats(const ExpertsPlan &p) { return route_floats(p.experts, p.groups) + 2 * p.top; }
-__global__ __launch_bounds__(kThreads) void route_kernel(const ExpertsPlan p, Routed *__restrict__ routed, float *__restrict__ weights, uint32_t *__restrict__ count) {
+__global__ __launch_bounds__(kThreads) void route_kernel(const ExpertsPlan p, const uint32_t run, Routed *__restrict__ routed, float *__restrict__ weights, uint32_t *__restrict__ count) {
     extern __shared__ float lds[];
-    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r0 = blockIdx.x * kRouteRows, n = min(kRouteRows, p.rows - r0);
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r0 = blockIdx.x * run, n = min(run, p.rows - r0);
     float *mine = lds + wave * route_wave_floats(p);
     uint32_t *chosen = reinterpret_cast<uint32_t *>(mine + route_floats(p.experts, p.groups));
     float *weight = reinterpret_cast<float *>(chosen + p.top);
-    uint32_t *seen = reinterpret_cast<uint32_t *>(lds + kWaves * route_wave_floats(p)), *base = seen + p.experts, *place = base + p.experts, *whose = place + kRouteRows * p.top; // [kRouteRows][top]
+    uint32_t *seen = reinterpret_cast<uint32_t *>(lds + kWaves * route_wave_floats(p)), *base = seen + p.experts, *place = base + p.experts, *whose = place + run * p.top; // [run][top]
     for (uint32_t e = threadIdx.x; e < p.experts; e += kThreads) seen[e] = 0;
     __syncthreads();
-    for (uint32_t i = wave; i < kRouteRows; i += kWaves) { // (the same trips for every wave: the choice has barriers)
+    for (uint32_t i = wave; i < run; i += kWaves) { // (the same trips for every wave: the choice has barriers)
         const uint32_t row = r0 + min(i, n - 1);
         choose_experts<64>(p, row, mine, chosen, weight, lane);
         if (i < n)
@@ -493,7 +487,8 @@ struct Scratch {
 };
 
 size_t route_bytes(const ExpertsPlan &p) { return (route_floats(p.experts, p.groups) + 2 * (size_t)p.top) * 4; }
-size_t many_route_bytes(const ExpertsPlan &p) { return (kWaves * (size_t)route_wave_floats(p) + 2 * (size_t)p.experts + 2 * (size_t)kRouteRows * p.top) * 4; }
+constexpr uint32_t kMaxRun = 16;
+size_t many_route_bytes(const ExpertsPlan &p) { return (kWaves * (size_t)route_wave_floats(p) + 2 * (size_t)p.experts + 2 * (size_t)kMaxRun * p.top) * 4; }
 bool vector_rows(const ExpertsPlan &p) {
     const uint32_t vw = p.fmt == kFmtBF16 ? 8 : 4;
     return p.width % vw == 0 && p.ff % vw == 0 && aligned16(p.gate_up) && aligned16(p.down) && aligned16(p.h);
@@ -611,7 +606,8 @@ int launch_experts(cg_backend *be, const ExpertsPlan &p, float *y, int *y_fmt) {
     {
         ProfScope prof(be, CG_K_GATHER, 4.0 * p.rows * p.experts + 20.0 * n);
         hipLaunchKernelGGL(clear_kernel, dim3((p.experts + kThreads - 1) / kThreads), dim3(kThreads), 0, be->stream, count, p.experts);
-        hipLaunchKernelGGL(route_kernel, dim3((p.rows + kRouteRows - 1) / kRouteRows), dim3(kThreads), many_route_bytes(p), be->stream, p, routed, weights, count);
+        const uint32_t run = std::min(kMaxRun, (uint32_t)kWaves * std::max(1u, p.rows / (4 * be->compute_units * kWaves)));
+        hipLaunchKernelGGL(route_kernel, dim3((p.rows + run - 1) / run), dim3(kThreads), many_route_bytes(p), be->stream, p, run, routed, weights, count);
         hipLaunchKernelGGL(route_lists_kernel, dim3((uint32_t)((n + kThreads - 1) / kThreads)), dim3(kThreads), (size_t)(p.experts + 1) * 8, be->stream, p.experts, (uint32_t)n, tm,
                            max_tiles, routed, count, list, tiles);
         if (int rc = launched("route")) return rc;

@@ -10,11 +10,6 @@ namespace {
 
 constexpr int kThreads = 256, kWaves = 4;
 
-__device__ __forceinline__ float wave_sum(float v) {
-#pragma unroll
-    for (int d = 32; d > 0; d >>= 1) v += __shfl_xor(v, d, 64);
-    return v;
-}
 __device__ __forceinline__ uint32_t round_bf16(float v) { return asu(v) + 0x7FFFu + ((asu(v) >> 16) & 1u); } // (bits above 15 hold the pattern)
 __device__ __forceinline__ float element(const Table &t, int64_t i) {
     return t.fmt == kFmtBF16 ? asf((uint32_t)static_cast<const uint16_t *>(t.p)[i] << 16) : static_cast<const float *>(t.p)[i];
@@ -41,12 +36,12 @@ __global__ __launch_bounds__(kThreads) void pair_embedding_kernel(const PairEmbe
 }
 
 // ---- grouped norm and filter -----------------------------------------------------------------------------------------
-// A workgroup takes `run` tokens of a sequence and one group of columns: first the scales of these tokens' rows and of the
-// taps - 1 before them (a wave per row), then, with a thread per VW columns, the filter along the tokens; what the filter
-// looks back on stays in registers.  TAPS: at most so many.
-template <int VW, int TAPS> __global__ __launch_bounds__(kThreads) void conv_rows_kernel(const ConvRowsPlan p) {
+// A workgroup takes `run` tokens of a sequence and `cols` columns of a group (blockIdx.y: group and part of it): the scales of
+// these tokens' rows and of the taps - 1 before them (a wave per row, four rows' pieces in flight), then, with a thread per VW
+// columns, the filter along the tokens; what the filter looks back on stays in registers.  TAPS: at most so many.
+template <int VW, int TAPS> __global__ __launch_bounds__(kThreads) void conv_rows_kernel(const ConvRowsPlan p, const uint32_t parts) {
     extern __shared__ float scale[]; // [run + taps - 1]
-    const uint32_t past = p.taps - 1, cols = p.width / p.groups, c0 = blockIdx.y * cols;
+    const uint32_t past = p.taps - 1, size = p.width / p.groups, group = blockIdx.y / parts, part = blockIdx.y - group * parts, g0 = group * size;
     const uint32_t runs = (p.S + p.run - 1) / p.run, b = blockIdx.x / runs, s0 = (blockIdx.x - b * runs) * p.run, n = min(p.run, p.S - s0);
     const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     auto load = [&](const float *q, float(&v)[VW]) {
@@ -57,25 +52,55 @@ template <int VW, int TAPS> __global__ __launch_bounds__(kThreads) void conv_row
             v[0] = *q;
         }
     };
-    for (uint32_t i = wave; i < n + past; i += kWaves) {
-        const int32_t s = (int32_t)(s0 + i) - (int32_t)past;
-        if (s < 0) continue;
-        const float *x = p.x.p + ((int64_t)b * p.S + s) * p.x.pitch + c0;
-        float m = 0.0f;
-#pragma unroll 4
-        for (uint32_t k = lane * VW; k < cols; k += 64 * VW) {
-            float v[VW];
-            load(x + k, v);
+    // this thread's columns, its share of the filters asked for first
+    const uint32_t per = ((size + parts - 1) / parts + VW - 1) / VW * VW, c_end = g0 + min(size, (part + 1) * per);
+    uint32_t c = g0 + part * per + threadIdx.x * VW;
+    float gamma[2][VW], w[2][TAPS][VW]; // tap t counts from the present back
+    auto ask_filters = [&](uint32_t at) {
+        at = min(at, p.width - VW);
 #pragma unroll
-            for (int j = 0; j < VW; j++) m = fmaf(v[j], v[j], m);
+        for (int f = 0; f < 2; f++) {
+            if (f >= p.n) break;
+            load(p.out[f].gamma + at, gamma[f]);
+#pragma unroll
+            for (int j = 0; j < VW; j++) {
+                if (TAPS == 4 && VW == 4 && p.taps == 4 && p.out[f].conv) {
+                    const float4 t = *reinterpret_cast<const float4 *>(p.out[f].conv + (int64_t)(at + j) * 4);
+                    w[f][0][j] = t.w, w[f][1 % TAPS][j] = t.z, w[f][2 % TAPS][j] = t.y, w[f][3 % TAPS][j] = t.x;
+                } else {
+#pragma unroll
+                    for (int t = 0; t < TAPS; t++) w[f][t][j] = p.out[f].conv && t < (int)p.taps ? p.out[f].conv[(int64_t)(at + j) * p.taps + (p.taps - 1 - t)] : 0.0f;
+                }
+            }
         }
-        m = wave_sum(m);
-        if (lane == 0) scale[i] = 1.0f / sqrtf(m / (float)cols + p.eps);
+    };
+    ask_filters(c);
+    constexpr int ROWS = 4; // of a wave at a time
+    for (uint32_t i0 = wave; i0 < n + past; i0 += kWaves * ROWS) {
+        float m[ROWS] = {};
+        for (uint32_t k = lane * VW; k < size; k += 64 * VW) {
+            float v[ROWS][VW];
+#pragma unroll
+            for (int e = 0; e < ROWS; e++) { // (clamped: rows that are not there are not stored)
+                const int32_t s = (int32_t)(s0 + min(i0 + e * kWaves, n + past - 1)) - (int32_t)past;
+                load(p.x.p + ((int64_t)b * p.S + max(s, 0)) * p.x.pitch + g0 + k, v[e]);
+            }
+#pragma unroll
+            for (int e = 0; e < ROWS; e++)
+#pragma unroll
+                for (int j = 0; j < VW; j++) m[e] = fmaf(v[e][j], v[e][j], m[e]);
+        }
+#pragma unroll
+        for (int e = 0; e < ROWS; e++) {
+            const uint32_t i = i0 + e * kWaves;
+            const float sum = wave_total(m[e]);
+            if (lane == 0 && i < n + past) scale[i] = 1.0f / sqrtf(sum / (float)size + p.eps);
+        }
     }
     __syncthreads();
-    for (uint32_t k = threadIdx.x * VW; k < cols; k += kThreads * VW) {
-        const uint32_t c = c0 + k;
-        // z of token s0 - past + i
+    for (; c < c_end; c += kThreads * VW) {
+        if (c >= g0 + part * per + kThreads * VW) ask_filters(c);
+        // z of token s0 - past + i, for the tokens in front of the sequence's new ones from its state
         auto unit = [&](uint32_t i, float(&v)[VW]) {
             const int32_t s = (int32_t)(s0 + i) - (int32_t)past;
             if (s >= 0) {
@@ -91,25 +116,13 @@ template <int VW, int TAPS> __global__ __launch_bounds__(kThreads) void conv_row
         };
         // the inputs behind the sequence's end become its state
         auto keep = [&](int32_t s, const float(&v)[VW]) {
-            const int32_t at = s - (int32_t)(p.S - past);
+            const int32_t at = s - ((int32_t)p.S - (int32_t)past);
             if (at < 0) return;
             float *o = p.state_out + ((int64_t)b * past + at) * p.width + c;
             if constexpr (VW == 4) *reinterpret_cast<float4 *>(o) = make_float4(v[0], v[1], v[2], v[3]);
             else *o = v[0];
         };
-        float gamma[2][VW], w[2][TAPS][VW], z[TAPS][VW];
-#pragma unroll
-        for (int f = 0; f < 2; f++) {
-            if (f >= p.n) break;
-#pragma unroll
-            for (int j = 0; j < VW; j++) {
-                gamma[f][j] = p.out[f].gamma[c + j];
-#pragma unroll
-                for (int t = 0; t < TAPS; t++) // tap t of TAPS counts from the present back: the ring's order
-                    w[f][t][j] = p.out[f].conv && t < (int)p.taps ? p.out[f].conv[(int64_t)(c + j) * p.taps + (p.taps - 1 - t)] : 0.0f;
-            }
-        }
-        // z[t]: the input t tokens back
+        float z[TAPS][VW]; // the input t tokens back
 #pragma unroll
         for (int t = 0; t < TAPS; t++)
 #pragma unroll
@@ -120,41 +133,49 @@ template <int VW, int TAPS> __global__ __launch_bounds__(kThreads) void conv_row
                 unit(past - t, z[t - 1]); // (moved one back below)
                 if (s0 + n == p.S && (int32_t)s0 - t < 0) keep((int32_t)s0 - t, z[t - 1]);
             }
-        for (uint32_t i = 0; i < n; i++) {
+        constexpr int AHEAD = 4; // rows asked for together
+        for (uint32_t i0 = 0; i0 < n; i0 += AHEAD) {
+            float next[AHEAD][VW];
 #pragma unroll
-            for (int t = TAPS - 1; t >= 1; t--)
+            for (int e = 0; e < AHEAD; e++) unit(past + min(i0 + e, n - 1), next[e]);
 #pragma unroll
-                for (int j = 0; j < VW; j++) z[t][j] = z[t - 1][j];
-            unit(past + i, z[0]);
-            const uint32_t s = s0 + i;
-            if (past) keep((int32_t)s, z[0]);
-            const int64_t r = (int64_t)b * p.S + s;
+            for (int e = 0; e < AHEAD; e++) {
+                const uint32_t s = s0 + i0 + e;
+                if (i0 + e >= n) break;
 #pragma unroll
-            for (int f = 0; f < 2; f++) {
-                if (f >= p.n) break;
-                float h[VW];
+                for (int t = TAPS - 1; t >= 1; t--)
 #pragma unroll
-                for (int j = 0; j < VW; j++) {
-                    float a = 0.0f;
+                    for (int j = 0; j < VW; j++) z[t][j] = z[t - 1][j];
 #pragma unroll
-                    for (int t = TAPS - 1; t >= 0; t--) a = fmaf(w[f][t][j], z[t][j], a);
-                    h[j] = (a + z[0][j]) * gamma[f][j];
-                }
-                const int64_t o = r * p.width + c;
-                if (p.out[f].fmt == kFmtBF16) {
-                    uint16_t *d = static_cast<uint16_t *>(p.out[f].dst) + o;
-                    if constexpr (VW == 4)
-                        *reinterpret_cast<uint2 *>(d) =
-                            make_uint2((round_bf16(h[0]) >> 16) | (round_bf16(h[1]) & 0xFFFF0000u), (round_bf16(h[2]) >> 16) | (round_bf16(h[3]) & 0xFFFF0000u));
-                    else *d = (uint16_t)(round_bf16(h[0]) >> 16);
-                } else {
-                    float *d = static_cast<float *>(p.out[f].dst) + o;
-                    if (p.out[f].round) {
+                for (int j = 0; j < VW; j++) z[0][j] = next[e][j];
+                if (past) keep((int32_t)s, z[0]);
+                const int64_t o = ((int64_t)b * p.S + s) * p.width + c;
 #pragma unroll
-                        for (int j = 0; j < VW; j++) h[j] = asf(round_bf16(h[j]) & 0xFFFF0000u);
+                for (int f = 0; f < 2; f++) {
+                    if (f >= p.n) break;
+                    float h[VW];
+#pragma unroll
+                    for (int j = 0; j < VW; j++) {
+                        float a = 0.0f;
+#pragma unroll
+                        for (int t = TAPS - 1; t >= 0; t--) a = fmaf(w[f][t][j], z[t][j], a);
+                        h[j] = (a + z[0][j]) * gamma[f][j];
                     }
-                    if constexpr (VW == 4) *reinterpret_cast<float4 *>(d) = make_float4(h[0], h[1], h[2], h[3]);
-                    else *d = h[0];
+                    if (p.out[f].fmt == kFmtBF16) {
+                        uint16_t *d = static_cast<uint16_t *>(p.out[f].dst) + o;
+                        if constexpr (VW == 4)
+                            *reinterpret_cast<uint2 *>(d) =
+                                make_uint2((round_bf16(h[0]) >> 16) | (round_bf16(h[1]) & 0xFFFF0000u), (round_bf16(h[2]) >> 16) | (round_bf16(h[3]) & 0xFFFF0000u));
+                        else *d = (uint16_t)(round_bf16(h[0]) >> 16);
+                    } else {
+                        float *d = static_cast<float *>(p.out[f].dst) + o;
+                        if (p.out[f].round) {
+#pragma unroll
+                            for (int j = 0; j < VW; j++) h[j] = asf(round_bf16(h[j]) & 0xFFFF0000u);
+                        }
+                        if constexpr (VW == 4) *reinterpret_cast<float4 *>(d) = make_float4(h[0], h[1], h[2], h[3]);
+                        else *d = h[0];
+                    }
                 }
             }
         }
@@ -202,7 +223,7 @@ template <int VW> __global__ __launch_bounds__(kThreads) void side_sum_kernel(co
 #pragma unroll
         for (int j = 0; j < VW; j++) m = fmaf(v[j], v[j], m);
     }
-    m = wave_sum(m);
+    m = wave_total(m);
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = m;
     __syncthreads();
     const float f = scale / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)width + eps);
@@ -236,23 +257,25 @@ int launch_pair_embedding(cg_backend *be, const PairEmbeddingPlan &p) {
 
 int launch_conv_rows(cg_backend *be, ConvRowsPlan p) {
     const uint32_t cols = p.width / p.groups, past = p.taps - 1;
-    // short runs while the device is not full
+    // short runs while the device is not full, and a group's columns over several workgroups
     p.run = 1;
-    while (p.run < 16 && (uint64_t)p.B * p.groups * ((p.S + p.run * 2 - 1) / (p.run * 2)) >= 4ull * be->compute_units) p.run *= 2;
+    while (p.run < 16 && (uint64_t)p.B * p.groups * ((p.S + p.run * 2 - 1) / (p.run * 2)) >= 8ull * be->compute_units) p.run *= 2;
+    uint32_t split = 1;
+    while (cols / (split * 2) >= 128 && (uint64_t)p.B * p.S * p.groups * split * 2 <= be->compute_units) split *= 2;
     double bytes = 4.0;
     bool vec = cols % 4 == 0 && p.x.pitch % 4 == 0 && aligned16(p.x.p) && aligned16(p.state) && aligned16(p.state_out);
     for (int f = 0; f < p.n; f++) {
         bytes += p.out[f].fmt == kFmtBF16 ? 2.0 : 4.0;
-        vec = vec && aligned16(p.out[f].dst);
+        vec = vec && aligned16(p.out[f].dst) && aligned16(p.out[f].gamma) && aligned16(p.out[f].conv);
     }
     ProfScope prof(be, CG_K_REDUCE, bytes * p.B * p.S * p.width);
     const uint32_t runs = (p.S + p.run - 1) / p.run;
-    const dim3 grid(p.B * runs, p.groups);
+    const dim3 grid(p.B * runs, p.groups * split);
     const size_t lds = (p.run + past) * 4;
     hipStream_t s = be->stream;
 #define CG_CONV(T)                                                                                       \
-    if (vec) hipLaunchKernelGGL((conv_rows_kernel<4, T>), grid, dim3(kThreads), lds, s, p);               \
-    else hipLaunchKernelGGL((conv_rows_kernel<1, T>), grid, dim3(kThreads), lds, s, p)
+    if (vec) hipLaunchKernelGGL((conv_rows_kernel<4, T>), grid, dim3(kThreads), lds, s, p, split);        \
+    else hipLaunchKernelGGL((conv_rows_kernel<1, T>), grid, dim3(kThreads), lds, s, p, split)
     if (p.taps <= 1) { CG_CONV(1); }
     else if (p.taps <= 2) { CG_CONV(2); }
     else if (p.taps <= 3) { CG_CONV(3); }

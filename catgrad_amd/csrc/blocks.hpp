@@ -141,12 +141,21 @@ struct AttentionPlan {
     bool bias, unit_heads, mix_scores, zero_sink;
     uint32_t rot_dims;          // 0: no rotation
     double rot_log2;            // log2 of its base
+    const float2 *rot_fine, *rot_coarse; // tables (RotTable); set by launch_attention
     Rows q, k, v;
     const float *q_norm, *k_norm, *talk;
     float *keys, *values;       // row 0 of the cached rows of (b 0, kv head 0); the new rows follow the cached ones
     int64_t k_block, v_block;   // elements from one (b, kv head) to the next
     float *out;                 // [B * S, heads * vdim]
 };
+#ifdef __HIPCC__
+// {cos, sin} of pair i at a position
+__device__ __forceinline__ float2 rotation_at(const AttentionPlan &p, uint64_t position, uint32_t i) {
+    const uint32_t pairs = p.rot_dims / 2;
+    const float2 a = p.rot_fine[(position % kRotFine) * pairs + i], b = p.rot_coarse[(position / kRotFine) * pairs + i];
+    return make_float2(fmaf(a.x, b.x, -a.y * b.y), fmaf(a.x, b.y, a.y * b.x));
+}
+#endif
 int launch_attention(cg_backend *be, const AttentionPlan &p);
 // More than a few new tokens, on the matrix instructions (q: the prepared queries); kDeclined: sizes it does not take.
 int launch_attention_tiles(cg_backend *be, const AttentionPlan &p, const float *q);

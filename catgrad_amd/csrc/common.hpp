@@ -112,6 +112,18 @@ struct DeferredWrite;
 struct Buffer;
 }
 
+namespace cg {
+// {cos, sin} of position * base^(-2 i / dims): of the positions 0 .. kRotFine - 1 and of the multiples of kRotFine, [.., dims / 2]
+// each; a position's pair is the product of two of them as complex numbers.
+constexpr uint32_t kRotFine = 1024;
+struct RotTable {
+    uint32_t dims;
+    double log2_base;
+    Buffer *fine, *coarse;
+    uint32_t coarse_n;
+};
+} // namespace cg
+
 struct cg_backend {
     std::recursive_mutex mu; // held by every entry point for the duration of the call
     std::atomic<long> live_tensors{0}; // heap handles that name this backend (see alloc_tensor)
@@ -144,6 +156,7 @@ struct cg_backend {
     size_t const_bytes = 0;
     cg::Buffer *iota = nullptr; // 0, 1, 2, ... : every arange is a view of it
     int64_t iota_len = 0;
+    std::vector<cg::RotTable> rot_tables; // of the rotations that attention blocks have asked for
     bool fuse = true; // defer element-wise ops and fuse them (CG_FUSE=0 switches it off)
     bool aot = true;  // use the compiled kernels for listed programs (CG_AOT=0: interpreter only)
     uint64_t programs_compiled = 0, programs_interpreted = 0; // launches of fused programs, by kernel kind
@@ -290,6 +303,7 @@ cg_tensor *alloc_tensor(cg_backend *be);
 int ensure_concrete(cg_tensor *t);
 // A dense copy of any view.
 int materialize(cg_backend *be, const cg_tensor *x, cg_tensor **out);
+void buffer_release(Buffer *b);
 
 // ---- helpers for the entry points -------------------------------------------------------
 struct Consume { // the consumed reference of a tensor argument (move semantics of the ABI)

@@ -290,6 +290,20 @@ __device__ __forceinline__ uint32_t apply(uint32_t a, uint32_t b, uint32_t c, ui
     return 0u;
 }
 
+// Sum over the 64 lanes of a wave, for every lane: inside rows of 16 lanes by shifts, then from row to row, all without LDS.
+template <int CTRL, int ROWS> __device__ __forceinline__ float add_shifted(float v) {
+    return v + asf((uint32_t)__builtin_amdgcn_update_dpp(0, (int)asu(v), CTRL, ROWS, 0xF, true));
+}
+__device__ __forceinline__ float wave_total(float v) {
+    v = add_shifted<0x111, 0xF>(v); // row_shr 1, 2, 4, 8
+    v = add_shifted<0x112, 0xF>(v);
+    v = add_shifted<0x114, 0xF>(v);
+    v = add_shifted<0x118, 0xF>(v);
+    v = add_shifted<0x142, 0xA>(v); // the first row's sum into the second, the third's into the fourth
+    v = add_shifted<0x143, 0xC>(v); // the lower half's into the upper
+    return asf((uint32_t)__builtin_amdgcn_readlane((int)asu(v), 63));
+}
+
 // Offset (in elements) of row `row` of a view whose outer axes are described by
 // (od, odiv, os), innermost first.
 __device__ __forceinline__ int64_t row_offset(uint32_t row, uint32_t nouter, const uint32_t *od, const FastDiv *odiv,

@@ -118,7 +118,7 @@ void drop_packed(Buffer *b) {
     b->packed.clear();
 }
 
-static void buffer_release(Buffer *b) {
+void buffer_release(Buffer *b) {
     while (b && b->rc.fetch_sub(1) == 1) {
         if (b->ptr) b->be->pool.free(b->ptr, b->cls);
         if (b->side) b->be->pool.free(b->side, b->side_cls);
@@ -1220,6 +1220,11 @@ static void const_memo_clear(cg_backend *be) {
     buffer_release(be->iota);
     be->iota = nullptr;
     be->iota_len = 0;
+    for (RotTable &t : be->rot_tables) {
+        buffer_release(t.fine);
+        buffer_release(t.coarse);
+    }
+    be->rot_tables.clear();
 }
 
 static void const_memo_insert(cg_backend *be, const std::string &key, Buffer *b) {
@@ -2205,8 +2210,9 @@ int cg_pool_stats(cg_backend *b, size_t *bytes_in_use, size_t *bytes_cached) {
     if (b && b->owner_gone) return fail(CG_ERR_ARG, "backend used after cg_backend_destroy");
     if (!b) return fail(CG_ERR_ARG, "null backend");
     b->pool.stats(bytes_in_use, bytes_cached);
-    // what the backend keeps for itself (iota, results of constant programs) counts as cached
+    // what the backend keeps for itself (iota, rotations, results of constant programs) counts as cached
     size_t kept = b->const_bytes + (b->iota ? b->iota->cls : 0);
+    for (const RotTable &t : b->rot_tables) kept += t.fine->cls + t.coarse->cls;
     if (bytes_in_use) *bytes_in_use -= kept < *bytes_in_use ? kept : *bytes_in_use;
     if (bytes_cached) *bytes_cached += kept;
     return CG_OK;

@@ -69,11 +69,17 @@ class LayeredModel : public Model {
     void expect(const std::string &name, const Shape &s) {
         if (dims(name) != s) throw InterpreterError("parameter " + name + " does not have the shape the configuration asks for");
     }
-    // (computed at once: a view of a deferred tensor would compute it again for itself)
+    // Computed at once: a view of a deferred tensor would compute it again for itself.  A small matrix is part of one that is
+    // large enough for the backend to keep it in two bytes a value.
+    static constexpr size_t kNarrowFrom = 65536;
     Tensor stored_form(Tensor t) {
-        t = i_.backend.cast(std::move(t), weights_);
-        i_.backend.realize(t);
-        return t;
+        Backend &be = i_.backend;
+        const Shape s = t.shape();
+        const bool small = weights_ != CG_F32 && s.size() == 2 && s[0] * s[1] < kNarrowFrom;
+        if (small) t = be.concat(be.cast(std::move(t), CG_F32), be.zeros(Shape{(kNarrowFrom + s[1] - 1) / s[1], s[1]}, CG_F32), 0);
+        t = be.cast(std::move(t), weights_);
+        be.realize(t);
+        return small ? be.slice(std::move(t), 0, 0, s[0]) : t;
     }
     void store(const std::string &name) { i_.parameters[name] = stored_form(std::move(i_.parameters[name])); }
 
