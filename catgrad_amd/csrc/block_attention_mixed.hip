@@ -15,6 +15,7 @@
 #include "device_utils.hpp"
 
 #include <algorithm>
+#include <type_traits>
 
 namespace cg {
 namespace {
@@ -203,17 +204,21 @@ template <int DT> __device__ __forceinline__ f32x4 scores(const f32x4 (&q)[DT], 
     return a + b;
 }
 
-// DT / VT: 16-wide pieces of a key / a value row (EXACT: without a rest).  QREG: the queries stay in registers; else they are read for every key tile.
-template <int HPW, int DT, int VT, bool QREG, bool EXACT>
+// DT / VT: 16-wide pieces of a key / a value row (EXACT: without a rest).  QREG: the queries stay in registers; else they are
+// read for every key tile.  SHARED: a wave's heads have one kv head; its next keys and values are asked for as soon as the
+// registers of these are free.  A wave whose heads are not all there computes its last one again in their place: their rows of
+// the buffers meet zeros in the mixing, and nobody stores what they come to.
+template <int HPW, int DT, int VT, bool QREG, bool EXACT, bool SHARED>
 __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(const AttentionPlan p, const float *__restrict__ q, const uint32_t tiles, const uint32_t splits,
                                                                                 float *__restrict__ dst, float2 *__restrict__ stats) {
     extern __shared__ float lds[]; // three buffers of scores [heads rounded up to 16][16][16], talk [heads rounded up][the same + 4]
     constexpr int RT = (HPW * kTileWaves + 15) / 16; // row tiles of the mixing product: the heads rounded up to 16
-    constexpr bool EARLY_K = HPW * VT + (QREG ? HPW * DT : 0) + DT + VT <= 40, EARLY_V = EARLY_K; // registers for what is asked for at a tile's start
+    constexpr uint32_t BUFFER = RT * 16 * kHeadPitch, TALK = RT * 16 + 4;
+    // (where registers are short keys or values are asked for when they are needed)
+    constexpr bool TIGHT = HPW * VT + (QREG ? HPW * DT : DT) + DT + VT > 40, AHEAD_K = SHARED && QREG, AHEAD_V = SHARED && !TIGHT;
     const uint32_t wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, li = lane & 15, lg = lane >> 4;
     const uint32_t tile = tiles - 1 - blockIdx.x / splits, split = blockIdx.x % splits, b = blockIdx.y, s0 = tile * kRowsT;
-    const uint32_t h0 = wave * HPW, rep = p.heads / p.kv_heads, tiles16 = RT, buffer = tiles16 * 16 * kHeadPitch;
-    const bool shared = min(h0 + HPW - 1, p.heads - 1) / rep == min(h0, p.heads - 1) / rep; // one kv head for all of this wave's heads
+    const uint32_t h0 = wave * HPW, rep = p.heads / p.kv_heads;
     const uint32_t first_row = p.cached + s0, last_row = p.cached + min(s0 + kRowsT, p.S) - 1, last = p.cached + p.S - 1;
     uint32_t lo = first_visible(p, first_row);
     const uint32_t ntiles = (last_row + 1 - lo + kKeysT - 1) / kKeysT, per = (ntiles + splits - 1) / splits;
@@ -221,108 +226,113 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
     lo += from * kKeysT;
 
     f32x4 qf[QREG ? HPW : 1][DT], out[HPW][VT];
-    float slope[HPW], top[HPW], l[HPW]; // of row li, l of this lane's keys
-    const uint32_t talk_pitch = tiles16 * 16 + 4;
-    float *talk = lds + 3 * buffer;
+    float top[HPW], l[HPW]; // of row li, l of this lane's keys
+    float *talk = lds + 3 * BUFFER;
+    auto head_of = [&](int i) { return min(h0 + i, p.heads - 1); };
 #pragma unroll
     for (int i = 0; i < HPW; i++) {
-        const uint32_t h = min(h0 + i, p.heads - 1);
-        if constexpr (QREG) load_q<DT>(p, q, b, s0, li, lg, h, qf[i]);
-        slope[i] = p.bias ? slope_of(h, p.heads) : 0.0f;
+        if constexpr (QREG) load_q<DT>(p, q, b, s0, li, lg, head_of(i), qf[i]);
         top[i] = p.zero_sink ? 0.0f : kNone;
         l[i] = 0.0f;
 #pragma unroll
         for (int c = 0; c < VT; c++) out[i][c] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
     }
-    for (uint32_t i = threadIdx.x; i < tiles16 * 16 * tiles16 * 16; i += kTileWaves * 64) {
-        const uint32_t h = i / (tiles16 * 16), g = i % (tiles16 * 16);
-        talk[h * talk_pitch + g] = h < p.heads && g < p.heads ? p.talk[(int64_t)h * p.heads + g] : 0.0f;
+    for (uint32_t i = threadIdx.x; i < RT * 16 * RT * 16; i += kTileWaves * 64) {
+        const uint32_t h = i / (RT * 16), g = i % (RT * 16);
+        talk[h * TALK + g] = h < p.heads && g < p.heads ? p.talk[(int64_t)h * p.heads + g] : 0.0f;
     }
-    for (uint32_t i = p.heads * kHeadPitch + threadIdx.x; i < buffer; i += kTileWaves * 64) // heads that are not there
-        lds[i] = lds[buffer + i] = lds[2 * buffer + i] = 0.0f;
+    for (uint32_t i = HPW * kTileWaves * kHeadPitch + threadIdx.x; i < BUFFER; i += kTileWaves * 64) // rows that no wave writes
+        lds[i] = lds[BUFFER + i] = lds[2 * BUFFER + i] = 0.0f;
     __syncthreads();
-    auto load_k = [&](uint32_t g, uint32_t key, f32x4(&f)[DT]) {
+    f32x4 k[DT];
+    float v[4][VT];
+    const uint32_t koff = EXACT ? 4 * lg : 0;
+    auto load_k = [&](uint32_t g, uint32_t key) {
         const float *base = p.keys + ((int64_t)b * p.kv_heads + g) * p.k_block + (int64_t)key * p.dim; // (the same for the whole wave)
-        const uint32_t row = min(li, last - key) * p.dim;
+        const uint32_t row = min(li, last - key) * p.dim + koff;
 #pragma unroll
-        for (int c = 0; c < DT; c++) f[c] = *reinterpret_cast<const f32x4 *>(base + (row + (EXACT ? 16 * c + 4 * lg : min(16 * c + 4 * lg, p.dim - 4)))); // (clamped: the query is zero there)
+        for (int c = 0; c < DT; c++) k[c] = *reinterpret_cast<const f32x4 *>(base + (row + (EXACT ? 16 * c : min(16 * c + 4 * lg, p.dim - 4)))); // (clamped: the query is zero there)
     };
-    uint32_t b0 = 0, b1 = 2, b2 = 1; // buffers of this iteration's scores, mixing, values
-    for (uint32_t it = 0; it < n + 2; it++) {
-        const bool do_s = it < n && h0 < p.heads, do_v = it >= 2 && h0 < p.heads;
+    auto load_v = [&](uint32_t g, uint32_t key) {
+        const float *base = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)key * p.vdim;
+#pragma unroll
+        for (int t = 0; t < 4; t++) {
+            const uint32_t row = min(4 * lg + t, last - key) * p.vdim + (EXACT ? li : 0);
+#pragma unroll
+            for (int c = 0; c < VT; c++) v[t][c] = base[row + (EXACT ? 16 * c : min(16 * c + li, p.vdim - 1))]; // (clamped: columns that nobody stores)
+        }
+    };
+    uint32_t b0 = 0, b1 = 2 * BUFFER, b2 = BUFFER; // buffers of this iteration's scores, mixing, values
+    // scores of key tile `it`, mixing of the one before, soft-max and values of the one before that
+    auto step = [&](uint32_t it, auto do_s, auto do_m, auto do_v) {
         const uint32_t js = lo + it * kKeysT, jv = lo + (it - 2) * kKeysT;
-        f32x4 k[DT];
-        float v[4][VT];
-        auto load_v = [&](uint32_t g) {
-            const float *base = p.values + ((int64_t)b * p.kv_heads + g) * p.v_block + (int64_t)jv * p.vdim;
+        f32x4 x[HPW];
+        if constexpr (do_v) {
 #pragma unroll
-            for (int t = 0; t < 4; t++) {
-                const uint32_t row = min(4 * lg + t, last - jv) * p.vdim;
+            for (int i = 0; i < HPW; i++) x[i] = *reinterpret_cast<const f32x4 *>(lds + b2 + (h0 + i) * kHeadPitch + li * kRowPitch + 4 * lg);
+        }
+        if constexpr (do_s) { // scores of this wave's heads (of keys that a row does not see as well)
 #pragma unroll
-                for (int c = 0; c < VT; c++) v[t][c] = base[row + (EXACT ? 16 * c + li : min(16 * c + li, p.vdim - 1))]; // (clamped: columns that nobody stores)
-            }
-        };
-        if (do_s && EARLY_K) load_k(h0 / rep, js, k);
-        if (do_v && EARLY_V) load_v(h0 / rep);
-        if (it >= 1 && it < n + 1) {
-            // talk [heads, heads] . scores [heads, 256 columns]: a wave owns whole columns and writes them back in place
+            for (int i = 0; i < HPW; i++) {
+                if (!SHARED || (!AHEAD_K && i == 0)) load_k(head_of(i) / rep, js);
+                if constexpr (!QREG) load_q<DT>(p, q, b, s0, li, lg, head_of(i), qf[0]);
+                f32x4 a = scores<DT>(qf[QREG ? i : 0], k);
+                if (p.bias) {
+                    const float slope = slope_of(head_of(i), p.heads), d = (float)(int)(first_row + 4 * lg - js - li);
 #pragma unroll
-            for (uint32_t e = 0; e < kRowsT / kTileWaves; e++) {
-                float *w = lds + b1 * buffer + (wave * (kRowsT / kTileWaves) + e) * kRowPitch + li;
-                f32x4 acc[RT];
-#pragma unroll
-                for (int a = 0; a < RT; a++) acc[a] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll
-                for (int c = 0; c < RT; c++) {
-                    f32x4 f[RT];
-#pragma unroll
-                    for (int a = 0; a < RT; a++) f[a] = *reinterpret_cast<const f32x4 *>(talk + (16 * a + li) * talk_pitch + 16 * c + 4 * lg);
-#pragma unroll
-                    for (int t = 0; t < 4; t++) {
-                        const float x = w[(16 * c + 4 * lg + t) * kHeadPitch];
-#pragma unroll
-                        for (int a = 0; a < RT; a++) acc[a] = mfma(f[a][t], x, acc[a]);
-                    }
+                    for (int r = 0; r < 4; r++) a[r] = fmaf(-slope, d + (float)r, a[r]);
                 }
+                float *w = lds + b0 + (h0 + i) * kHeadPitch + li;
+#pragma unroll
+                for (int r = 0; r < 4; r++) w[(4 * lg + r) * kRowPitch] = a[r];
+                if constexpr (TIGHT) __builtin_amdgcn_sched_barrier(0); // (one head's queries at a time)
+            }
+            if constexpr (AHEAD_K) load_k(head_of(0) / rep, lo + min(it + 1, n - 1) * kKeysT);
+        }
+        if constexpr (do_m) { // talk [heads, heads] . scores [heads, 256 columns]: a wave owns whole columns and writes them back in place
+            constexpr int E = kRowsT / kTileWaves;
+            float *w = lds + b1 + wave * E * kRowPitch + li;
+            f32x4 acc[E][RT];
+#pragma unroll
+            for (int e = 0; e < E; e++)
+#pragma unroll
+                for (int a = 0; a < RT; a++) acc[e][a] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+            for (int c = 0; c < RT; c++) {
+                f32x4 f[RT];
+#pragma unroll
+                for (int a = 0; a < RT; a++) f[a] = *reinterpret_cast<const f32x4 *>(talk + (16 * a + li) * TALK + 16 * c + 4 * lg);
+#pragma unroll
+                for (int t = 0; t < 4; t++)
+#pragma unroll
+                    for (int e = 0; e < E; e++) {
+                        const float y = w[(16 * c + 4 * lg + t) * kHeadPitch + e * kRowPitch];
+#pragma unroll
+                        for (int a = 0; a < RT; a++) acc[e][a] = mfma(f[a][t], y, acc[e][a]);
+                    }
+            }
+#pragma unroll
+            for (int e = 0; e < E; e++)
 #pragma unroll
                 for (int a = 0; a < RT; a++)
 #pragma unroll
-                    for (int r = 0; r < 4; r++) {
-                        w[(16 * a + 4 * lg + r) * kHeadPitch] = acc[a][r]; // (heads that are not there: zero)
-                    }
-            }
+                    for (int r = 0; r < 4; r++) w[(16 * a + 4 * lg + r) * kHeadPitch + e * kRowPitch] = acc[e][a][r];
         }
-        if (do_s) { // scores of this wave's heads (of keys that a row does not see as well)
-#pragma unroll
-            for (int i = 0; i < HPW; i++) {
-                const uint32_t h = h0 + i;
-                if (h >= p.heads) break;
-                if (i > 0 ? !shared : !EARLY_K) load_k(h / rep, js, k);
-                if constexpr (!QREG) load_q<DT>(p, q, b, s0, li, lg, h, qf[0]);
-                const f32x4 a = scores<DT>(qf[QREG ? i : 0], k);
-                float *w = lds + b0 * buffer + h * kHeadPitch + li;
-                const float d = (float)(int)(first_row + 4 * lg - js - li);
-#pragma unroll
-                for (int r = 0; r < 4; r++) w[(4 * lg + r) * kRowPitch] = fmaf(-slope[i], d + (float)r, a[r]);
-            }
-        }
-        if (do_v) { // mixed scores -> weights . values; a lane has four keys of row li
+        if constexpr (do_v) { // mixed scores -> weights . values; a lane has four keys of row li
             const bool whole = jv + kKeysT - 1 <= first_row && (!p.window || last_row - jv < p.window);
+            const int32_t d0 = (int32_t)(first_row + li) - (int32_t)(jv + 4 * lg);
+            bool moves = false;
 #pragma unroll
-            for (int i = 0; i < HPW; i++) {
-                const uint32_t h = h0 + i;
-                if (h >= p.heads) break;
-                if (i > 0 ? !shared : !EARLY_V) load_v(h / rep);
-                f32x4 x = *reinterpret_cast<const f32x4 *>(lds + b2 * buffer + h * kHeadPitch + li * kRowPitch + 4 * lg);
-                bool moves = false;
+            for (int i = 0; i < HPW; i++)
 #pragma unroll
                 for (int t = 0; t < 4; t++) {
-                    const int32_t d = (int32_t)(first_row + li) - (int32_t)(jv + 4 * lg + t);
-                    x[t] = whole || (d >= 0 && (!p.window || (uint32_t)d < p.window)) ? x[t] * kLog2e : -INFINITY;
-                    moves = moves || x[t] - top[i] > kSlack;
+                    x[i][t] = whole || (d0 >= t && (!p.window || (uint32_t)(d0 - t) < p.window)) ? x[i][t] * kLog2e : -INFINITY;
+                    moves = moves || x[i][t] - top[i] > kSlack;
                 }
-                if (__any(moves)) {
-                    float up = fmaxf(fmaxf(x[0], x[1]), fmaxf(x[2], x[3]));
+            if (__any(moves)) {
+#pragma unroll
+                for (int i = 0; i < HPW; i++) {
+                    float up = fmaxf(fmaxf(x[i][0], x[i][1]), fmaxf(x[i][2], x[i][3]));
                     up = fmaxf(up, __shfl_xor(up, 16, 64));
                     up = fmaxf(top[i], fmaxf(up, __shfl_xor(up, 32, 64)));
                     const float f = __builtin_amdgcn_exp2f(top[i] - up);
@@ -335,20 +345,42 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
                         for (int c = 0; c < VT; c++) out[i][c][r] *= fr;
                     }
                 }
+            }
 #pragma unroll
-                for (int t = 0; t < 4; t++) x[t] = __builtin_amdgcn_exp2f(x[t] - top[i]);
-                l[i] += (x[0] + x[1]) + (x[2] + x[3]);
+            for (int i = 0; i < HPW; i++) {
+                if (!SHARED || (!AHEAD_V && i == 0)) load_v(head_of(i) / rep, jv);
+#pragma unroll
+                for (int t = 0; t < 4; t++) x[i][t] = __builtin_amdgcn_exp2f(x[i][t] - top[i]);
+                l[i] += (x[i][0] + x[i][1]) + (x[i][2] + x[i][3]);
 #pragma unroll
                 for (int t = 0; t < 4; t++)
 #pragma unroll
-                    for (int c = 0; c < VT; c++) out[i][c] = mfma(x[t], v[t][c], out[i][c]);
+                    for (int c = 0; c < VT; c++) out[i][c] = mfma(x[i][t], v[t][c], out[i][c]);
+                if constexpr (TIGHT) __builtin_amdgcn_sched_barrier(0);
             }
+            if constexpr (AHEAD_V) load_v(head_of(0) / rep, min(jv + kKeysT, lo + (n - 1) * kKeysT));
         }
-        __syncthreads();
+        // one barrier for what this wave has read and written in LDS; loads from memory stay on their way
+        asm volatile("" ::: "memory");
+        __builtin_amdgcn_s_waitcnt(0xC07F); // lgkmcnt(0)
+        __builtin_amdgcn_s_barrier();
+        asm volatile("" ::: "memory");
         const uint32_t t = b2;
         b2 = b1;
         b1 = b0;
         b0 = t;
+    };
+    if (n) { // (an empty part of the keys: nothing)
+        const std::true_type yes{};
+        const std::false_type no{};
+        if constexpr (AHEAD_K) load_k(head_of(0) / rep, lo);
+        if constexpr (AHEAD_V) load_v(head_of(0) / rep, lo);
+        step(0, yes, no, no);
+        if (n > 1) step(1, yes, yes, no);
+        for (uint32_t it = 2; it < n; it++) step(it, yes, yes, yes);
+        if (n == 1) step(1, no, yes, no);
+        else step(n, no, yes, yes);
+        step(n + 1, no, no, yes);
     }
     const uint64_t rows = (uint64_t)p.B * p.S;
 #pragma unroll
@@ -723,12 +755,19 @@ int mixed_rows(cg_backend *be, const AttentionPlan &p, uint32_t row0, uint32_t r
     return launched("attention_mixed_rows");
 }
 
-template <int HPW, int DT, int VT, bool QREG, bool EXACT = false> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t splits, float *dst, float2 *stats) {
+template <int HPW, int DT, int VT, bool QREG, bool EXACT, bool SHARED>
+int launch_tiles(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t splits, float *dst, float2 *stats) {
     const uint32_t tiles = (p.S + kRowsT - 1) / kRowsT;
     const size_t h16 = (HPW * kTileWaves + 15) / 16 * 16, lds = (3 * h16 * kHeadPitch + h16 * (h16 + 4)) * 4;
-    if (int rc = allow_lds(reinterpret_cast<const void *>(&attention_mixed_tiles_kernel<HPW, DT, VT, QREG, EXACT>), lds)) return rc;
-    hipLaunchKernelGGL((attention_mixed_tiles_kernel<HPW, DT, VT, QREG, EXACT>), dim3(tiles * splits, p.B), dim3(kTileWaves * 64), lds, be->stream, p, q, tiles, splits, dst, stats);
+    if (int rc = allow_lds(reinterpret_cast<const void *>(&attention_mixed_tiles_kernel<HPW, DT, VT, QREG, EXACT, SHARED>), lds)) return rc;
+    hipLaunchKernelGGL((attention_mixed_tiles_kernel<HPW, DT, VT, QREG, EXACT, SHARED>), dim3(tiles * splits, p.B), dim3(kTileWaves * 64), lds, be->stream, p, q, tiles, splits, dst,
+                       stats);
     return CG_OK;
+}
+template <int HPW, int DT, int VT, bool QREG, bool EXACT = false>
+int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t splits, float *dst, float2 *stats) {
+    if (HPW == 1 || p.heads / p.kv_heads % HPW == 0) return launch_tiles<HPW, DT, VT, QREG, EXACT, true>(be, p, q, splits, dst, stats);
+    return launch_tiles<HPW, DT, VT, QREG, EXACT, HPW == 1>(be, p, q, splits, dst, stats);
 }
 template <int HPW> int run_tiles(cg_backend *be, const AttentionPlan &p, const float *q, uint32_t splits, float *dst, float2 *stats) {
     const uint32_t d = p.dim, v = p.vdim;
