@@ -9,8 +9,7 @@
 //                 expert_tile_kernel    products on the matrix instructions: rows gathered through the lists, the activation
 //                                       in the store of the first; 16 / 32 values of k per row and stage by loads straight
 //                                       into a ring of LDS stages, one barrier a stage
-#include "blocks.hpp"
-#include "device_utils.hpp"
+#include "block_stream.hpp"
 
 #include <algorithm>
 
@@ -19,8 +18,6 @@ namespace {
 
 constexpr int kThreads = 256, kWaves = 4;
 
-__device__ __forceinline__ float bf16_lo(uint32_t w) { return asf(w << 16); }
-__device__ __forceinline__ float bf16_hi(uint32_t w) { return asf(w & 0xFFFF0000u); }
 __device__ __forceinline__ uint32_t round_bf16(float v) { return asu(v) + 0x7FFFu + ((asu(v) >> 16) & 1u); } // (bits above 15 hold the pattern)
 __device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float activation(float g, float u, float limit, float slope) {
@@ -86,50 +83,6 @@ __device__ void choose_experts(const ExpertsPlan &p, uint32_t row, float *lds, u
 }
 
 // ---- a few rows ------------------------------------------------------------------------------------------------------
-// sum over k of the row of n values in memory (words or bfloat16 patterns, 16 bytes at a time) with x in LDS or memory
-template <bool BF16, bool VEC> struct Streamed {
-    static constexpr uint32_t W = VEC ? (BF16 ? 8 : 4) : 1;
-    uint4 v;
-    __device__ __forceinline__ void load(const void *row, uint32_t k) {
-        if constexpr (VEC) {
-            typedef uint32_t u4 __attribute__((ext_vector_type(4)));
-            const u4 t = __builtin_nontemporal_load(reinterpret_cast<const u4 *>(static_cast<const char *>(row) + (uint64_t)k * (BF16 ? 2 : 4)));
-            v = make_uint4(t[0], t[1], t[2], t[3]);
-        } else {
-            v.x = BF16 ? (uint32_t)static_cast<const uint16_t *>(row)[k] << 16 : static_cast<const uint32_t *>(row)[k];
-        }
-    }
-    __device__ __forceinline__ float dot(const float (&x)[W], float s) const {
-        if constexpr (!VEC) {
-            return fmaf(asf(v.x), x[0], s);
-        } else if constexpr (BF16) {
-            const uint32_t w[4] = {v.x, v.y, v.z, v.w};
-#pragma unroll
-            for (int i = 0; i < 4; i++) {
-                s = fmaf(bf16_lo(w[i]), x[2 * i], s);
-                s = fmaf(bf16_hi(w[i]), x[2 * i + 1], s);
-            }
-            return s;
-        } else {
-            s = fmaf(asf(v.x), x[0], s);
-            s = fmaf(asf(v.y), x[1], s);
-            s = fmaf(asf(v.z), x[2], s);
-            return fmaf(asf(v.w), x[3], s);
-        }
-    }
-    static __device__ __forceinline__ void input(const float *x, uint64_t k, float (&o)[W]) {
-        if constexpr (VEC) {
-#pragma unroll
-            for (uint32_t i = 0; i < W; i += 4) {
-                const float4 t = *reinterpret_cast<const float4 *>(x + k + i);
-                o[i] = t.x, o[i + 1] = t.y, o[i + 2] = t.z, o[i + 3] = t.w;
-            }
-        } else {
-            o[0] = x[k];
-        }
-    }
-};
-
 // blockIdx.x: columns (four waves, one after the other), blockIdx.y: row * top + choice
 template <bool BF16, bool VEC, int STEPS>
 __global__ __launch_bounds__(kThreads) void expert_first_kernel(const ExpertsPlan p, const uint32_t per_wave, float *__restrict__ hidden, uint32_t *__restrict__ chosen_out) {

@@ -1,7 +1,6 @@
 // What stands around a decoder layer's products: embeddings of tokens and token pairs, grouped norms with short filters over
 // time, and the vectors that tokens add to their rows.
-#include "blocks.hpp"
-#include "device_utils.hpp"
+#include "block_stream.hpp"
 
 #include <algorithm>
 
@@ -54,7 +53,10 @@ template <int VW, int TAPS> __global__ __launch_bounds__(kThreads) void conv_row
     };
     // this thread's columns, its share of the filters asked for first
     const uint32_t per = ((size + parts - 1) / parts + VW - 1) / VW * VW, c_end = g0 + min(size, (part + 1) * per);
-    uint32_t c = g0 + part * per + threadIdx.x * VW;
+    // few columns: the workgroup's waves take parts of the run
+    const uint32_t across = min(kThreads, ((per + VW - 1) / VW + 63) / 64 * 64), subs = kThreads / across, sub = threadIdx.x / across;
+    const uint32_t sub_run = (n + subs - 1) / subs, i_first = min(n, sub * sub_run), i_end = min(n, i_first + sub_run);
+    const uint32_t c_first = g0 + part * per + (threadIdx.x - sub * across) * VW;
     float gamma[2][VW], w[2][TAPS][VW]; // tap t counts from the present back
     auto ask_filters = [&](uint32_t at) {
         at = min(at, p.width - VW);
@@ -74,7 +76,7 @@ template <int VW, int TAPS> __global__ __launch_bounds__(kThreads) void conv_row
             }
         }
     };
-    ask_filters(c);
+    ask_filters(c_first);
     constexpr int ROWS = 4; // of a wave at a time
     for (uint32_t i0 = wave; i0 < n + past; i0 += kWaves * ROWS) {
         float m[ROWS] = {};
@@ -98,8 +100,9 @@ template <int VW, int TAPS> __global__ __launch_bounds__(kThreads) void conv_row
         }
     }
     __syncthreads();
-    for (; c < c_end; c += kThreads * VW) {
-        if (c >= g0 + part * per + kThreads * VW) ask_filters(c);
+    if (sub >= subs || i_first == i_end) return;
+    for (uint32_t c = c_first; c < c_end; c += across * VW) {
+        if (c != c_first) ask_filters(c);
         // z of token s0 - past + i, for the tokens in front of the sequence's new ones from its state
         auto unit = [&](uint32_t i, float(&v)[VW]) {
             const int32_t s = (int32_t)(s0 + i) - (int32_t)past;
@@ -130,18 +133,19 @@ template <int VW, int TAPS> __global__ __launch_bounds__(kThreads) void conv_row
 #pragma unroll
         for (int t = TAPS - 1; t >= 1; t--)
             if (t <= (int)past) {
-                unit(past - t, z[t - 1]); // (moved one back below)
-                if (s0 + n == p.S && (int32_t)s0 - t < 0) keep((int32_t)s0 - t, z[t - 1]);
+                const int32_t s = (int32_t)(s0 + i_first) - t;
+                unit(past + i_first - t, z[t - 1]); // (moved one back below)
+                if (s0 + i_end == p.S && s < 0) keep(s, z[t - 1]);
             }
         constexpr int AHEAD = 4; // rows asked for together
-        for (uint32_t i0 = 0; i0 < n; i0 += AHEAD) {
+        for (uint32_t i0 = i_first; i0 < i_end; i0 += AHEAD) {
             float next[AHEAD][VW];
 #pragma unroll
-            for (int e = 0; e < AHEAD; e++) unit(past + min(i0 + e, n - 1), next[e]);
+            for (int e = 0; e < AHEAD; e++) unit(past + min(i0 + e, i_end - 1), next[e]);
 #pragma unroll
             for (int e = 0; e < AHEAD; e++) {
                 const uint32_t s = s0 + i0 + e;
-                if (i0 + e >= n) break;
+                if (i0 + e >= i_end) break;
 #pragma unroll
                 for (int t = TAPS - 1; t >= 1; t--)
 #pragma unroll
@@ -200,6 +204,78 @@ __global__ __launch_bounds__(kThreads) void side_gate_kernel(float *__restrict__
         id = 0;
     }
     g[i] = gelu(g[i]) * element(table, (int64_t)id * table.pitch + first + k);
+}
+
+// The same for a few rows with the product in front: a wave per (row, value).
+template <bool BF16, bool VEC>
+__global__ __launch_bounds__(kThreads) void side_first_kernel(const Rows x, const Weight w, const Tokens ids, const Table table, const uint32_t vocab, const uint32_t first,
+                                                              float *__restrict__ g, uint32_t *fault) {
+    typedef Streamed<BF16, VEC> St;
+    constexpr uint32_t W = St::W, SPAN = 64 * W, EB = BF16 ? 2 : 4;
+    const uint32_t lane = threadIdx.x & 63, i = blockIdx.x * kWaves + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), r = blockIdx.y;
+    if (i >= w.n) return;
+    uint32_t id = token_at(ids, r);
+    if (id >= vocab) {
+        *fault = kFaultIndexRange;
+        id = 0;
+    }
+    const float e = element(table, (int64_t)id * table.pitch + first + i);
+    const char *row = static_cast<const char *>(w.p) + (int64_t)i * w.pitch * EB;
+    const float *xr = x.p + (int64_t)r * x.pitch;
+    float a = 0.0f;
+#pragma unroll 4
+    for (uint32_t k = lane * W; k < w.k; k += SPAN) {
+        St s;
+        s.load(row, k);
+        float v[W];
+        St::input(xr, k, v);
+        a = s.dot(v, a);
+    }
+    a = wave_total(a);
+    if (lane == 0) g[(int64_t)r * w.n + i] = gelu(a) * e;
+}
+
+// The rest for a few rows in one launch, a workgroup per row: LANES lanes share a row of w (all of it in 16-byte pieces), its
+// product with g ends in the last of them, and stays there until the row's mean square is known.  WORK: rows of w per LANES lanes.
+constexpr int kSideThreads = 1024;
+template <bool BF16, int LANES, int WORK>
+__global__ __launch_bounds__(kSideThreads) void side_second_kernel(const Rows x, const float *__restrict__ g, const Weight w, const float *__restrict__ norm, const float eps,
+                                                                   const float scale, float *__restrict__ out) {
+    typedef Streamed<BF16, true> St;
+    constexpr uint32_t W = St::W, EB = BF16 ? 2 : 4, PER = kSideThreads / LANES;
+    __shared__ float red[kSideThreads / 64];
+    const uint32_t sub = threadIdx.x % LANES, n0 = threadIdx.x / LANES, k = min(sub * W, w.k - W);
+    const int64_t r = blockIdx.x;
+    St s[WORK];
+#pragma unroll
+    for (int i = 0; i < WORK; i++) s[i].load(static_cast<const char *>(w.p) + (int64_t)min(n0 + i * PER, w.n - 1) * w.pitch * EB, k);
+    float v[W], y[WORK], m = 0.0f;
+    St::input(g + r * w.k, k, v);
+#pragma unroll
+    for (uint32_t j = 0; j < W; j++) v[j] = sub * W < w.k ? v[j] : 0.0f;
+#pragma unroll
+    for (int i = 0; i < WORK; i++) {
+        float a = s[i].dot(v, 0.0f);
+        if (LANES >= 2) a = add_shifted<0x111, 0xF>(a);
+        if (LANES >= 4) a = add_shifted<0x112, 0xF>(a);
+        if (LANES >= 8) a = add_shifted<0x114, 0xF>(a);
+        if (LANES >= 16) a = add_shifted<0x118, 0xF>(a);
+        y[i] = a;
+        if (sub == LANES - 1 && n0 + i * PER < w.n) m = fmaf(a, a, m);
+    }
+    m = wave_total(m);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = m;
+    __syncthreads();
+    m = 0.0f;
+#pragma unroll
+    for (int i = 0; i < kSideThreads / 64; i++) m += red[i];
+    const float f = scale / sqrtf(m / (float)w.n + eps);
+    if (sub != LANES - 1) return;
+#pragma unroll
+    for (int i = 0; i < WORK; i++) {
+        const uint32_t n = n0 + i * PER;
+        if (n < w.n) out[r * w.n + n] = fmaf(y[i] * f, norm[n], x.p[r * x.pitch + n]);
+    }
 }
 
 // out = x + scale * y / sqrt(mean(y^2) + eps) * norm; a workgroup per row
@@ -293,6 +369,48 @@ int launch_side_gate(cg_backend *be, float *g, const Tokens &ids, const Table &t
     hipLaunchKernelGGL(side_gate_kernel, dim3((uint32_t)((n + kThreads - 1) / kThreads)), dim3(kThreads), 0, be->stream, g, ids, table, vocab, first, dim, rows,
                        be->fault_dev);
     return launched("side_gate");
+}
+
+int launch_side_first(cg_backend *be, const Rows &x, uint32_t rows, const Weight &w, const Tokens &ids, const Table &table, uint32_t vocab, uint32_t first, float *g) {
+    const bool bf16 = w.fmt == kFmtBF16;
+    const uint32_t vw = bf16 ? 8 : 4;
+    const bool vec = w.k % vw == 0 && w.pitch % vw == 0 && aligned16(w.p) && x.pitch % 4 == 0 && aligned16(x.p);
+    ProfScope prof(be, CG_K_GEMM_SKINNY, (double)w.n * w.k * (bf16 ? 2.0 : 4.0) + 4.0 * rows * ((double)w.k + w.n));
+    const dim3 grid((w.n + kWaves - 1) / kWaves, rows);
+#define CG_FIRST(BF, VE) hipLaunchKernelGGL((side_first_kernel<BF, VE>), grid, dim3(kThreads), 0, be->stream, x, w, ids, table, vocab, first, g, be->fault_dev)
+    if (bf16 && vec) CG_FIRST(true, true);
+    else if (bf16) CG_FIRST(true, false);
+    else if (vec) CG_FIRST(false, true);
+    else CG_FIRST(false, false);
+#undef CG_FIRST
+    return launched("side_first");
+}
+
+template <bool BF16, int LANES> static int side_second(cg_backend *be, const Rows &x, const float *g, uint32_t rows, const Weight &w, const float *norm, float eps, float scale, float *out) {
+    const uint32_t work = (w.n + kSideThreads / LANES - 1) / (kSideThreads / LANES);
+#define CG_SECOND(WK) hipLaunchKernelGGL((side_second_kernel<BF16, LANES, WK>), dim3(rows), dim3(kSideThreads), 0, be->stream, x, g, w, norm, eps, scale, out)
+    if (work <= 4) CG_SECOND(4);
+    else if (work <= 8) CG_SECOND(8);
+    else if (work <= 16) CG_SECOND(16);
+    else return kDeclined;
+#undef CG_SECOND
+    return launched("side_second");
+}
+
+constexpr uint64_t kSideBytes = 64 << 10; // of a matrix that one compute unit reads sooner than two launches pass
+
+int launch_side_second(cg_backend *be, const Rows &x, const float *g, uint32_t rows, const Weight &w, const float *norm, float eps, float scale, float *out) {
+    const bool bf16 = w.fmt == kFmtBF16;
+    const uint32_t vw = bf16 ? 8 : 4, pieces = (w.k + vw - 1) / vw;
+    if (w.k % vw || w.pitch % vw || !aligned16(w.p) || !aligned16(g) || pieces > 16 || (uint64_t)w.n * w.k * (bf16 ? 2 : 4) > kSideBytes) return kDeclined;
+    ProfScope prof(be, CG_K_GEMM_SKINNY, (double)w.n * w.k * (bf16 ? 2.0 : 4.0) + 4.0 * rows * ((double)w.k + 2.0 * w.n));
+#define CG_SIDE(L) return bf16 ? side_second<true, L>(be, x, g, rows, w, norm, eps, scale, out) : side_second<false, L>(be, x, g, rows, w, norm, eps, scale, out)
+    if (pieces <= 1) CG_SIDE(1);
+    if (pieces <= 2) CG_SIDE(2);
+    if (pieces <= 4) CG_SIDE(4);
+    if (pieces <= 8) CG_SIDE(8);
+    CG_SIDE(16);
+#undef CG_SIDE
 }
 
 int launch_side_sum(cg_backend *be, const Rows &x, const float *y, const float *norm, uint32_t rows, uint32_t width, float eps, float scale, float *out) {

@@ -318,13 +318,13 @@ __device__ __forceinline__ float blocks_sum(float v) {
 
 // A workgroup holds all of its waves' activations in registers (STEPS of 64 lanes' worth each) and walks column groups.
 template <bool BF16, int STEPS, int WAVES>
-__global__ __launch_bounds__(WAVES * 64) void four_rows_linear_kernel(const ProductInput in, const uint32_t rows, const Weight w, const uint32_t iters,
-                                                                      const float *__restrict__ bias, const float scale, float *__restrict__ out) {
+__device__ __forceinline__ void four_rows_linear(const ProductInput &in, const uint32_t rows, const Weight &w, const uint32_t block, const uint32_t iters,
+                                                 const float *__restrict__ bias, const float scale, float *__restrict__ out) {
     constexpr uint32_t W = Frag<BF16>::W, SPAN = 16 * W;
     __shared__ f32x4 sums[2][WAVES][4];
     __shared__ float squares[WAVES][4];
     const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, j = lane & 3, k0 = wave * SPAN + (lane >> 2) * W;
-    const uint32_t g0 = blockIdx.x * iters, groups = (w.n + 3) / 4, g1 = min(g0 + iters, groups);
+    const uint32_t g0 = block * iters, groups = (w.n + 3) / 4, g1 = min(g0 + iters, groups);
     Frag<BF16> wt[STEPS];
     auto ask = [&](uint32_t g) {
         const uint32_t n = min(g * 4 + j, w.n - 1);
@@ -377,6 +377,24 @@ __global__ __launch_bounds__(WAVES * 64) void four_rows_linear_kernel(const Prod
             if (m < rows && n < w.n) out[(int64_t)m * w.n + n] = s * rstd + (bias ? bias[n] : 0.0f);
         }
     }
+}
+
+template <bool BF16, int STEPS, int WAVES>
+__global__ __launch_bounds__(WAVES * 64) void four_rows_linear_kernel(const ProductInput in, const uint32_t rows, const Weight w, const uint32_t iters,
+                                                                      const float *__restrict__ bias, const float scale, float *__restrict__ out) {
+    four_rows_linear<BF16, STEPS, WAVES>(in, rows, w, blockIdx.x, iters, bias, scale, out);
+}
+// two products, the first on the first blocks0 workgroups
+struct FourRowsJob {
+    ProductInput in;
+    Weight w;
+    float *out;
+    uint32_t iters;
+};
+template <bool BF16, int STEPS, int WAVES>
+__global__ __launch_bounds__(WAVES * 64) void four_rows_linear2_kernel(const FourRowsJob j0, const FourRowsJob j1, const uint32_t blocks0, const uint32_t rows) {
+    if (blockIdx.x < blocks0) four_rows_linear<BF16, STEPS, WAVES>(j0.in, rows, j0.w, blockIdx.x, j0.iters, nullptr, 1.0f, j0.out);
+    else four_rows_linear<BF16, STEPS, WAVES>(j1.in, rows, j1.w, blockIdx.x - blocks0, j1.iters, nullptr, 1.0f, j1.out);
 }
 
 // One branch of the residual sum: the sums of the polynomial's terms (or the plain sum) and the row sums they are scaled by.
@@ -708,12 +726,16 @@ static bool four_rows(const ProductInput &in, uint32_t rows, const Weight &w) {
            (!in.x2.p || (in.x2.pitch % 4 == 0 && aligned16(in.x2.p)));
 }
 
+static uint32_t column_groups(cg_backend *be, const Weight &w, uint32_t *iters) { // workgroups, which walk several groups when there are many
+    const uint32_t groups = (w.n + 3) / 4, resident = (uint32_t)be->compute_units * 8;
+    *iters = std::max(1u, (groups + resident - 1) / resident);
+    return (groups + *iters - 1) / *iters;
+}
 template <bool BF16, int STEPS, int WAVES>
-static void four_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows, const Weight &w, const float *bias, float scale, float *out) {
-    const uint32_t groups = (w.n + 3) / 4, resident = (uint32_t)be->compute_units * 8; // workgroups that walk several groups when there are many
-    const uint32_t iters = std::max(1u, (groups + resident - 1) / resident);
-    hipLaunchKernelGGL((four_rows_linear_kernel<BF16, STEPS, WAVES>), dim3((groups + iters - 1) / iters), dim3(WAVES * 64), 0, be->stream, in, rows, w, iters,
-                       bias, scale, out);
+static void launch_four_rows(cg_backend *be, const ProductInput &in, uint32_t rows, const Weight &w, const float *bias, float scale, float *out) {
+    uint32_t iters;
+    const uint32_t blocks = column_groups(be, w, &iters);
+    hipLaunchKernelGGL((four_rows_linear_kernel<BF16, STEPS, WAVES>), dim3(blocks), dim3(WAVES * 64), 0, be->stream, in, rows, w, iters, bias, scale, out);
 }
 
 int launch_few_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows, const Weight &w, const float *bias, float scale, float *out) {
@@ -722,11 +744,11 @@ int launch_few_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows
         ProfScope prof(be, CG_K_GEMM_SKINNY, (double)w.n * w.k * (bf16 ? 2.0 : 4.0) + 4.0 * rows * ((double)in.k + w.n));
         const uint32_t steps = (in.k + (bf16 ? 511 : 255)) / (bf16 ? 512 : 256); // of a workgroup of four waves
 #define CG_FOUR(BF)                                                                              \
-    if (steps <= 1) four_rows_linear<BF, 1, 4>(be, in, rows, w, bias, scale, out);               \
-    else if (steps <= 2) four_rows_linear<BF, 2, 4>(be, in, rows, w, bias, scale, out);          \
-    else if (steps <= 4) four_rows_linear<BF, 4, 4>(be, in, rows, w, bias, scale, out);          \
-    else if (steps <= 8) four_rows_linear<BF, 4, 8>(be, in, rows, w, bias, scale, out);          \
-    else four_rows_linear<BF, 8, 8>(be, in, rows, w, bias, scale, out)
+    if (steps <= 1) launch_four_rows<BF, 1, 4>(be, in, rows, w, bias, scale, out);               \
+    else if (steps <= 2) launch_four_rows<BF, 2, 4>(be, in, rows, w, bias, scale, out);          \
+    else if (steps <= 4) launch_four_rows<BF, 4, 4>(be, in, rows, w, bias, scale, out);          \
+    else if (steps <= 8) launch_four_rows<BF, 4, 8>(be, in, rows, w, bias, scale, out);          \
+    else launch_four_rows<BF, 8, 8>(be, in, rows, w, bias, scale, out)
         if (bf16) { CG_FOUR(true); }
         else { CG_FOUR(false); }
 #undef CG_FOUR
@@ -755,6 +777,34 @@ int launch_few_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows
 #undef CG_LIN_NC
 #undef CG_LIN
     return rc ? rc : launched("few_rows_linear");
+}
+
+template <bool BF16, int STEPS, int WAVES> static void launch_four_rows2(cg_backend *be, FourRowsJob (&j)[2], uint32_t rows) {
+    const uint32_t b0 = column_groups(be, j[0].w, &j[0].iters), b1 = column_groups(be, j[1].w, &j[1].iters);
+    hipLaunchKernelGGL((four_rows_linear2_kernel<BF16, STEPS, WAVES>), dim3(b0 + b1), dim3(WAVES * 64), 0, be->stream, j[0], j[1], b0, rows);
+}
+
+int launch_few_rows_linear2(cg_backend *be, const ProductInput (&in)[2], uint32_t rows, const Weight (&w)[2], float *const (&out)[2]) {
+    const bool bf16 = w[0].fmt == kFmtBF16;
+    FourRowsJob j[2];
+    double bytes = 0.0;
+    for (int i = 0; i < 2; i++) {
+        if (!four_rows(in[i], rows, w[i]) || in[i].gamma || in[i].poly || w[i].fmt != w[0].fmt || in[i].k != in[0].k || in[i].k > (bf16 ? 8192u : 4096u)) return kDeclined;
+        j[i] = {in[i], w[i], out[i], 1};
+        bytes += (double)w[i].n * w[i].k * (bf16 ? 2.0 : 4.0) + 4.0 * rows * ((double)in[i].k + w[i].n);
+    }
+    ProfScope prof(be, CG_K_GEMM_SKINNY, bytes);
+    const uint32_t steps = (in[0].k + (bf16 ? 511 : 255)) / (bf16 ? 512 : 256); // of a workgroup of four waves
+#define CG_FOUR(BF)                                                  \
+    if (steps <= 1) launch_four_rows2<BF, 1, 4>(be, j, rows);        \
+    else if (steps <= 2) launch_four_rows2<BF, 2, 4>(be, j, rows);   \
+    else if (steps <= 4) launch_four_rows2<BF, 4, 4>(be, j, rows);   \
+    else if (steps <= 8) launch_four_rows2<BF, 4, 8>(be, j, rows);   \
+    else launch_four_rows2<BF, 8, 8>(be, j, rows)
+    if (bf16) { CG_FOUR(true); }
+    else { CG_FOUR(false); }
+#undef CG_FOUR
+    return launched("four_rows_linear2");
 }
 
 template <bool BF16, int NG> static bool four_rows_residual(cg_backend *be, const Rows &x, const ResidualBranch *br, int n, uint32_t rows, uint32_t width, float *out) {

@@ -577,20 +577,19 @@ int cg_block_conv_linear(cg_backend *b, const cg_conv_linear_args *a, cg_tensor 
         p.state_out = so->buf ? static_cast<float *>(so->buf->ptr) : nullptr;
         rc = launch_conv_rows(b, p);
     }
+    ProductInput pi[2];
     for (size_t i = 0; i < a->n && !rc; i++) {
         const int64_t yd[3] = {B, S, in[i].w.n};
         rc = new_dense(b, CG_F32, yd, 3, &o[i]);
-        if (rc) break;
-        float *dst = static_cast<float *>(o[i]->buf->ptr);
-        if (few) {
-            ProductInput pi;
-            pi.x = {static_cast<const float *>(in[i].x->buf->ptr), W};
-            pi.k1 = pi.k = (uint32_t)W;
-            rc = launch_few_rows_linear(b, pi, (uint32_t)rows, in[i].w, nullptr, 1.0f, dst);
-        } else {
-            rc = operand_product(b, in[i].x, in[i].tiles, in[i].w, in[i].wv, dst);
-        }
+        pi[i].x = {static_cast<const float *>(in[i].x->buf->ptr), W};
+        pi[i].k1 = pi[i].k = (uint32_t)W;
     }
+    auto dst = [&](size_t i) { return static_cast<float *>(o[i]->buf->ptr); };
+    int both = kDeclined;
+    if (!rc && few && a->n == 2) both = launch_few_rows_linear2(b, pi, (uint32_t)rows, {in[0].w, in[1].w}, {dst(0), dst(1)});
+    if (both != kDeclined) rc = both;
+    for (size_t i = 0; i < a->n && !rc && both == kDeclined; i++)
+        rc = few ? launch_few_rows_linear(b, pi[i], (uint32_t)rows, in[i].w, nullptr, 1.0f, dst(i)) : operand_product(b, in[i].x, in[i].tiles, in[i].w, in[i].wv, dst(i));
     if (rc) {
         release(so);
         release(o[0]);
@@ -653,10 +652,16 @@ int cg_block_token_side(cg_backend *b, const cg_token_side_args *a, cg_tensor **
         if (few_rows_slots((uint64_t)rows, (uint64_t)staged_pitch(w.k) * 4)) return launch_few_rows_linear(b, p, (uint32_t)rows, w, nullptr, 1.0f, static_cast<float *>(dst));
         return general_product(b, h, p, (uint32_t)rows, w, wv, static_cast<float *>(dst));
     };
-    if (!rc) rc = product(x, gate, gv, g);
-    if (!rc) rc = launch_side_gate(b, static_cast<float *>(g), ids, table, (uint32_t)vocab, (uint32_t)a->first, (uint32_t)dim, (uint32_t)rows);
-    if (!rc) rc = product({static_cast<const float *>(g), dim}, proj, pv, y);
-    if (!rc) rc = launch_side_sum(b, x, static_cast<const float *>(y), norm, (uint32_t)rows, (uint32_t)W, a->eps, a->scale, static_cast<float *>(o->buf->ptr));
+    const bool few = rows <= kFewRows;
+    if (!rc && few) rc = launch_side_first(b, x, (uint32_t)rows, gate, ids, table, (uint32_t)vocab, (uint32_t)a->first, static_cast<float *>(g));
+    if (!rc && !few) rc = product(x, gate, gv, g);
+    if (!rc && !few) rc = launch_side_gate(b, static_cast<float *>(g), ids, table, (uint32_t)vocab, (uint32_t)a->first, (uint32_t)dim, (uint32_t)rows);
+    int second = kDeclined;
+    if (!rc && few)
+        second = launch_side_second(b, x, static_cast<const float *>(g), (uint32_t)rows, proj, norm, a->eps, a->scale, static_cast<float *>(o->buf->ptr));
+    if (second != kDeclined) rc = second;
+    if (!rc && second == kDeclined) rc = product({static_cast<const float *>(g), dim}, proj, pv, y);
+    if (!rc && second == kDeclined) rc = launch_side_sum(b, x, static_cast<const float *>(y), norm, (uint32_t)rows, (uint32_t)W, a->eps, a->scale, static_cast<float *>(o->buf->ptr));
     if (rc) {
         release(o);
         return rc;

@@ -40,6 +40,8 @@ inline uint32_t staged_pitch(uint32_t k) { return (k + 7) / 8 * 8; } // floats o
 
 // out[r, n] = scale * in[r, :] . w[n, :] + bias[n], rows <= kFewRows
 int launch_few_rows_linear(cg_backend *be, const ProductInput &in, uint32_t rows, const Weight &w, const float *bias, float scale, float *out);
+// Two such products of operands of the same width without norms or biases in one launch; kDeclined: not at once.
+int launch_few_rows_linear2(cg_backend *be, const ProductInput (&in)[2], uint32_t rows, const Weight (&w)[2], float *const (&out)[2]);
 // out[r, n] = x[r, n] + sum_i sigmoid(gate_i[r, n] + gate_bias_i[n]) * (in_i[r, :] . w_i[n, :]), rows <= kFewRows
 struct ResidualBranch {
     ProductInput in;
@@ -110,6 +112,9 @@ struct ConvRowsPlan {
 int launch_conv_rows(cg_backend *be, ConvRowsPlan p);
 
 int launch_side_gate(cg_backend *be, float *g, const Tokens &ids, const Table &table, uint32_t vocab, uint32_t first, uint32_t dim, uint32_t rows);
+// A few rows: g[r] = gelu(x[r] . w^T) * the rows' vectors; then out = x + scale * norm(g . w^T) (kDeclined: sizes it does not take).
+int launch_side_first(cg_backend *be, const Rows &x, uint32_t rows, const Weight &w, const Tokens &ids, const Table &table, uint32_t vocab, uint32_t first, float *g);
+int launch_side_second(cg_backend *be, const Rows &x, const float *g, uint32_t rows, const Weight &w, const float *norm, float eps, float scale, float *out);
 int launch_side_sum(cg_backend *be, const Rows &x, const float *y, const float *norm, uint32_t rows, uint32_t width, float eps, float scale, float *out);
 
 // ---- mixtures of experts ---------------------------------------------------------------------------------------------
