@@ -287,7 +287,7 @@ __global__ __launch_bounds__(kThreads) void route_lists_kernel(const uint32_t ex
     }
 }
 
-constexpr uint32_t kTileN = 128, kStages = 4, kXcds = 8, kGroupM = 8;
+constexpr uint32_t kTileN = 128, kStages = 4;
 typedef float float16v __attribute__((ext_vector_type(16)));
 typedef float float4v __attribute__((ext_vector_type(4)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -315,11 +315,8 @@ template <bool BF16, bool FIRST, int MT> __global__ __launch_bounds__(kThreads) 
     extern __shared__ float lds_dyn[];
     typedef __attribute__((address_space(3))) char lds_char;
     lds_char *const lds = (lds_char *)lds_dyn;
-    // a run of tiles per XCD, down a column of kGroupM row tiles (mostly one expert's) first
-    const uint32_t ntiles = gridDim.x, xcd = blockIdx.x % kXcds, q8 = ntiles / kXcds, r8 = ntiles % kXcds, tiles_m = ntiles / a.tiles_n;
-    const uint32_t lin = xcd * q8 + min(xcd, r8) + blockIdx.x / kXcds, group = lin / (kGroupM * a.tiles_n), in_group = lin % (kGroupM * a.tiles_n);
-    const uint32_t gsize = min(tiles_m - group * kGroupM, kGroupM);
-    const uint32_t tile = group * kGroupM + in_group % gsize, n0 = in_group / gsize * OUT_N;
+    // (tiles in order: the empty ones at the end cost every XCD the same, and an XCD's tiles share two columns of weights)
+    const uint32_t tile = blockIdx.x / a.tiles_n, n0 = (blockIdx.x - tile * a.tiles_n) * OUT_N;
     const uint4 job = a.tiles[tile];
     const uint32_t m = job.z, nk = (a.K + STAGE_K - 1) / STAGE_K;
     if (m == 0) return;
