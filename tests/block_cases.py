@@ -451,7 +451,7 @@ def run_grouped_linear(be, rows, K, groups, n, dt):
 EXPERTS = [  # rows, width, experts, top, groups, keep, ff, K of the branch (0: none), dtype
     (1, 32, 8, 2, 2, 1, 24, 40, "f32"), (1, 32, 8, 3, 4, 2, 24, 40, "bf16"), (4, 64, 16, 4, 4, 2, 48, 64, "f32"), (8, 520, 12, 3, 3, 2, 136, 264, "bf16"),
     (3, 30, 6, 2, 2, 1, 10, 14, "f32"), (3, 30, 6, 2, 2, 1, 10, 14, "bf16"), (1, 1024, 32, 8, 4, 2, 384, 1024, "bf16"), (4, 2048, 32, 8, 4, 2, 256, 512, "bf16"),
-    (9, 32, 8, 2, 2, 1, 24, 40, "f32"), (40, 64, 16, 4, 4, 2, 48, 64, "f32"), (300, 128, 16, 4, 2, 1, 96, 128, "bf16"), (300, 128, 16, 4, 2, 1, 96, 128, "f32"),
+    (9, 32, 8, 2, 2, 1, 24, 40, "f32"), (40, 64, 16, 4, 4, 2, 48, 64, "f32"), (300, 128, 14, 3, 2, 1, 88, 128, "bf16"), (300, 128, 14, 3, 2, 1, 88, 128, "f32"),
     (70, 30, 6, 2, 2, 1, 10, 14, "f32"), (70, 30, 6, 2, 2, 1, 10, 14, "bf16"), (33, 64, 5, 5, 1, 1, 40, 0, "f32"), (2, 64, 5, 5, 1, 1, 40, 0, "f32"),
     (100, 64, 4, 1, 4, 1, 32, 48, "bf16"), (1, 64, 4, 1, 4, 1, 32, 48, "f32"), (2, 64, 4, 2, 4, 2, 32, 48, "f32"), (1, 64, 1, 1, 1, 1, 32, 48, "f32"),
     (50, 64, 1, 1, 1, 1, 32, 48, "f32"), (50, 72, 200, 6, 8, 3, 24, 48, "f32"), (2, 72, 200, 6, 8, 3, 24, 48, "f32"), (1100, 256, 8, 2, 2, 2, 200, 64, "bf16"),

@@ -23,7 +23,7 @@ CONFIGS = {
     "attention_only": config_of([attention_layer(8, 2, 16, 16, None, rot=16), attention_layer(2, 1, 32, 8, None, rot=0)], 64, 32),
     "single_members": config_of([attention_layer(4, 2, 16, 16, experts(4, 2, 24, groups=4, keep=3), rot=8)] * 2, 41, 32, groups=8),
     "all_experts": config_of([attention_layer(4, 2, 16, 16, experts(4, 4, 24, groups=2, keep=2), rot=8)], 41, 32, taps=8),
-    "wider": config_of([attention_layer(8, 4, 32, 40, experts(16, 4, 96, groups=4, keep=2, limit=7.0), rot=16, base=1e5)] * 2, 300, 192,
+    "wider": config_of([attention_layer(10, 5, 32, 40, experts(12, 3, 88, groups=4, keep=2, limit=7.0), rot=16, base=1e5)] * 2, 300, 160,
                        loop={"start": 0, "stop": 2, "times": 2}, side=32, buckets=251, mul_prev=101, mul_cur=13),
 }
 
