@@ -1,8 +1,10 @@
 // Causal attention of new tokens behind a cache, with a window, a distance bias, a query temperature, norms over whole
-// projections and head mixing after the soft-max (cg_block_attention).
+// projections, rotations, unit heads, a sink, and head mixing after the soft-max or before it (cg_block_attention; the latter's
+// kernels are in block_attention_mixed.hip).
 //
 //   attention_prepare_kernel  more than a few new tokens, a workgroup per token: the query row normed and scaled, the key and
 //                             value rows into the cache (then block_attention_tiles.hip, for the sizes it takes)
+//   attention_turn_*_kernel   the same with rotations and unit heads
 //   attention_scores_kernel   a workgroup per (token, kv head, 128 keys): scores, and their maximum and sum per head; with a
 //                             few new tokens the preparation as well
 //   attention_mix_kernel      the same split: soft-max weights of every head, mixed, times the values of the kv head

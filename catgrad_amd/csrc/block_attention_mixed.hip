@@ -179,7 +179,7 @@ constexpr float kSlack = 24.0f;                           // a row's `top` moves
 
 __device__ __forceinline__ f32x4 mfma(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
-// Workgroup ids go to the eight XCDs in turn: the last rows, which see the most keys, go first.
+// Queries of 16 rows, zero beyond a row's end.
 template <int DT> __device__ __forceinline__ void load_q(const AttentionPlan &p, const float *q, uint32_t b, uint32_t s0, uint32_t li, uint32_t lg, uint32_t h, f32x4 (&f)[DT]) {
     const uint32_t s = min(s0 + li, p.S - 1);
     const float *row = q + (((int64_t)b * p.S + s) * p.heads + h) * p.dim;
@@ -217,7 +217,7 @@ __global__ __launch_bounds__(kTileWaves * 64) void attention_mixed_tiles_kernel(
     // (where registers are short keys or values are asked for when they are needed)
     constexpr bool TIGHT = HPW * VT + (QREG ? HPW * DT : DT) + DT + VT > 40, AHEAD_K = SHARED && QREG, AHEAD_V = SHARED && !TIGHT;
     const uint32_t wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, li = lane & 15, lg = lane >> 4;
-    const uint32_t tile = tiles - 1 - blockIdx.x / splits, split = blockIdx.x % splits, b = blockIdx.y, s0 = tile * kRowsT;
+    const uint32_t tile = tiles - 1 - blockIdx.x / splits /* the last rows see the most keys: first */, split = blockIdx.x % splits, b = blockIdx.y, s0 = tile * kRowsT;
     const uint32_t h0 = wave * HPW, rep = p.heads / p.kv_heads;
     const uint32_t first_row = p.cached + s0, last_row = p.cached + min(s0 + kRowsT, p.S) - 1, last = p.cached + p.S - 1;
     uint32_t lo = first_visible(p, first_row);
